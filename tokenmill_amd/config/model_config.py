@@ -603,6 +603,141 @@ class LuzevikConfig:
                     raise ConfigError(f"layers[{i}]: {mlp['top']} of {mlp['experts']} experts")
 
 
+@dataclass(frozen=True)
+class KasovikLayer:
+    type: str                       # "retention" | "parallel"
+    mixer: dict                     # the mixer's sizes and constants, as config.json gives them
+    mlp: dict | None                # {"ff", "limit"} | None
+    weights_of: int | None = None   # the layer (with tensors of its own) whose tensors this one uses
+
+
+@dataclass
+class KasovikConfig:
+    """The Kasovik decoder: token embedding times a constant plus a row per pair of neighbouring tokens; layers with one norm
+    whose result both the mixer and the feed-forward read; a mixer that is either a retention (fixed decays, rotated queries and
+    keys) or two mixers side by side, window attention with a sink whose values are its keys and a gated delta rule with a decay
+    per key channel, added with constant weights; a dense feed-forward with a clamped gate and biases, or none; layers that use
+    an earlier layer's tensors; the output head is the embedding table. Every size and constant that can differ between two
+    models is read from config.json (the widths inside the narrow projections are their tensors'); the model has no position
+    limit of its own (``max_positions`` if the file gives one)."""
+
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    embedding_scale: float
+    pair_buckets: int
+    pair_mul_prev: int
+    pair_mul_cur: int
+    layers: tuple[KasovikLayer, ...]
+    max_position_embeddings: int | None = None
+    eos_token_ids: tuple[int, ...] = field(default_factory=tuple)
+
+    architecture = "Kasovik"
+    MIXERS = ("retention", "parallel")
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @classmethod
+    def from_dict(cls, raw: dict, generation: dict | None = None) -> "KasovikConfig":
+        norm, embedding = _require(raw, "norm"), _require(raw, "embedding")
+        pairs = _require(embedding, "bigram")
+        layers: list[KasovikLayer] = []
+        for i, entry in enumerate(_require(raw, "layers")):
+            kind = entry.get("type")
+            if kind not in cls.MIXERS:
+                raise ConfigError(f"layers[{i}]: type '{kind}' is not one of {list(cls.MIXERS)}")
+            mixer = entry.get("mixer")
+            if not isinstance(mixer, dict):
+                raise ConfigError(f"layers[{i}] has no 'mixer' sizes")
+            if kind == "retention":
+                wanted = [(mixer, k, "retention") for k in ("heads", "dim", "vdim", "decay")]
+            else:
+                left, right = mixer.get("left"), mixer.get("right")
+                if not isinstance(left, dict) or not isinstance(right, dict):
+                    raise ConfigError(f"layers[{i}]: a parallel mixer has 'left' and 'right' sizes")
+                wanted = [(mixer, k, "parallel mixer") for k in ("left_scale", "right_scale")] + \
+                    [(left, k, "left mixer") for k in ("heads", "kv_heads", "dim", "vdim", "scale")] + \
+                    [(right, k, "right mixer") for k in ("heads", "kv_heads", "dim", "vdim", "conv")]
+            for where, key, what in wanted:
+                if where.get(key) is None:
+                    raise ConfigError(f"layers[{i}]: the {what} has no '{key}'")
+            mlp = entry.get("mlp")
+            if mlp is not None:
+                if mlp.get("kind", "dense") != "dense":
+                    raise ConfigError(f"layers[{i}]: feed-forward kind '{mlp.get('kind')}' is not 'dense'")
+                for key in ("ff", "limit"):
+                    if mlp.get(key) is None:
+                        raise ConfigError(f"layers[{i}]: the feed-forward has no '{key}'")
+                mlp = {"ff": int(mlp["ff"]), "limit": float(mlp["limit"])}
+            source = entry.get("weights_of")
+            if source is not None:
+                source = int(source)
+                if not 0 <= source < i:
+                    raise ConfigError(f"layers[{i}]: weights_of must name an earlier layer")
+                other = layers[source]
+                if (other.type, other.mixer, other.mlp) != (kind, mixer, mlp):
+                    raise ConfigError(f"layers[{i}]: the sizes must equal those of layer {source}, whose weights it uses")
+                if other.weights_of is not None:
+                    source = other.weights_of
+            layers.append(KasovikLayer(kind, dict(mixer), mlp, source))
+        most = raw.get("max_positions")
+        cfg = cls(vocab_size=int(_require(raw, "vocab")), hidden_size=int(_require(raw, "width")), norm_eps=float(_require(norm, "eps")),
+                  embedding_scale=float(_require(embedding, "scale")), pair_buckets=int(_require(pairs, "buckets")),
+                  pair_mul_prev=int(_require(pairs, "mul_prev")), pair_mul_cur=int(_require(pairs, "mul_cur")), layers=tuple(layers),
+                  max_position_embeddings=int(most) if most is not None else None,
+                  eos_token_ids=collect_eos_ids(([generation] if generation else []) + [raw]))
+        cfg.validate()
+        return cfg
+
+    def validate(self) -> None:
+        for name in ("vocab_size", "hidden_size", "pair_buckets"):
+            if getattr(self, name) <= 0:
+                raise ConfigError(f"{name} must be positive, got {getattr(self, name)}")
+        for name in ("pair_mul_prev", "pair_mul_cur"):
+            if not 0 <= getattr(self, name) < 1 << 31:
+                raise ConfigError(f"{name} must be at least 0 and below 2^31, got {getattr(self, name)}")
+        if self.max_position_embeddings is not None and self.max_position_embeddings <= 0:
+            raise ConfigError("max_positions must be positive")
+        if not self.norm_eps > 0:
+            raise ConfigError("norm.eps must be positive")
+        if not self.layers:
+            raise ConfigError("a model needs at least one layer")
+        for i, layer in enumerate(self.layers):
+            m = layer.mixer
+            if layer.type == "retention":
+                for key in ("heads", "dim", "vdim"):
+                    if int(m[key]) <= 0:
+                        raise ConfigError(f"layers[{i}]: {key} must be positive")
+                if len(m["decay"]) != int(m["heads"]):
+                    raise ConfigError(f"layers[{i}]: {len(m['decay'])} decays for {m['heads']} heads")
+                rot = m.get("rot")
+                if rot:
+                    dims = int(rot.get("dims", 0))
+                    if dims < 0 or dims % 2 or dims > int(m["dim"]):
+                        raise ConfigError(f"layers[{i}]: rot.dims {dims} must be even and at most {m['dim']}")
+                    if dims and not float(rot.get("base", 0)) > 0:
+                        raise ConfigError(f"layers[{i}]: rot.base must be positive")
+            else:
+                for side in ("left", "right"):
+                    part = m[side]
+                    for key in ("heads", "kv_heads", "dim", "vdim"):
+                        if int(part[key]) <= 0:
+                            raise ConfigError(f"layers[{i}]: {side}.{key} must be positive")
+                    if int(part["heads"]) % int(part["kv_heads"]):
+                        raise ConfigError(f"layers[{i}]: {side}: {part['heads']} heads do not divide into {part['kv_heads']} kv_heads")
+                if int(m["left"]["dim"]) != int(m["left"]["vdim"]):
+                    raise ConfigError(f"layers[{i}]: left: the values are the keys, so vdim must equal dim")
+                size = (m["left"].get("mask") or {}).get("size")
+                if size is not None and int(size) < 1:
+                    raise ConfigError(f"layers[{i}]: left: mask.size must be at least 1")
+                if int(m["right"]["conv"]) < 1:
+                    raise ConfigError(f"layers[{i}]: right.conv must be at least 1")
+            if layer.mlp is not None and (layer.mlp["ff"] <= 0 or not layer.mlp["limit"] > 0):
+                raise ConfigError(f"layers[{i}]: the feed-forward's ff and limit must be positive")
+
+
 def read_json(path: Path) -> dict:
     try:
         return json.loads(path.read_text())

@@ -42,32 +42,34 @@ int tm_attn_paged_generic(const void* q, int q_stride, void* out, int out_stride
                           int dtype, hipStream_t stream);
 
 // The same with keys and values of different sizes (D, DV), scores capped smoothly at +-softcap (0: as they are) and a gate
-// per (token, head) (float32, rows ldg apart; null: none) whose sigmoid multiplies the head's result.
+// per (token, head) (float32, rows ldg apart; null: none) whose sigmoid multiplies the head's result;
+// sink (float32 [H]; null: none): one more term exp(sink[h]) in the denominator of head h's softmax, with no key behind it.
 int tm_attn_paged_generic_ext(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                               const int* block_tables, int table_width, const int* seq_of_token, const int* positions, int T, int H,
                               int KVH, int D, int DV, int page, float scale, int window, float softcap, const float* gate, int ldg,
-                              int dtype, hipStream_t stream);
+                              const float* sink, int dtype, hipStream_t stream);
 
-// The matrix-unit attention kernels with capped scores (softcap > 0: s <- softcap * tanh(s / softcap); 0: as the plain entries).
+// The matrix-unit attention kernels with capped scores (softcap > 0: s <- softcap * tanh(s / softcap); 0: as the plain entries)
+// and a sink per head (as above; null: none).
 int tm_attn_prefill_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                              const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH, int D, int page,
-                             float scale, int window, float softcap, hipStream_t stream);
+                             float scale, int window, float softcap, const float* sink, hipStream_t stream);
 int tm_attn_prefill_shared_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                                const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH, int D, int page,
-                               float scale, int window, float softcap, hipStream_t stream);
+                               float scale, int window, float softcap, const float* sink, hipStream_t stream);
 int tm_attn_prefill_f32_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                             const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH, int D, int page,
-                            float scale, int window, float softcap, hipStream_t stream);
+                            float scale, int window, float softcap, const float* sink, hipStream_t stream);
 int tm_attn_decode_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                             const int* block_tables, int table_width, const int* context_lens, float* part_o, float* part_ml,
                             int max_chunks, int S, int H, int KVH, int D, int page, float scale, int window, float softcap,
-                            hipStream_t stream);
+                            const float* sink, hipStream_t stream);
 
 // q and k normed over the whole projection, rotated and stored (attention_prepare.hip): see the head of that file.
 int tm_whole_norm_rope_store(const float* proj, int ld, void* q_out, int dtype, int T, int H, int G, int D, int Dv, int rot,
                              int interleaved, const float* q_w, const float* k_w, float eps, const float* cos_t, const float* sin_t,
                              const int* positions, const int* slots, void* k_pool, void* v_pool, int page, int has_kv,
-                             int per_head, hipStream_t stream);
+                             int per_head, int unit, int v_is_k, hipStream_t stream);
 int tm_head_gate(void* x, int dtype, const float* gate, int ldg, int T, int H, int Dv, hipStream_t stream);
 
 int tm_gemm_skinny(const void* A, int lda, const void* W, const void* bias, int bias_dtype, void* C, int ldc, int M,
@@ -180,20 +182,20 @@ int tm_attn_sigmoid_prefill(const void* q, int q_stride, void* out, int out_stri
 // Gated linear attention (gla.hip): the decays from the gate projection, the recurrence over a step's rows request by
 // request with the state [slots, H, D, Dv] in 32-bit, and the per-head norm of the result times silu(gate).
 int tm_gla_decay(const float* z, float* a, float tau, long long n, hipStream_t stream);
-int tm_gla_scan(const void* proj, int ld, int q_off, int k_off, int v_off, int dtype, const float* decay, float* o,
+int tm_gla_scan(const void* proj, int ld, int q_off, int k_off, int v_off, int dtype, const float* decay, int ldd, float* o,
                 float* state, const int* cu_q_lens, const int* state_slots, int S, int H, int D, int Dv, float q_scale,
                 hipStream_t stream);
 // Whether tm_gla_scan takes o == nullptr for these operands (only the states are advanced): rows in whole 16-byte pieces.
 int tm_gla_scan_in_pieces(int dtype, const void* proj, int ld, int q_off, int k_off, const float* decay, int D);
 int tm_gla_out_gate(const float* o, const void* gate, int ldg, int dtype, const float* w, void* y, int T, int H, int Dv,
-                    float eps, hipStream_t stream);
+                    float eps, int sigmoid, hipStream_t stream);
 // The decays straight from the narrow projection x [T, K] (rows ldx apart), W [N, K], bias [N] of the model's type:
 // a = sigmoid(x W^T + b)^(1/tau), 32-bit. And a long portion in segments (see gla.hip): the product of each segment's
 // decays, and the chain over a request's segments that turns the segments' local states into their true start states
 // and the request's new state.
 int tm_gla_gate_decay(const void* x, int ldx, const void* W, const void* bias, int dtype, float* a, int T, int N, int K,
                       float tau, hipStream_t stream);
-int tm_gla_segment_decay(const float* decay, const int* cu_seg, float* P, int n_seg, int HD, hipStream_t stream);
+int tm_gla_segment_decay(const float* decay, int ldd, const int* cu_seg, float* P, int n_seg, int HD, hipStream_t stream);
 int tm_gla_combine(float* state, const int* state_slots, const int* first_seg, const float* P, const float* local,
                    float* start, int S, int HD, int Dv, hipStream_t stream);
 
@@ -216,17 +218,29 @@ int tm_poly_norm(const float* z, const float* coef, void* out, int dtype, int T,
 
 // The gated delta rule and two sublayers side by side (delta_rule.hip): see the head of that file.
 int tm_delta_prepare(const void* proj, int ld, const void* conv_w, const void* conv_state, const float* ba, int ldba,
-                     const float* a_log, const float* dt_bias, const int* cu_q_lens, const int* state_slots, const int* seq_of_token,
-                     float* out, int ldo, int T, int H, int G, int D, int Dv, int taps, float unit_eps, int dtype, hipStream_t stream);
+                     const float* z, int ldz, const float* a_log, const float* dt_bias, const int* cu_q_lens, const int* state_slots,
+                     const int* seq_of_token, float* out, int ldo, int T, int H, int G, int D, int Dv, int taps, float unit_eps, int dtype, hipStream_t stream);
 int tm_delta_conv_state(const void* proj, int ld, void* state, const int* cu_q_lens, const int* state_slots, int S, int C, int taps,
                         int dtype, hipStream_t stream);
 int tm_delta_scan(const float* rows, int ld, float* o, float* state, const int* cu_q_lens, const int* state_slots, int S, int H, int G,
-                  int D, int Dv, int row_dv, int use_v, hipStream_t stream);
+                  int D, int Dv, int row_dv, int use_v, int per_channel, hipStream_t stream);
 int tm_delta_combine(const float* trans, const float* local, float* start, float* state, const int* state_slots, const int* first_seg,
                      int S, int H, int D, int Dv, hipStream_t stream);
 int tm_pair_norm_mean(const void* a, const void* b, const float* wa, const float* wb, void* out, int T, int W, float eps, int dtype,
                       hipStream_t stream);
 int tm_gelu_mul(const void* gu, void* out, int dtype, int T, int I, hipStream_t stream);
+// out[t, i] = g sigmoid(alpha g) (u + 1) with g = min(gu[t, i], limit), u = gu[t, I + i] held to +-limit, in 32-bit.
+int tm_clamped_glu(const void* gu, void* out, int dtype, int T, int I, float alpha, float limit, hipStream_t stream);
+// Embedding rows with a row per pair of neighbouring tokens (embedding_pairs.hip): see the head of that file.
+int tm_embed_pairs(const void* table, const void* pairs, int dtype, const int* ids, const int* positions, const int* cu_q_lens,
+                   const int* state_slots, const int* seq_of_token, int* prev_state, float* out, int T, int hidden, int vocab,
+                   float scale, int buckets, long long mul_prev, long long mul_cur, hipStream_t stream);
+// A weighted sum of up to three results added to the residual stream, and the RMS norm of the sum (sum_norm.hip): see there.
+int tm_sum_norm(float* resid, const void* y0, float s0, const void* y1, float s1, const void* y2, float s2, const int* rows,
+                const void* w, int w_dtype, void* out, int dtype, int R, int hidden, float eps, hipStream_t stream);
+// q, k and v of a retention as 32-bit rows, q and k rotated, k scaled (retention.hip): see there.
+int tm_retention_prepare(const void* proj, int ld, int dtype, const float* cos_t, const float* sin_t, int rot, const int* positions,
+                         float* rows, int ldr, int T, int H, int D, int Dv, float k_scale, hipStream_t stream);
 int tm_embed_gather_scaled(const void* table, int dtype, const int* ids, float* out, int T, int hidden, int vocab, float scale,
                            hipStream_t stream);
 

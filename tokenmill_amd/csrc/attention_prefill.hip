@@ -188,7 +188,7 @@ __global__ __launch_bounds__(64 * KS) void attn_prefill_mfma_kernel(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
     const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ tiles, int n_tiles, int pair, int H, int KVH, int page_shift,
-    float scale_log2, float cap_in, float cap_out, int window) {
+    float scale_log2, float cap_in, float cap_out, int window, const float* __restrict__ sink) {
     constexpr int NDC = D / 32, NDT = D / 16;
     __shared__ float s_m[KS][16], s_l[KS][16];
     __shared__ float s_o[KS][16][D + 1];
@@ -298,6 +298,7 @@ __global__ __launch_bounds__(64 * KS) void attn_prefill_mfma_kernel(
                     o0 = fmaf(s_o[w][col][d], f, o0);
                     o1 = fmaf(s_o[w][col][d + 1], f, o1);
                 }
+                if (sink) ll += __builtin_amdgcn_exp2f(sink[h0 + hh] * 1.4426950408889634f - mm);      // a term of the denominator without a key
                 const float inv = 1.f / ll;
                 *(uint32_t*)(out + (size_t)(row0 + col) * out_stride + (size_t)(h0 + hh) * D + d) = pk_bf16(o0 * inv, o1 * inv);
             }
@@ -315,7 +316,8 @@ template <int D> struct PrefillShape { static constexpr int HPW = D <= 64 ? 4 : 
 template <int D, int HPW>
 static void launch_split_keys(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                               const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH,
-                              int page_shift, float scale_log2, float cap_in, float cap_out, int window, hipStream_t stream) {
+                              int page_shift, float scale_log2, float cap_in, float cap_out, int window, const float* sink,
+                              hipStream_t stream) {
     constexpr int KS = PrefillShape<D>::KS;
     const int splits = (H / KVH + HPW - 1) / HPW;
     // fold the table in two once the folded launch still gives every CU a block
@@ -323,14 +325,15 @@ static void launch_split_keys(const void* q, int q_stride, void* out, int out_st
     dim3 grid(pair ? (n_tiles + 1) / 2 : n_tiles, KVH * splits);
     attn_prefill_mfma_kernel<D, HPW, KS><<<grid, 64 * KS, 0, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_tables,
-        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window);
+        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, sink);
 }
 
-// softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax
+// softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax; sink (float32 [H]) or null: one more term
+// exp(sink[h]) in the denominator of head h's softmax, with no key behind it
 extern "C" int tm_attn_prefill_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                         const void* v_pool, const int* block_tables, int table_width, const int* tiles,
                                         int n_tiles, int H, int KVH, int D, int page, float scale, int window, float softcap,
-                                        hipStream_t stream) {
+                                        const float* sink, hipStream_t stream) {
     if (n_tiles <= 0) return TM_OK;
     if (!(softcap >= 0.f)) return TM_ERR_ARG;
     const float cap_in = softcap > 0.f ? scale / softcap : 0.f, cap_out = softcap > 0.f ? softcap / scale : 0.f;
@@ -344,7 +347,7 @@ extern "C" int tm_attn_prefill_mfma_cap(const void* q, int q_stride, void* out, 
     const float scale_log2 = scale * 1.4426950408889634f;
     if ((long long)KVH * ((G + 1) / 2) > 65535) return TM_ERR_ARG;
 #define TM_SPLIT_ARGS q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, \
-                      page_shift, scale_log2, cap_in, cap_out, window, stream
+                      page_shift, scale_log2, cap_in, cap_out, window, sink, stream
 #define TM_PREFILL_CASE(DD)                                                                                       \
     case DD: {                                                                                                    \
         constexpr int HPW = PrefillShape<DD>::HPW;                                                                \
@@ -373,5 +376,5 @@ extern "C" int tm_attn_prefill_mfma(const void* q, int q_stride, void* out, int 
                                     int n_tiles, int H, int KVH, int D, int page, float scale, int window,
                                     hipStream_t stream) {
     return tm_attn_prefill_mfma_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, D,
-                                    page, scale, window, 0.f, stream);
+                                    page, scale, window, 0.f, nullptr, stream);
 }

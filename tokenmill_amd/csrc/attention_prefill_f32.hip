@@ -30,7 +30,8 @@ template <int D>
 __global__ __launch_bounds__(64 * AF_SPLIT) void attn_prefill_f32_kernel(
     const float* __restrict__ q, int q_stride, float* __restrict__ out, int out_stride,
     const float* __restrict__ k_pool, const float* __restrict__ v_pool, const int* __restrict__ block_tables,
-    int table_width, const int* __restrict__ tiles, int H, int KVH, int page_shift, float scale, int window, float softcap) {
+    int table_width, const int* __restrict__ tiles, int H, int KVH, int page_shift, float scale, int window, float softcap,
+    const float* __restrict__ sink) {
     constexpr int DQ = D / 4;           // values of a key (or query) a lane holds
     constexpr int NDT = D / 16;         // 16-row tiles of d
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / TM_WAVE);
@@ -153,6 +154,7 @@ __global__ __launch_bounds__(64 * AF_SPLIT) void attn_prefill_f32_kernel(
             sw[w] = (mw[w] == -INFINITY) ? 0.f : expf(mw[w] - top);     // a token always sees its own key: top is finite
             sum += l_s[w][tok] * sw[w];
         }
+        if (sink) sum += expf(sink[h] - top);                             // a term of the denominator without a key
         const float inv = 1.f / sum;
         float* orow = out + (size_t)(row0 + tok) * out_stride + (size_t)h * D;
         for (int d = (threadIdx.x & 15) * 4; d < D; d += 64) {
@@ -171,11 +173,12 @@ __global__ __launch_bounds__(64 * AF_SPLIT) void attn_prefill_f32_kernel(
 // q float32 [T, >= H*D] rows, out float32 [T, >= H*D]; pools float32, K [pages, page, KVH, D], V [pages, KVH, D, page];
 // tiles int32 [n_tiles][4] = (request index, first row, tokens (1..16), position of the first token).
 // Needs D % 16 == 0 (at most 128), page a power of two >= 16, 16-byte aligned q, out and pools, strides % 4 == 0.
-// softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax.
+// softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax; sink (float32 [H]) or null: one more term
+// exp(sink[h]) in the denominator of head h's softmax, with no key behind it.
 extern "C" int tm_attn_prefill_f32_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                        const void* v_pool, const int* block_tables, int table_width, const int* tiles,
                                        int n_tiles, int H, int KVH, int D, int page, float scale, int window, float softcap,
-                                       hipStream_t stream) {
+                                       const float* sink, hipStream_t stream) {
     if (n_tiles <= 0) return TM_OK;
     if (!(softcap >= 0.f)) return TM_ERR_ARG;
     if (H <= 0 || KVH <= 0 || H % KVH || page < 16 || (page & (page - 1)) || window < 0 || table_width <= 0 ||
@@ -190,7 +193,7 @@ extern "C" int tm_attn_prefill_f32_cap(const void* q, int q_stride, void* out, i
     case DD:                                                                                                      \
         attn_prefill_f32_kernel<DD><<<grid, 64 * AF_SPLIT, 0, stream>>>(                                          \
             (const float*)q, q_stride, (float*)out, out_stride, (const float*)k_pool, (const float*)v_pool,       \
-            block_tables, table_width, tiles, H, KVH, page_shift, scale, window, softcap);                                 \
+            block_tables, table_width, tiles, H, KVH, page_shift, scale, window, softcap, sink);                           \
         break
     switch (D) {
         TM_PREFILL_F32_CASE(16);
@@ -214,5 +217,5 @@ extern "C" int tm_attn_prefill_f32(const void* q, int q_stride, void* out, int o
                                    int n_tiles, int H, int KVH, int D, int page, float scale, int window,
                                    hipStream_t stream) {
     return tm_attn_prefill_f32_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, D,
-                                   page, scale, window, 0.f, stream);
+                                   page, scale, window, 0.f, nullptr, stream);
 }

@@ -224,7 +224,7 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
     const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ tiles, int n_tiles, int pair, int H, int KVH, int page_shift,
-    float scale_log2, float cap_in, float cap_out, int window) {
+    float scale_log2, float cap_in, float cap_out, int window, const float* __restrict__ sink) {
     constexpr int NDC = D / 32, NDT = D / 16, THREADS = 64 * WAVES, STAGE = SharedShape<D>::STAGE, HPW = SharedPlan<D>::HPW;
     extern __shared__ __align__(16) unsigned char stages[];          // two stages
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / TM_WAVE);
@@ -308,6 +308,7 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
             lsum += __shfl_xor(lsum, 16, TM_WAVE);
             lsum += __shfl_xor(lsum, 32, TM_WAVE);
             if (r >= valid) continue;
+            if (sink) lsum += __builtin_amdgcn_exp2f(sink[h0 + hh] * 1.4426950408889634f - st.m[hh]);      // a term of the denominator without a key
             const float inv = 1.f / lsum;
             bf16_t* orow = out + (size_t)(row0 + r) * out_stride + (size_t)(h0 + hh) * D + 4 * g;
 #pragma unroll
@@ -324,7 +325,8 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
 template <int D, int WAVES>
 static int launch_shared(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                          const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH,
-                         int page_shift, float scale_log2, float cap_in, float cap_out, int window, hipStream_t stream) {
+                         int page_shift, float scale_log2, float cap_in, float cap_out, int window, const float* sink,
+                         hipStream_t stream) {
     constexpr int lds = 2 * SharedShape<D>::STAGE;
     static bool raised = false;
     if (lds > 48 * 1024 && !raised) {
@@ -338,7 +340,7 @@ static int launch_shared(const void* q, int q_stride, void* out, int out_stride,
     dim3 grid(pair ? (n_tiles + 1) / 2 : n_tiles, KVH);
     attn_prefill_shared_kernel<D, WAVES><<<grid, 64 * WAVES, lds, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_tables,
-        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window);
+        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, sink);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
@@ -351,11 +353,12 @@ extern "C" int tm_attn_prefill_shared_takes(int H, int KVH, int D) {
     return G <= 8 * (D <= 64 ? SharedPlan<64>::HPW : SharedPlan<128>::HPW);
 }
 
-// softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax
+// softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax; sink (float32 [H]) or null: one more term
+// exp(sink[h]) in the denominator of head h's softmax, with no key behind it
 extern "C" int tm_attn_prefill_shared_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                           const void* v_pool, const int* block_tables, int table_width, const int* tiles,
                                           int n_tiles, int H, int KVH, int D, int page, float scale, int window, float softcap,
-                                          hipStream_t stream) {
+                                          const float* sink, hipStream_t stream) {
     if (n_tiles <= 0) return TM_OK;
     if (!(softcap >= 0.f)) return TM_ERR_ARG;
     const float cap_in = softcap > 0.f ? scale / softcap : 0.f, cap_out = softcap > 0.f ? softcap / scale : 0.f;
@@ -369,7 +372,7 @@ extern "C" int tm_attn_prefill_shared_cap(const void* q, int q_stride, void* out
     while ((1 << page_shift) < page) ++page_shift;
     const float scale_log2 = scale * 1.4426950408889634f;
 #define TM_SHARED_ARGS q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, \
-                       page_shift, scale_log2, cap_in, cap_out, window, stream
+                       page_shift, scale_log2, cap_in, cap_out, window, sink, stream
 #define TM_SHARED_CASE(DD)                                                          \
     case DD:                                                                        \
         if (need <= 2) return launch_shared<DD, 2>(TM_SHARED_ARGS);                 \
@@ -394,5 +397,5 @@ extern "C" int tm_attn_prefill_shared(const void* q, int q_stride, void* out, in
                                       int n_tiles, int H, int KVH, int D, int page, float scale, int window,
                                       hipStream_t stream) {
     return tm_attn_prefill_shared_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH,
-                                      D, page, scale, window, 0.f, stream);
+                                      D, page, scale, window, 0.f, nullptr, stream);
 }

@@ -2,15 +2,17 @@
 //
 //   S <- g_t S;   u_t = beta_t (v_t - S^T k_t);   S <- S + k_t u_t^T;   o_t = S^T q_t
 //
-// with one decay g_t in (0, 1) and one step size beta_t in (0, 1) per token and head, unit vectors q_t (times D^-1/2) and
-// k_t, advanced token by token in the order of the positions, within a step's portion and from one step to the next (the
+// with a decay g_t in (0, 1) per token and head, or one per token, head and key channel (it then multiplies the rows of S one by
+// one), a step size beta_t in (0, 1) per token and head, unit vectors q_t (times D^-1/2) and k_t, advanced token by token in the order of the positions, within a step's portion and from one step to the next (the
 // state lives in the request's state slot between steps). H value heads share G <= H query/key heads (head h reads q/k
 // head h / (H / G)).
 //
 //   tm_delta_prepare     per token: the short causal convolution over time of the q | k | v channels of the stacked
 //                        projection (the rows before the step's first from the request's convolution state), silu, the two
 //                        unit norms, k . q, beta = sigmoid(b) and g = exp(-exp(A_log) softplus(a + dt_bias)); all written
-//                        as one 32-bit row [q (G D) | k (G D) | v (H Dv) | beta (H) | g (H) | k.q (G)]
+//                        as one 32-bit row [q (G D) | k (G D) | v (H Dv) | beta (H) | g (H) | k.q (G)]; with a decay per key
+//                        channel its logarithm comes from a [H, D] row z of its own, a = z + dt_bias, A_log per head, and the
+//                        decays stand behind the rest, [... | k.q (G) | g (H D)] (the H floats of g before k.q stay unused)
 //   tm_delta_conv_state  then the convolution state becomes the last taps - 1 projection rows the request has seen
 //   tm_delta_scan        the recurrence over those rows; writes o in 32-bit
 //   tm_delta_combine     chains the segments of a long portion (each scanned from zero and from the identity) into every
@@ -19,7 +21,8 @@
 //
 // The columns of S are independent of each other: with d_k = S^T k and d_q = S^T q taken on the state as the token finds it,
 //   u = beta (v - g d_k),   o = g d_q + u (k . q),   S <- g S + k u^T
-// is the same recurrence with one round of sums a token instead of two. The scan is dealt over (request, head, 16 columns)
+// is the same recurrence with one round of sums a token instead of two (with a decay per channel S is decayed before the sums,
+// and g falls out of the first two lines). The scan is dealt over (request, head, 16 columns)
 // blocks; a lane keeps a sixteenth of a column's D rows in registers, and a column's sixteen partial sums are added in a fixed
 // order; a request's rows reach its block through LDS, a tile of tokens at a time. A token's result depends on its
 // request's state and tokens only, never on the step's other rows; how the prompt was cut changes it by 32-bit rounding at
@@ -48,13 +51,20 @@ __device__ __forceinline__ float delta_conv_channel(const T* __restrict__ proj, 
     return silu_f32(acc);
 }
 
-// grid (T, G + ceil(H Dv / 256)); a block is a token and either one q/k head (a thread a channel of q and of k; the head's three
-// sums by the block's fixed tree) or 256 channels of v; the first block of v also makes the token's step sizes and decays. Few
-// tokens still make many blocks, and a thread's loads are a handful.
+// grid (T, G + ceil(H Dv / 256) [+ ceil(H D / 256)]); a block is a token and either one q/k head (a thread a channel of q and of
+// k; the head's three sums by the block's fixed tree) or 256 channels of v; the first block of v also makes the token's step
+// sizes and its decays per head; with decays per channel (z) the last blocks make 256 of those each. Few tokens still make many
+// blocks, and a thread's loads are a handful.
+__device__ __forceinline__ float delta_decay(float a, float a_log) {
+    const float sp = fmaxf(a, 0.f) + log1pf(expf(-fabsf(a)));                    // softplus
+    return expf(-expf(a_log) * sp);
+}
+
 template <typename T>
 __global__ __launch_bounds__(DP_THREADS) void delta_prepare_kernel(const T* __restrict__ proj, int ld, const T* __restrict__ conv_w,
                                                                    const T* __restrict__ conv_state, const float* __restrict__ ba,
-                                                                   int ldba, const float* __restrict__ a_log,
+                                                                   int ldba, const float* __restrict__ z, int ldz,
+                                                                   const float* __restrict__ a_log,
                                                                    const float* __restrict__ dt_bias, const int* __restrict__ cu,
                                                                    const int* __restrict__ slots, const int* __restrict__ seq_of_token,
                                                                    float* __restrict__ out, int ldo, int H, int G, int D, int Dv,
@@ -80,39 +90,43 @@ __global__ __launch_bounds__(DP_THREADS) void delta_prepare_kernel(const T* __re
         if (c == 0) o[C + 2 * H + unit] = qk * iq * ik;
         return;
     }
+    const int v_units = (H * Dv + DP_THREADS - 1) / DP_THREADS;
+    if (unit >= G + v_units) {
+        const int n = (unit - G - v_units) * DP_THREADS + threadIdx.x;
+        if (n < H * D) o[C + 2 * H + G + n] = delta_decay(z[(size_t)t * ldz + n] + dt_bias[n], a_log[n / D]);
+        return;
+    }
     const int c = 2 * G * D + (unit - G) * DP_THREADS + threadIdx.x;
     if (c < C) o[c] = delta_conv_channel<T>(proj, ld, conv_w, st, C, taps, first, i, c);
     if (unit == G)
         for (int h = threadIdx.x; h < H; h += DP_THREADS) {
             const float b = ba[(size_t)t * ldba + h];
-            const float a = ba[(size_t)t * ldba + H + h] + dt_bias[h];
-            const float sp = fmaxf(a, 0.f) + log1pf(expf(-fabsf(a)));            // softplus
             o[C + h] = 1.0f / (1.0f + expf(-b));
-            o[C + H + h] = expf(-expf(a_log[h]) * sp);
+            if (!z) o[C + H + h] = delta_decay(ba[(size_t)t * ldba + H + h] + dt_bias[h], a_log[h]);
         }
 }
 
 extern "C" int tm_delta_prepare(const void* proj, int ld, const void* conv_w, const void* conv_state, const float* ba, int ldba,
-                                const float* a_log, const float* dt_bias, const int* cu_q_lens, const int* state_slots,
+                                const float* z, int ldz, const float* a_log, const float* dt_bias, const int* cu_q_lens, const int* state_slots,
                                 const int* seq_of_token, float* out, int ldo, int T, int H, int G, int D, int Dv, int taps,
                                 float unit_eps, int dtype, hipStream_t stream) {
     if (!proj || !conv_w || !ba || !a_log || !dt_bias || !cu_q_lens || !state_slots || !seq_of_token || !out || T < 0 || H <= 0 ||
         G <= 0 || H % G || D <= 0 || D > DP_THREADS || Dv <= 0 || taps < 1 || taps > DR_MAX_TAPS || (taps > 1 && !conv_state) ||
-        ldba < 2 * H || !(unit_eps > 0.f))
+        ldba < (z ? H : 2 * H) || (z && ldz < H * D) || !(unit_eps > 0.f))
         return TM_ERR_ARG;
     const long long C = 2LL * G * D + (long long)H * Dv;
-    const long long units = G + ((long long)H * Dv + DP_THREADS - 1) / DP_THREADS;
-    if (ld < C || ldo < C + 2 * H + G || units > 65535) return TM_ERR_ARG;
+    const long long units = G + ((long long)H * Dv + DP_THREADS - 1) / DP_THREADS + (z ? ((long long)H * D + DP_THREADS - 1) / DP_THREADS : 0);
+    if (ld < C || ldo < C + 2 * H + G + (z ? (long long)H * D : 0) || units > 65535) return TM_ERR_ARG;
     if (dtype != TM_F32 && dtype != TM_BF16) return TM_ERR_ARG;
     if (T == 0) return TM_OK;
     const dim3 grid(T, (unsigned)units);
     if (dtype == TM_F32)
         delta_prepare_kernel<float><<<grid, DP_THREADS, 0, stream>>>((const float*)proj, ld, (const float*)conv_w, (const float*)conv_state,
-                                                                     ba, ldba, a_log, dt_bias, cu_q_lens, state_slots, seq_of_token, out,
+                                                                     ba, ldba, z, ldz, a_log, dt_bias, cu_q_lens, state_slots, seq_of_token, out,
                                                                      ldo, H, G, D, Dv, taps, unit_eps);
     else
         delta_prepare_kernel<bf16_t><<<grid, DP_THREADS, 0, stream>>>((const bf16_t*)proj, ld, (const bf16_t*)conv_w,
-                                                                      (const bf16_t*)conv_state, ba, ldba, a_log, dt_bias, cu_q_lens,
+                                                                      (const bf16_t*)conv_state, ba, ldba, z, ldz, a_log, dt_bias, cu_q_lens,
                                                                       state_slots, seq_of_token, out, ldo, H, G, D, Dv, taps, unit_eps);
     TM_CHECK_LAUNCH();
     return TM_OK;
@@ -177,8 +191,9 @@ __device__ __forceinline__ float row16_sum(float v) {
 // consecutive threads consecutive floats, into registers while the tile before is worked on (CPM: floats of a token a thread
 // fetches at most), and put it down in the other of two buffers. VEC: R is a multiple of 4, so a lane reads its q and k from
 // LDS as float4. o null: only the states are wanted. use_v 0: the values count as zero and the state's Dv columns need not be the
-// rows' row_dv (a scan from the identity gives the product of the tokens' transitions g (I - beta k k^T)).
-template <int RMAX, int CPM, bool VEC>
+// rows' row_dv (a scan from the identity gives the product of the tokens' transitions g (I - beta k k^T)). CH: a decay per key
+// channel; the tile's rows are then D floats longer, [... | v | g].
+template <int RMAX, int CPM, bool VEC, bool CH>
 __global__ __launch_bounds__(DR_THREADS) void delta_scan_kernel(const float* __restrict__ rows, int ld, float* __restrict__ o,
                                                                float* __restrict__ state, const int* __restrict__ cu_q_lens,
                                                                const int* __restrict__ state_slots, int H, int G, int D, int Dv,
@@ -193,7 +208,7 @@ __global__ __launch_bounds__(DR_THREADS) void delta_scan_kernel(const float* __r
     const bool col = e < Dv;
     const int t0 = cu_q_lens[s], t1 = cu_q_lens[s + 1];
     if (t1 <= t0) return;                                                 // the whole block
-    const int C = 2 * G * D + H * row_dv, W = 2 * D + 4 + DR_COLS;
+    const int C = 2 * G * D + H * row_dv, WV = 2 * D + 4 + DR_COLS, W = WV + (CH ? D : 0);
     // where in a prepared row the floats come from that this thread fetches of every token (-1: none)
     int from[CPM];
 #pragma unroll
@@ -205,7 +220,8 @@ __global__ __launch_bounds__(DR_THREADS) void delta_scan_kernel(const float* __r
         else if (c == 2 * D) at = C + h;
         else if (c == 2 * D + 1) at = C + H + h;
         else if (c == 2 * D + 2) at = C + 2 * H + g;
-        else if (use_v && c >= 2 * D + 4 && c < W && blockIdx.x * DR_COLS + (c - 2 * D - 4) < Dv)
+        else if (CH && c >= WV && c < W) at = C + 2 * H + G + h * D + (c - WV);
+        else if (use_v && c >= 2 * D + 4 && c < WV && blockIdx.x * DR_COLS + (c - 2 * D - 4) < Dv)
             at = 2 * G * D + h * row_dv + blockIdx.x * DR_COLS + (c - 2 * D - 4);
         from[j] = at;
     }
@@ -248,6 +264,10 @@ __global__ __launch_bounds__(DR_THREADS) void delta_scan_kernel(const float* __r
                     if (i < R) {
                         const float4 q4 = *(const float4*)(row + d0 + i), k4 = *(const float4*)(row + D + d0 + i);
                         kk[i] = k4.x, kk[i + 1] = k4.y, kk[i + 2] = k4.z, kk[i + 3] = k4.w;
+                        if (CH) {
+                            const float4 g4 = *(const float4*)(row + WV + d0 + i);
+                            S[i] *= g4.x, S[i + 1] *= g4.y, S[i + 2] *= g4.z, S[i + 3] *= g4.w;
+                        }
                         dk += S[i] * k4.x, dq += S[i] * q4.x;
                         dk += S[i + 1] * k4.y, dq += S[i + 1] * q4.y;
                         dk += S[i + 2] * k4.z, dq += S[i + 2] * q4.z;
@@ -259,6 +279,7 @@ __global__ __launch_bounds__(DR_THREADS) void delta_scan_kernel(const float* __r
                     const bool in = i < R && d0 + i < D;
                     kk[i] = in ? row[D + d0 + i] : 0.f;
                     if (in) {
+                        if (CH) S[i] *= row[WV + d0 + i];
                         dk += S[i] * kk[i];
                         dq += S[i] * row[d0 + i];
                     }
@@ -266,11 +287,11 @@ __global__ __launch_bounds__(DR_THREADS) void delta_scan_kernel(const float* __r
             }
             dk = row16_sum(dk);
             dq = row16_sum(dq);
-            const float beta = row[2 * D], decay = row[2 * D + 1], kq = row[2 * D + 2], v = row[2 * D + 4 + mine];
+            const float beta = row[2 * D], decay = CH ? 1.f : row[2 * D + 1], kq = row[2 * D + 2], v = row[2 * D + 4 + mine];
             const float u = beta * (v - decay * dk);
 #pragma unroll
             for (int i = 0; i < RMAX; ++i)
-                if (i < R) S[i] = decay * S[i] + kk[i] * u;
+                if (i < R) S[i] = (CH ? S[i] : decay * S[i]) + kk[i] * u;
             if (o && col && part == 0) out[(size_t)tt * H * Dv] = decay * dq + u * kq;
         }
         which ^= 1;
@@ -281,26 +302,30 @@ __global__ __launch_bounds__(DR_THREADS) void delta_scan_kernel(const float* __r
 }
 
 extern "C" int tm_delta_scan(const float* rows, int ld, float* o, float* state, const int* cu_q_lens, const int* state_slots, int S,
-                             int H, int G, int D, int Dv, int row_dv, int use_v, hipStream_t stream) {
+                             int H, int G, int D, int Dv, int row_dv, int use_v, int per_channel, hipStream_t stream) {
     if (!rows || !state || !cu_q_lens || !state_slots || S < 0 || H <= 0 || G <= 0 || H % G || D <= 0 || D > 256 || Dv <= 0 ||
         row_dv <= 0 || (use_v && row_dv != Dv) || (o && !use_v) || H > 65535 || S > 65535 ||
-        (long long)ld < 2LL * G * D + (long long)H * row_dv + 2 * H + G)
+        (long long)ld < 2LL * G * D + (long long)H * row_dv + 2 * H + G + (per_channel ? (long long)H * D : 0))
         return TM_ERR_ARG;
     if (S == 0) return TM_OK;
     const dim3 grid((Dv + DR_COLS - 1) / DR_COLS, H, S);
-    const int W = 2 * D + 4 + DR_COLS;
-    const size_t lds = (size_t)2 * DR_TT * W * sizeof(float);              // 68 KB at most
+    const int W = (per_channel ? 3 : 2) * D + 4 + DR_COLS;
+    const size_t lds = (size_t)2 * DR_TT * W * sizeof(float);              // 68 KB at most, 101 KB with decays per channel
     const bool vec = D % (4 * DR_PARTS) == 0;
-#define DR_GO(RM, CPM_)                                                                                                          \
+#define DR_GO(RM, CPM_, CH_)                                                                                                     \
     do {                                                                                                                         \
-        auto kernel = vec ? delta_scan_kernel<RM, CPM_, true> : delta_scan_kernel<RM, CPM_, false>;                              \
+        auto kernel = vec ? delta_scan_kernel<RM, CPM_, true, CH_> : delta_scan_kernel<RM, CPM_, false, CH_>;                    \
         if (lds > 64 * 1024 && hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) \
             return TM_ERR_LAUNCH;                                                                                                \
         kernel<<<grid, DR_THREADS, lds, stream>>>(rows, ld, o, state, cu_q_lens, state_slots, H, G, D, Dv, row_dv, use_v);       \
     } while (0)
-    if (D <= 64) DR_GO(4, 1);                       // W <= 148
-    else if (D <= 128) DR_GO(8, 2);                 // W <= 276
-    else DR_GO(16, 3);                              // W <= 532
+    if (per_channel) {
+        if (D <= 64) DR_GO(4, 1, true);             // W <= 212
+        else if (D <= 128) DR_GO(8, 2, true);       // W <= 404
+        else DR_GO(16, 4, true);                    // W <= 788
+    } else if (D <= 64) DR_GO(4, 1, false);         // W <= 148
+    else if (D <= 128) DR_GO(8, 2, false);          // W <= 276
+    else DR_GO(16, 3, false);                       // W <= 532
 #undef DR_GO
     TM_CHECK_LAUNCH();
     return TM_OK;

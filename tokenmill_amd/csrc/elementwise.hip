@@ -536,6 +536,61 @@ extern "C" int tm_gelu_mul(const void* gu, void* out, int dtype, int T, int I, h
     return TM_OK;
 }
 
+// out[t, i] = g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = up held to +-limit: the clamped gated activation, computed in
+// 32-bit and rounded once; gu [T, 2I] (gate columns, then up columns). Eight elements a thread where the rows come in whole
+// pieces of eight.
+__device__ __forceinline__ float clamped_glu_f32(float g, float u, float alpha, float limit) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+}
+
+template <typename T, int N>
+__global__ __launch_bounds__(256) void clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, float alpha,
+                                                          float limit) {
+    const size_t t = blockIdx.y;
+    const int i = (blockIdx.x * 256 + threadIdx.x) * N;
+    if (i >= I) return;
+    const T* gr = gu + t * 2 * I + i;
+    T* o = out + t * I + i;
+    if constexpr (N == 1) {
+        Elem<T>::store(o, clamped_glu_f32(Elem<T>::load(gr), Elem<T>::load(gr + I), alpha, limit));
+    } else {
+        __align__(16) T g[N], u[N], r[N];
+#pragma unroll
+        for (int p = 0; p < (int)(N * sizeof(T) / 16); ++p) {
+            ((uint4*)g)[p] = ((const uint4*)gr)[p];
+            ((uint4*)u)[p] = ((const uint4*)(gr + I))[p];
+        }
+#pragma unroll
+        for (int j = 0; j < N; ++j) Elem<T>::store(r + j, clamped_glu_f32(Elem<T>::load(g + j), Elem<T>::load(u + j), alpha, limit));
+#pragma unroll
+        for (int p = 0; p < (int)(N * sizeof(T) / 16); ++p) ((uint4*)o)[p] = ((const uint4*)r)[p];
+    }
+}
+
+template <typename T>
+static void launch_clamped_glu(const void* gu, void* out, int T_rows, int I, float alpha, float limit, hipStream_t stream) {
+    const bool pieces = I % 8 == 0 && ((uintptr_t)gu % 16) == 0 && ((uintptr_t)out % 16) == 0;
+    for (int t0 = 0; t0 < T_rows; t0 += 65535) {
+        const int rows = T_rows - t0 < 65535 ? T_rows - t0 : 65535;
+        const T* src = (const T*)gu + (size_t)t0 * 2 * I;
+        T* dst = (T*)out + (size_t)t0 * I;
+        if (pieces) clamped_glu_kernel<T, 8><<<dim3((I / 8 + 255) / 256, rows), 256, 0, stream>>>(src, dst, I, alpha, limit);
+        else clamped_glu_kernel<T, 1><<<dim3((I + 255) / 256, rows), 256, 0, stream>>>(src, dst, I, alpha, limit);
+    }
+}
+
+extern "C" int tm_clamped_glu(const void* gu, void* out, int dtype, int T, int I, float alpha, float limit, hipStream_t stream) {
+    if (T <= 0) return TM_OK;
+    if (I <= 0 || !gu || !out || !(limit > 0.f)) return TM_ERR_ARG;
+    if (dtype == TM_F32) launch_clamped_glu<float>(gu, out, T, I, alpha, limit, stream);
+    else if (dtype == TM_BF16) launch_clamped_glu<bf16_t>(gu, out, T, I, alpha, limit, stream);
+    else return TM_ERR_ARG;
+    TM_CHECK_LAUNCH();
+    return TM_OK;
+}
+
 extern "C" int tm_gelu_tanh(const void* in, void* out, int dtype, long long n, hipStream_t stream) {
     return launch_activation<ACT_GELU_TANH>(in, out, dtype, n, stream);
 }

@@ -7,7 +7,9 @@
 // (the state lives in the request's state slot between steps). Three kernels:
 //   gla_decay     a = sigmoid(z)^(1/tau) from the gate projection z, as exp(logsigmoid(z) / tau), 32-bit
 //   gla_scan      the recurrence; reads q, k, v from the rows of the stacked projection, writes o in 32-bit
-//   gla_out_gate  y = w * o / rms(o) (per head, over Dv) * silu(g), rounded once to the model's type
+//   gla_out_gate  y = w * o / rms(o) (per head, over Dv) * silu(g) (or sigmoid(g); w null: no weight), rounded once to the
+//                 model's type
+// The decays may also be the same for every token (ldd = 0): a retention.
 // Everything that enters the recurrence is 32-bit. The columns of S are independent of each other, so the scan is
 // dealt over (request, head, 16 columns) wavefronts; a lane keeps a quarter of a column's D rows in registers, and a
 // column's four partial dot products are added in a fixed order. A token's result depends on its request's state
@@ -39,7 +41,7 @@ extern "C" int tm_gla_decay(const float* z, float* a, float tau, long long n, hi
 // p * R .. p * R + R - 1 of its column, R = ceil(D / GLA_PARTS) <= RMAX.
 template <typename T, int RMAX>
 __global__ __launch_bounds__(TM_WAVE) void gla_scan_kernel(const T* __restrict__ proj, int ld, int q_off, int k_off, int v_off,
-                                                          const float* __restrict__ decay, float* __restrict__ o,
+                                                          const float* __restrict__ decay, int ldd, float* __restrict__ o,
                                                           float* __restrict__ state, const int* __restrict__ cu_q_lens,
                                                           const int* __restrict__ state_slots, int H, int D, int Dv,
                                                           float q_scale) {
@@ -59,7 +61,7 @@ __global__ __launch_bounds__(TM_WAVE) void gla_scan_kernel(const T* __restrict__
         const T* row = proj + (size_t)t * ld;
         const T* qr = row + q_off + h * D + d0;
         const T* kr = row + k_off + h * D + d0;
-        const float* ar = decay + ((size_t)t * H + h) * D + d0;
+        const float* ar = decay + (size_t)t * ldd + h * D + d0;
         const float v = col ? Elem<T>::load(row + v_off + h * Dv + e) : 0.f;
         float acc = 0.f;
 #pragma unroll
@@ -86,7 +88,7 @@ __global__ __launch_bounds__(TM_WAVE) void gla_scan_kernel(const T* __restrict__
 // other's loads); OUT = false leaves q and the results out (the scan that only builds the segments' local states).
 template <typename T, int RMAX, int PARTS, bool OUT>
 __global__ __launch_bounds__(TM_WAVE) void gla_scan_vec_kernel(const T* __restrict__ proj, int ld, int q_off, int k_off, int v_off,
-                                                              const float* __restrict__ decay, float* __restrict__ o,
+                                                              const float* __restrict__ decay, int ldd, float* __restrict__ o,
                                                               float* __restrict__ state, const int* __restrict__ cu_q_lens,
                                                               const int* __restrict__ state_slots, int H, int D, int Dv,
                                                               float q_scale) {
@@ -110,7 +112,7 @@ __global__ __launch_bounds__(TM_WAVE) void gla_scan_vec_kernel(const T* __restri
     const size_t head_q = (size_t)q_off + h * D + d0, head_k = (size_t)k_off + h * D + d0;
     {
         const T* row = proj + (size_t)t0 * ld;
-        const float* ar = decay + ((size_t)t0 * H + h) * D + d0;
+        const float* ar = decay + (size_t)t0 * ldd + h * D + d0;
 #pragma unroll
         for (int i = 0; i < NQ; ++i)
             if (i < nq) {
@@ -126,7 +128,7 @@ __global__ __launch_bounds__(TM_WAVE) void gla_scan_vec_kernel(const T* __restri
         const int tn = t + 1 < t1 ? t + 1 : t;            // the last token asks for itself again
         {
             const T* row = proj + (size_t)tn * ld;
-            const float* ar = decay + ((size_t)tn * H + h) * D + d0;
+            const float* ar = decay + (size_t)tn * ldd + h * D + d0;
 #pragma unroll
             for (int i = 0; i < NQ; ++i)
                 if (i < nq) {
@@ -184,14 +186,14 @@ static bool gla_scan_in_pieces(const void* proj, int ld, int q_off, int k_off, c
 }
 
 template <typename T>
-static int launch_gla_scan(const void* proj, int ld, int q_off, int k_off, int v_off, const float* decay, float* o, float* state,
-                           const int* cu, const int* slots, int S, int H, int D, int Dv, float q_scale, hipStream_t stream) {
+static int launch_gla_scan(const void* proj, int ld, int q_off, int k_off, int v_off, const float* decay, int ldd, float* o,
+                           float* state, const int* cu, const int* slots, int S, int H, int D, int Dv, float q_scale, hipStream_t stream) {
     const dim3 grid((Dv + GLA_COLS - 1) / GLA_COLS, H, S);
     const int R = (D + GLA_PARTS - 1) / GLA_PARTS;
     // o == nullptr: only the states are wanted (the first scan of a portion in segments)
 #define GLA_VEC(RM, P, OUT_)                                                                                                     \
     gla_scan_vec_kernel<T, RM, P, OUT_><<<dim3((Dv + TM_WAVE / P - 1) / (TM_WAVE / P), H, S), TM_WAVE, 0, stream>>>(              \
-        (const T*)proj, ld, q_off, k_off, v_off, decay, o, state, cu, slots, H, D, Dv, q_scale)
+        (const T*)proj, ld, q_off, k_off, v_off, decay, ldd, o, state, cu, slots, H, D, Dv, q_scale)
     if (D / 8 <= 32 && gla_scan_in_pieces<T>(proj, ld, q_off, k_off, decay, D, 8)) {           // eight lanes a column
         if (D / 8 <= 16) { if (o) GLA_VEC(16, 8, true); else GLA_VEC(16, 8, false); }
         else { if (o) GLA_VEC(32, 8, true); else GLA_VEC(32, 8, false); }
@@ -207,13 +209,13 @@ static int launch_gla_scan(const void* proj, int ld, int q_off, int k_off, int v
 #undef GLA_VEC
     if (!o) return TM_ERR_ARG;                                  // the scan without results exists for rows in 16-byte pieces only
     if (R <= 16)
-        gla_scan_kernel<T, 16><<<grid, TM_WAVE, 0, stream>>>((const T*)proj, ld, q_off, k_off, v_off, decay, o, state, cu, slots, H,
+        gla_scan_kernel<T, 16><<<grid, TM_WAVE, 0, stream>>>((const T*)proj, ld, q_off, k_off, v_off, decay, ldd, o, state, cu, slots, H,
                                                             D, Dv, q_scale);
     else if (R <= 32)
-        gla_scan_kernel<T, 32><<<grid, TM_WAVE, 0, stream>>>((const T*)proj, ld, q_off, k_off, v_off, decay, o, state, cu, slots, H,
+        gla_scan_kernel<T, 32><<<grid, TM_WAVE, 0, stream>>>((const T*)proj, ld, q_off, k_off, v_off, decay, ldd, o, state, cu, slots, H,
                                                             D, Dv, q_scale);
     else
-        gla_scan_kernel<T, 64><<<grid, TM_WAVE, 0, stream>>>((const T*)proj, ld, q_off, k_off, v_off, decay, o, state, cu, slots, H,
+        gla_scan_kernel<T, 64><<<grid, TM_WAVE, 0, stream>>>((const T*)proj, ld, q_off, k_off, v_off, decay, ldd, o, state, cu, slots, H,
                                                             D, Dv, q_scale);
     TM_CHECK_LAUNCH();
     return TM_OK;
@@ -234,17 +236,17 @@ extern "C" int tm_gla_scan_in_pieces(int dtype, const void* proj, int ld, int q_
 }
 
 // proj rows hold q [H, D] at q_off, k [H, D] at k_off, v [H, Dv] at v_off (element offsets into a row of ld elements);
-// decay float32 [T, H, D]; o float32 [T, H, Dv]; state float32 [slots, H, D, Dv]; request s of the step owns rows
+// decay float32 [T, H, D] (rows ldd = H * D apart), or with ldd = 0 one row [H, D] for every token; o float32 [T, H, Dv]; state float32 [slots, H, D, Dv]; request s of the step owns rows
 // cu_q_lens[s] .. cu_q_lens[s + 1] - 1 and the state row state_slots[s].
-extern "C" int tm_gla_scan(const void* proj, int ld, int q_off, int k_off, int v_off, int dtype, const float* decay, float* o,
+extern "C" int tm_gla_scan(const void* proj, int ld, int q_off, int k_off, int v_off, int dtype, const float* decay, int ldd, float* o,
                            float* state, const int* cu_q_lens, const int* state_slots, int S, int H, int D, int Dv,
                            float q_scale, hipStream_t stream) {
     if (S <= 0) return TM_OK;
     if (H <= 0 || D <= 0 || D > 256 || Dv <= 0 || H > 65535 || S > 65535 || !proj || !decay || !state || !cu_q_lens ||
-        !state_slots || q_off < 0 || k_off < 0 || v_off < 0 || ld < q_off + H * D || ld < k_off + H * D || ld < v_off + H * Dv)
+        !state_slots || (ldd != 0 && ldd != H * D) || q_off < 0 || k_off < 0 || v_off < 0 || ld < q_off + H * D || ld < k_off + H * D || ld < v_off + H * Dv)
         return TM_ERR_ARG;
-    if (dtype == TM_F32) return launch_gla_scan<float>(proj, ld, q_off, k_off, v_off, decay, o, state, cu_q_lens, state_slots, S, H, D, Dv, q_scale, stream);
-    if (dtype == TM_BF16) return launch_gla_scan<bf16_t>(proj, ld, q_off, k_off, v_off, decay, o, state, cu_q_lens, state_slots, S, H, D, Dv, q_scale, stream);
+    if (dtype == TM_F32) return launch_gla_scan<float>(proj, ld, q_off, k_off, v_off, decay, ldd, o, state, cu_q_lens, state_slots, S, H, D, Dv, q_scale, stream);
+    if (dtype == TM_BF16) return launch_gla_scan<bf16_t>(proj, ld, q_off, k_off, v_off, decay, ldd, o, state, cu_q_lens, state_slots, S, H, D, Dv, q_scale, stream);
     return TM_ERR_ARG;
 }
 
@@ -252,7 +254,7 @@ extern "C" int tm_gla_scan(const void* proj, int ld, int q_off, int k_off, int v
 template <typename T>
 __global__ __launch_bounds__(TM_WAVE) void gla_out_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate, int ldg,
                                                               const float* __restrict__ w, T* __restrict__ y, int H, int Dv,
-                                                              float eps) {
+                                                              float eps, int sigmoid) {
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const float* orow = o + ((size_t)t * H + h) * Dv;
     const T* grow = gate + (size_t)t * ldg + (size_t)h * Dv;
@@ -263,19 +265,20 @@ __global__ __launch_bounds__(TM_WAVE) void gla_out_gate_kernel(const float* __re
     const float r = 1.0f / sqrtf(ss / (float)Dv + eps);
     for (int e = lane; e < Dv; e += TM_WAVE) {
         const float g = Elem<T>::load(grow + e);
-        Elem<T>::store(yrow + e, (w[e] * (orow[e] * r)) * (g / (1.f + expf(-g))));
+        const float v = w ? w[e] * (orow[e] * r) : orow[e] * r;
+        Elem<T>::store(yrow + e, v * ((sigmoid ? 1.f : g) / (1.f + expf(-g))));
     }
 }
 
 extern "C" int tm_gla_out_gate(const float* o, const void* gate, int ldg, int dtype, const float* w, void* y, int T, int H, int Dv,
-                               float eps, hipStream_t stream) {
+                               float eps, int sigmoid, hipStream_t stream) {
     if (T <= 0) return TM_OK;
-    if (H <= 0 || H > 65535 || Dv <= 0 || ldg < H * Dv || !o || !gate || !w || !y || !(eps > 0.f)) return TM_ERR_ARG;
+    if (H <= 0 || H > 65535 || Dv <= 0 || ldg < H * Dv || !o || !gate || !y || !(eps > 0.f)) return TM_ERR_ARG;
     const dim3 grid(T, H);
     if (dtype == TM_F32)
-        gla_out_gate_kernel<float><<<grid, TM_WAVE, 0, stream>>>(o, (const float*)gate, ldg, w, (float*)y, H, Dv, eps);
+        gla_out_gate_kernel<float><<<grid, TM_WAVE, 0, stream>>>(o, (const float*)gate, ldg, w, (float*)y, H, Dv, eps, sigmoid);
     else if (dtype == TM_BF16)
-        gla_out_gate_kernel<bf16_t><<<grid, TM_WAVE, 0, stream>>>(o, (const bf16_t*)gate, ldg, w, (bf16_t*)y, H, Dv, eps);
+        gla_out_gate_kernel<bf16_t><<<grid, TM_WAVE, 0, stream>>>(o, (const bf16_t*)gate, ldg, w, (bf16_t*)y, H, Dv, eps, sigmoid);
     else
         return TM_ERR_ARG;
     TM_CHECK_LAUNCH();
@@ -331,12 +334,12 @@ extern "C" int tm_gla_gate_decay(const void* x, int ldx, const void* W, const vo
 // and then every segment is scanned again from its true start B_c, all segments at once (tm_gla_scan once more).
 // The chain over tokens becomes a chain over segments plus two scans that fill the chip.
 // ------------------------------------------------------------------------------------------------------------------
-__global__ __launch_bounds__(256) void gla_segment_decay_kernel(const float* __restrict__ decay, const int* __restrict__ cu_seg,
+__global__ __launch_bounds__(256) void gla_segment_decay_kernel(const float* __restrict__ decay, int ldd, const int* __restrict__ cu_seg,
                                                                float* __restrict__ P, int HD) {
     const int j = blockIdx.x * 256 + threadIdx.x, c = blockIdx.y;
     if (j >= HD) return;
     float p = 1.f;
-    for (int t = cu_seg[c]; t < cu_seg[c + 1]; ++t) p *= decay[(size_t)t * HD + j];
+    for (int t = cu_seg[c]; t < cu_seg[c + 1]; ++t) p *= decay[(size_t)t * ldd + j];
     P[(size_t)c * HD + j] = p;
 }
 
@@ -360,10 +363,10 @@ __global__ __launch_bounds__(256) void gla_combine_kernel(float* __restrict__ st
     *st = S;
 }
 
-extern "C" int tm_gla_segment_decay(const float* decay, const int* cu_seg, float* P, int n_seg, int HD, hipStream_t stream) {
+extern "C" int tm_gla_segment_decay(const float* decay, int ldd, const int* cu_seg, float* P, int n_seg, int HD, hipStream_t stream) {
     if (n_seg <= 0) return TM_OK;
-    if (!decay || !cu_seg || !P || HD <= 0 || n_seg > 65535) return TM_ERR_ARG;
-    gla_segment_decay_kernel<<<dim3((HD + 255) / 256, n_seg), 256, 0, stream>>>(decay, cu_seg, P, HD);
+    if (!decay || !cu_seg || !P || HD <= 0 || n_seg > 65535 || (ldd != 0 && ldd != HD)) return TM_ERR_ARG;
+    gla_segment_decay_kernel<<<dim3((HD + 255) / 256, n_seg), 256, 0, stream>>>(decay, ldd, cu_seg, P, HD);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }

@@ -53,6 +53,7 @@ struct TmAttentionOp {          // resid += o(attention(rope(qkv(norm(resid)))))
     int write;                  // 0: this call reads a cache that another call writes
     float softcap;              // > 0: a scaled score s becomes softcap * tanh(s / softcap) before the softmax
     int outside;                // 1: q always comes projected, encoded and stored (TmStream.qkv); `qkv` and `norm` are not looked at
+    const float* sink;          // [H]: one more term exp(sink[h]) in the denominator of head h's softmax, with no key behind it; or null
 };
 
 struct TmFfnOp {                // resid += down(silu(gate(n)) * up(n)), n = norm(resid)

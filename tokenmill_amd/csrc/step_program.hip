@@ -357,17 +357,17 @@ struct Run {
                     HD % 4 == 0 && aligned(attn, 8)) {
                     ++p->taken[TM_PREFILL_SHARED_KEYS];
                     rc = tm_attn_prefill_shared_cap(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->prefill_tiles,
-                                                    s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.softcap, stream);
+                                                    s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.softcap, a.sink, stream);
                 } else {
                     ++p->taken[TM_PREFILL_SPLIT_KEYS];
                     rc = tm_attn_prefill_mfma_cap(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->prefill_tiles,
-                                                  s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.softcap, stream);
+                                                  s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.softcap, a.sink, stream);
                 }
                 done_prefill = true;
             } else if (tp && s->n_tiles > 0 && s->prefill_tiles && dtype == TM_F32 && a.D % 16 == 0 && a.D >= 16 &&
                        a.D <= 128 && page_ok && q_stride % 4 == 0 && aligned(q, 16)) {
                 rc = tm_attn_prefill_f32_cap(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->prefill_tiles, s->n_tiles, a.H,
-                                             a.KVH, a.D, a.page, a.scale, a.window, a.softcap, stream);
+                                             a.KVH, a.D, a.page, a.scale, a.window, a.softcap, a.sink, stream);
                 done_prefill = true;
             }
             if (rc) return rc;
@@ -378,20 +378,20 @@ struct Run {
                 rc = tm_attn_decode_mfma_cap(q_dec, q_stride, out_dec, HD, a.k_pool, a.v_pool, tables + (size_t)(S - nd) * W, W,
                                              s->context_lens + (S - nd), split ? part_o : nullptr, split ? part_ml : nullptr,
                                              tm_decode_chunks(s->max_decode_context), nd, a.H, a.KVH, a.D, a.page, a.scale, a.window,
-                                             a.softcap, stream);
+                                             a.softcap, a.sink, stream);
                 done_decode = true;
             }
             if (rc) return rc;
             if (tp && !done_prefill && nd && !done_decode) {
                 rc = tm_attn_paged_generic_ext(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->seq_of_token, s->positions, T,
-                                               a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.softcap, nullptr, 0, dtype, stream);
+                                               a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.softcap, nullptr, 0, a.sink, dtype, stream);
             } else {
                 if (tp && !done_prefill)
                     rc = tm_attn_paged_generic_ext(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->seq_of_token, s->positions,
-                                                   tp, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.softcap, nullptr, 0, dtype, stream);
+                                                   tp, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.softcap, nullptr, 0, a.sink, dtype, stream);
                 if (!rc && nd && !done_decode)
                     rc = tm_attn_paged_generic_ext(q_dec, q_stride, out_dec, HD, a.k_pool, a.v_pool, tables, W, s->seq_of_token + tp,
-                                                   s->positions + tp, nd, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.softcap, nullptr, 0,
+                                                   s->positions + tp, nd, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.softcap, nullptr, 0, a.sink,
                                                    dtype, stream);
             }
             if (rc) return rc;

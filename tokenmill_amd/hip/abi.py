@@ -31,7 +31,7 @@ class TmAttentionOp(Structure):
     _fields_ = [("norm", TmNorm), ("qkv", TmLinear), ("o", TmLinear), ("cos_t", c_void_p), ("sin_t", c_void_p),
                 ("k_pool", c_void_p), ("v_pool", c_void_p), ("H", c_int), ("KVH", c_int), ("D", c_int), ("scale", c_float),
                 ("window", c_int), ("rot", c_int), ("max_positions", c_int), ("page", c_int), ("group", c_int),
-                ("write", c_int), ("softcap", c_float), ("outside", c_int)]
+                ("write", c_int), ("softcap", c_float), ("outside", c_int), ("sink", c_void_p)]
 
 
 class TmFfnOp(Structure):

@@ -604,14 +604,15 @@ def attn_decode_mfma_supported(dtype, H: int, KVH: int, D: int, page: int) -> bo
 def attn_decode_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                      block_tables: torch.Tensor, context_lens: torch.Tensor, H: int, KVH: int, D: int, scale: float,
                      window: int, max_context: int, workspace: tuple[torch.Tensor, torch.Tensor] | None = None,
-                     split: bool | None = None, softcap: float = 0.0):
+                     split: bool | None = None, softcap: float = 0.0, sink: torch.Tensor | None = None):
     """Attention of one new token per request over its cache (the token's own key included); ``softcap`` > 0: a scaled
-    score s becomes softcap * tanh(s / softcap).
+    score s becomes softcap * tanh(s / softcap); ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator.
     q: [S, >= H*D] rows (unit inner stride), out [S, H*D] view; block_tables int32 [S, W];
     context_lens int32 [S] (new token counted); max_context >= every context length. ``split``: None runs
     the kernel the library's rule names for this many requests (contexts split over blocks and merged, or one
     block a request and kv head); True / False name it (each kernel alone, in tests)."""
-    _gpu(q, out, k_pool, v_pool, block_tables, context_lens)
+    _gpu(q, out, k_pool, v_pool, block_tables, context_lens, sink)
+    _check_sink(sink, H)
     S = q.shape[0]
     page = _check_pools(k_pool, v_pool, KVH, D, torch.bfloat16, "attn_decode")
     _need(attn_decode_mfma_supported(q.dtype, H, KVH, D, page), "attn_decode: unsupported head size, group or page size")
@@ -642,7 +643,7 @@ def attn_decode_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v
     _check(library().tm_attn_decode_mfma_cap(_p(q), c_int(q_stride), _p(out), c_int(out_stride), _p(k_pool), _p(v_pool),
                                              _p(block_tables), c_int(W), _p(context_lens), _p(part_o), _p(part_ml),
                                              c_int(chunks), c_int(S), c_int(H), c_int(KVH), c_int(D), c_int(page),
-                                             c_float(scale), c_int(window), c_float(softcap), _stream()), "attn_decode_mfma")
+                                             c_float(scale), c_int(window), c_float(softcap), _p(sink), _stream()), "attn_decode_mfma")
     return out
 
 
@@ -656,13 +657,15 @@ def attn_prefill_mfma_supported(dtype, H: int, KVH: int, D: int, page: int) -> b
 
 def attn_prefill_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                       block_tables: torch.Tensor, tiles: torch.Tensor, H: int, KVH: int, D: int, scale: float,
-                      window: int, shared: bool = False, softcap: float = 0.0) -> torch.Tensor:
-    """Attention of prompt portions over the cache (``softcap`` > 0: a scaled score s becomes softcap * tanh(s / softcap)). q: [T, >= H*D] rows, out [T, H*D]; tiles int32
+                      window: int, shared: bool = False, softcap: float = 0.0, sink: torch.Tensor | None = None) -> torch.Tensor:
+    """Attention of prompt portions over the cache (``softcap`` > 0: a scaled score s becomes softcap * tanh(s / softcap);
+    ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator). q: [T, >= H*D] rows, out [T, H*D]; tiles int32
     [n, 4] = (request index, first row, tokens (1..16), position of the first token) cover the rows
     to compute; every row of a tile belongs to one request at consecutive positions. ``shared``: the kernel
     that stages a tile's keys and values through LDS for all heads of a kv head, instead of the one whose
     wavefronts split the key blocks (each kernel alone, in tests; a step's choice is the library's)."""
-    _gpu(q, out, k_pool, v_pool, block_tables, tiles)
+    _gpu(q, out, k_pool, v_pool, block_tables, tiles, sink)
+    _check_sink(sink, H)
     T = q.shape[0]
     page = _check_pools(k_pool, v_pool, KVH, D, torch.bfloat16, "attn_prefill")
     _need(attn_prefill_mfma_supported(q.dtype, H, KVH, D, page), "attn_prefill: unsupported head size or page size")
@@ -684,7 +687,7 @@ def attn_prefill_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, 
     _check(entry(_p(q), c_int(q_stride), _p(out), c_int(out_stride), _p(k_pool), _p(v_pool),
                  _p(block_tables), c_int(block_tables.shape[1]), _p(tiles),
                  c_int(tiles.shape[0]), c_int(H), c_int(KVH), c_int(D), c_int(page),
-                 c_float(scale), c_int(window), c_float(softcap), _stream()), "attn_prefill_shared" if shared else "attn_prefill_mfma")
+                 c_float(scale), c_int(window), c_float(softcap), _p(sink), _stream()), "attn_prefill_shared" if shared else "attn_prefill_mfma")
     return out
 
 
@@ -695,10 +698,11 @@ def attn_prefill_f32_supported(dtype, H: int, KVH: int, D: int, page: int) -> bo
 
 def attn_prefill_f32(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                      block_tables: torch.Tensor, tiles: torch.Tensor, H: int, KVH: int, D: int, scale: float,
-                     window: int, softcap: float = 0.0) -> torch.Tensor:
+                     window: int, softcap: float = 0.0, sink: torch.Tensor | None = None) -> torch.Tensor:
     """Attention of prompt portions over the cache in true 32-bit (32-bit MFMA). Operands as for
     ``attn_prefill_mfma``, all float32."""
-    _gpu(q, out, k_pool, v_pool, block_tables, tiles)
+    _gpu(q, out, k_pool, v_pool, block_tables, tiles, sink)
+    _check_sink(sink, H)
     T = q.shape[0]
     page = _check_pools(k_pool, v_pool, KVH, D, torch.float32, "attn_prefill_f32")
     _need(attn_prefill_f32_supported(q.dtype, H, KVH, D, page), "attn_prefill_f32: unsupported head size or page size")
@@ -715,7 +719,7 @@ def attn_prefill_f32(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v
     _check(library().tm_attn_prefill_f32_cap(_p(q), c_int(q_stride), _p(out), c_int(out_stride), _p(k_pool), _p(v_pool),
                                              _p(block_tables), c_int(block_tables.shape[1]), _p(tiles),
                                              c_int(tiles.shape[0]), c_int(H), c_int(KVH), c_int(D), c_int(page),
-                                             c_float(scale), c_int(window), c_float(softcap), _stream()), "attn_prefill_f32")
+                                             c_float(scale), c_int(window), c_float(softcap), _p(sink), _stream()), "attn_prefill_f32")
     return out
 
 
@@ -1188,7 +1192,7 @@ def gla_scan(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torc
              cu_q_lens: torch.Tensor, state_slots: torch.Tensor, num_seqs: int, H: int, D: int, Dv: int, q_scale: float) -> torch.Tensor:
     """The recurrence S = diag(decay_t) S + k_t v_t^T, o_t = S^T (q_scale * q_t) over the rows of each request of the
     step in order, from and to the request's state row (``o`` None where ``gla_scan_states_only``: the states alone). proj [T, ld] holds q, k [H*D] and v [H*Dv] at the given column
-    offsets; decay float32 [T, H*D]; o float32 [T, H*Dv]; state float32 [slots, H, D, Dv]; cu_q_lens int32 [S+1];
+    offsets; decay float32 [T, H*D] (or [1, H*D]: every token's); o float32 [T, H*Dv]; state float32 [slots, H, D, Dv]; cu_q_lens int32 [S+1];
     state_slots int32 [S]."""
     _gpu(proj, decay, o, state, cu_q_lens, state_slots)
     T, ld_cols = proj.shape
@@ -1196,7 +1200,8 @@ def gla_scan(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torc
     _need(0 < D <= 256 and Dv > 0 and H > 0, "gla_scan: key size up to 256")
     for off, n in ((q_off, H * D), (k_off, H * D), (v_off, H * Dv)):
         _need(0 <= off and off + n <= ld_cols, "gla_scan: q, k, v lie inside a row of proj")
-    _need(decay.dtype == torch.float32 and decay.is_contiguous() and tuple(decay.shape) == (T, H * D), f"gla_scan: decay float32 [{T}, {H * D}]")
+    _need(decay.dtype == torch.float32 and decay.is_contiguous() and decay.shape[0] in (T, 1) and decay.shape[1] == H * D,
+          f"gla_scan: decay float32 [{T}, {H * D}] or [1, {H * D}]")
     if o is not None:
         _need(o.dtype == torch.float32 and o.is_contiguous() and tuple(o.shape) == (T, H * Dv), f"gla_scan: o float32 [{T}, {H * Dv}]")
     else:
@@ -1208,24 +1213,26 @@ def gla_scan(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, decay: torc
     _need(num_seqs <= 65535, "gla_scan: at most 65,535 requests a step")
     ld = proj.stride(0) if T > 1 else max(ld_cols, proj.stride(0))
     _check(library().tm_gla_scan(_p(proj), c_int(ld), c_int(q_off), c_int(k_off), c_int(v_off), c_int(code(proj.dtype)), _p(decay),
-                                 _p(o), _p(state), _p(cu_q_lens), _p(state_slots), c_int(num_seqs), c_int(H), c_int(D), c_int(Dv),
+                                 c_int(0 if decay.shape[0] == 1 else H * D), _p(o), _p(state), _p(cu_q_lens), _p(state_slots), c_int(num_seqs), c_int(H), c_int(D), c_int(Dv),
                                  c_float(q_scale), _stream()), "gla_scan")
     return o
 
 
-def gla_out_gate(o: torch.Tensor, gate: torch.Tensor, w: torch.Tensor, y: torch.Tensor, H: int, Dv: int, eps: float) -> torch.Tensor:
-    """y[t, h] = w * o[t, h] / rms(o[t, h]) * silu(gate[t, h]). o float32 [T, H*Dv]; gate [T, >= H*Dv] (a view with unit
+def gla_out_gate(o: torch.Tensor, gate: torch.Tensor, w: torch.Tensor | None, y: torch.Tensor, H: int, Dv: int, eps: float,
+                 sigmoid: bool = False) -> torch.Tensor:
+    """y[t, h] = w * o[t, h] / rms(o[t, h]) * silu(gate[t, h]) (``sigmoid``: * sigmoid(gate); w None: no weight). o float32 [T, H*Dv]; gate [T, >= H*Dv] (a view with unit
     inner stride) and y [T, H*Dv] of the model's type; w float32 [Dv]."""
     _gpu(o, gate, w, y)
     T = o.shape[0]
     _need(o.dtype == torch.float32 and o.is_contiguous() and tuple(o.shape) == (T, H * Dv), f"gla_out_gate: o float32 [{T}, {H * Dv}]")
     _need(gate.stride(1) == 1 and gate.shape[0] == T and gate.shape[1] >= H * Dv and gate.dtype == y.dtype, "gla_out_gate: gate [T, >= H*Dv] of y's type")
     _need(y.is_contiguous() and tuple(y.shape) == (T, H * Dv), f"gla_out_gate: y [{T}, {H * Dv}]")
-    _need(w.dtype == torch.float32 and tuple(w.shape) == (Dv,) and w.is_contiguous(), f"gla_out_gate: w float32 [{Dv}]")
+    if w is not None:
+        _need(w.dtype == torch.float32 and tuple(w.shape) == (Dv,) and w.is_contiguous(), f"gla_out_gate: w float32 [{Dv}]")
     _need(eps > 0, "gla_out_gate: eps must be positive")
     ldg = gate.stride(0) if T > 1 else max(gate.stride(0), H * Dv)
     _check(library().tm_gla_out_gate(_p(o), _p(gate), c_int(ldg), c_int(code(y.dtype)), _p(w), _p(y), c_int(T), c_int(H), c_int(Dv),
-                                     c_float(eps), _stream()), "gla_out_gate")
+                                     c_float(eps), c_int(1 if sigmoid else 0), _stream()), "gla_out_gate")
     return y
 
 
@@ -1281,14 +1288,14 @@ def gla_gate_decay(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None, 
 
 
 def gla_segment_decay(decay: torch.Tensor, cu_seg: torch.Tensor, n_seg: int, out: torch.Tensor) -> torch.Tensor:
-    """out[c, j] = product over the rows cu_seg[c] .. cu_seg[c + 1] - 1 of decay[t, j]. decay float32 [T, HD]."""
+    """out[c, j] = product over the rows cu_seg[c] .. cu_seg[c + 1] - 1 of decay[t, j]. decay float32 [T, HD] (or [1, HD]: every row's)."""
     _gpu(decay, cu_seg, out)
     T, HD = decay.shape
     _need(decay.dtype == torch.float32 and decay.is_contiguous(), "gla_segment_decay: decay is contiguous float32 [T, HD]")
     _need(out.dtype == torch.float32 and out.is_contiguous() and tuple(out.shape) == (n_seg, HD), f"gla_segment_decay: out float32 [{n_seg}, {HD}]")
     _ints(cu_seg, n_seg + 1, "cu_seg")
     _need(n_seg <= 65535, "gla_segment_decay: at most 65,535 segments")
-    _check(library().tm_gla_segment_decay(_p(decay), _p(cu_seg), _p(out), c_int(n_seg), c_int(HD), _stream()), "gla_segment_decay")
+    _check(library().tm_gla_segment_decay(_p(decay), c_int(0 if T == 1 else HD), _p(cu_seg), _p(out), c_int(n_seg), c_int(HD), _stream()), "gla_segment_decay")
     return out
 
 
@@ -1700,16 +1707,21 @@ def moe_experts(x: torch.Tensor, routed, w_gate_up: torch.Tensor, w_down: torch.
 def whole_norm_rope_store(proj: torch.Tensor, q_out: torch.Tensor, H: int, G: int, D: int, Dv: int, q_w: torch.Tensor | None,
                           k_w: torch.Tensor | None, eps: float, cos: torch.Tensor | None, sin: torch.Tensor | None, interleaved: bool,
                           positions: torch.Tensor | None, slots: torch.Tensor | None, k_pool: torch.Tensor | None,
-                          v_pool: torch.Tensor | None, has_kv: bool = True, per_head: bool = False) -> torch.Tensor:
+                          v_pool: torch.Tensor | None, has_kv: bool = True, per_head: bool = False, unit: bool = False,
+                          v_is_k: bool = False) -> torch.Tensor:
     """proj float32 [T, >= H*D (+ G*D + G*Dv)]: q (and k) are divided by the root mean square of the whole projection (all
     heads of a token at once) and multiplied by q_w [H*D] / k_w [G*D] (float32; None: no norm), the first 2 * cos.shape[1]
     channels of every head rotated by the token's position (pairs (j, j + rot/2), or (2j, 2j + 1) if ``interleaved``); q goes
     to q_out [T, H*D], k and v to the tokens' cache slots. ``has_kv`` False: the row holds no k and v (a layer that reads
     another layer's cache). ``per_head``: every head of q and of k is normed by itself over its D channels, with weights [D] that
-    the heads share."""
+    the heads share. ``unit``: q and k are normed without weights. ``v_is_k``: the row holds no v; a value is the projected k
+    before its norm and rotation (D = Dv)."""
     _gpu(proj, q_out, q_w, k_w, cos, sin, positions, slots, k_pool, v_pool)
     T = proj.shape[0]
-    width = H * D + (G * (D + Dv) if has_kv else 0)
+    width = H * D + (G * (D if v_is_k else D + Dv) if has_kv else 0)
+    _need(not v_is_k or (has_kv and D == Dv), "whole_norm_rope_store: values that are the keys have the keys' size")
+    _need(not unit or (q_w is None and k_w is None), "whole_norm_rope_store: a norm without weights has none")
+    _need(eps > 0, "whole_norm_rope_store: eps must be positive")
     _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= width,
           f"whole_norm_rope_store: proj is float32 [T, >= {width}]")
     _need(tuple(q_out.shape) == (T, H * D) and q_out.is_contiguous(), f"whole_norm_rope_store: q_out is contiguous [T, {H * D}]")
@@ -1734,18 +1746,21 @@ def whole_norm_rope_store(proj: torch.Tensor, q_out: torch.Tensor, H: int, G: in
                                               c_int(D), c_int(Dv), c_int(rot), c_int(1 if interleaved else 0), _p(q_w), _p(k_w),
                                               c_float(eps), _p(cos), _p(sin), _p(positions), _p(slots if write else None),
                                               _p(k_pool if write else None), _p(v_pool if write else None), c_int(page),
-                                              c_int(1 if has_kv else 0), c_int(1 if per_head else 0), _stream()), "whole_norm_rope_store")
+                                              c_int(1 if has_kv else 0), c_int(1 if per_head else 0), c_int(1 if unit else 0),
+                                              c_int(1 if v_is_k else 0), _stream()), "whole_norm_rope_store")
     return q_out
 
 
 def attn_paged_softmax(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, block_tables: torch.Tensor,
                        seq_of_token: torch.Tensor, positions: torch.Tensor, H: int, G: int, D: int, Dv: int, scale: float,
-                       window: int = 0, softcap: float = 0.0, gate: torch.Tensor | None = None) -> torch.Tensor:
+                       window: int = 0, softcap: float = 0.0, gate: torch.Tensor | None = None,
+                       sink: torch.Tensor | None = None) -> torch.Tensor:
     """Softmax attention of every token of the step over its request's cached keys (its own included), a token and a head a
     wavefront: keys of D channels, values of Dv; a score s becomes softcap * tanh(s / softcap) if ``softcap`` > 0; head h of
-    token t is multiplied by sigmoid(gate[t, h]) (gate: a float32 view [T, >= H] with unit inner stride; None: no gate).
-    q [T, >= H*D] with unit inner stride, out [T, H*Dv]."""
-    _gpu(q, out, k_pool, v_pool, block_tables, seq_of_token, positions, gate)
+    token t is multiplied by sigmoid(gate[t, h]) (gate: a float32 view [T, >= H] with unit inner stride; None: no gate);
+    ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator. q [T, >= H*D] with unit inner stride, out [T, H*Dv]."""
+    _gpu(q, out, k_pool, v_pool, block_tables, seq_of_token, positions, gate, sink)
+    _check_sink(sink, H)
     T = q.shape[0]
     _need(q.stride(1) == 1 and q.shape[1] >= H * D and out.is_contiguous() and tuple(out.shape) == (T, H * Dv),
           f"attention: q [T, >={H * D}] unit inner stride, out contiguous [T, {H * Dv}]")
@@ -1766,7 +1781,7 @@ def attn_paged_softmax(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor,
     _check(library().tm_attn_paged_generic_ext(_p(q), c_int(q_stride), _p(out), c_int(H * Dv), _p(k_pool), _p(v_pool), _p(block_tables),
                                                c_int(block_tables.shape[1]), _p(seq_of_token), _p(positions), c_int(T), c_int(H),
                                                c_int(G), c_int(D), c_int(Dv), c_int(page), c_float(scale), c_int(window),
-                                               c_float(softcap), _p(gate), c_int(ldg), code(q.dtype), _stream()), "attn_paged_generic_ext")
+                                               c_float(softcap), _p(gate), c_int(ldg), _p(sink), code(q.dtype), _stream()), "attn_paged_generic_ext")
     return out
 
 
@@ -1869,20 +1884,23 @@ DELTA_MAX_KEY_DIM = 256
 DELTA_MAX_CHANNELS = 1 << 22        # convolved channels of a token (q | k | v)
 
 
-def delta_row_width(H: int, G: int, D: int, Dv: int) -> int:
-    """Floats of a prepared row [q | k | v | beta | g | k.q], rounded up to whole 16-byte pieces."""
-    return -(-(2 * G * D + H * Dv + 2 * H + G) // 4) * 4
+def delta_row_width(H: int, G: int, D: int, Dv: int, per_channel: bool = False) -> int:
+    """Floats of a prepared row [q | k | v | beta | g | k.q], rounded up to whole 16-byte pieces; with a decay per key channel
+    [q | k | v | beta | - | k.q | g (H D)]."""
+    return -(-(2 * G * D + H * Dv + 2 * H + G + (H * D if per_channel else 0)) // 4) * 4
 
 
 def delta_prepare(proj: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Tensor | None, ba: torch.Tensor, a_log: torch.Tensor,
                   dt_bias: torch.Tensor, cu_q_lens: torch.Tensor, state_slots: torch.Tensor, seq_of_token: torch.Tensor, num_seqs: int,
-                  out: torch.Tensor, H: int, G: int, D: int, Dv: int, unit_eps: float = 1e-6) -> torch.Tensor:
+                  out: torch.Tensor, H: int, G: int, D: int, Dv: int, unit_eps: float = 1e-6, z: torch.Tensor | None = None) -> torch.Tensor:
     """The rows the delta-rule recurrence reads, from the projections of a step. proj [T, >= C] (C = 2 G D + H Dv: the q, k and v
     channels first) in the model's type; conv_w [C, taps] and conv_state [slots, taps - 1, C] of the same type (the rows before a
     request's first row of the step come from its state; the state itself is advanced by ``delta_conv_state``); ba float32
     [T, >= 2H] = [b | a]; a_log, dt_bias float32 [H]. Per token: y = silu(conv(.)), q = y_q / sqrt(sum y_q^2 + eps) / sqrt(D),
     k = y_k / sqrt(sum y_k^2 + eps), beta = sigmoid(b), g = exp(-exp(a_log) softplus(a + dt_bias)); out float32
-    [T, delta_row_width] = [q | k | v | beta | g | k.q]."""
+    [T, delta_row_width] = [q | k | v | beta | g | k.q]. With ``z`` (float32 [T, >= H D]) there is a decay per key channel,
+    g = exp(-exp(a_log_h) softplus(z + dt_bias)), dt_bias [H D]; ba then holds b alone, and out is [q | k | v | beta | - | k.q | g]."""
+    _gpu(z)
     _gpu(proj, conv_w, conv_state, ba, a_log, dt_bias, cu_q_lens, state_slots, seq_of_token, out)
     T = proj.shape[0]
     C = 2 * G * D + H * Dv
@@ -1894,19 +1912,24 @@ def delta_prepare(proj: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Te
     if taps > 1:
         _need(conv_state is not None and conv_state.dim() == 3 and tuple(conv_state.shape[1:]) == (taps - 1, C)
               and conv_state.is_contiguous() and conv_state.dtype == proj.dtype, f"delta_prepare: conv_state is [slots, {taps - 1}, {C}] of proj's type")
-    _need(ba.dtype == torch.float32 and ba.dim() == 2 and ba.shape[0] == T and ba.shape[1] >= 2 * H and ba.stride(1) == 1,
-          f"delta_prepare: ba is float32 [T, >= {2 * H}]")
-    for name, v in (("a_log", a_log), ("dt_bias", dt_bias)):
-        _need(v.dtype == torch.float32 and tuple(v.shape) == (H,) and v.is_contiguous(), f"delta_prepare: {name} is float32 [{H}]")
+    _need(ba.dtype == torch.float32 and ba.dim() == 2 and ba.shape[0] == T and ba.shape[1] >= (H if z is not None else 2 * H)
+          and ba.stride(1) == 1, f"delta_prepare: ba is float32 [T, >= {H if z is not None else 2 * H}]")
+    ldz = 0
+    if z is not None:
+        _need(z.dtype == torch.float32 and z.dim() == 2 and z.shape[0] == T and z.shape[1] >= H * D and z.stride(1) == 1,
+              f"delta_prepare: z is float32 [T, >= {H * D}]")
+        ldz = z.stride(0) if T > 1 else max(z.stride(0), z.shape[1])
+    for name, v, n in (("a_log", a_log, H), ("dt_bias", dt_bias, H * D if z is not None else H)):
+        _need(v.dtype == torch.float32 and tuple(v.shape) == (n,) and v.is_contiguous(), f"delta_prepare: {name} is float32 [{n}]")
     ldo = out.shape[1] if out.dim() == 2 else 0
-    _need(out.dtype == torch.float32 and out.dim() == 2 and out.shape[0] == T and out.is_contiguous() and ldo >= C + 2 * H + G,
-          "delta_prepare: out is contiguous float32 [T, >= C + 2H + G]")
+    _need(out.dtype == torch.float32 and out.dim() == 2 and out.shape[0] == T and out.is_contiguous()
+          and ldo >= delta_row_width(H, G, D, Dv, z is not None), "delta_prepare: out is contiguous float32 [T, delta_row_width]")
     _ints(cu_q_lens, num_seqs + 1, "cu_q_lens")
     _ints(state_slots, num_seqs, "state_slots")
     _ints(seq_of_token, T, "seq_of_token")
     ld = proj.stride(0) if T > 1 else max(proj.stride(0), proj.shape[1])
     ldba = ba.stride(0) if T > 1 else max(ba.stride(0), ba.shape[1])
-    _check(library().tm_delta_prepare(_p(proj), c_int(ld), _p(conv_w), _p(conv_state), _p(ba), c_int(ldba), _p(a_log), _p(dt_bias),
+    _check(library().tm_delta_prepare(_p(proj), c_int(ld), _p(conv_w), _p(conv_state), _p(ba), c_int(ldba), _p(z), c_int(ldz), _p(a_log), _p(dt_bias),
                                       _p(cu_q_lens), _p(state_slots), _p(seq_of_token), _p(out), c_int(ldo), c_int(T), c_int(H), c_int(G),
                                       c_int(D), c_int(Dv), c_int(taps), c_float(unit_eps), c_int(code(proj.dtype)), _stream()),
            "delta_prepare")
@@ -1929,16 +1952,17 @@ def delta_conv_state(proj: torch.Tensor, C: int, conv_state: torch.Tensor, cu_q_
 
 
 def delta_scan(rows: torch.Tensor, o: torch.Tensor | None, state: torch.Tensor, cu_q_lens: torch.Tensor, state_slots: torch.Tensor,
-               num_seqs: int, H: int, G: int, D: int, Dv: int, transitions_of: int | None = None) -> torch.Tensor | None:
+               num_seqs: int, H: int, G: int, D: int, Dv: int, transitions_of: int | None = None, per_channel: bool = False) -> torch.Tensor | None:
     """The recurrence over the rows of ``delta_prepare``, request by request in the order of the step's rows:
     S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q. state float32 [slots, H, D, Dv] (row state_slots[s] is read and
     written); o float32 [T, H * Dv], or None where only the states are wanted. ``transitions_of`` = the rows' value size: the
     values count as zero and the state has ``Dv`` columns of its own (from the identity, Dv = D, a run of tokens leaves the
-    product of its transitions g (I - beta k k^T))."""
+    product of its transitions g (I - beta k k^T)). ``per_channel``: the rows hold a decay per key channel."""
     _gpu(rows, o, state, cu_q_lens, state_slots)
     T = rows.shape[0]
     row_dv = Dv if transitions_of is None else transitions_of
-    _need(rows.dtype == torch.float32 and rows.dim() == 2 and rows.is_contiguous() and rows.shape[1] >= 2 * G * D + H * row_dv + 2 * H + G,
+    _need(rows.dtype == torch.float32 and rows.dim() == 2 and rows.is_contiguous()
+          and rows.shape[1] >= 2 * G * D + H * row_dv + 2 * H + G + (H * D if per_channel else 0),
           "delta_scan: rows are those of delta_prepare")
     if o is not None:
         _need(transitions_of is None, "delta_scan: a scan without values has no results")
@@ -1950,7 +1974,7 @@ def delta_scan(rows: torch.Tensor, o: torch.Tensor | None, state: torch.Tensor, 
     _ints(state_slots, num_seqs, "state_slots")
     _check(library().tm_delta_scan(_p(rows), c_int(rows.shape[1]), _p(o), _p(state), _p(cu_q_lens), _p(state_slots), c_int(num_seqs),
                                    c_int(H), c_int(G), c_int(D), c_int(Dv), c_int(row_dv), c_int(0 if transitions_of is not None else 1),
-                                   _stream()), "delta_scan")
+                                   c_int(1 if per_channel else 0), _stream()), "delta_scan")
     return o
 
 
@@ -1984,4 +2008,100 @@ def pair_norm_mean(a: torch.Tensor, b: torch.Tensor, wa: torch.Tensor, wb: torch
     _need(eps > 0, "pair_norm_mean: eps must be positive")
     _check(library().tm_pair_norm_mean(_p(a), _p(b), _p(wa), _p(wb), _p(out), c_int(T), c_int(W), c_float(eps), c_int(code(a.dtype)),
                                        _stream()), "pair_norm_mean")
+    return out
+
+
+# -------------------------------------------------------------------------------------------- pair embedding, sums with a norm, retention, clamped gate
+
+def embed_pairs(table: torch.Tensor, pairs: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor, cu_q_lens: torch.Tensor,
+                state_slots: torch.Tensor, seq_of_token: torch.Tensor, num_seqs: int, prev_state: torch.Tensor, out: torch.Tensor,
+                scale: float, mul_prev: int, mul_cur: int) -> torch.Tensor:
+    """out[t] = table[id_t] * scale + pairs[(id_(t-1) * mul_prev + id_t * mul_cur) mod buckets] as 32-bit rows, the last row of
+    ``pairs`` [buckets + 1, hidden] at position 0. The token before a request's first row of the step comes from ``prev_state``
+    (int32 [slots, 1]), which becomes the request's last token of the step."""
+    _gpu(table, pairs, ids, positions, cu_q_lens, state_slots, seq_of_token, prev_state, out)
+    T = ids.numel()
+    vocab, hidden = table.shape
+    _need(table.is_contiguous() and pairs.is_contiguous() and pairs.dtype == table.dtype and pairs.dim() == 2 and pairs.shape[1] == hidden
+          and pairs.shape[0] >= 2, "embed_pairs: table [V, hidden] and pairs [buckets + 1, hidden] of one type")
+    _need(out.dtype == torch.float32 and tuple(out.shape) == (T, hidden) and out.is_contiguous(), f"embed_pairs: out is float32 [{T}, {hidden}]")
+    _need(prev_state.dtype == torch.int32 and prev_state.is_contiguous() and prev_state.dim() == 2 and prev_state.shape[1] == 1,
+          "embed_pairs: prev_state is int32 [slots, 1]")
+    _ints(ids, T, "ids")
+    _ints(positions, T, "positions")
+    _ints(seq_of_token, T, "seq_of_token")
+    _ints(cu_q_lens, num_seqs + 1, "cu_q_lens")
+    _ints(state_slots, num_seqs, "state_slots")
+    _need(abs(mul_prev) < 1 << 31 and abs(mul_cur) < 1 << 31, "embed_pairs: multipliers below 2^31")
+    _check(library().tm_embed_pairs(_p(table), _p(pairs), c_int(code(table.dtype)), _p(ids), _p(positions), _p(cu_q_lens), _p(state_slots),
+                                    _p(seq_of_token), _p(prev_state), _p(out), c_int(T), c_int(hidden), c_int(vocab), c_float(scale),
+                                    c_int(pairs.shape[0] - 1), c_longlong(mul_prev), c_longlong(mul_cur), _stream()), "embed_pairs")
+    return out
+
+
+def sum_norm(resid: torch.Tensor, parts: list, w: torch.Tensor | None, out: torch.Tensor | None, eps: float,
+             rows: torch.Tensor | None = None) -> torch.Tensor | None:
+    """v = resid + sum of scale * y over ``parts`` [(y, scale), ...] (one to three, [T, hidden] of one type); with ``rows`` None
+    every row runs and v is written back to resid (float32 [T, hidden]); out = v / sqrt(mean(v^2) + eps) * w (out None: the add
+    alone). With ``rows`` (int32 [R]) only those rows are read, resid stays as it is and out is [R, hidden]."""
+    T, hidden = resid.shape
+    _need(1 <= len(parts) <= 3, "sum_norm: one to three results")
+    ys = [y for y, _ in parts]
+    _gpu(resid, w, out, rows, *ys)
+    _need(resid.dtype == torch.float32 and resid.is_contiguous(), "sum_norm: resid is contiguous float32")
+    for y in ys:
+        _need(y.is_contiguous() and tuple(y.shape) == (T, hidden) and y.dtype == ys[0].dtype, f"sum_norm: the results are contiguous [{T}, {hidden}] of one type")
+    n = T if rows is None else rows.numel()
+    if rows is not None:
+        _ints(rows, n, "rows")
+        _need(out is not None, "sum_norm: rows are only read for a norm")
+    if out is not None:
+        _need(out.is_contiguous() and tuple(out.shape) == (n, hidden) and out.dtype == ys[0].dtype, f"sum_norm: out is [{n}, {hidden}] of the results' type")
+        _need(w is not None and w.is_contiguous() and tuple(w.shape) == (hidden,), f"sum_norm: w is [{hidden}]")
+    scales = [float(s) for _, s in parts] + [0.0] * (3 - len(parts))
+    ys = ys + [None] * (3 - len(ys))
+    _check(library().tm_sum_norm(_p(resid), _p(ys[0]), c_float(scales[0]), _p(ys[1]), c_float(scales[1]), _p(ys[2]), c_float(scales[2]),
+                                 _p(rows), _p(w if out is not None else None), c_int(code(w.dtype) if w is not None else 0), _p(out),
+                                 c_int(code(parts[0][0].dtype)), c_int(n), c_int(hidden), c_float(eps), _stream()), "sum_norm")
+    return out
+
+
+def retention_row_width(H: int, D: int, Dv: int) -> int:
+    """Floats of a row [q | k | v] of a retention, rounded up to whole 16-byte pieces."""
+    return -(-H * (2 * D + Dv) // 4) * 4
+
+
+def retention_prepare(proj: torch.Tensor, cos: torch.Tensor | None, sin: torch.Tensor | None, positions: torch.Tensor, rows: torch.Tensor,
+                      H: int, D: int, Dv: int, k_scale: float) -> torch.Tensor:
+    """rows float32 [T, retention_row_width] = [q | k * k_scale | v] from proj [T, >= H (2 D + Dv)] (q, k, v in this order), the first
+    2 * cos.shape[1] channels of every head of q and k turned by the token's position (pairs half that width apart)."""
+    _gpu(proj, cos, sin, positions, rows)
+    T = proj.shape[0]
+    width = H * (2 * D + Dv)
+    _need(proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= width, f"retention_prepare: proj is [T, >= {width}]")
+    _need(rows.dtype == torch.float32 and rows.is_contiguous() and rows.dim() == 2 and rows.shape[0] == T and rows.shape[1] >= width,
+          f"retention_prepare: rows is float32 [{T}, >= {width}]")
+    rot = 0
+    if cos is not None:
+        rot = 2 * cos.shape[1]
+        _need(sin is not None and cos.dtype == sin.dtype == torch.float32 and cos.shape == sin.shape and cos.is_contiguous()
+              and sin.is_contiguous() and rot <= D, "retention_prepare: cos/sin float32 [max_pos, rot/2], rot <= D")
+    _ints(positions, T, "positions")
+    ld = proj.stride(0) if T > 1 else max(proj.stride(0), proj.shape[1])
+    _check(library().tm_retention_prepare(_p(proj), c_int(ld), c_int(code(proj.dtype)), _p(cos), _p(sin), c_int(rot), _p(positions), _p(rows),
+                                          c_int(rows.shape[1]), c_int(T), c_int(H), c_int(D), c_int(Dv), c_float(k_scale), _stream()),
+           "retention_prepare")
+    return rows
+
+
+def clamped_glu(gu: torch.Tensor, out: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
+    """out[t, i] = g sigmoid(alpha g) (u + 1), g = min(gu[t, i], limit), u = gu[t, I + i] held to +-limit, computed in 32-bit;
+    gu [T, 2I], out [T, I]."""
+    _gpu(gu, out)
+    T, two_i = gu.shape
+    _need(two_i % 2 == 0 and tuple(out.shape) == (T, two_i // 2) and gu.is_contiguous() and out.is_contiguous() and gu.dtype == out.dtype,
+          "clamped_glu: gu [T, 2I] and out [T, I] of one type, contiguous")
+    _need(limit > 0, "clamped_glu: limit must be positive")
+    _check(library().tm_clamped_glu(_p(gu), _p(out), c_int(code(gu.dtype)), c_int(T), c_int(two_i // 2), c_float(alpha), c_float(limit),
+                                    _stream()), "clamped_glu")
     return out

@@ -143,11 +143,12 @@ class StepProgram:
         return self._added(self._lib.tm_program_add_embedding(self._handle, ctypes.byref(op)), part)
 
     def attention(self, part, norm, qkv, o, rotation, cache, num_heads: int, num_kv_heads: int, head_dim: int,
-                  scale: float, window: int | None, softcap: float = 0.0) -> int | None:
+                  scale: float, window: int | None, softcap: float = 0.0, sink: torch.Tensor | None = None) -> int | None:
         """resid += o(attention(rotate(qkv(norm(resid))))) over the paged cache ``cache`` (a ``KVCacheView``).
         ``rotation``: (cos, sin, rotary width, positions) of a rotary encoding, or () for none. ``softcap`` > 0: a scaled
         score s becomes softcap * tanh(s / softcap). ``qkv`` None: the operation has no projection of its own and is only
-        ever handed q (its keys and values encoded and stored by the caller); ``norm`` is then not looked at."""
+        ever handed q (its keys and values encoded and stored by the caller); ``norm`` is then not looked at.
+        ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator of head h's softmax."""
         outside = qkv is None
         n, q, out = self._norm(None if outside else norm), (TmLinear() if outside else self._linear(qkv)), self._linear(o)
         if n is None or q is None or out is None or getattr(cache, "k", None) is None or getattr(cache, "v", None) is None:
@@ -159,10 +160,12 @@ class StepProgram:
         else:
             cos = sin = None
             rot = n_pos = 0
-        self._keep.append((cache.k, cache.v))
+        if sink is not None and (sink.dtype != torch.float32 or tuple(sink.shape) != (num_heads,) or not sink.is_contiguous() or not sink.is_cuda):
+            return None
+        self._keep.append((cache.k, cache.v, sink))
         op = TmAttentionOp(n, q, out, cos, sin, cache.k.data_ptr(), cache.v.data_ptr(), num_heads, num_kv_heads, head_dim,
                            float(scale), window or 0, rot, n_pos, cache.k.shape[1], cache.group, 1 if cache.write else 0,
-                           float(softcap or 0.0), 1 if outside else 0)
+                           float(softcap or 0.0), 1 if outside else 0, sink.data_ptr() if sink is not None else None)
         return self._added(self._lib.tm_program_add_attention(self._handle, ctypes.byref(op)), part)
 
     def feed_forward(self, part, norm, gate_up, down, intermediate: int) -> int | None:

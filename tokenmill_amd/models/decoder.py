@@ -25,12 +25,17 @@ class DecoderModel:
     def __init__(self, config, embedding: Part, layers: list, final_norm: Norm, head: Part,
                  run: list[LayerCall] | None = None,
                  names: tuple[str, str, str, str] = ("model.embed_tokens.", "model.layers.{i}.", "model.norm.", ""),
-                 ignorable: tuple[str, ...] = ()):
+                 ignorable: tuple[str, ...] = (), layer_numbers: list[int] | None = None):
+        """``layer_numbers``: what stands for {i} in the tensor names of each layer, where that is not its index here (a
+        checkpoint numbers the calls of the run list, and some calls use another's layer)."""
         self.config = config
         self.embedding, self.layers, self.final_norm, self.head = embedding, layers, final_norm, head
         self.run = run if run is not None else [LayerCall(i) for i in range(len(layers))]
         self.names = names
         self.ignorable = ignorable
+        self.layer_numbers = list(layer_numbers) if layer_numbers is not None else list(range(len(layers)))
+        if len(self.layer_numbers) != len(layers):
+            raise ValueError(f"{len(self.layer_numbers)} layer numbers for {len(layers)} layers")
         self.dtype: torch.dtype | None = None
         self.device = None
         for j, call in enumerate(self.run):
@@ -47,7 +52,7 @@ class DecoderModel:
     def _prefixed(self):
         emb, layer, norm, head = self.names
         yield self.embedding, emb
-        for i, block in enumerate(self.layers):
+        for i, block in zip(self.layer_numbers, self.layers):
             yield block, layer.format(i=i)
         yield self.final_norm, norm
         yield self.head, head
@@ -69,8 +74,11 @@ class DecoderModel:
     # --- what the cache manager must provide -------------------------------------------------------
 
     def cache_specs(self) -> list[KVCacheSpec | StateSpec | None]:
-        """One entry per run call: the cache its mixer needs, or None for a call that reads another's."""
-        return [None if c.cache_of is not None else self._cache_spec(self.layers[c.layer]) for c in self.run]
+        """One entry per run call: the cache its mixer needs, or None for a call that reads another's; and, if the embedding
+        keeps state of its own, one entry more behind them."""
+        specs = [None if c.cache_of is not None else self._cache_spec(self.layers[c.layer]) for c in self.run]
+        own = self.embedding.cache_spec() if hasattr(self.embedding, "cache_spec") else None
+        return specs + [own] if own is not None else specs
 
     @staticmethod
     def _cache_spec(layer):
@@ -88,10 +96,14 @@ class DecoderModel:
         from tokenmill_amd.hip.program import StepProgram
         program = StepProgram(self.dtype, self.embedding.hidden, self.device, tune)
         emb, head, norm = self.embedding, self.head, self.final_norm
+        state = caches[len(self.run)] if len(caches) > len(self.run) else None        # the embedding's own, if it keeps any
         if getattr(emb, "emit", lambda p: None)(program) is None:
             def embed(flow, step):
                 # an embedding that adds something by position is handed the positions too
-                rows = emb.forward(step.token_ids, step.positions) if getattr(emb, "by_position", False) else emb.forward(step.token_ids)
+                if state is not None:
+                    rows = emb.forward_step(step, state)
+                else:
+                    rows = emb.forward(step.token_ids, step.positions) if getattr(emb, "by_position", False) else emb.forward(step.token_ids)
                 flow.resid, flow.delta = rows, None
             program.foreign(emb, embed)
         for j, call in enumerate(self.run):

@@ -4,12 +4,14 @@
   * biases on q, k and v;
   * an RMS norm of q and of k over the WHOLE projection (all heads of a token at once, one weight per channel of the
     projection), before the rotation; or instead an RMS norm of every head of q and of k by itself, with one weight per
-    channel of a head that the heads share;
+    channel of a head that the heads share, or (``norm_weights`` False) without weights;
   * a rotation of the first channels of each head, pairs a half apart or neighbouring, with whatever frequencies the
     ``RotaryEmbedding`` was built with;
   * scores capped smoothly: s <- cap * tanh(s / cap);
   * a gate per head: head h of a token is multiplied by sigmoid((W_g x)_h), x the mixer's input;
   * a sliding window;
+  * a sink per head (``sink``): one more term exp(sink_h) in the softmax's denominator, with no key and no value;
+  * values that are the keys (``keys_are_values``): v = k as projected, before its norm and rotation, and no matrix of their own;
   * no keys and values of its own (``own_kv`` False): the mixer reads the cache that another layer writes, with its
     own queries.
 
@@ -35,15 +37,17 @@ class SoftmaxAttention(Mixer):
     def __init__(self, hidden: int, num_heads: int, num_kv_heads: int, head_dim: int, v_head_dim: int, scale: float,
                  rotary: RotaryEmbedding | None = None, whole_norm_eps: float | None = None, qkv_bias: bool = False,
                  softcap: float | None = None, head_gate: bool = False, window: int | None = None, own_kv: bool = True,
-                 head_norm_eps: float | None = None,
+                 head_norm_eps: float | None = None, norm_weights: bool = True, sink: bool = False, keys_are_values: bool = False,
                  names: tuple[str, str, str, str] = ("q", "k", "v", "o"),
                  extra_names: tuple[str, str, str] = ("q.norm", "k.norm", "g"),
-                 suffixes: tuple[str, str] = ("", ".b")):
+                 suffixes: tuple[str, str] = ("", ".b"), sink_name: str = "sink"):
         """``whole_norm_eps``: None for no norm of q and k over the whole projection; ``head_norm_eps``: None for no norm head
         by head (one of the two at most). ``softcap``: None or 0 for none. ``extra_names``: the checkpoint's names of the two
         norm weights and of the gate's matrix, under the mixer's prefix."""
         if whole_norm_eps is not None and head_norm_eps is not None:
             raise ValueError("q and k are normed over the whole projection or head by head, not both")
+        if keys_are_values and (head_dim != v_head_dim or not own_kv):
+            raise ValueError("values that are the keys have the keys' size, in a mixer with keys of its own")
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads do not divide into {num_kv_heads} kv heads")
         if head_dim % 4 or not 0 < head_dim <= MAX_HEAD_DIM or not 0 < v_head_dim <= MAX_HEAD_DIM:
@@ -60,11 +64,13 @@ class SoftmaxAttention(Mixer):
         self.head_norm_eps = head_norm_eps
         self.norm_eps = whole_norm_eps if whole_norm_eps is not None else head_norm_eps     # None: q and k are not normed
         self.softcap, self.window, self.own_kv = float(softcap or 0.0), window, own_kv
+        self.norm_weights, self.has_sink, self.sink_name, self.keys_are_values = norm_weights, sink, sink_name, keys_are_values
+        self.unit_norm = self.norm_eps is not None and not norm_weights
         self.q_size, self.k_size, self.v_size = num_heads * head_dim, num_kv_heads * head_dim, num_kv_heads * v_head_dim
         sizes, stacked = [self.q_size], [names[0]]
         if own_kv:
-            sizes += [self.k_size, self.v_size]
-            stacked += [names[1], names[2]]
+            sizes += [self.k_size] if keys_are_values else [self.k_size, self.v_size]
+            stacked += [names[1]] if keys_are_values else [names[1], names[2]]
         # the gate's rows ride behind q|k|v in the one product where that product has no biases (the gate has none)
         self.gate_stacked = head_gate and not qkv_bias
         self.gate_at = sum(sizes)
@@ -78,6 +84,7 @@ class SoftmaxAttention(Mixer):
         self.extra_names = extra_names
         self.q_norm: torch.Tensor | None = None
         self.k_norm: torch.Tensor | None = None
+        self.sink: torch.Tensor | None = None   # float32 [H]
         self._own: dict = {}                    # per cache: the library's attention operation as a program of its own
 
     def _linears(self):
@@ -88,7 +95,9 @@ class SoftmaxAttention(Mixer):
         for lin in self._linears():
             specs.update(lin.tensor_specs(prefix))
         qn, kn, _ = self.extra_names
-        if self.norm_eps is not None:
+        if self.has_sink:
+            specs[prefix + self.sink_name] = TensorSpec((self.num_heads,))
+        if self.norm_eps is not None and self.norm_weights:
             per_head = self.head_norm_eps is not None
             specs[prefix + qn] = TensorSpec((self.head_dim if per_head else self.q_size,), init="ones")
             if self.own_kv:
@@ -99,7 +108,8 @@ class SoftmaxAttention(Mixer):
         for lin in self._linears():
             lin.load(tensors, prefix)
         qn, kn, _ = self.extra_names
-        if self.norm_eps is not None:               # the vectors that meet 32-bit statistics are kept in 32-bit
+        self.sink = tensors[prefix + self.sink_name].float().contiguous() if self.has_sink else None
+        if self.norm_eps is not None and self.norm_weights:     # the vectors that meet 32-bit statistics are kept in 32-bit
             self.q_norm = tensors[prefix + qn].float().contiguous()
             self.k_norm = tensors[prefix + kn].float().contiguous() if self.own_kv else None
         if self.rotary is not None:
@@ -160,7 +170,7 @@ class SoftmaxAttention(Mixer):
                                       rot.cos if rot is not None else None, rot.sin if rot is not None else None,
                                       bool(rot is not None and rot.interleaved), step.positions, group.slot_mapping,
                                       cache.k if self.own_kv else None, cache.v if self.own_kv else None, has_kv=self.own_kv,
-                                      per_head=self.head_norm_eps is not None)
+                                      per_head=self.head_norm_eps is not None, unit=self.unit_norm, v_is_k=self.keys_are_values)
         if D == Dv:
             # keys and values of one size: the kernel library's own attention operation, which is handed q and chooses the
             # kernels of a step (prompt portions and single tokens on the matrix unit where it takes the sizes), then
@@ -180,7 +190,7 @@ class SoftmaxAttention(Mixer):
         if key not in self._own:
             program = StepProgram(dtype, self.hidden, cache.k.device)
             op = program.attention(self, None, None, self.o, (), cache, self.num_heads, self.num_kv_heads, self.head_dim, self.scale,
-                                   self.window, self.softcap)
+                                   self.window, self.softcap, self.sink)
             self._own[key] = (program, op, cache) if op is not None else None
         entry = self._own[key]
         return entry[:2] if entry is not None else None
@@ -189,4 +199,4 @@ class SoftmaxAttention(Mixer):
         """Keys and values of different sizes: a token and a head a wavefront."""
         H, G, D, Dv = self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim
         ops.attn_paged_softmax(q, out, cache.k, cache.v, group.block_tables, step.seq_of_token, step.positions, H, G, D, Dv,
-                               self.scale, self.window or 0, self.softcap, gate)
+                               self.scale, self.window or 0, self.softcap, gate, sink=self.sink)

@@ -239,3 +239,56 @@ class GatedResidualBlock(Block):
             from tokenmill_amd.parts.norm import GatedAdd
             GatedAdd(None, 1.0).add_normed(resid, y)
         return None
+
+
+class SharedNormBlock(Block):
+    """One norm, and both sublayers read its result:
+
+        h = norm(x);   x += mixer(h) + ffn(h)            (``ffn`` None: the mixer alone)
+
+    A mixer of several results (``forward_parts``) brings them with their weights. Everything that goes into the stream stays
+    pending together (``WeightedAdd``), so the norm of the next block adds it all and norms the sum in one kernel."""
+
+    def __init__(self, norm: Norm, mixer: Mixer, ffn: FeedForward | None = None, names: tuple[str, str, str] = ("norm1", "mix.", "mlp.")):
+        self.norm, self.mixer, self.ffn, self.names = norm, mixer, ffn, names
+
+    def _parts(self):
+        return [(p, n) for p, n in zip((self.norm, self.mixer, self.ffn), self.names) if p is not None]
+
+    def tensor_specs(self, prefix: str):
+        specs = {}
+        for part, name in self._parts():
+            specs.update(part.tensor_specs(prefix + name))
+        return specs
+
+    def load(self, tensors, prefix: str) -> None:
+        for part, name in self._parts():
+            part.load(tensors, prefix + name)
+
+    def prepare(self, pack_weights: bool) -> None:
+        for part, _ in self._parts():
+            part.prepare(pack_weights)
+
+    def _results(self, x: NormedInput, step: StepContext, cache):
+        """(first result, how it and the others go into the stream)."""
+        from tokenmill_amd.parts.norm import WeightedAdd
+        h = x.tensor()
+        split = getattr(self.mixer, "forward_parts", None)
+        parts = split(h, step, cache) if split is not None else [(self.mixer.forward(h, step, cache), 1.0)]
+        if self.ffn is not None:
+            parts = [*parts, (self.ffn.forward(h, step), 1.0)]
+        (first, scale), *others = parts
+        return first, WeightedAdd(scale, others)
+
+    def emit(self, program, cache) -> None:
+        def run(flow, step):
+            x = NormedInput(self.norm, flow.resid, flow.delta, program.dtype, delta_norm=flow.delta_norm)
+            flow.delta, flow.delta_norm = self._results(x, step, cache)
+        program.foreign(self.mixer, run)
+
+    def forward(self, resid: torch.Tensor, delta: torch.Tensor | None, step: StepContext, cache,
+                dtype: torch.dtype) -> None:
+        """The block by itself: resid float32 [T, hidden] is updated in place with everything; nothing is left pending."""
+        first, way = self._results(NormedInput(self.norm, resid, delta, dtype), step, cache)
+        way.add_normed(resid, first)
+        return None

@@ -5,7 +5,7 @@ import torch
 
 from tokenmill_amd import profiling
 from tokenmill_amd.hip import ops
-from tokenmill_amd.parts.base import Part
+from tokenmill_amd.parts.base import Part, StateSpec, StateView, StepContext
 from tokenmill_amd.parts.linear import Linear
 from tokenmill_amd.weights.loader import TensorSpec
 
@@ -24,14 +24,38 @@ class LearnedPositions(Part):
         self.weight = tensors[f"{prefix}{self.name}"]
 
 
+class PairRows(Part):
+    """A table with a row per bucket of token pairs, added (unscaled) to a token's embedding row: bucket
+    (previous token * mul_prev + token * mul_cur) mod buckets, and one row more, the last, for a request's first token. The
+    previous token is per-request state: one int32 a request, carried from step to step."""
+
+    def __init__(self, buckets: int, hidden: int, mul_prev: int, mul_cur: int, name: str = "weight"):
+        if buckets < 1:
+            raise ValueError("a table of token pairs has at least one bucket")
+        self.buckets, self.hidden, self.mul_prev, self.mul_cur, self.name = buckets, hidden, int(mul_prev), int(mul_cur), name
+        self.weight: torch.Tensor | None = None
+
+    def tensor_specs(self, prefix: str):
+        return {f"{prefix}{self.name}": TensorSpec((self.buckets + 1, self.hidden))}
+
+    def load(self, tensors, prefix: str) -> None:
+        self.weight = tensors[f"{prefix}{self.name}"]
+
+    def state_spec(self) -> StateSpec:
+        return StateSpec((1,), torch.int32)
+
+
 class TokenEmbedding(Part):
     """x = E[ids] * scale (``scale`` 1 unless the model says otherwise); rows are widened into the 32-bit residual stream.
-    With ``places`` (a ``LearnedPositions``) the row of the token's position is added, in 32-bit."""
+    With ``places`` (a ``LearnedPositions``) the row of the token's position is added, with ``pairs`` (a ``PairRows``) the
+    row of the token and the one before it, in 32-bit."""
 
-    def __init__(self, vocab: int, hidden: int, name: str = "weight", places: LearnedPositions | None = None, scale: float = 1.0):
-        if places is not None and scale != 1.0:
-            raise ValueError("an embedding with position rows has no scale")
+    def __init__(self, vocab: int, hidden: int, name: str = "weight", places: LearnedPositions | None = None, scale: float = 1.0,
+                 pairs: PairRows | None = None):
+        if places is not None and (scale != 1.0 or pairs is not None):
+            raise ValueError("an embedding with position rows has no scale and no rows of pairs")
         self.vocab, self.hidden, self.name, self.places, self.scale = vocab, hidden, name, places, float(scale)
+        self.pairs = pairs
         self.weight: torch.Tensor | None = None
 
     @property
@@ -39,24 +63,31 @@ class TokenEmbedding(Part):
         """Does ``forward`` need the tokens' positions beside their ids?"""
         return self.places is not None
 
+    def cache_spec(self) -> StateSpec | None:
+        """State the embedding keeps per request (the token before), or None."""
+        return self.pairs.state_spec() if self.pairs is not None else None
+
+    def _tables(self):
+        return [p for p in (self.places, self.pairs) if p is not None]
+
     def tensor_specs(self, prefix: str):
         specs = {f"{prefix}{self.name}": TensorSpec((self.vocab, self.hidden))}
-        if self.places is not None:
-            specs.update(self.places.tensor_specs(prefix))
+        for part in self._tables():
+            specs.update(part.tensor_specs(prefix))
         return specs
 
     def load(self, tensors, prefix: str) -> None:
         self.weight = tensors[f"{prefix}{self.name}"]
-        if self.places is not None:
-            self.places.load(tensors, prefix)
+        for part in self._tables():
+            part.load(tensors, prefix)
 
     def emit(self, program) -> int | None:
-        if self.places is not None or self.scale != 1.0:
+        if self._tables() or self.scale != 1.0:
             return None                         # the library's operation gathers token rows only, as they are
         return program.embedding(self, self.weight)
 
     def cost(self, label, step, rows):
-        return rows * self.hidden * (self.weight.element_size() * (2 if self.places is not None else 1) + 4), 0
+        return rows * self.hidden * (self.weight.element_size() * (1 + len(self._tables())) + 4), 0
 
     def forward(self, token_ids: torch.Tensor, positions: torch.Tensor | None = None) -> torch.Tensor:
         out = torch.empty((token_ids.numel(), self.hidden), dtype=torch.float32, device=token_ids.device)
@@ -64,6 +95,14 @@ class TokenEmbedding(Part):
             if self.places is not None:
                 return ops.embed_gather_pos(self.weight, self.places.weight, token_ids, positions, out)
             return ops.embed_gather(self.weight, token_ids, out, self.scale)
+
+    def forward_step(self, step: StepContext, cache: StateView) -> torch.Tensor:
+        """The rows of an embedding that keeps state, for a step's tokens; the state moves on to the step's last tokens."""
+        pairs = self.pairs
+        out = torch.empty((step.num_tokens, self.hidden), dtype=torch.float32, device=step.token_ids.device)
+        with profiling.label("embed", lambda: self.cost("embed", None, step.num_tokens)):
+            return ops.embed_pairs(self.weight, pairs.weight, step.token_ids, step.positions, step.cu_q_lens, step.state_slots,
+                                   step.seq_of_token, step.num_seqs, cache.state, out, self.scale, pairs.mul_prev, pairs.mul_cur)
 
 
 class OutputHead(Part):

@@ -121,20 +121,25 @@ class DenseFeedForward(FeedForward):
 
 
 class GatedFeedForward(FeedForward):
-    """down(act(gate(x)) * up(x)) without biases, gate and up stacked into one product. ``activation``: "gelu_tanh", the
-    tanh form of GELU, or "silu"; it is computed in 32-bit on the gate's rounded result and the product with up is rounded
-    once. (``SwiGLU`` is the "silu" case as one operation of the kernel library's step program, for models whose blocks
+    """down(act(gate(x)) * up(x)), gate and up stacked into one product, with or without biases (``bias``). ``activation``:
+    "gelu_tanh", the tanh form of GELU, or "silu"; it is computed in 32-bit on the gate's rounded result and the product with up
+    is rounded once. "clamped_glu": down(g sigmoid(1.702 g) (u + 1)) with g = min(gate(x), limit) and u = up(x) held to +-limit
+    (``limit``), in 32-bit and rounded once. (``SwiGLU`` is the "silu" case as one operation of the kernel library's step program, for models whose blocks
     describe themselves to it.)"""
 
-    ACTIVATIONS = ("gelu_tanh", "silu")
+    ACTIVATIONS = ("gelu_tanh", "silu", "clamped_glu")
+    ALPHA = 1.702           # of the clamped gate's sigmoid: the mechanism's own constant
 
     def __init__(self, hidden: int, intermediate: int, activation: str = "gelu_tanh", names: tuple[str, str, str] = ("gate", "up", "down"),
-                 suffixes: tuple[str, str] = ("", ".b")):
+                 suffixes: tuple[str, str] = ("", ".b"), bias: bool = False, limit: float | None = None):
         if activation not in self.ACTIVATIONS:
             raise ValueError(f"activation '{activation}' is not one of {sorted(self.ACTIVATIONS)}")
+        if (activation == "clamped_glu") != (limit is not None) or (limit is not None and not limit > 0):
+            raise ValueError("a clamped gate has a positive limit, the others have none")
         self.hidden, self.intermediate, self.activation = hidden, intermediate, activation
-        self.gate_up = Linear(hidden, [intermediate, intermediate], list(names[:2]), bias=False, suffixes=suffixes)
-        self.down = Linear(intermediate, hidden, names[2], bias=False, suffixes=suffixes)
+        self.limit = float(limit) if limit is not None else None
+        self.gate_up = Linear(hidden, [intermediate, intermediate], list(names[:2]), bias=bias, suffixes=suffixes)
+        self.down = Linear(intermediate, hidden, names[2], bias=bias, suffixes=suffixes)
 
     def tensor_specs(self, prefix: str):
         return {**self.gate_up.tensor_specs(prefix), **self.down.tensor_specs(prefix)}
@@ -156,6 +161,9 @@ class GatedFeedForward(FeedForward):
         with profiling.label("gate_up", lambda: self.gate_up.cost(x.shape[0])):
             gu = self.gate_up.forward(x)
             a = torch.empty((x.shape[0], self.intermediate), dtype=x.dtype, device=x.device)
-            (ops.gelu_mul if self.activation == "gelu_tanh" else ops.silu_mul)(gu, a)
+            if self.activation == "clamped_glu":
+                ops.clamped_glu(gu, a, self.limit, self.ALPHA)
+            else:
+                (ops.gelu_mul if self.activation == "gelu_tanh" else ops.silu_mul)(gu, a)
         with profiling.label("down", lambda: self.down.cost(x.shape[0])):
             return self.down.forward(a)

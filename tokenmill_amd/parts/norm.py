@@ -35,6 +35,43 @@ class RMSNorm(Norm):
         return self.weight, self.eps
 
 
+class WeightedAdd:
+    """What a sublayer's result passes on its way into the residual stream when other results go with it:
+    resid += scale * y + sum of scale_i * y_i. ``others`` [(y_i, scale_i), ...]: results of sublayers side by side. It stands
+    where a norm behind a sublayer stands (``Flow.delta_norm``), so the norm in front of the next sublayer can add them all and
+    do its own work in one kernel."""
+
+    def __init__(self, scale: float = 1.0, others: list | None = None):
+        self.scale, self.others = float(scale), list(others or [])
+
+    def parts(self, y: torch.Tensor) -> list:
+        return [(y, self.scale), *self.others]
+
+    def select(self, rows: torch.Tensor) -> "WeightedAdd":
+        """The same for some rows only."""
+        idx = rows.long()
+        return WeightedAdd(self.scale, [(y.index_select(0, idx), s) for y, s in self.others])
+
+    def moved(self, y: torch.Tensor, rows: int) -> int:
+        """Bytes of the results that an add over ``rows`` rows reads."""
+        return rows * y.shape[1] * y.element_size() * (1 + len(self.others))
+
+    def add_normed(self, resid, y) -> None:
+        with profiling.label("norm", lambda: (resid.numel() * 8 + self.moved(y, y.shape[0]), 0)):
+            parts = self.parts(y)
+            for i in range(0, len(parts), 3):               # the kernel adds up to three at a time
+                ops.sum_norm(resid, parts[i:i + 3], None, None, 1.0)
+
+
+def _settled(resid: torch.Tensor, delta: torch.Tensor, delta_norm, rows: torch.Tensor):
+    """A copy of ``rows`` of the stream with a pending result added the way ``delta_norm`` says: for a norm that wants only some
+    rows, cannot do that add itself, and must leave the stream as it is."""
+    resid = resid.index_select(0, rows.long())
+    way = delta_norm.select(rows) if hasattr(delta_norm, "select") else delta_norm
+    way.add_normed(resid, delta.index_select(0, rows.long()))
+    return resid
+
+
 class GroupRMSNorm(Norm):
     """RMS norm in groups: the row is cut into ``groups`` equal consecutive parts, each part is divided by its own
     sqrt(mean(part^2) + eps), and the whole is multiplied by the weight; all of it in 32-bit, the result rounded
@@ -75,14 +112,15 @@ class GroupRMSNorm(Norm):
         if delta is not None and delta_norm is not None:
             if isinstance(delta_norm, GroupRMSNorm) and (delta_norm.groups, delta_norm.eps) == (self.groups, self.eps):
                 post = delta_norm.weight
+            elif isinstance(delta_norm, WeightedAdd) and self.groups == 1 and len(delta_norm.others) <= 2:
+                with profiling.label("norm", lambda: (n * self.hidden * (4 + (4 if rows is None else 0) + out.element_size())
+                                                      + delta_norm.moved(delta, n), 0)):
+                    return ops.sum_norm(resid, delta_norm.parts(delta), self.weight, out, self.eps, rows)
             elif rows is None:
                 delta_norm.add_normed(resid, delta)
                 delta = None
             else:
-                # only some rows are wanted and the residual is to stay as it is: the pending result's norm on a copy
-                resid = resid.index_select(0, rows.long())
-                delta_norm.add_normed(resid, delta.index_select(0, rows.long()))
-                delta, rows = None, None
+                resid, delta, rows = _settled(resid, delta, delta_norm, rows), None, None
         added = 0 if delta is None else (4 if rows is None else 0) + delta.element_size()
         with profiling.label("norm", lambda: self._cost(n, out.element_size(), added)):
             return ops.group_norm(resid, delta, post, self.weight, out, self.groups, self.eps, rows)
@@ -110,9 +148,7 @@ class PassThrough(Norm):
                 delta_norm.add_normed(resid, delta)
                 delta = None
             else:
-                resid = resid.index_select(0, rows.long())
-                delta_norm.add_normed(resid, delta.index_select(0, rows.long()))
-                delta, rows = None, None
+                resid, delta, rows = _settled(resid, delta, delta_norm, rows), None, None
         added = 0 if delta is None else (4 if rows is None else 0) + delta.element_size()
         with profiling.label("norm", lambda: (n * self.hidden * (4 + out.element_size() + added), 0)):
             return ops.group_norm(resid, delta, post, None, out, groups, eps, rows)
@@ -165,10 +201,8 @@ class LayerNorm(Norm):
             elif rows is None:
                 delta_norm.add_normed(resid, delta)
                 delta = None
-            else:       # only some rows are wanted and the residual is to stay as it is: the pending result's way in on a copy
-                resid = resid.index_select(0, rows.long())
-                delta_norm.add_normed(resid, delta.index_select(0, rows.long()))
-                delta, rows = None, None
+            else:
+                resid, delta, rows = _settled(resid, delta, delta_norm, rows), None, None
         added = 0 if delta is None else (4 if rows is None else 0) + delta.element_size() * (2 if gate is not None else 1)
         with profiling.label("norm", lambda: self._cost(n, out.element_size(), added)):
             return ops.layer_norm(resid, delta, gate, mult, self.weight, self.bias, out, self.eps, rows)

@@ -1,7 +1,13 @@
-"""Two mixers side by side: both read the same input, each result is RMS-normed over the model's width with a weight of
-its own, and the mixer's result is half their sum,
+"""Two mixers side by side: both read the same input. Either each result is RMS-normed over the model's width with a weight
+of its own, and the mixer's result is half their sum,
 
-    y = (rms_norm(left(h); w_left) + rms_norm(right(h); w_right)) / 2.
+    y = (rms_norm(left(h); w_left) + rms_norm(right(h); w_right)) / 2,
+
+or the results are added with two constant weights (``scales``),
+
+    y = scale_left * left(h) + scale_right * right(h),
+
+which a block that takes several results at once (``forward_parts``) adds into the residual stream in 32-bit.
 
 The two may be any mixers of which at most one keeps pages and at most one keeps state slots (an attention beside a
 recurrence): the layer's cache is then the pages of the one with the state of the other beside them.
@@ -28,10 +34,15 @@ def _split(spec):
 
 
 class ParallelMixer(Mixer):
-    def __init__(self, hidden: int, left: Mixer, right: Mixer, norm_eps: float, prefixes: tuple[str, str] = ("left.", "right."),
-                 norm_names: tuple[str, str] = ("left.out", "right.out")):
-        self.hidden, self.left, self.right, self.norm_eps = hidden, left, right, float(norm_eps)
-        self.prefixes, self.norm_names = prefixes, norm_names
+    def __init__(self, hidden: int, left: Mixer, right: Mixer, norm_eps: float | None = None,
+                 prefixes: tuple[str, str] = ("left.", "right."), norm_names: tuple[str, str] = ("left.out", "right.out"),
+                 scales: tuple[float, float] | None = None):
+        if (norm_eps is None) == (scales is None):
+            raise ValueError("the two results are either normed or weighted by constants")
+        self.hidden, self.left, self.right = hidden, left, right
+        self.norm_eps = float(norm_eps) if norm_eps is not None else None
+        self.scales = (float(scales[0]), float(scales[1])) if scales is not None else None
+        self.prefixes, self.norm_names = prefixes, norm_names if scales is None else ()
         (lk, ls), (rk, rs) = _split(left.cache_spec()), _split(right.cache_spec())
         if (lk is not None and rk is not None) or (ls is not None and rs is not None):
             raise ValueError("of two mixers side by side, one may keep pages and one may keep state")
@@ -54,8 +65,9 @@ class ParallelMixer(Mixer):
     def load(self, tensors, prefix: str) -> None:
         self.left.load(tensors, prefix + self.prefixes[0])
         self.right.load(tensors, prefix + self.prefixes[1])
-        self.w_left = tensors[prefix + self.norm_names[0]].float().contiguous()
-        self.w_right = tensors[prefix + self.norm_names[1]].float().contiguous()
+        if self.scales is None:
+            self.w_left = tensors[prefix + self.norm_names[0]].float().contiguous()
+            self.w_right = tensors[prefix + self.norm_names[1]].float().contiguous()
 
     def prepare(self, pack_weights: bool) -> None:
         self.left.prepare(pack_weights)
@@ -74,10 +86,24 @@ class ParallelMixer(Mixer):
             return StateView(cache.state) if which == self.state_of and cache.state is not None else None
         return cache if which == self.state_of else None
 
+    def _both(self, x: torch.Tensor, step: StepContext, cache):
+        return self.left.forward(x, step, self._cache_for(0, cache)), self.right.forward(x, step, self._cache_for(1, cache))
+
+    def forward_parts(self, x, step: StepContext, cache) -> list:
+        """[(result [T, hidden], its weight), ...]: what is to be added into the residual stream."""
+        if self.scales is None:
+            return [(self.forward(x, step, cache), 1.0)]
+        a, b = self._both(as_tensor(x), step, cache)
+        return [(a, self.scales[0]), (b, self.scales[1])]
+
     def forward(self, x, step: StepContext, cache, residual: torch.Tensor | None = None):
-        x = as_tensor(x)
-        a = self.left.forward(x, step, self._cache_for(0, cache))
-        b = self.right.forward(x, step, self._cache_for(1, cache))
+        if self.scales is not None:
+            from tokenmill_amd.parts.norm import WeightedAdd
+            (a, s), other = self.forward_parts(x, step, cache)
+            total = torch.zeros(a.shape, dtype=torch.float32, device=a.device)
+            WeightedAdd(s, [other]).add_normed(total, a)
+            return total if a.dtype == torch.float32 else ops.convert(total, torch.empty_like(a))
+        a, b = self._both(as_tensor(x), step, cache)
         out = torch.empty_like(a)
         with profiling.label("norm", lambda: (3 * a.numel() * a.element_size(), 0)):
             return ops.pair_norm_mean(a, b, self.w_left, self.w_right, out, self.norm_eps)

@@ -1,0 +1,111 @@
+"""Retention: a recurrent mixer with a matrix of state per request and head and one fixed decay per head.
+
+    q_t, k_t = rotate(W_q h_t), rotate(W_k h_t) / sqrt(D)     [heads, D]
+    v_t, g_t = W_v h_t, W_g h_t                               [heads, Dv]
+    S_t = decay_h S_(t-1) + k_t v_t^T                         [D, Dv] per head, 32-bit, zero at a request's first token
+    o_t = S_t^T q_t
+    y_t = W_o (concat over heads of unit_rms(o_t) * silu(g_t))
+
+with the rotation of ``rotary`` (by the token's position, over the first channels of a head) or none. The state is the mixer's
+cache: a ``StateSpec`` slot per request, advanced in token order inside a step's portion and carried from step to step. What
+lies between the projections and the norm of the result is 32-bit. It is gated linear attention with decays that do not
+change from token to token, and runs that recurrence's kernels. A step of single tokens works on the step's device tensors
+alone, so it can be recorded into a HIP graph.
+"""
+from __future__ import annotations
+
+import torch
+
+from tokenmill_amd import profiling
+from tokenmill_amd.hip import ops
+from tokenmill_amd.parts.base import Mixer, StateSpec, StateView, StepContext, as_tensor, step_segments
+from tokenmill_amd.parts.gla import MAX_KEY_DIM
+from tokenmill_amd.parts.linear import Linear
+from tokenmill_amd.parts.position import RotaryEmbedding
+
+
+class Retention(Mixer):
+    def __init__(self, hidden: int, num_heads: int, key_dim: int, value_dim: int, decay: list[float], norm_eps: float,
+                 rotary: RotaryEmbedding | None = None, names: tuple[str, ...] = ("q", "k", "v", "g", "o"),
+                 suffixes: tuple[str, str] = ("", ".b")):
+        if not 0 < key_dim <= MAX_KEY_DIM or value_dim <= 0:
+            raise ValueError(f"key size {key_dim}: the recurrence kernel takes up to {MAX_KEY_DIM}")
+        if len(decay) != num_heads:
+            raise ValueError(f"{len(decay)} decays for {num_heads} heads")
+        if rotary is not None and (rotary.interleaved or rotary.rotary_dim > key_dim):
+            raise ValueError("a retention rotates pairs half the rotated width apart, inside a head")
+        self.hidden, self.num_heads, self.key_dim, self.value_dim = hidden, num_heads, key_dim, value_dim
+        self.norm_eps, self.rotary, self.decay_values = float(norm_eps), rotary, [float(d) for d in decay]
+        self.k_size, self.v_size = num_heads * key_dim, num_heads * value_dim
+        self.proj = Linear(hidden, [self.k_size, self.k_size, self.v_size, self.v_size], list(names[:4]), bias=False, suffixes=suffixes)
+        self.o = Linear(self.v_size, hidden, names[4], bias=False, suffixes=suffixes)
+        self.decay: torch.Tensor | None = None          # float32 [1, H * D]: every token's
+
+    def tensor_specs(self, prefix: str):
+        return {**self.proj.tensor_specs(prefix), **self.o.tensor_specs(prefix)}
+
+    def load(self, tensors, prefix: str) -> None:
+        self.proj.load(tensors, prefix)
+        self.o.load(tensors, prefix)
+        if self.rotary is not None:
+            self.rotary.load(tensors, prefix)
+        per_head = torch.tensor(self.decay_values, dtype=torch.float32)
+        self.decay = per_head.repeat_interleave(self.key_dim)[None].contiguous().to(self.o.weight.device)
+
+    def prepare(self, pack_weights: bool) -> None:
+        self.proj.prepare(pack_weights)
+        self.o.prepare(pack_weights)
+
+    def cache_spec(self):
+        return StateSpec((self.num_heads, self.key_dim, self.value_dim), torch.float32)
+
+    def cost(self, label: str, step: StepContext | None, rows: int) -> tuple[int, int]:
+        if label == "qkv":
+            return self.proj.cost(rows)
+        if label == "o_proj":
+            return self.o.cost(rows)
+        # the recurrence: q, k, v and the result once; the state read and written once per request; per token and head
+        # D * Dv multiply-adds for the state and as many for the result
+        e = self.proj.weight.element_size()
+        seqs = step.num_seqs if step is not None else 1
+        moved = rows * ((2 * self.k_size + self.v_size) * e + self.v_size * 4) + 2 * seqs * self.num_heads * self.key_dim * self.value_dim * 4
+        return moved, 4 * rows * self.num_heads * self.key_dim * self.value_dim
+
+    # Rows of a request's portion from which the recurrence runs in segments of this many rows (see ``_scan``)
+    SEGMENT = 64
+
+    def forward(self, x, step: StepContext, cache: StateView, residual: torch.Tensor | None = None):
+        x = as_tensor(x)
+        T = x.shape[0]
+        H, D, Dv, rot = self.num_heads, self.key_dim, self.value_dim, self.rotary
+        if rot is not None and step.max_context_len > rot.max_positions:
+            raise ValueError(f"position {step.max_context_len - 1} is beyond the rotary table ({rot.max_positions} positions)")
+        with profiling.label("qkv", lambda: self.cost("qkv", step, T)):
+            proj = self.proj.forward(x)                                          # [T, q | k | v | g]
+        o = torch.empty((T, self.v_size), dtype=torch.float32, device=x.device)
+        y = torch.empty((T, self.v_size), dtype=x.dtype, device=x.device)
+        with profiling.label("recurrence", lambda: self.cost("attention", step, T)):
+            rows = torch.empty((T, ops.retention_row_width(H, D, Dv)), dtype=torch.float32, device=x.device)
+            ops.retention_prepare(proj, rot.cos if rot is not None else None, rot.sin if rot is not None else None, step.positions, rows,
+                                  H, D, Dv, D ** -0.5)
+            self._scan(rows, o, cache.state, step)
+            ops.gla_out_gate(o, proj[:, 2 * self.k_size + self.v_size:], None, y, H, Dv, self.norm_eps)
+        with profiling.label("o_proj", lambda: self.o.cost(T)):
+            return self.o.forward(y)
+
+    def _scan(self, rows, o, state, step: StepContext) -> None:
+        """The recurrence over the step's rows: one scan from the requests' states, or for a long portion (as in gated linear
+        attention) two scans of its segments side by side with a chain of the segments' states between them."""
+        H, D, Dv, ks = self.num_heads, self.key_dim, self.value_dim, self.k_size
+        if step.max_q_len < 2 * self.SEGMENT:
+            ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, o, state, step.cu_q_lens, step.state_slots, step.num_seqs, H, D, Dv, 1.0)
+            return
+        cu_seg, ids, first, n_seg = step_segments(step, self.SEGMENT, rows.device)
+        local = torch.zeros((n_seg, H, D, Dv), dtype=torch.float32, device=rows.device)
+        states_only = ops.gla_scan_states_only(rows, 0, ks, self.decay, D)       # else o is written and overwritten below
+        ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, None if states_only else o, local, cu_seg, ids, n_seg, H, D, Dv, 1.0)
+        products = torch.empty((n_seg, ks), dtype=torch.float32, device=rows.device)
+        ops.gla_segment_decay(self.decay, cu_seg, n_seg, products)
+        start = torch.empty_like(local)
+        ops.gla_combine(state, step.state_slots, first, products, local, start, step.num_seqs)
+        ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, o, start, cu_seg, ids, n_seg, H, D, Dv, 1.0)
