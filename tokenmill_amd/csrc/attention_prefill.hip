@@ -42,7 +42,7 @@ __device__ __forceinline__ __amdgpu_buffer_rsrc_t uniform_buffer(const void* bas
 // lane: lane 2 i + t holds the page of tile t of block kb + i * KS. A tile that holds no key any
 // query of this wavefront may see (beyond the newest key, or wholly behind the window) is replaced
 // by the nearest tile that does: its table entry may name no page. The caller masks every score of
-// such a tile by the key's real position, so what is loaded in its place only has to be finite.
+// such a tile by the key's real position and clears its values (the tile in its place may hold keys beyond the newest one).
 template <int KS>
 __device__ __forceinline__ int2 lane_pages(int kb, int lane, int first_tile, int last_tile,
                                            const int* __restrict__ table, int page_shift) {
@@ -79,13 +79,14 @@ template <int D, int HPW>
 __device__ __forceinline__ void attend_block(KVBlock<D>& blk, HeadState<D, HPW>& st, const PFrag (&qf)[HPW][D / 32],
                                              int key0, int nh, const TileView& tv, int g, float scale_log2, float cap_in, float cap_out) {
     constexpr int NDC = D / 32, NDT = D / 16;
-    // values of keys nobody may see (beyond the newest key) can hold anything: clear them
-    if (key0 + 31 > tv.last_key) {
+    // values of keys nobody may see (beyond the newest key, or behind every window: see lane_pages) can hold anything: clear them
+    if (key0 + 31 > tv.last_key || key0 < tv.first_key) {
+        auto seen = [&](int k) { return k <= tv.last_key && k >= tv.first_key; };
 #pragma unroll
         for (int t = 0; t < 2; ++t) {
             const int k0 = key0 + 16 * t + 4 * g;
-            const uint32_t keep0 = ((k0 <= tv.last_key) ? 0x0000ffffu : 0u) | ((k0 + 1 <= tv.last_key) ? 0xffff0000u : 0u);
-            const uint32_t keep1 = ((k0 + 2 <= tv.last_key) ? 0x0000ffffu : 0u) | ((k0 + 3 <= tv.last_key) ? 0xffff0000u : 0u);
+            const uint32_t keep0 = (seen(k0) ? 0x0000ffffu : 0u) | (seen(k0 + 1) ? 0xffff0000u : 0u);
+            const uint32_t keep1 = (seen(k0 + 2) ? 0x0000ffffu : 0u) | (seen(k0 + 3) ? 0xffff0000u : 0u);
 #pragma unroll
             for (int dt = 0; dt < NDT; ++dt) {
                 blk.v[dt][t][0] &= keep0;
@@ -219,6 +220,7 @@ __global__ __launch_bounds__(64 * KS) void attn_prefill_mfma_kernel(
         tv.my_lo = (window > 0 && tv.my_pos - window + 1 > 0) ? tv.my_pos - window + 1 : 0;
         tv.last_lo = (window > 0 && tv.last_key - window + 1 > 0) ? tv.last_key - window + 1 : 0;
         const int first_key = (window > 0 && pos0 - window + 1 > 0) ? pos0 - window + 1 : 0;
+        tv.first_key = first_key;
         const int kb0 = first_key / 32, kb1 = tv.last_key / 32;
         const int first_tile = first_key / 16, last_tile = tv.last_key / 16;
 

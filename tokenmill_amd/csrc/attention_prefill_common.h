@@ -53,6 +53,7 @@ struct HeadState {
 struct TileView {
     int pos0;               // position of the tile's first query
     int last_key;           // newest key any query of the tile sees
+    int first_key;          // oldest key any query of the tile sees (0 without a window)
     int last_lo;            // oldest key the tile's last query sees (0 without a window)
     int my_pos, my_lo;      // this lane's query column: its position and the oldest key it sees
 };

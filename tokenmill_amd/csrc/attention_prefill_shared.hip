@@ -101,10 +101,10 @@ struct StageCopy {
         }
     }
 
-    // Store what was loaded into a stage of LDS. `keys` of the stage's 64 positions exist: the values of the
-    // others (beyond the newest key; they can hold anything) are cleared here, once for all wavefronts, so that
+    // Store what was loaded into a stage of LDS. Of the stage's 64 positions [from, keys) can be seen: the values of the
+    // others (beyond the newest key, or behind every window, where another tile stands in; they can hold anything) are cleared here, once for all wavefronts, so that
     // the products need no mask (their weights are zero, but zero times anything is not).
-    __device__ __forceinline__ void store(unsigned char* stage, int tid, int keys) const {
+    __device__ __forceinline__ void store(unsigned char* stage, int tid, int from, int keys) const {
 #pragma unroll
         for (int i = 0; i < ITERS; ++i) {
             const int idx = tid + i * THREADS;
@@ -113,11 +113,13 @@ struct StageCopy {
             *(u32x4_t*)(stage + stage_row(kk) * SharedShape<D>::K_STRIDE + pc * 16) = k[i];
             const int j = idx / (2 * D), d = (idx % (2 * D)) / 2, half = idx & 1;
             u32x4_t val = v[i];
-            if (keys < PS_KEYS) {                                    // block-uniform: a tile's last stage only
+            if (keys < PS_KEYS || from > 0) {                        // block-uniform: a tile's last stage, and its first with a window
                 const int first = 16 * j + 8 * half;
 #pragma unroll
-                for (int w = 0; w < 4; ++w)
-                    val[w] &= ((first + 2 * w < keys) ? 0x0000ffffu : 0u) | ((first + 2 * w + 1 < keys) ? 0xffff0000u : 0u);
+                for (int w = 0; w < 4; ++w) {
+                    const int k0 = first + 2 * w, k1 = k0 + 1;
+                    val[w] &= ((k0 < keys && k0 >= from) ? 0x0000ffffu : 0u) | ((k1 < keys && k1 >= from) ? 0xffff0000u : 0u);
+                }
             }
             *(u32x4_t*)(stage + SharedShape<D>::K_BYTES + d * SharedShape<D>::V_STRIDE + j * 32 + half * 16) = val;
         }
@@ -249,6 +251,7 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
         tv.my_lo = (window > 0 && tv.my_pos - window + 1 > 0) ? tv.my_pos - window + 1 : 0;
         tv.last_lo = (window > 0 && tv.last_key - window + 1 > 0) ? tv.last_key - window + 1 : 0;
         const int first_key = (window > 0 && pos0 - window + 1 > 0) ? pos0 - window + 1 : 0;
+        tv.first_key = first_key;
         const int sb0 = first_key / PS_KEYS, sb1 = tv.last_key / PS_KEYS;
         const int first_tile = first_key / 16, last_tile = tv.last_key / 16;
 
@@ -278,7 +281,7 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
         TilePlaces places = lane_places(base, lane, first_tile, last_tile, table, page_shift, kvh, KVH, D);
         StageCopy<D, THREADS> copy;
         copy.load(places, 0, kp, vp, KVH, page_shift, tid);
-        copy.store(stages, tid, tv.last_key + 1 - sb0 * PS_KEYS);
+        copy.store(stages, tid, first_key - sb0 * PS_KEYS, tv.last_key + 1 - sb0 * PS_KEYS);
         __syncthreads();
         for (int sb = sb0; sb <= sb1; ++sb) {
             const int cur = (sb - sb0) & 1;
@@ -296,7 +299,7 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
                     attend_shared<D, HPW>(stages + cur * STAGE, sub, st, qf, key0, tv, r, g, scale_log2, cap_in, cap_out);
                 }
             }
-            copy.store(stages + (cur ^ 1) * STAGE, tid, tv.last_key + 1 - next * PS_KEYS);
+            copy.store(stages + (cur ^ 1) * STAGE, tid, first_key - next * PS_KEYS, tv.last_key + 1 - next * PS_KEYS);
             __syncthreads();
         }
 

@@ -37,9 +37,9 @@ class GatedDeltaRule(Mixer):
     def __init__(self, hidden: int, num_heads: int, num_kv_heads: int, key_dim: int, value_dim: int, taps: int, norm_eps: float,
                  names: tuple[str, ...] = ("q", "k", "v", "g", "b", "a", "o"), conv_suffix: str = ".conv",
                  other_names: tuple[str, str, str] = ("A_log", "dt_bias", "norm"), suffixes: tuple[str, str] = ("", ".b"),
-                 channel_decay: bool = False, narrow_gate: bool = False, drawn_rank: int = 16):
+                 channel_decay: bool = False, narrow_gate: bool = False, drawn_rank: int | None = None):
         """``channel_decay`` / ``narrow_gate``: see above; the narrow projection "a" is stored as "a1" and "a2", "g" as "g1" and
-        "g2". ``drawn_rank``: their width in a model drawn at random."""
+        "g2". ``drawn_rank``: their width in a model drawn at random (a head's key size unless given)."""
         if num_heads <= 0 or num_kv_heads <= 0 or num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads do not divide into {num_kv_heads} query/key heads")
         if not 0 < key_dim <= ops.DELTA_MAX_KEY_DIM or value_dim <= 0:
@@ -54,7 +54,7 @@ class GatedDeltaRule(Mixer):
             raise ValueError(f"{self.channels} convolved channels: the kernel takes up to {ops.DELTA_MAX_CHANNELS}")
         n = dict(zip(("q", "k", "v", "g", "b", "a", "o"), names))
         self.names, self.conv_suffix, self.other_names = n, conv_suffix, other_names
-        self.channel_decay, self.narrow_gate, self.drawn_rank, self.suffixes = channel_decay, narrow_gate, drawn_rank, suffixes
+        self.channel_decay, self.narrow_gate, self.drawn_rank, self.suffixes = channel_decay, narrow_gate, drawn_rank or key_dim, suffixes
         self.decays = num_heads * key_dim if channel_decay else num_heads
         self.proj: Linear | None = None         # q | k | v, then the gate or the narrow projections' first halves
         self.decay2: Linear | None = None       # the second halves
