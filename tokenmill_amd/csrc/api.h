@@ -235,6 +235,14 @@ int tm_clamped_glu(const void* gu, void* out, int dtype, int T, int I, float alp
 int tm_embed_pairs(const void* table, const void* pairs, int dtype, const int* ids, const int* positions, const int* cu_q_lens,
                    const int* state_slots, const int* seq_of_token, int* prev_state, float* out, int T, int hidden, int vocab,
                    float scale, int buckets, long long mul_prev, long long mul_cur, hipStream_t stream);
+// A recurrence over prompt portions in chunks of 64 tokens on the 32-bit matrix unit (chunk_scan.hip): see the head of that file.
+int tm_delta_chunks(const float* rows, int ld, const int* cu_chunk, int n_chunks, float* Wm, float* Qm, float* Km, float* Pm, float* gam,
+                    float* u0, int H, int G, int D, int DP, int Dv, int per_channel, hipStream_t stream);
+int tm_retention_chunks(const float* rows, int ld, const int* cu_chunk, int n_chunks, const float* decay, float* Qm, float* Km, float* Pm,
+                        float* gam, int H, int D, int DP, hipStream_t stream);
+int tm_chunk_chain(const float* Wm, const float* Qm, const float* Km, const float* Pm, const float* gam, const float* u0, int ldu, float* o,
+                   float* state, const int* cu_chunk, const int* first_chunk, const int* state_slots, int S, int H, int D, int DP, int Dv,
+                   hipStream_t stream);
 // A weighted sum of up to three results added to the residual stream, and the RMS norm of the sum (sum_norm.hip): see there.
 int tm_sum_norm(float* resid, const void* y0, float s0, const void* y1, float s1, const void* y2, float s2, const int* rows,
                 const void* w, int w_dtype, void* out, int dtype, int R, int hidden, float eps, hipStream_t stream);

@@ -2105,3 +2105,76 @@ def clamped_glu(gu: torch.Tensor, out: torch.Tensor, limit: float, alpha: float)
     _check(library().tm_clamped_glu(_p(gu), _p(out), c_int(code(gu.dtype)), c_int(T), c_int(two_i // 2), c_float(alpha), c_float(limit),
                                     _stream()), "clamped_glu")
     return out
+
+
+# -------------------------------------------------------------------------------------------- recurrences in chunks
+
+CHUNK = 64                  # tokens of a chunk
+CHUNK_MAX_KEY_DIM = 128
+
+
+def _chunk_space(n: int, H: int, D: int, device, w: bool):
+    """(padded key size, W or None, G Q, K^T, P, G_n) for n chunks of H heads."""
+    _need(0 < D <= CHUNK_MAX_KEY_DIM, f"chunks: key sizes up to {CHUNK_MAX_KEY_DIM}")
+    DP = 64 if D <= 64 else 128
+    tile = CHUNK * DP
+    parts = 3 if w else 2
+    space = torch.empty(n * H * (parts * tile + CHUNK * CHUNK + DP), dtype=torch.float32, device=device)
+    views, at = [], 0
+    for size in [tile] * parts + [CHUNK * CHUNK, DP]:
+        views.append(space[at:at + n * H * size])
+        at += n * H * size
+    return (DP, views[0] if w else None, *views[-4:])
+
+
+def _check_chunks(cu_chunk: torch.Tensor, n: int, first_chunk: torch.Tensor, state_slots: torch.Tensor, num_seqs: int) -> None:
+    _ints(cu_chunk, n + 1, "cu_chunk")
+    _ints(first_chunk, num_seqs + 1, "first_chunk")
+    _ints(state_slots, num_seqs, "state_slots")
+    _need(0 < n <= 65535 and 0 < num_seqs <= 65535, "chunks: up to 65,535 chunks and requests a call")
+
+
+def delta_chunk_scan(rows: torch.Tensor, o: torch.Tensor, state: torch.Tensor, cu_chunk: torch.Tensor, first_chunk: torch.Tensor, n: int,
+                     state_slots: torch.Tensor, num_seqs: int, H: int, G: int, D: int, Dv: int, per_channel: bool) -> torch.Tensor:
+    """``delta_scan`` for long portions: the recurrence in chunks of at most 64 rows (chunk c: rows cu_chunk[c] .. cu_chunk[c + 1] - 1;
+    request s owns the chunks first_chunk[s] .. first_chunk[s + 1] - 1), keys of up to 128 channels. The same operands otherwise;
+    rows of o that belong to no chunk are not written."""
+    _gpu(rows, o, state, cu_chunk, first_chunk, state_slots)
+    T = rows.shape[0]
+    _need(rows.dtype == torch.float32 and rows.dim() == 2 and rows.is_contiguous() and rows.shape[1] >= delta_row_width(H, G, D, Dv, per_channel),
+          "delta_chunk_scan: rows are those of delta_prepare")
+    _need(o.dtype == torch.float32 and o.is_contiguous() and tuple(o.shape) == (T, H * Dv), f"delta_chunk_scan: o is float32 [{T}, {H * Dv}]")
+    _need(state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (H, D, Dv),
+          f"delta_chunk_scan: state is float32 [slots, {H}, {D}, {Dv}]")
+    _need(H % G == 0 and H > 0 and Dv > 0, "delta_chunk_scan: sizes the kernel does not take")
+    _check_chunks(cu_chunk, n, first_chunk, state_slots, num_seqs)
+    DP, Wm, Qm, Km, Pm, gam = _chunk_space(n, H, D, rows.device, w=True)
+    u0 = torch.empty((n * CHUNK, H * Dv), dtype=torch.float32, device=rows.device)
+    _check(library().tm_delta_chunks(_p(rows), c_int(rows.shape[1]), _p(cu_chunk), c_int(n), _p(Wm), _p(Qm), _p(Km), _p(Pm), _p(gam), _p(u0),
+                                     c_int(H), c_int(G), c_int(D), c_int(DP), c_int(Dv), c_int(1 if per_channel else 0), _stream()),
+           "delta_chunks")
+    _check(library().tm_chunk_chain(_p(Wm), _p(Qm), _p(Km), _p(Pm), _p(gam), _p(u0), c_int(H * Dv), _p(o), _p(state), _p(cu_chunk),
+                                    _p(first_chunk), _p(state_slots), c_int(num_seqs), c_int(H), c_int(D), c_int(DP), c_int(Dv), _stream()),
+           "chunk_chain")
+    return o
+
+
+def retention_chunk_scan(rows: torch.Tensor, decay: torch.Tensor, o: torch.Tensor, state: torch.Tensor, cu_chunk: torch.Tensor,
+                         first_chunk: torch.Tensor, n: int, state_slots: torch.Tensor, num_seqs: int, H: int, D: int, Dv: int) -> torch.Tensor:
+    """A retention over the rows of ``retention_prepare`` in chunks, as ``delta_chunk_scan``; decay float32 [1, H * D] (a head's D
+    values equal)."""
+    _gpu(rows, decay, o, state, cu_chunk, first_chunk, state_slots)
+    T, ld = rows.shape
+    _need(rows.dtype == torch.float32 and rows.is_contiguous() and ld >= H * (2 * D + Dv), "retention_chunk_scan: rows are those of retention_prepare")
+    _need(decay.dtype == torch.float32 and decay.is_contiguous() and decay.numel() == H * D, f"retention_chunk_scan: decay is float32 [{H * D}]")
+    _need(o.dtype == torch.float32 and o.is_contiguous() and tuple(o.shape) == (T, H * Dv), f"retention_chunk_scan: o is float32 [{T}, {H * Dv}]")
+    _need(state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (H, D, Dv),
+          f"retention_chunk_scan: state is float32 [slots, {H}, {D}, {Dv}]")
+    _check_chunks(cu_chunk, n, first_chunk, state_slots, num_seqs)
+    DP, _, Qm, Km, Pm, gam = _chunk_space(n, H, D, rows.device, w=False)
+    _check(library().tm_retention_chunks(_p(rows), c_int(ld), _p(cu_chunk), c_int(n), _p(decay), _p(Qm), _p(Km), _p(Pm), _p(gam), c_int(H),
+                                         c_int(D), c_int(DP), _stream()), "retention_chunks")
+    _check(library().tm_chunk_chain(_p(None), _p(Qm), _p(Km), _p(Pm), _p(gam), _p(rows[:, 2 * H * D:]), c_int(ld), _p(o), _p(state),
+                                    _p(cu_chunk), _p(first_chunk), _p(state_slots), c_int(num_seqs), c_int(H), c_int(D), c_int(DP), c_int(Dv),
+                                    _stream()), "chunk_chain")
+    return o

@@ -191,12 +191,16 @@ class GatedDeltaRule(Mixer):
         with profiling.label("o_proj", lambda: self.o.cost(T)):
             return self.o.forward(y)
 
-    # Rows of a request's portion from which the recurrence runs in segments of this many rows (see ``_scan``)
+    # Rows of a request's portion from which the recurrence runs in chunks on the matrix unit, or (keys it does not take) in
+    # segments of this many rows (see ``_scan``)
+    CHUNKS_FROM = 32
     SEGMENT = 128
 
     def _scan(self, rows, o, matrices, step: StepContext) -> None:
         """The recurrence over the step's rows. A step whose longest portion is short (single tokens, small portions) is one
-        scan from the requests' states. A long portion is cut into segments of ``SEGMENT`` rows: the recurrence is linear in
+        scan from the requests' states. Longer portions run in chunks of 64 rows as products of small matrices
+        (``ops.delta_chunk_scan``), and the step's single tokens, if it has any, as a scan beside them. With keys of more channels
+        than that takes, a long portion is cut into segments of ``SEGMENT`` rows: the recurrence is linear in
         the state, S_end = M S_start + B over any run of tokens, so every segment is first scanned twice side by side with all
         others, from a zero state (B: what its own rows build) and, without values, from the identity (M: the product of its
         tokens' transitions g (I - beta k k^T)); a chain over the segments gives each segment's true start state and the
@@ -205,6 +209,13 @@ class GatedDeltaRule(Mixer):
         otherwise than in the plain chain: the two agree up to 32-bit rounding."""
         H, G, D, Dv = self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim
         ch = self.channel_decay
+        if step.max_q_len >= self.CHUNKS_FROM and D <= ops.CHUNK_MAX_KEY_DIM:
+            cu_chunk, _, first, n = step_segments(step, ops.CHUNK, rows.device, portions_only=True)
+            portions = step.num_seqs - step.num_decode
+            ops.delta_chunk_scan(rows, o, matrices, cu_chunk, first, n, step.state_slots, portions, H, G, D, Dv, ch)
+            if step.num_decode:
+                ops.delta_scan(rows, o, matrices, step.cu_q_lens[portions:], step.state_slots[portions:], step.num_decode, H, G, D, Dv, per_channel=ch)
+            return
         if step.max_q_len < 2 * self.SEGMENT:
             ops.delta_scan(rows, o, matrices, step.cu_q_lens, step.state_slots, step.num_seqs, H, G, D, Dv, per_channel=ch)
             return

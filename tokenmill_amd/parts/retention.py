@@ -71,7 +71,9 @@ class Retention(Mixer):
         moved = rows * ((2 * self.k_size + self.v_size) * e + self.v_size * 4) + 2 * seqs * self.num_heads * self.key_dim * self.value_dim * 4
         return moved, 4 * rows * self.num_heads * self.key_dim * self.value_dim
 
-    # Rows of a request's portion from which the recurrence runs in segments of this many rows (see ``_scan``)
+    # Rows of a request's portion from which the recurrence runs in chunks on the matrix unit, or (keys it does not take) in
+    # segments of this many rows (see ``_scan``)
+    CHUNKS_FROM = 32
     SEGMENT = 64
 
     def forward(self, x, step: StepContext, cache: StateView, residual: torch.Tensor | None = None):
@@ -94,9 +96,19 @@ class Retention(Mixer):
             return self.o.forward(y)
 
     def _scan(self, rows, o, state, step: StepContext) -> None:
-        """The recurrence over the step's rows: one scan from the requests' states, or for a long portion (as in gated linear
-        attention) two scans of its segments side by side with a chain of the segments' states between them."""
+        """The recurrence over the step's rows: one scan from the requests' states; for longer portions chunks of 64 rows as
+        products of small matrices (``ops.retention_chunk_scan``), with a scan of the step's single tokens beside them; or, with
+        keys of more channels than that takes, (as in gated linear attention) two scans of a portion's segments side by side with a
+        chain of the segments' states between them."""
         H, D, Dv, ks = self.num_heads, self.key_dim, self.value_dim, self.k_size
+        if step.max_q_len >= self.CHUNKS_FROM and D <= ops.CHUNK_MAX_KEY_DIM:
+            cu_chunk, _, first, n = step_segments(step, ops.CHUNK, rows.device, portions_only=True)
+            portions = step.num_seqs - step.num_decode
+            ops.retention_chunk_scan(rows, self.decay, o, state, cu_chunk, first, n, step.state_slots, portions, H, D, Dv)
+            if step.num_decode:
+                ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, o, state, step.cu_q_lens[portions:], step.state_slots[portions:], step.num_decode,
+                             H, D, Dv, 1.0)
+            return
         if step.max_q_len < 2 * self.SEGMENT:
             ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, o, state, step.cu_q_lens, step.state_slots, step.num_seqs, H, D, Dv, 1.0)
             return
