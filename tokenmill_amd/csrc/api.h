@@ -243,6 +243,16 @@ int tm_retention_chunks(const float* rows, int ld, const int* cu_chunk, int n_ch
 int tm_chunk_chain(const float* Wm, const float* Qm, const float* Km, const float* Pm, const float* gam, const float* u0, int ldu, float* o,
                    float* state, const int* cu_chunk, const int* first_chunk, const int* state_slots, int S, int H, int D, int DP, int Dv,
                    hipStream_t stream);
+// Single tokens through a recurrent mixer in one launch, from the projections to what the output projection reads
+// (recurrence_step.hip): see the head of that file. tm_delta_step_takes: whether the sizes are taken.
+int tm_retention_step(const void* proj, int ld, int dtype, const float* cos_t, const float* sin_t, int rot, const int* positions,
+                      const float* decay, float* state, const int* state_slots, void* y, int n, int H, int D, int Dv, float k_scale,
+                      float eps, hipStream_t stream);
+int tm_delta_step_takes(int H, int G, int D, int Dv);
+int tm_delta_step(const void* proj, int ld, const void* conv_w, void* conv_state, const float* ba, int ldba, const float* z, int ldz,
+                  const float* a_log, const float* dt_bias, const void* gate, int ldg, int sigmoid, const float* norm_w, float* state,
+                  const int* state_slots, void* y, int n, int H, int G, int D, int Dv, int taps, float unit_eps, float eps, int dtype,
+                  hipStream_t stream);
 // A weighted sum of up to three results added to the residual stream, and the RMS norm of the sum (sum_norm.hip): see there.
 int tm_sum_norm(float* resid, const void* y0, float s0, const void* y1, float s1, const void* y2, float s2, const int* rows,
                 const void* w, int w_dtype, void* out, int dtype, int R, int hidden, float eps, hipStream_t stream);

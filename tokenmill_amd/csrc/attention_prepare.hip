@@ -111,6 +111,55 @@ __global__ __launch_bounds__(AP_THREADS) void whole_norm_rope_store_kernel(
     }
 }
 
+// Heads normed by themselves: a wavefront a token and head of q or k (grid (T, ceil((H + G) / 4)), four heads a block), so that a
+// step of few tokens is one short round. The same sums in the same order as above; a lane has the channels lane, lane + 64, ... of
+// its head (D <= 256), the rotated partner of a channel comes from the lanes' own copy in LDS.
+#define AP_MAX_DIM 256
+template <typename T>
+__global__ __launch_bounds__(AP_THREADS) void head_norm_rope_store_kernel(
+    const float* __restrict__ proj, int ld, T* __restrict__ q_out, int H, int G, int D, int Dv, int rot, int interleaved,
+    const float* __restrict__ q_w, const float* __restrict__ k_w, float eps, const float* __restrict__ cos_t,
+    const float* __restrict__ sin_t, const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ k_pool,
+    T* __restrict__ v_pool, int page, int has_kv, int v_is_k) {
+    __shared__ float row_s[AP_THREADS / TM_WAVE][AP_MAX_DIM];
+    const int t = blockIdx.x, wave = threadIdx.x / TM_WAVE, lane = threadIdx.x % TM_WAVE;
+    const int hh = blockIdx.y * (AP_THREADS / TM_WAVE) + wave, Q = H * D, K = has_kv ? G * D : 0;
+    if (hh >= H + (has_kv ? G : 0)) return;                 // (no barrier below: a wavefront reads what it wrote itself)
+    const bool is_q = hh < H;
+    const float* x = proj + (size_t)t * ld + hh * D;        // q heads, then k heads, lie one behind the other in the row
+    const float* w = is_q ? q_w : k_w;
+    float* xs = row_s[wave];
+    float ss = 0.f;
+    for (int d = lane; d < D; d += TM_WAVE) {
+        const float v = x[d];
+        ss += v * v;
+        xs[d] = v;
+    }
+    const int slot = (has_kv && slots) ? slots[t] : -1;
+    const bool store = has_kv && k_pool && slot >= 0;
+    const float r = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
+    T* to = is_q ? q_out + (size_t)t * Q + hh * D : store ? k_pool + (size_t)slot * K + (hh - H) * D : nullptr;
+    const int half = cos_t ? rot / 2 : 0;
+    if (to) {
+        const float* cs = half ? cos_t + (size_t)positions[t] * half : nullptr;
+        const float* sn = half ? sin_t + (size_t)positions[t] * half : nullptr;
+        for (int j = lane; j < half; j += TM_WAVE) {
+            const int a = interleaved ? 2 * j : j, b = interleaved ? 2 * j + 1 : j + half;
+            const float x1 = w ? w[a] * (xs[a] * r) : xs[a] * r, x2 = w ? w[b] * (xs[b] * r) : xs[b] * r;
+            float y1, y2;
+            rotate_pair(x1, x2, cs[j], sn[j], y1, y2);
+            Elem<T>::store(to + a, y1);
+            Elem<T>::store(to + b, y2);
+        }
+        for (int d = 2 * half + lane; d < D; d += TM_WAVE) Elem<T>::store(to + d, w ? w[d] * (xs[d] * r) : xs[d] * r);
+    }
+    if (!is_q && store) {                                   // the wavefront of a k head also stores the values of that head
+        const float* v = v_is_k ? nullptr : proj + (size_t)t * ld + Q + K + (hh - H) * Dv;
+        T* vo = v_pool + ((size_t)(slot / page) * G + (hh - H)) * Dv * page + slot % page;
+        for (int d = lane; d < Dv; d += TM_WAVE) Elem<T>::store(vo + (size_t)d * page, v ? v[d] : xs[d]);
+    }
+}
+
 extern "C" int tm_whole_norm_rope_store(const float* proj, int ld, void* q_out, int dtype, int T, int H, int G, int D, int Dv,
                                         int rot, int interleaved, const float* q_w, const float* k_w, float eps,
                                         const float* cos_t, const float* sin_t, const int* positions, const int* slots,
@@ -126,6 +175,21 @@ extern "C" int tm_whole_norm_rope_store(const float* proj, int ld, void* q_out, 
     if (has_kv && (q_w == nullptr) != (k_w == nullptr)) return TM_ERR_ARG;
     if (cos_t && rot && (!sin_t || !positions)) return TM_ERR_ARG;
     if (k_pool && (!has_kv || !slots || !v_pool || page <= 0)) return TM_ERR_ARG;
+    if (dtype != TM_F32 && dtype != TM_BF16) return TM_ERR_ARG;
+    if (per_head && (unit || q_w) && D <= AP_MAX_DIM) {
+        const int per = AP_THREADS / TM_WAVE;
+        const dim3 grid(T, (H + (has_kv ? G : 0) + per - 1) / per);
+        if (dtype == TM_F32)
+            head_norm_rope_store_kernel<float><<<grid, AP_THREADS, 0, stream>>>(proj, ld, (float*)q_out, H, G, D, Dv, rot, interleaved, q_w,
+                                                                               k_w, eps, cos_t, sin_t, positions, slots, (float*)k_pool,
+                                                                               (float*)v_pool, page, has_kv, v_is_k);
+        else
+            head_norm_rope_store_kernel<bf16_t><<<grid, AP_THREADS, 0, stream>>>(proj, ld, (bf16_t*)q_out, H, G, D, Dv, rot, interleaved, q_w,
+                                                                                k_w, eps, cos_t, sin_t, positions, slots, (bf16_t*)k_pool,
+                                                                                (bf16_t*)v_pool, page, has_kv, v_is_k);
+        TM_CHECK_LAUNCH();
+        return TM_OK;
+    }
     if (dtype == TM_F32)
         whole_norm_rope_store_kernel<float><<<T, AP_THREADS, 0, stream>>>(proj, ld, (float*)q_out, H, G, D, Dv, rot, interleaved, q_w,
                                                                           k_w, eps, cos_t, sin_t, positions, slots, (float*)k_pool,

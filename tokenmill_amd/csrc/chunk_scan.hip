@@ -17,6 +17,10 @@
 //   tm_retention_chunks  likewise P, G Q, (G_n / G K)^T and G_n, from the rows of tm_retention_prepare
 //   tm_chunk_chain       the chain over a request's chunks: writes o and the request's new state
 //
+// The chain's operands are stored in the order its lanes take them: a matrix [rows, inner] as tiles of 16 x 16, tile after tile along
+// the inner dimension, and in a tile the four consecutive inner elements of lane (row + 16 * quarter) behind each other, so that a
+// wavefront's load of a tile is one run of 1,024 bytes (`cs_at`). U0 likewise as it lies in the results' lanes.
+//
 // No ratio of decays is ever above one or taken of two underflowed numbers: logarithms are summed inside sub-blocks of 16 tokens,
 // a pair of tokens of one sub-block takes the exponential of their difference, and across sub-blocks each side brings a factor of
 // at most one (from its own token to a sub-block border between the two). All of it is 32-bit; a token's result depends on its
@@ -27,10 +31,16 @@
 #define CS_C 64                              // tokens of a chunk
 #define CS_SUB 16                            // tokens of a sub-block
 #define CS_A_STRIDE 68                       // floats between rows of A in LDS (16-byte aligned)
+#define CS_I_STRIDE 20                       // and of the inverses of its diagonal blocks
 #define CS_PREP 512
 #define CS_CHAIN 256
 
 typedef float cs_f32x4 __attribute__((ext_vector_type(4)));
+
+// Where element (row, inner) of a matrix with `tiles` tiles along its inner dimension is stored
+__device__ __forceinline__ int cs_at(int row, int inner, int tiles) {
+    return (((row >> 4) * tiles + (inner >> 4)) * 64 + ((inner >> 2) & 3) * 16 + (row & 15)) * 4 + (inner & 3);
+}
 
 __device__ __forceinline__ cs_f32x4 cs_mfma(float a, float b, cs_f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
@@ -84,31 +94,75 @@ __global__ __launch_bounds__(CS_PREP) void delta_chunks_kernel(const float* __re
     }
     __syncthreads();
     float* Pg = Pm + at * CS_C * CS_C;
-    // pairs of one sub-block: a thread a pair
-    for (int p = tid; p < 4 * CS_SUB * CS_SUB; p += CS_PREP) {
-        const int I = p >> 8, t = CS_SUB * I + ((p >> 4) & 15), s = CS_SUB * I + (p & 15);
-        float a = 0.f, b = 0.f;
-        if (s <= t) {
-            for (int d = 0; d < DP; d += 4) {
-                const cs_f32x4 kt = *(const cs_f32x4*)(Ks + t * LD + d), qt = *(const cs_f32x4*)(Qs + t * LD + d);
-                const cs_f32x4 ks = *(const cs_f32x4*)(Ks + s * LD + d);
-                const cs_f32x4 lt = *(const cs_f32x4*)(Ls + t * LD + d), lsv = *(const cs_f32x4*)(Ls + s * LD + d);
+    const int wave = __builtin_amdgcn_readfirstlane(tid / TM_WAVE), lane = tid % TM_WAVE, r = lane % 16, g = lane / 16;
+    if (wave < 5) {
+        // pairs of one sub-block: four lanes (a quarter of the channels each) take two tokens t and four tokens s; a sub-block
+        // has 20 such blocks on and below its diagonal: quads of s per pair of t: 1 1 2 2 3 3 4 4
+        const int task = tid / 4, part = tid % 4, I = task / 20, k = task % 20;
+        const int tp = k < 2 ? k : k < 6 ? 2 + (k - 2) / 2 : k < 12 ? 4 + (k - 6) / 3 : 6 + (k - 12) / 4;
+        const int sq = k < 2 ? 0 : k < 6 ? (k - 2) % 2 : k < 12 ? (k - 6) % 3 : (k - 12) % 4;
+        const int t0 = CS_SUB * I + 2 * tp, s0 = CS_SUB * I + 4 * sq;
+        float pa[2][4], pb[2][4];
 #pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    const float e = ks[i] * __builtin_amdgcn_exp2f(lt[i] - lsv[i]);
-                    a += kt[i] * e;
-                    b += qt[i] * e;
-                }
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) pa[i][j] = pb[i][j] = 0.f;
+#pragma unroll 1
+        for (int d = 4 * part; d < DP; d += 16) {
+            cs_f32x4 kt[2], qt[2], lt[2];
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                kt[i] = *(const cs_f32x4*)(Ks + (t0 + i) * LD + d);
+                qt[i] = *(const cs_f32x4*)(Qs + (t0 + i) * LD + d);
+                lt[i] = *(const cs_f32x4*)(Ls + (t0 + i) * LD + d);
+            }
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const cs_f32x4 ks = *(const cs_f32x4*)(Ks + (s0 + j) * LD + d), lsv = *(const cs_f32x4*)(Ls + (s0 + j) * LD + d);
+#pragma unroll
+                for (int i = 0; i < 2; ++i)
+#pragma unroll
+                    for (int m = 0; m < 4; ++m) {
+                        // (a pair with s after t is dropped below; its exponent is held to zero so that it stays finite)
+                        const float e = ks[m] * __builtin_amdgcn_exp2f(fminf(lt[i][m] - lsv[m], 0.f));
+                        pa[i][j] += kt[i][m] * e;
+                        pb[i][j] += qt[i][m] * e;
+                    }
             }
         }
-        As[t * CS_A_STRIDE + s] = s < t ? beta[t] * a : 0.f;
-        Pg[t * CS_C + s] = b;
-    }
-    // pairs of two sub-blocks I > J: a wavefront two of them, on the matrix unit
-    {
-        const int wave = __builtin_amdgcn_readfirstlane(tid / TM_WAVE), lane = tid % TM_WAVE, r = lane % 16, g = lane / 16;
-        if (wave < 6) {
-            const int I = wave < 1 ? 1 : wave < 3 ? 2 : 3, J = wave < 1 ? 0 : wave < 3 ? wave - 1 : wave - 3;
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                pa[i][j] += __shfl_xor(pa[i][j], 1, TM_WAVE);
+                pa[i][j] += __shfl_xor(pa[i][j], 2, TM_WAVE);
+                pb[i][j] += __shfl_xor(pb[i][j], 1, TM_WAVE);
+                pb[i][j] += __shfl_xor(pb[i][j], 2, TM_WAVE);
+            }
+        if (part < 2) {                                 // lane 0 writes A's two rows, lane 1 P's
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                const int t = t0 + i;
+                cs_f32x4 v;
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+                    v[j] = part == 0 ? (s0 + j < t ? beta[t] * pa[i][j] : 0.f) : (s0 + j <= t ? pb[i][j] : 0.f);
+                if (part == 0) *(cs_f32x4*)(As + t * CS_A_STRIDE + s0) = v;
+                else *(cs_f32x4*)(Pg + cs_at(t, s0, 4)) = v;
+            }
+        } else if (sq == tp / 2) {                      // and the quads behind the diagonal's are zeros
+            for (int z = s0 + 4; z < CS_SUB * (I + 1); z += 4)
+#pragma unroll
+                for (int i = 0; i < 2; ++i) {
+                    if (part == 2) *(cs_f32x4*)(As + (t0 + i) * CS_A_STRIDE + z) = cs_f32x4{0.f, 0.f, 0.f, 0.f};
+                    else *(cs_f32x4*)(Pg + cs_at(t0 + i, z, 4)) = cs_f32x4{0.f, 0.f, 0.f, 0.f};
+                }
+        }
+    } else {
+        // pairs of two sub-blocks I > J on the matrix unit: three wavefronts, two of the six products each
+#pragma unroll 1
+        for (int p = 2 * (wave - 5); p < 2 * (wave - 5) + 2; ++p) {
+            const int I = p < 1 ? 1 : p < 3 ? 2 : 3, J = p < 1 ? 0 : p < 3 ? p - 1 : p - 3;
             const int tr = CS_SUB * I + r, sr = CS_SUB * J + r;
             cs_f32x4 accA = {0.f, 0.f, 0.f, 0.f}, accP = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll 2
@@ -130,75 +184,94 @@ __global__ __launch_bounds__(CS_PREP) void delta_chunks_kernel(const float* __re
             for (int i = 0; i < 4; ++i) {
                 const int t = CS_SUB * I + 4 * g + i, s = CS_SUB * J + r;
                 As[t * CS_A_STRIDE + s] = beta[t] * accA[i];
-                Pg[t * CS_C + s] = accP[i];
+                Pg[cs_at(t, s, 4)] = accP[i];
             }
         }
     }
     // what the chain reads of the tokens themselves
     float* Qg = Qm + at * CS_C * DP;
     float* Kg = Km + at * CS_C * DP;
-    for (int idx = tid; idx < CS_C * DP; idx += CS_PREP) {
-        const int t = idx / DP, d = idx % DP;
-        float before = Ls[t * LD + d];
-        for (int M = 0; M < t / CS_SUB; ++M) before += tot[M * DP + d];
-        Qg[idx] = Qs[t * LD + d] * __builtin_amdgcn_exp2f(before);
+    // (a wavefront writes tile after tile: idx / 64 is the tile, the lane its place in it)
+    for (int tile = wave; tile < 4 * (DP / 16); tile += CS_PREP / TM_WAVE) {
+        const int I = tile / (DP / 16), t = CS_SUB * I + r, d = 16 * (tile % (DP / 16)) + 4 * g;
+        cs_f32x4 v = *(const cs_f32x4*)(Ls + t * LD + d);
+        for (int M = 0; M < I; ++M) v += *(const cs_f32x4*)(tot + M * DP + d);
+        const cs_f32x4 q4 = *(const cs_f32x4*)(Qs + t * LD + d);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = q4[i] * __builtin_amdgcn_exp2f(v[i]);
+        *(cs_f32x4*)(Qg + (tile * 64 + lane) * 4) = v;
     }
-    for (int idx = tid; idx < CS_C * DP; idx += CS_PREP) {
-        const int d = idx / CS_C, t = idx % CS_C, I = t / CS_SUB;
-        float after = tot[I * DP + d] - Ls[t * LD + d];
-        for (int M = I + 1; M < 4; ++M) after += tot[M * DP + d];
-        Kg[idx] = Ks[t * LD + d] * __builtin_amdgcn_exp2f(after);
+    for (int tile = wave; tile < 4 * (DP / 16); tile += CS_PREP / TM_WAVE) {
+        const int I = tile % 4, d = 16 * (tile / 4) + r;
+        float rest = tot[I * DP + d];
+        for (int M = I + 1; M < 4; ++M) rest += tot[M * DP + d];
+        cs_f32x4 v;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int t = CS_SUB * I + 4 * g + i;
+            v[i] = Ks[t * LD + d] * __builtin_amdgcn_exp2f(rest - Ls[t * LD + d]);
+        }
+        *(cs_f32x4*)(Kg + (tile * 64 + lane) * 4) = v;
     }
     for (int d = tid; d < DP; d += CS_PREP)
         gam[at * DP + d] = __builtin_amdgcn_exp2f(tot[d] + tot[DP + d] + tot[2 * DP + d] + tot[3 * DP + d]);
     __syncthreads();
-    // (I + A) X = B (G K) and = B V, a thread a column, from the first token on; the columns of the first DP threads are W's
+    // the inverses of I + A's four 16x16 blocks on the diagonal: a wavefront a block, a lane a column, from the first row on
+    float* inv = Qs;                                    // [4][16][CS_I_STRIDE]: the queries are no longer needed
+    if (wave < 4 && lane < 16) {
+        const float* a = As + CS_SUB * wave * CS_A_STRIDE + CS_SUB * wave;
+        float x[CS_SUB];
+#pragma unroll
+        for (int t = 0; t < CS_SUB; ++t) {
+            float v = t == lane ? 1.f : 0.f;
+#pragma unroll
+            for (int s = 0; s < t; ++s) v -= a[t * CS_A_STRIDE + s] * x[s];
+            x[t] = v;
+        }
+#pragma unroll
+        for (int t = 0; t < CS_SUB; ++t) inv[(CS_SUB * wave + t) * CS_I_STRIDE + lane] = x[t];
+    }
+    __syncthreads();
+    // (I + A) X = B (G K) and = B V in blocks of 16 rows, a wavefront 16 columns at a time: X_I = inv_I (B_I - sum over J < I of
+    // A_IJ X_J). A block of X lies in the lanes as the next product takes it. The first DP columns are W's.
     float* Wg = Wm + at * CS_C * DP;
-    for (int col = tid; col < DP + Dv; col += CS_PREP) {
-        const bool is_w = __builtin_amdgcn_readfirstlane(col) < DP;      // the same for a wavefront's lanes (DP is a multiple of 64)
-        float x[CS_C];
-        if (is_w) {
-            float before = 0.f;
+    const int v_tiles = (Dv + 15) / 16;
+    float* ug = u0 + at * v_tiles * CS_C * 16;
+    for (int tile = wave; tile < DP / 16 + v_tiles; tile += CS_PREP / TM_WAVE) {
+        const bool is_w = tile < DP / 16;
+        const int e = (is_w ? tile : tile - DP / 16) * 16 + r;
+        const int ev = e < Dv ? e : Dv - 1;             // a column beyond the last repeats it; nobody stores what comes of it
+        cs_f32x4 X[4];
+        float before = 0.f;
 #pragma unroll
-            for (int t = 0; t < CS_C; ++t) {
-                x[t] = beta[t] * (Ks[t * LD + col] * __builtin_amdgcn_exp2f(before + Ls[t * LD + col]));
-                if (t % CS_SUB == CS_SUB - 1) before += tot[t / CS_SUB * DP + col];
+        for (int I = 0; I < 4; ++I) {
+            cs_f32x4 acc;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int t = CS_SUB * I + 4 * g + i;
+                if (is_w) {
+                    acc[i] = beta[t] * (Ks[t * LD + e] * __builtin_amdgcn_exp2f(before + Ls[t * LD + e]));
+                } else {                                // rows beyond the chunk's last: the last one again, with a beta of zero
+                    const int tc = t < n ? t : n - 1;
+                    acc[i] = beta[t] * rows[(size_t)(row0 + tc) * ld + 2 * G * D + h * Dv + ev];
+                }
             }
-        } else {
-            // rows beyond the chunk's last: the last one again, with a beta of zero
-            const float* v = rows + (size_t)row0 * ld + 2 * G * D + h * Dv + (col - DP);
-            int off = 0;
+            if (is_w) before += tot[I * DP + e];
 #pragma unroll
-            for (int t = 0; t < CS_C; ++t) {
-                x[t] = beta[t] * v[off];
-                off += t + 1 < n ? ld : 0;
-                asm volatile("" : "+v"(off));            // (else 64 offsets are made ahead and held)
+            for (int J = 0; J < I; ++J) {
+                const cs_f32x4 a4 = *(const cs_f32x4*)(As + (CS_SUB * I + r) * CS_A_STRIDE + CS_SUB * J + 4 * g);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc = cs_mfma(-a4[i], X[J][i], acc);
             }
-        }
+            const cs_f32x4 t4 = *(const cs_f32x4*)(inv + (CS_SUB * I + r) * CS_I_STRIDE + 4 * g);
+            X[I] = cs_f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int t = 1; t < CS_C; ++t) {
-            float p0 = 0.f, p1 = 0.f;
+            for (int i = 0; i < 4; ++i) X[I] = cs_mfma(t4[i], acc[i], X[I]);
+            if (is_w) {
 #pragma unroll
-            for (int s = 0; s < t; s += 4) {             // A is zero from its diagonal on
-                const cs_f32x4 a = *(const cs_f32x4*)(As + t * CS_A_STRIDE + s);
-                p0 += a[0] * x[s];
-                p1 += a[1] * x[s + 1];
-                p0 += a[2] * x[s + 2];
-                p1 += a[3] * x[s + 3];
-            }
-            x[t] -= p0 + p1;
-        }
-        if (is_w) {
-#pragma unroll
-            for (int t = 0; t < CS_C; ++t) Wg[t * DP + col] = -x[t];
-        } else {
-            float* u = u0 + (size_t)c * CS_C * H * Dv + (size_t)h * Dv + (col - DP);
-            int off = 0;
-#pragma unroll
-            for (int t = 0; t < CS_C; ++t) {
-                u[off] = x[t];
-                off += H * Dv;
-                asm volatile("" : "+v"(off));
+                for (int i = 0; i < 4; ++i) Wg[cs_at(CS_SUB * I + 4 * g + i, e, DP / 16)] = -X[I][i];
+            } else {
+                *(cs_f32x4*)(ug + (((tile - DP / 16) * 4 + I) * 64 + lane) * 4) = X[I];
             }
         }
     }
@@ -207,8 +280,8 @@ __global__ __launch_bounds__(CS_PREP) void delta_chunks_kernel(const float* __re
 static size_t delta_chunks_lds(int DP) { return ((size_t)3 * CS_C * (DP + 4) + CS_C * CS_A_STRIDE + 4 * DP + CS_C) * sizeof(float); }
 
 // rows as tm_delta_prepare writes them; chunk c holds the rows cu_chunk[c] .. cu_chunk[c + 1] - 1 (1 to 64 of one request). Km, Qm,
-// Wm float [n, H, 64 * DP] (Km as [DP][64]), Pm [n, H, 64, 64], gam [n, H, DP] with DP = 64 or 128 >= D, u0 [64 n, H Dv]
-// (a chunk's 64 rows each, zeros behind its tokens).
+// Wm float [n, H, 64 * DP], Pm [n, H, 64 * 64], gam [n, H, DP] with DP = 64 or 128 >= D, u0
+// [n, H, ceil(Dv / 16), 64 * 16]; matrices in the chain's order.
 extern "C" int tm_delta_chunks(const float* rows, int ld, const int* cu_chunk, int n_chunks, float* Wm, float* Qm, float* Km, float* Pm,
                                float* gam, float* u0, int H, int G, int D, int DP, int Dv, int per_channel, hipStream_t stream) {
     if (n_chunks <= 0) return TM_OK;
@@ -277,18 +350,24 @@ __global__ __launch_bounds__(CS_CHAIN) void retention_chunks_kernel(const float*
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int t = 16 * I + 4 * g + i, s = 16 * J + r;
-            Pg[t * CS_C + s] = s <= t ? acc[i] * pw[t - s] : 0.f;
+            Pg[cs_at(t, s, 4)] = s <= t ? acc[i] * pw[t - s] : 0.f;
         }
     }
     float* Qg = Qm + at * CS_C * DP;
     float* Kg = Km + at * CS_C * DP;
-    for (int idx = tid; idx < CS_C * DP; idx += CS_CHAIN) {
-        const int t = idx / DP, d = idx % DP;
-        Qg[idx] = Qs[t * LD + d] * pw[t + 1];
+    for (int tile = wave; tile < 4 * (DP / 16); tile += CS_CHAIN / TM_WAVE) {
+        const int t = 16 * (tile / (DP / 16)) + r, d = 16 * (tile % (DP / 16)) + 4 * g;
+        *(cs_f32x4*)(Qg + (tile * 64 + lane) * 4) = *(const cs_f32x4*)(Qs + t * LD + d) * pw[t + 1];
     }
-    for (int idx = tid; idx < CS_C * DP; idx += CS_CHAIN) {
-        const int d = idx / CS_C, t = idx % CS_C;
-        Kg[idx] = t < n ? Ks[t * LD + d] * pw[n - 1 - t] : 0.f;
+    for (int tile = wave; tile < 4 * (DP / 16); tile += CS_CHAIN / TM_WAVE) {
+        const int d = 16 * (tile / 4) + r;
+        cs_f32x4 v;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int t = 16 * (tile % 4) + 4 * g + i;
+            v[i] = t < n ? Ks[t * LD + d] * pw[n - 1 - t] : 0.f;
+        }
+        *(cs_f32x4*)(Kg + (tile * 64 + lane) * 4) = v;
     }
     for (int d = tid; d < DP; d += CS_CHAIN) gam[at * DP + d] = pw[n];
 }
@@ -318,50 +397,48 @@ extern "C" int tm_retention_chunks(const float* rows, int ld, const int* cu_chun
 
 // ------------------------------------------------------------------------------------------------ the chain
 
-// What a wavefront reads of a chunk, in the operands' places: rows r of its 16 tokens (or of its tiles of key channels), sixteen
-// bytes at channel (or token) 4 g of every tile of 16.
+// What a wavefront reads of a chunk, in the operands' places.
 template <int NDT, bool HAS_W>
 struct ChunkRegs {
     static constexpr int NJ = NDT / 4;                  // tiles of 16 key channels of a wavefront's share of the state
-    cs_f32x4 w[HAS_W ? NDT : 1], q[NDT], p[4], k[NJ][4], gam[NJ];
-    float u[4];
+    cs_f32x4 w[HAS_W ? NDT : 1], q[NDT], p[4], k[NJ][4], gam[NJ], u;
 };
 
+// Where a wavefront's operands of one (chunk, head) start.
 template <int NDT, bool HAS_W>
-__device__ __forceinline__ void load_chunk(ChunkRegs<NDT, HAS_W>& x, const float* __restrict__ Wm, const float* __restrict__ Qm,
-                                           const float* __restrict__ Km, const float* __restrict__ Pm, const float* __restrict__ gam,
-                                           const float* __restrict__ u0, int ldu, size_t at, int row0, int n, int wave, int r, int g,
-                                           bool col) {
-    constexpr int DP = 16 * NDT, NJ = ChunkRegs<NDT, HAS_W>::NJ;
-    const size_t mine = (at * CS_C + 16 * wave + r) * DP + 4 * g;
+struct ChunkPlaces {
+    const float *w, *q, *p, *k, *gam, *u;
+    int u_row[4];                                       // without W: offsets of the lane's four rows of values
+
+    __device__ __forceinline__ ChunkPlaces(const float* Wm, const float* Qm, const float* Km, const float* Pm, const float* gm, const float* u0,
+                                           int ldu, size_t at, int row0, int n, int wave, int r, int g) {
+        const int lane = 16 * g + r;
+        const size_t mine = (at * 4 + wave) * NDT * 256 + 4 * lane;
+        w = Wm + mine;
+        q = Qm + mine;
+        p = Pm + (at * 4 + wave) * 4 * 256 + 4 * lane;
+        k = Km + (at * NDT + wave * (NDT / 4)) * 4 * 256 + 4 * lane;
+        gam = gm + (at * NDT + wave * (NDT / 4)) * 16 + 4 * g;
+        u = HAS_W ? u0 + at * ldu + (wave * 64 + lane) * 4 : u0 + (size_t)row0 * ldu;
 #pragma unroll
-    for (int dt = 0; dt < NDT; ++dt) {
-        if (HAS_W) x.w[dt] = *(const cs_f32x4*)(Wm + mine + 16 * dt);
-        x.q[dt] = *(const cs_f32x4*)(Qm + mine + 16 * dt);
+        for (int i = 0; i < 4; ++i) {
+            const int t = 16 * wave + 4 * g + i;        // a row behind the chunk's tokens meets zeros everywhere: any will do
+            u_row[i] = (t < n ? t : n - 1) * ldu;
+        }
     }
-#pragma unroll
-    for (int tt = 0; tt < 4; ++tt)
-        if (tt <= wave) x.p[tt] = *(const cs_f32x4*)(Pm + (at * CS_C + 16 * wave + r) * CS_C + 16 * tt + 4 * g);
-#pragma unroll
-    for (int j = 0; j < NJ; ++j) {
-        const int dt = wave * NJ + j;
-#pragma unroll
-        for (int tt = 0; tt < 4; ++tt) x.k[j][tt] = *(const cs_f32x4*)(Km + (at * DP + 16 * dt + r) * CS_C + 16 * tt + 4 * g);
-        x.gam[j] = *(const cs_f32x4*)(gam + at * DP + 16 * dt + 4 * g);
+    __device__ __forceinline__ cs_f32x4 load_u() const {
+        return HAS_W ? *(const cs_f32x4*)u : cs_f32x4{u[u_row[0]], u[u_row[1]], u[u_row[2]], u[u_row[3]]};
     }
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        const int t = 16 * wave + 4 * g + i;
-        x.u[i] = (col && t < n) ? u0[(size_t)(row0 + t) * ldu] : 0.f;
-    }
-}
+};
 
 // grid (H, ceil(Dv / 16), requests); a block is four wavefronts and 16 columns of a request's and head's state. A wavefront owns 16
 // of a chunk's tokens (rows of U and O) and a quarter of the state's rows. The matrix unit leaves a 16x16 result with four
 // consecutive rows in a lane, and takes its second operand one row a lane: with the rows of every product's inner sum dealt the
 // same way (row 16 tile + 4 g + i to lane group g, instruction i) a result is the next product's operand as it lies. U and S go
-// through LDS (column by column, so that a lane's four rows are one piece) because every wavefront needs all their rows. The next
-// chunk's operands are asked for before the current chunk is worked on.
+// through LDS (column by column, so that a lane's four rows are one piece) because every wavefront needs all their rows. An
+// operand's registers are filled with the next chunk's as soon as its products are issued (the last chunk asks for itself again), a
+// few loads at a time between the products: asked for in one go they hold up the products behind them. Every load is unconditional:
+// behind a test the compiler waits for what is on its way.
 // Neighbouring blocks are heads, so that (heads in multiples of eight) the blocks that read one head's chunks share an L2.
 template <int NDT, bool HAS_W>
 __global__ __launch_bounds__(CS_CHAIN) void chunk_chain_kernel(const float* __restrict__ Wm, const float* __restrict__ Qm,
@@ -379,7 +456,8 @@ __global__ __launch_bounds__(CS_CHAIN) void chunk_chain_kernel(const float* __re
     const int c0 = first_chunk[s], c1 = first_chunk[s + 1];
     if (c1 <= c0) return;                                           // the whole block
     float* st = state + (((size_t)state_slots[s] * H + h) * D) * Dv + (col ? e : 0);
-    const float* u_col = u0 + (size_t)h * Dv + (col ? e : 0);
+    const float* u_mine = HAS_W ? u0 + (size_t)blockIdx.y * CS_C * 16 : u0 + (size_t)h * Dv + (col ? e : 0);
+    if (HAS_W) ldu = gridDim.y * CS_C * 16;                         // from one (chunk, head) to the next
     cs_f32x4 S[NJ];
 #pragma unroll
     for (int j = 0; j < NJ; ++j) {
@@ -388,53 +466,84 @@ __global__ __launch_bounds__(CS_CHAIN) void chunk_chain_kernel(const float* __re
         for (int i = 0; i < 4; ++i) S[j][i] = (col && d0 + i < D) ? st[(size_t)(d0 + i) * Dv] : 0.f;
         *(cs_f32x4*)(Ss + r * SLD + d0) = S[j];
     }
-    ChunkRegs<NDT, HAS_W> now, next;
-    int row0 = cu_chunk[c0], row1 = cu_chunk[c0 + 1];
-    load_chunk<NDT, HAS_W>(now, Wm, Qm, Km, Pm, gam, u_col, ldu, (size_t)c0 * H + h, HAS_W ? c0 * CS_C : row0, row1 - row0, wave, r, g, col);
-    __syncthreads();
-    for (int c = c0; c < c1; ++c) {
-        const int n = row1 - row0;
-        const int cn = c + 1 < c1 ? c + 1 : c;                      // the last chunk asks for itself again
-        const int nrow0 = cu_chunk[cn], nrow1 = cu_chunk[cn + 1];
-        load_chunk<NDT, HAS_W>(next, Wm, Qm, Km, Pm, gam, u_col, ldu, (size_t)cn * H + h, HAS_W ? cn * CS_C : nrow0,
-                                 nrow1 - nrow0, wave, r, g, col);
-        // U = U0 + W S, O = (G Q) S
-        cs_f32x4 U = {now.u[0], now.u[1], now.u[2], now.u[3]}, O = {0.f, 0.f, 0.f, 0.f};
+    ChunkRegs<NDT, HAS_W> x;
+    int row0 = cu_chunk[c0], n = cu_chunk[c0 + 1] - row0;
+    {
+        const ChunkPlaces<NDT, HAS_W> at(Wm, Qm, Km, Pm, gam, u_mine, ldu, (size_t)c0 * H + h, row0, n, wave, r, g);
+        x.u = at.load_u();                                          // in the order in which the loop uses and asks for them again
 #pragma unroll
         for (int dt = 0; dt < NDT; ++dt) {
-            const cs_f32x4 s4 = *(const cs_f32x4*)(Ss + r * SLD + 16 * dt + 4 * g);
+            if (HAS_W) x.w[dt] = *(const cs_f32x4*)(at.w + 256 * dt);
+            x.q[dt] = *(const cs_f32x4*)(at.q + 256 * dt);
+        }
+#pragma unroll
+        for (int tt = 0; tt < 4; ++tt) {
+            x.p[tt] = *(const cs_f32x4*)(at.p + 256 * tt);          // (beyond the diagonal: not looked at)
+#pragma unroll
+            for (int j = 0; j < NJ; ++j) x.k[j][tt] = *(const cs_f32x4*)(at.k + (4 * j + tt) * 256);
+        }
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) x.gam[j] = *(const cs_f32x4*)(at.gam + 16 * j);
+    }
+    __syncthreads();
+    for (int c = c0; c < c1; ++c) {
+        const int cn = c + 1 < c1 ? c + 1 : c;
+        const int nrow0 = cu_chunk[cn], nn = cu_chunk[cn + 1] - nrow0;
+        const ChunkPlaces<NDT, HAS_W> next(Wm, Qm, Km, Pm, gam, u_mine, ldu, (size_t)cn * H + h, nrow0, nn, wave, r, g);
+        // U = U0 + W S, O = (G Q) S
+        cs_f32x4 U = x.u, O = {0.f, 0.f, 0.f, 0.f};
+        x.u = next.load_u();
+        cs_f32x4 s4 = *(const cs_f32x4*)(Ss + r * SLD + 4 * g);
+#pragma unroll
+        for (int dt = 0; dt < NDT; ++dt) {
+            const cs_f32x4 ahead = *(const cs_f32x4*)(Ss + r * SLD + 16 * (dt + 1 < NDT ? dt + 1 : dt) + 4 * g);
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                if (HAS_W) U = cs_mfma(now.w[dt][i], s4[i], U);
-                O = cs_mfma(now.q[dt][i], s4[i], O);
+                if (HAS_W) U = cs_mfma(x.w[dt][i], s4[i], U);
+                O = cs_mfma(x.q[dt][i], s4[i], O);
             }
+            if (HAS_W) x.w[dt] = *(const cs_f32x4*)(next.w + 256 * dt);
+            x.q[dt] = *(const cs_f32x4*)(next.q + 256 * dt);
+            s4 = ahead;
+            __builtin_amdgcn_sched_barrier(0);
         }
         *(cs_f32x4*)(Us + r * ULD + 16 * wave + 4 * g) = U;
         __syncthreads();                                            // U is whole, and every wavefront has read S
         // S <- G_n S + (G_n / G K)^T U, O += P U
+        cs_f32x4 u4 = *(const cs_f32x4*)(Us + r * ULD + 4 * g);
 #pragma unroll
-        for (int j = 0; j < NJ; ++j) S[j] = now.gam[j] * S[j];
+        for (int j = 0; j < NJ; ++j) {
+            S[j] = x.gam[j] * S[j];
+            x.gam[j] = *(const cs_f32x4*)(next.gam + 16 * j);
+        }
 #pragma unroll
         for (int tt = 0; tt < 4; ++tt) {
-            const cs_f32x4 u4 = *(const cs_f32x4*)(Us + r * ULD + 16 * tt + 4 * g);
+            const cs_f32x4 ahead = *(const cs_f32x4*)(Us + r * ULD + 16 * (tt < 3 ? tt + 1 : tt) + 4 * g);
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                if (tt <= wave) O = cs_mfma(now.p[tt][i], u4[i], O);
+            for (int i = 0; i < 4; ++i)
 #pragma unroll
-                for (int j = 0; j < NJ; ++j) S[j] = cs_mfma(now.k[j][tt][i], u4[i], S[j]);
+                for (int j = 0; j < NJ; ++j) S[j] = cs_mfma(x.k[j][tt][i], u4[i], S[j]);
+            if (tt <= wave) {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) O = cs_mfma(x.p[tt][i], u4[i], O);
             }
+            x.p[tt] = *(const cs_f32x4*)(next.p + 256 * tt);
+#pragma unroll
+            for (int j = 0; j < NJ; ++j) x.k[j][tt] = *(const cs_f32x4*)(next.k + (4 * j + tt) * 256);
+            u4 = ahead;
+            __builtin_amdgcn_sched_barrier(0);
         }
 #pragma unroll
         for (int j = 0; j < NJ; ++j) *(cs_f32x4*)(Ss + r * SLD + 16 * (wave * NJ + j) + 4 * g) = S[j];
+        float* out = o + ((size_t)row0 * H + h) * Dv + e;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int t = 16 * wave + 4 * g + i;
-            if (col && t < n) o[((size_t)(row0 + t) * H + h) * Dv + e] = O[i];
+            if (col && t < n) out[(size_t)t * H * Dv] = O[i];
         }
         __syncthreads();                                            // S is whole, and every wavefront has read U
-        now = next;
         row0 = nrow0;
-        row1 = nrow1;
+        n = nn;
     }
 #pragma unroll
     for (int j = 0; j < NJ; ++j)
@@ -446,14 +555,14 @@ __global__ __launch_bounds__(CS_CHAIN) void chunk_chain_kernel(const float* __re
 }
 
 // The chunks first_chunk[s] .. first_chunk[s + 1] - 1 of every request s, in order, from and to the request's row of state
-// [slots, H, D, Dv]. Wm null: U is U0 itself (a retention: u0 are the values, a row a token of
-// the step); else u0 holds 64 rows a chunk. u0: column h Dv + e of rows ldu apart; o [T, H Dv].
+// [slots, H, D, Dv]. Wm null: U is U0 itself (a retention: u0 are the values, column
+// h Dv + e of rows ldu apart, a row a token of the step); else u0 is tm_delta_chunks' own. o [T, H Dv].
 extern "C" int tm_chunk_chain(const float* Wm, const float* Qm, const float* Km, const float* Pm, const float* gam, const float* u0,
                               int ldu, float* o, float* state, const int* cu_chunk, const int* first_chunk, const int* state_slots,
                               int S, int H, int D, int DP, int Dv, hipStream_t stream) {
     if (S <= 0) return TM_OK;
     if (!Qm || !Km || !Pm || !gam || !u0 || !o || !state || !cu_chunk || !first_chunk || !state_slots || H <= 0 || D <= 0 || D > DP ||
-        Dv <= 0 || S > 65535 || (Dv + 15) / 16 > 65535 || ldu < H * Dv)
+        Dv <= 0 || S > 65535 || (Dv + 15) / 16 > 65535 || (!Wm && ldu < H * Dv))
         return TM_ERR_ARG;
     const dim3 grid(H, (Dv + 15) / 16, S);
 #define CS_GO(NDT_, W_)                                                                                                              \

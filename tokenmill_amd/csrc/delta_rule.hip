@@ -51,59 +51,90 @@ __device__ __forceinline__ float delta_conv_channel(const T* __restrict__ proj, 
     return silu_f32(acc);
 }
 
-// grid (T, G + ceil(H Dv / 256) [+ ceil(H D / 256)]); a block is a token and either one q/k head (a thread a channel of q and of
-// k; the head's three sums by the block's fixed tree) or 256 channels of v; the first block of v also makes the token's step
-// sizes and its decays per head; with decays per channel (z) the last blocks make 256 of those each. Few tokens still make many
-// blocks, and a thread's loads are a handful.
 __device__ __forceinline__ float delta_decay(float a, float a_log) {
     const float sp = fmaxf(a, 0.f) + log1pf(expf(-fabsf(a)));                    // softplus
     return expf(-expf(a_log) * sp);
 }
 
-template <typename T>
+// grid (ceil(T / TT), G + ceil(H Dv / 256) [+ ceil(H D / 256)]); a block is TT tokens and either one q/k head or 256 channels of v; the
+// first block of v also makes the tokens' step sizes and their decays per head; with decays per channel (z) the last blocks make
+// 256 of those each. TT = 1: few tokens still make many blocks.
+template <typename T, int TT>
 __global__ __launch_bounds__(DP_THREADS) void delta_prepare_kernel(const T* __restrict__ proj, int ld, const T* __restrict__ conv_w,
                                                                    const T* __restrict__ conv_state, const float* __restrict__ ba,
                                                                    int ldba, const float* __restrict__ z, int ldz,
                                                                    const float* __restrict__ a_log,
                                                                    const float* __restrict__ dt_bias, const int* __restrict__ cu,
                                                                    const int* __restrict__ slots, const int* __restrict__ seq_of_token,
-                                                                   float* __restrict__ out, int ldo, int H, int G, int D, int Dv,
+                                                                   float* __restrict__ out, int ldo, int tokens, int H, int G, int D, int Dv,
                                                                    int taps, float unit_eps) {
-    __shared__ float red[DP_THREADS / TM_WAVE];
-    const int t = blockIdx.x, unit = blockIdx.y;
-    const int s = seq_of_token[t];
-    const int first = cu[s], i = t - first;                  // the token's place among its request's rows of this step
-    const int C = 2 * G * D + H * Dv;
-    const T* st = conv_state + (size_t)slots[s] * (taps - 1) * C;
-    float* o = out + (size_t)t * ldo;
-    if (unit < G) {                                          // D <= 256: a thread has one channel of the head's q and one of its k
-        const int c = threadIdx.x;
-        const bool in = c < D;
-        const float q = in ? delta_conv_channel<T>(proj, ld, conv_w, st, C, taps, first, i, unit * D + c) : 0.f;
-        const float k = in ? delta_conv_channel<T>(proj, ld, conv_w, st, C, taps, first, i, G * D + unit * D + c) : 0.f;
-        const float sq = block_sum<DP_THREADS>(q * q, red), sk = block_sum<DP_THREADS>(k * k, red), qk = block_sum<DP_THREADS>(q * k, red);
-        const float iq = (1.0f / sqrtf((float)D)) / sqrtf(sq + unit_eps), ik = 1.0f / sqrtf(sk + unit_eps);
-        if (in) {
-            o[unit * D + c] = q * iq;
-            o[G * D + unit * D + c] = k * ik;
-        }
-        if (c == 0) o[C + 2 * H + unit] = qk * iq * ik;
-        return;
-    }
+    const int unit = blockIdx.y, C = 2 * G * D + H * Dv;
     const int v_units = (H * Dv + DP_THREADS - 1) / DP_THREADS;
-    if (unit >= G + v_units) {
-        const int n = (unit - G - v_units) * DP_THREADS + threadIdx.x;
-        if (n < H * D) o[C + 2 * H + G + n] = delta_decay(z[(size_t)t * ldz + n] + dt_bias[n], a_log[n / D]);
+    if (unit < G) {
+        // a head's sums are those of its 64-channel pieces, added in order: with TT > 1 a wavefront a token makes one after the
+        // other, with TT = 1 the block's wavefronts a piece each
+        constexpr int PIECES = DP_THREADS / TM_WAVE, MINE = TT == 1 ? 1 : PIECES;        // D <= 256
+        __shared__ float red[PIECES][3];
+        const int wave = threadIdx.x / TM_WAVE, lane = threadIdx.x % TM_WAVE, t = blockIdx.x * TT + (TT == 1 ? 0 : wave);
+        if (TT > 1 && (wave >= TT || t >= tokens)) return;
+        const int s = seq_of_token[t], first = cu[s];
+        const T* st = conv_state + (size_t)slots[s] * (taps - 1) * C;
+        float* o = out + (size_t)t * ldo;
+        float q[MINE], k[MINE], sq = 0.f, sk = 0.f, qk = 0.f;
+#pragma unroll
+        for (int i = 0; i < MINE; ++i) {
+            const int c = lane + TM_WAVE * (TT == 1 ? wave : i);
+            q[i] = k[i] = 0.f;
+            if (c < D) {
+                q[i] = delta_conv_channel<T>(proj, ld, conv_w, st, C, taps, first, t - first, unit * D + c);
+                k[i] = delta_conv_channel<T>(proj, ld, conv_w, st, C, taps, first, t - first, G * D + unit * D + c);
+            }
+            if (TT == 1 || TM_WAVE * i < D) {
+                sq += wave_sum(q[i] * q[i]);
+                sk += wave_sum(k[i] * k[i]);
+                qk += wave_sum(q[i] * k[i]);
+            }
+        }
+        if constexpr (TT == 1) {
+            if (lane == 0) red[wave][0] = sq, red[wave][1] = sk, red[wave][2] = qk;
+            __syncthreads();
+            sq = red[0][0], sk = red[0][1], qk = red[0][2];
+#pragma unroll
+            for (int w = 1; w < PIECES; ++w) sq += red[w][0], sk += red[w][1], qk += red[w][2];
+        }
+        const float iq = (1.0f / sqrtf((float)D)) / sqrtf(sq + unit_eps), ik = 1.0f / sqrtf(sk + unit_eps);
+#pragma unroll
+        for (int i = 0; i < MINE; ++i) {
+            const int c = lane + TM_WAVE * (TT == 1 ? wave : i);
+            if (c < D) {
+                o[unit * D + c] = q[i] * iq;
+                o[G * D + unit * D + c] = k[i] * ik;
+            }
+        }
+        if (lane == 0 && (TT > 1 || wave == 0)) o[C + 2 * H + unit] = qk * iq * ik;
         return;
     }
-    const int c = 2 * G * D + (unit - G) * DP_THREADS + threadIdx.x;
-    if (c < C) o[c] = delta_conv_channel<T>(proj, ld, conv_w, st, C, taps, first, i, c);
-    if (unit == G)
-        for (int h = threadIdx.x; h < H; h += DP_THREADS) {
-            const float b = ba[(size_t)t * ldba + h];
-            o[C + h] = 1.0f / (1.0f + expf(-b));
-            if (!z) o[C + H + h] = delta_decay(ba[(size_t)t * ldba + H + h] + dt_bias[h], a_log[h]);
+#pragma unroll
+    for (int tt = 0; tt < TT; ++tt) {
+        const int t = blockIdx.x * TT + tt;
+        if (t >= tokens) return;
+        float* o = out + (size_t)t * ldo;
+        if (unit >= G + v_units) {
+            const int n = (unit - G - v_units) * DP_THREADS + threadIdx.x;
+            if (n < H * D) o[C + 2 * H + G + n] = delta_decay(z[(size_t)t * ldz + n] + dt_bias[n], a_log[n / D]);
+            continue;
         }
+        const int s = seq_of_token[t], first = cu[s];        // t - first: the token's place among its request's rows of this step
+        const int c = 2 * G * D + (unit - G) * DP_THREADS + threadIdx.x;
+        if (c < C)
+            o[c] = delta_conv_channel<T>(proj, ld, conv_w, conv_state + (size_t)slots[s] * (taps - 1) * C, C, taps, first, t - first, c);
+        if (unit == G)
+            for (int h = threadIdx.x; h < H; h += DP_THREADS) {
+                const float b = ba[(size_t)t * ldba + h];
+                o[C + h] = 1.0f / (1.0f + expf(-b));
+                if (!z) o[C + H + h] = delta_decay(ba[(size_t)t * ldba + H + h] + dt_bias[h], a_log[h]);
+            }
+    }
 }
 
 extern "C" int tm_delta_prepare(const void* proj, int ld, const void* conv_w, const void* conv_state, const float* ba, int ldba,
@@ -119,15 +150,18 @@ extern "C" int tm_delta_prepare(const void* proj, int ld, const void* conv_w, co
     if (ld < C || ldo < C + 2 * H + G + (z ? (long long)H * D : 0) || units > 65535) return TM_ERR_ARG;
     if (dtype != TM_F32 && dtype != TM_BF16) return TM_ERR_ARG;
     if (T == 0) return TM_OK;
-    const dim3 grid(T, (unsigned)units);
-    if (dtype == TM_F32)
-        delta_prepare_kernel<float><<<grid, DP_THREADS, 0, stream>>>((const float*)proj, ld, (const float*)conv_w, (const float*)conv_state,
-                                                                     ba, ldba, z, ldz, a_log, dt_bias, cu_q_lens, state_slots, seq_of_token, out,
-                                                                     ldo, H, G, D, Dv, taps, unit_eps);
-    else
-        delta_prepare_kernel<bf16_t><<<grid, DP_THREADS, 0, stream>>>((const bf16_t*)proj, ld, (const bf16_t*)conv_w,
-                                                                      (const bf16_t*)conv_state, ba, ldba, z, ldz, a_log, dt_bias, cu_q_lens,
-                                                                      state_slots, seq_of_token, out, ldo, H, G, D, Dv, taps, unit_eps);
+    const bool few = (long long)T * units <= 4096;           // a token a block while that many blocks run in a few rounds
+    const dim3 grid(few ? T : (T + 3) / 4, (unsigned)units);
+#define DP_GO(T_, TT_)                                                                                                            \
+    delta_prepare_kernel<T_, TT_><<<grid, DP_THREADS, 0, stream>>>((const T_*)proj, ld, (const T_*)conv_w, (const T_*)conv_state, ba, ldba, \
+                                                                   z, ldz, a_log, dt_bias, cu_q_lens, state_slots, seq_of_token, out, ldo, \
+                                                                   T, H, G, D, Dv, taps, unit_eps)
+    if (dtype == TM_F32) {
+        if (few) DP_GO(float, 1); else DP_GO(float, 4);
+    } else {
+        if (few) DP_GO(bf16_t, 1); else DP_GO(bf16_t, 4);
+    }
+#undef DP_GO
     TM_CHECK_LAUNCH();
     return TM_OK;
 }

@@ -2149,11 +2149,11 @@ def delta_chunk_scan(rows: torch.Tensor, o: torch.Tensor, state: torch.Tensor, c
     _need(H % G == 0 and H > 0 and Dv > 0, "delta_chunk_scan: sizes the kernel does not take")
     _check_chunks(cu_chunk, n, first_chunk, state_slots, num_seqs)
     DP, Wm, Qm, Km, Pm, gam = _chunk_space(n, H, D, rows.device, w=True)
-    u0 = torch.empty((n * CHUNK, H * Dv), dtype=torch.float32, device=rows.device)
+    u0 = torch.empty(n * H * -(-Dv // 16) * CHUNK * 16, dtype=torch.float32, device=rows.device)
     _check(library().tm_delta_chunks(_p(rows), c_int(rows.shape[1]), _p(cu_chunk), c_int(n), _p(Wm), _p(Qm), _p(Km), _p(Pm), _p(gam), _p(u0),
                                      c_int(H), c_int(G), c_int(D), c_int(DP), c_int(Dv), c_int(1 if per_channel else 0), _stream()),
            "delta_chunks")
-    _check(library().tm_chunk_chain(_p(Wm), _p(Qm), _p(Km), _p(Pm), _p(gam), _p(u0), c_int(H * Dv), _p(o), _p(state), _p(cu_chunk),
+    _check(library().tm_chunk_chain(_p(Wm), _p(Qm), _p(Km), _p(Pm), _p(gam), _p(u0), c_int(0), _p(o), _p(state), _p(cu_chunk),
                                     _p(first_chunk), _p(state_slots), c_int(num_seqs), c_int(H), c_int(D), c_int(DP), c_int(Dv), _stream()),
            "chunk_chain")
     return o
@@ -2178,3 +2178,78 @@ def retention_chunk_scan(rows: torch.Tensor, decay: torch.Tensor, o: torch.Tenso
                                     _p(cu_chunk), _p(first_chunk), _p(state_slots), c_int(num_seqs), c_int(H), c_int(D), c_int(DP), c_int(Dv),
                                     _stream()), "chunk_chain")
     return o
+
+
+# -------------------------------------------------------------------------------------------- single tokens of the recurrences
+
+def _rows_of(t: torch.Tensor, n: int, width: int, what: str) -> int:
+    """Row stride of a [n, >= width] view with unit inner stride."""
+    _need(t.dim() == 2 and t.shape[0] == n and t.shape[1] >= width and t.stride(1) == 1, f"{what} is [{n}, >= {width}] with unit inner stride")
+    return t.stride(0) if n > 1 else max(t.stride(0), t.shape[1])
+
+
+def _check_states(state: torch.Tensor, H: int, D: int, Dv: int, who: str) -> None:
+    _need(state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (H, D, Dv), f"{who}: state is float32 [slots, {H}, {D}, {Dv}]")
+
+
+def retention_step_takes(D: int, Dv: int) -> bool:
+    return 0 < D <= 256 and 0 < Dv <= 1024
+
+
+def retention_step(proj: torch.Tensor, cos: torch.Tensor | None, sin: torch.Tensor | None, positions: torch.Tensor, decay: torch.Tensor,
+                   state: torch.Tensor, state_slots: torch.Tensor, y: torch.Tensor, H: int, D: int, Dv: int, k_scale: float,
+                   eps: float) -> torch.Tensor:
+    """Single tokens, one a request: ``retention_prepare``, the recurrence over one row and ``gla_out_gate`` (silu, no weight) in one
+    launch. proj [n, >= 2 H (D + Dv)] = q | k | v | g; positions and state_slots int32 [n]; y [n, H * Dv] of proj's type."""
+    _gpu(proj, cos, sin, positions, decay, state, state_slots, y)
+    n = proj.shape[0]
+    ld = _rows_of(proj, n, 2 * H * (D + Dv), "retention_step: proj")
+    _need(retention_step_takes(D, Dv), "retention_step: sizes the kernel does not take")
+    _need(tuple(y.shape) == (n, H * Dv) and y.is_contiguous() and y.dtype == proj.dtype, f"retention_step: y is [{n}, {H * Dv}] of proj's type")
+    _need(decay.dtype == torch.float32 and decay.is_contiguous() and decay.numel() == H * D, f"retention_step: decay is float32 [{H * D}]")
+    rot = 0
+    if cos is not None:
+        rot = 2 * cos.shape[1]
+        _need(sin is not None and cos.dtype == sin.dtype == torch.float32 and cos.shape == sin.shape and cos.is_contiguous()
+              and sin.is_contiguous() and rot <= D, "retention_step: cos/sin float32 [max_pos, rot/2], rot <= D")
+    _check_states(state, H, D, Dv, "retention_step")
+    _ints(positions, n, "positions")
+    _ints(state_slots, n, "state_slots")
+    _check(library().tm_retention_step(_p(proj), c_int(ld), c_int(code(proj.dtype)), _p(cos), _p(sin), c_int(rot), _p(positions), _p(decay),
+                                       _p(state), _p(state_slots), _p(y), c_int(n), c_int(H), c_int(D), c_int(Dv), c_float(k_scale),
+                                       c_float(eps), _stream()), "retention_step")
+    return y
+
+
+def delta_step_takes(H: int, G: int, D: int, Dv: int) -> bool:
+    return bool(library().tm_delta_step_takes(c_int(H), c_int(G), c_int(D), c_int(Dv)))
+
+
+def delta_step(proj: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Tensor | None, ba: torch.Tensor, z: torch.Tensor | None,
+               a_log: torch.Tensor, dt_bias: torch.Tensor, gate: torch.Tensor, norm_w: torch.Tensor, state: torch.Tensor,
+               state_slots: torch.Tensor, y: torch.Tensor, H: int, G: int, D: int, Dv: int, unit_eps: float, eps: float,
+               sigmoid: bool) -> torch.Tensor:
+    """Single tokens, one a request: ``delta_prepare``, ``delta_conv_state``, the recurrence over one row and ``gla_out_gate`` in one
+    launch. proj [n, >= C], gate [n, >= H * Dv] and y [n, H * Dv] of one type; state_slots int32 [n]."""
+    _gpu(proj, conv_w, conv_state, ba, z, a_log, dt_bias, gate, norm_w, state, state_slots, y)
+    n, taps, C = proj.shape[0], conv_w.shape[1], 2 * G * D + H * Dv
+    ld, ldg = _rows_of(proj, n, C, "delta_step: proj"), _rows_of(gate, n, H * Dv, "delta_step: gate")
+    ldba = _rows_of(ba, n, H if z is not None else 2 * H, "delta_step: ba")
+    ldz = _rows_of(z, n, H * D, "delta_step: z") if z is not None else 0
+    _need(delta_step_takes(H, G, D, Dv), "delta_step: sizes the kernel does not take")
+    _need(tuple(conv_w.shape) == (C, taps) and conv_w.is_contiguous() and conv_w.dtype == proj.dtype == gate.dtype == y.dtype and 1 <= taps <= 16,
+          f"delta_step: conv_w is [{C}, taps] of proj's type, taps up to 16; gate and y of that type")
+    if taps > 1:
+        _need(conv_state is not None and conv_state.dim() == 3 and tuple(conv_state.shape[1:]) == (taps - 1, C) and conv_state.is_contiguous()
+              and conv_state.dtype == proj.dtype, f"delta_step: conv_state is [slots, {taps - 1}, {C}] of proj's type")
+    _need(ba.dtype == torch.float32 and (z is None or z.dtype == torch.float32), "delta_step: ba and z are float32")
+    for name, v, size in (("a_log", a_log, H), ("dt_bias", dt_bias, H * D if z is not None else H), ("norm_w", norm_w, Dv)):
+        _need(v.dtype == torch.float32 and tuple(v.shape) == (size,) and v.is_contiguous(), f"delta_step: {name} is float32 [{size}]")
+    _need(tuple(y.shape) == (n, H * Dv) and y.is_contiguous(), f"delta_step: y is [{n}, {H * Dv}]")
+    _check_states(state, H, D, Dv, "delta_step")
+    _ints(state_slots, n, "state_slots")
+    _check(library().tm_delta_step(_p(proj), c_int(ld), _p(conv_w), _p(conv_state), _p(ba), c_int(ldba), _p(z), c_int(ldz), _p(a_log),
+                                   _p(dt_bias), _p(gate), c_int(ldg), c_int(1 if sigmoid else 0), _p(norm_w), _p(state), _p(state_slots), _p(y),
+                                   c_int(n), c_int(H), c_int(G), c_int(D), c_int(Dv), c_int(taps), c_float(unit_eps), c_float(eps),
+                                   c_int(code(proj.dtype)), _stream()), "delta_step")
+    return y

@@ -178,16 +178,24 @@ class GatedDeltaRule(Mixer):
             gate = proj[:, self.gate_at:]
             if self.gate2 is not None:
                 gate = self.gate2.forward(gate)
-        o = torch.empty((T, self.v_size), dtype=torch.float32, device=x.device)
         y = torch.empty((T, self.v_size), dtype=x.dtype, device=x.device)
+        # the step's single tokens (its last rows and requests) go through one kernel from here to y, where it takes the sizes
+        singles = step.num_decode if ops.delta_step_takes(H, G, D, Dv) else 0
+        P, Tp = step.num_seqs - singles, T - singles
         with profiling.label("recurrence", lambda: self.cost("attention", step, T)):
-            rows = torch.empty((T, ops.delta_row_width(H, G, D, Dv, self.channel_decay)), dtype=torch.float32, device=x.device)
-            ops.delta_prepare(proj, self.conv_w, conv_state, steps, self.a_log, self.dt_bias, step.cu_q_lens, step.state_slots,
-                              step.seq_of_token, step.num_seqs, rows, H, G, D, Dv, UNIT_EPS, z=z)
-            if conv_state is not None:
-                ops.delta_conv_state(proj, self.channels, conv_state, step.cu_q_lens, step.state_slots, step.num_seqs)
-            self._scan(rows, o, matrices, step)
-            ops.gla_out_gate(o, gate, self.norm_w, y, H, Dv, self.norm_eps, sigmoid=self.narrow_gate)
+            if Tp:
+                o = torch.empty((Tp, self.v_size), dtype=torch.float32, device=x.device)
+                rows = torch.empty((Tp, ops.delta_row_width(H, G, D, Dv, self.channel_decay)), dtype=torch.float32, device=x.device)
+                ops.delta_prepare(proj[:Tp], self.conv_w, conv_state, steps[:Tp], self.a_log, self.dt_bias, step.cu_q_lens, step.state_slots,
+                                  step.seq_of_token, P, rows, H, G, D, Dv, UNIT_EPS, z=z[:Tp] if z is not None else None)
+                if conv_state is not None:
+                    ops.delta_conv_state(proj[:Tp], self.channels, conv_state, step.cu_q_lens, step.state_slots, P)
+                self._scan(rows, o, matrices, step, P)
+                ops.gla_out_gate(o, gate[:Tp], self.norm_w, y[:Tp], H, Dv, self.norm_eps, sigmoid=self.narrow_gate)
+            if singles:
+                ops.delta_step(proj[Tp:], self.conv_w, conv_state, steps[Tp:], z[Tp:] if z is not None else None, self.a_log, self.dt_bias,
+                               gate[Tp:], self.norm_w, matrices, step.state_slots[P:], y[Tp:], H, G, D, Dv, UNIT_EPS, self.norm_eps,
+                               self.narrow_gate)
         with profiling.label("o_proj", lambda: self.o.cost(T)):
             return self.o.forward(y)
 
@@ -196,34 +204,34 @@ class GatedDeltaRule(Mixer):
     CHUNKS_FROM = 32
     SEGMENT = 128
 
-    def _scan(self, rows, o, matrices, step: StepContext) -> None:
-        """The recurrence over the step's rows. A step whose longest portion is short (single tokens, small portions) is one
-        scan from the requests' states. Longer portions run in chunks of 64 rows as products of small matrices
-        (``ops.delta_chunk_scan``), and the step's single tokens, if it has any, as a scan beside them. With keys of more channels
-        than that takes, a long portion is cut into segments of ``SEGMENT`` rows: the recurrence is linear in
-        the state, S_end = M S_start + B over any run of tokens, so every segment is first scanned twice side by side with all
-        others, from a zero state (B: what its own rows build) and, without values, from the identity (M: the product of its
-        tokens' transitions g (I - beta k k^T)); a chain over the segments gives each segment's true start state and the
-        request's new state; and a third scan of all segments from those gives the results. Three scans that fill the chip and
-        a short chain of small products, instead of one chain over every token. The sums of a token's result are then ordered
-        otherwise than in the plain chain: the two agree up to 32-bit rounding."""
+    def _scan(self, rows, o, matrices, step: StepContext, num_seqs: int) -> None:
+        """The recurrence over the rows of the step's first ``num_seqs`` requests. A step whose longest portion is short (single
+        tokens, small portions) is one scan from the requests' states. Longer portions run in chunks of 64 rows as products of
+        small matrices (``ops.delta_chunk_scan``), and single tokens among the requests as a scan beside them. With keys of more
+        channels than that takes, a long portion is cut into segments of ``SEGMENT`` rows: the recurrence is linear in the state,
+        S_end = M S_start + B over any run of tokens, so every segment is first scanned twice side by side with all others, from a
+        zero state (B: what its own rows build) and, without values, from the identity (M: the product of its tokens' transitions
+        g (I - beta k k^T)); a chain over the segments gives each segment's true start state and the request's new state; and a
+        third scan of all segments from those gives the results. However the portions run, the sums of a token's result are only
+        ordered otherwise: the ways agree up to 32-bit rounding."""
         H, G, D, Dv = self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim
         ch = self.channel_decay
         if step.max_q_len >= self.CHUNKS_FROM and D <= ops.CHUNK_MAX_KEY_DIM:
             cu_chunk, _, first, n = step_segments(step, ops.CHUNK, rows.device, portions_only=True)
             portions = step.num_seqs - step.num_decode
+            singles = num_seqs - portions
             ops.delta_chunk_scan(rows, o, matrices, cu_chunk, first, n, step.state_slots, portions, H, G, D, Dv, ch)
-            if step.num_decode:
-                ops.delta_scan(rows, o, matrices, step.cu_q_lens[portions:], step.state_slots[portions:], step.num_decode, H, G, D, Dv, per_channel=ch)
+            if singles:
+                ops.delta_scan(rows, o, matrices, step.cu_q_lens[portions:], step.state_slots[portions:], singles, H, G, D, Dv, per_channel=ch)
             return
         if step.max_q_len < 2 * self.SEGMENT:
-            ops.delta_scan(rows, o, matrices, step.cu_q_lens, step.state_slots, step.num_seqs, H, G, D, Dv, per_channel=ch)
+            ops.delta_scan(rows, o, matrices, step.cu_q_lens, step.state_slots, num_seqs, H, G, D, Dv, per_channel=ch)
             return
-        cu_seg, ids, first, n_seg = step_segments(step, self.SEGMENT, rows.device)
+        cu_seg, ids, first, n_seg = step_segments(step, self.SEGMENT, rows.device, portions_only=num_seqs < step.num_seqs)
         local = torch.zeros((n_seg, H, D, Dv), dtype=torch.float32, device=rows.device)
         ops.delta_scan(rows, None, local, cu_seg, ids, n_seg, H, G, D, Dv, per_channel=ch)
         trans = torch.eye(D, dtype=torch.float32, device=rows.device).expand(n_seg, H, D, D).contiguous()
         ops.delta_scan(rows, None, trans, cu_seg, ids, n_seg, H, G, D, D, transitions_of=Dv, per_channel=ch)
         start = torch.empty_like(local)
-        ops.delta_combine(trans, local, start, matrices, step.state_slots, first, step.num_seqs)
+        ops.delta_combine(trans, local, start, matrices, step.state_slots, first, num_seqs)
         ops.delta_scan(rows, o, start, cu_seg, ids, n_seg, H, G, D, Dv, per_channel=ch)

@@ -84,20 +84,27 @@ class Retention(Mixer):
             raise ValueError(f"position {step.max_context_len - 1} is beyond the rotary table ({rot.max_positions} positions)")
         with profiling.label("qkv", lambda: self.cost("qkv", step, T)):
             proj = self.proj.forward(x)                                          # [T, q | k | v | g]
-        o = torch.empty((T, self.v_size), dtype=torch.float32, device=x.device)
         y = torch.empty((T, self.v_size), dtype=x.dtype, device=x.device)
+        cos, sin = (rot.cos, rot.sin) if rot is not None else (None, None)
+        # the step's single tokens (its last rows and requests) go through one kernel from here to y, where it takes the sizes
+        singles = step.num_decode if ops.retention_step_takes(D, Dv) else 0
+        P, Tp = step.num_seqs - singles, T - singles
         with profiling.label("recurrence", lambda: self.cost("attention", step, T)):
-            rows = torch.empty((T, ops.retention_row_width(H, D, Dv)), dtype=torch.float32, device=x.device)
-            ops.retention_prepare(proj, rot.cos if rot is not None else None, rot.sin if rot is not None else None, step.positions, rows,
-                                  H, D, Dv, D ** -0.5)
-            self._scan(rows, o, cache.state, step)
-            ops.gla_out_gate(o, proj[:, 2 * self.k_size + self.v_size:], None, y, H, Dv, self.norm_eps)
+            if Tp:
+                o = torch.empty((Tp, self.v_size), dtype=torch.float32, device=x.device)
+                rows = torch.empty((Tp, ops.retention_row_width(H, D, Dv)), dtype=torch.float32, device=x.device)
+                ops.retention_prepare(proj[:Tp], cos, sin, step.positions, rows, H, D, Dv, D ** -0.5)
+                self._scan(rows, o, cache.state, step, P)
+                ops.gla_out_gate(o, proj[:Tp, 2 * self.k_size + self.v_size:], None, y[:Tp], H, Dv, self.norm_eps)
+            if singles:
+                ops.retention_step(proj[Tp:], cos, sin, step.positions[Tp:], self.decay, cache.state, step.state_slots[P:], y[Tp:], H, D, Dv,
+                                   D ** -0.5, self.norm_eps)
         with profiling.label("o_proj", lambda: self.o.cost(T)):
             return self.o.forward(y)
 
-    def _scan(self, rows, o, state, step: StepContext) -> None:
-        """The recurrence over the step's rows: one scan from the requests' states; for longer portions chunks of 64 rows as
-        products of small matrices (``ops.retention_chunk_scan``), with a scan of the step's single tokens beside them; or, with
+    def _scan(self, rows, o, state, step: StepContext, num_seqs: int) -> None:
+        """The recurrence over the rows of the step's first ``num_seqs`` requests: one scan from the requests' states; for longer portions chunks of 64 rows as
+        products of small matrices (``ops.retention_chunk_scan``), with a scan of single tokens among the requests beside them; or, with
         keys of more channels than that takes, (as in gated linear attention) two scans of a portion's segments side by side with a
         chain of the segments' states between them."""
         H, D, Dv, ks = self.num_heads, self.key_dim, self.value_dim, self.k_size
@@ -105,19 +112,19 @@ class Retention(Mixer):
             cu_chunk, _, first, n = step_segments(step, ops.CHUNK, rows.device, portions_only=True)
             portions = step.num_seqs - step.num_decode
             ops.retention_chunk_scan(rows, self.decay, o, state, cu_chunk, first, n, step.state_slots, portions, H, D, Dv)
-            if step.num_decode:
-                ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, o, state, step.cu_q_lens[portions:], step.state_slots[portions:], step.num_decode,
-                             H, D, Dv, 1.0)
+            if num_seqs > portions:
+                ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, o, state, step.cu_q_lens[portions:], step.state_slots[portions:],
+                             num_seqs - portions, H, D, Dv, 1.0)
             return
         if step.max_q_len < 2 * self.SEGMENT:
-            ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, o, state, step.cu_q_lens, step.state_slots, step.num_seqs, H, D, Dv, 1.0)
+            ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, o, state, step.cu_q_lens, step.state_slots, num_seqs, H, D, Dv, 1.0)
             return
-        cu_seg, ids, first, n_seg = step_segments(step, self.SEGMENT, rows.device)
+        cu_seg, ids, first, n_seg = step_segments(step, self.SEGMENT, rows.device, portions_only=num_seqs < step.num_seqs)
         local = torch.zeros((n_seg, H, D, Dv), dtype=torch.float32, device=rows.device)
         states_only = ops.gla_scan_states_only(rows, 0, ks, self.decay, D)       # else o is written and overwritten below
         ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, None if states_only else o, local, cu_seg, ids, n_seg, H, D, Dv, 1.0)
         products = torch.empty((n_seg, ks), dtype=torch.float32, device=rows.device)
         ops.gla_segment_decay(self.decay, cu_seg, n_seg, products)
         start = torch.empty_like(local)
-        ops.gla_combine(state, step.state_slots, first, products, local, start, step.num_seqs)
+        ops.gla_combine(state, step.state_slots, first, products, local, start, num_seqs)
         ops.gla_scan(rows, 0, ks, 2 * ks, self.decay, o, start, cu_seg, ids, n_seg, H, D, Dv, 1.0)
