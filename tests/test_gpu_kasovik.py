@@ -293,8 +293,8 @@ def test_retention_whole_in_portions_token_by_token_and_beside_another(dt, H, D,
     mixer = Retention(64, H, D, Dv, decay, 1e-5, rotary=rotary)
     w = _weights(mixer, dt, 0.25, H * 5 + D)
     m = {"heads": H, "dim": D, "vdim": Dv, "decay": decay, "rot": {"base": 3e3, "dims": rot} if rot else None}
-    T = 300                                                # whole, the portion is scanned in segments; in pieces, as one chain
-    assert T >= 2 * mixer.SEGMENT
+    T = 300                                                # whole: chunks or (keys of 160) segments; in pieces, scans and chunks
+    assert T >= 2 * mixer.SEGMENT and mixer.CHUNKS_FROM <= 40
     torch.manual_seed(D)
     x = q(torch.randn(T, 64), dt)
     want = q(P.retention(x, m, w, "a.", 1e-5, torch.arange(T), dt), dt)
@@ -345,8 +345,8 @@ def test_delta_rule_with_a_decay_per_channel_whole_in_portions_token_by_token_an
     fixed["A_log"] = torch.rand(H, generator=g) * 5 - 5    # decays from a few tokens to hundreds
     w = _weights(mixer, dt, 0.25, H * 7 + D, **fixed)
     m = {"heads": H, "kv_heads": G_, "dim": D, "vdim": Dv, "conv": taps}
-    T = 300                                                # whole, the portion is scanned in segments; in pieces, as one chain
-    assert T >= 2 * mixer.SEGMENT > T - 113
+    T = 300                                                # whole: chunks or (keys of 160) segments; in pieces, scans and chunks
+    assert T >= 2 * mixer.SEGMENT > T - 113 and mixer.CHUNKS_FROM <= 40
     torch.manual_seed(D)
     x = q(torch.randn(T, 64), dt)
     want = q(P.delta_rule(x, m, w, "a.", 1e-5, dt), dt)
@@ -388,6 +388,142 @@ def test_channels_fade_by_their_own_decays(D):
             for h in range(H):
                 close(got[t, h], v[last, h] * g[h, ask] ** (t - last), torch.float32, f"channel {ask}, head {h}, token {t}")
         assert float(state[0].abs().max()) == 0.0
+
+
+def _delta_rows(T, H, G_, D, Dv, per_channel, g, decays):
+    """Rows as the recurrence takes them, made by hand: unit keys (some of them equal to the one before), decays drawn from
+    ``decays``."""
+    from tokenmill_amd.hip import ops
+    C = 2 * G_ * D + H * Dv
+    rows = torch.zeros(T, ops.delta_row_width(H, G_, D, Dv, per_channel))
+    qk = torch.randn(2, T, G_, D, generator=g)
+    qk[1, 3::7] = qk[1, 2:-1:7][:qk[1, 3::7].shape[0]]
+    qk = qk / qk.norm(dim=-1, keepdim=True)
+    rows[:, :G_ * D], rows[:, G_ * D:2 * G_ * D] = qk[0].reshape(T, -1), qk[1].reshape(T, -1)
+    rows[:, 2 * G_ * D:C] = torch.randn(T, H * Dv, generator=g)
+    rows[:, C:C + H] = torch.rand(T, H, generator=g)
+    rows[::5, C:C + H] = 1.0
+    pool = torch.tensor(decays)
+    if per_channel:
+        rows[:, C + 2 * H + G_:C + 2 * H + G_ + H * D] = pool[torch.randint(0, len(pool), (T, H * D), generator=g)]
+    else:
+        rows[:, C + H:C + 2 * H] = pool[torch.randint(0, len(pool), (T, H), generator=g)]
+    rows[:, C + 2 * H:C + 2 * H + G_] = (qk[0] * qk[1]).sum(-1)
+    return rows
+
+
+LENGTHS = [1, 64, 200, 65, 33, 128, 17]
+
+
+def _chunk_table(lengths):
+    cu, first, row = [0], [0], 0
+    for n in lengths:
+        for lo in range(0, n, 64):
+            row += min(64, n - lo)
+            cu.append(row)
+        first.append(len(cu) - 1)
+    return ints(cu), ints(first), len(cu) - 1
+
+
+@pytest.mark.parametrize("per_channel", [True, False])
+@pytest.mark.parametrize("H,G_,D,Dv", [(2, 1, 8, 6), (4, 2, 64, 48), (2, 2, 100, 130), (3, 1, 128, 16), (8, 4, 128, 128)])
+def test_delta_rule_in_chunks_is_the_scan(H, G_, D, Dv, per_channel):
+    """Portions of ragged lengths from states that are not zero: the chunks' products give the scan's results and states; with
+    decays that hardly forget, that forget at once, that underflow when they are multiplied, and that are zero."""
+    from tokenmill_amd.hip import ops
+    g = torch.Generator().manual_seed(D + Dv)
+    T, S = sum(LENGTHS), len(LENGTHS)
+    for decays in ([0.999, 0.9, 1.0], [0.5, 1e-6, 1e-30, 0.0, 1.0], [0.02, 0.05]):
+        rows = _delta_rows(T, H, G_, D, Dv, per_channel, g, decays).to(DEV)
+        start = torch.randn(S + 1, H, D, Dv, generator=g).to(DEV)
+        slots = torch.randperm(S, generator=g).to(torch.int32).to(DEV)
+        want_o, got_o = torch.empty((T, H * Dv), device=DEV), torch.full((T, H * Dv), math.nan, device=DEV)
+        want_s, got_s = start.clone(), start.clone()
+        ops.delta_scan(rows, want_o, want_s, ints([sum(LENGTHS[:i]) for i in range(S + 1)]), slots, S, H, G_, D, Dv, per_channel=per_channel)
+        cu, first, n = _chunk_table(LENGTHS)
+        ops.delta_chunk_scan(rows, got_o, got_s, cu, first, n, slots, S, H, G_, D, Dv, per_channel)
+        close(got_o.cpu(), want_o.cpu(), torch.float32, f"results, decays {decays}")
+        close(got_s.cpu(), want_s.cpu(), torch.float32, f"states, decays {decays}")
+        assert torch.equal(got_s[S], start[S]), "a slot of nobody's"
+
+
+@pytest.mark.parametrize("H,D,Dv", [(1, 8, 6), (3, 64, 40), (2, 100, 130), (4, 128, 256)])
+def test_retention_in_chunks_is_the_scan(H, D, Dv):
+    from tokenmill_amd.hip import ops
+    g = torch.Generator().manual_seed(D + Dv)
+    T, S = sum(LENGTHS), len(LENGTHS)
+    rows = (torch.randn(T, ops.retention_row_width(H, D, Dv), generator=g) * 0.3).to(DEV)
+    decay = torch.tensor([0.9990234375, 0.5, 1.0, 0.03][:H]).repeat_interleave(D)[None].contiguous().to(DEV)
+    start = torch.randn(S + 1, H, D, Dv, generator=g).to(DEV)
+    slots = torch.randperm(S, generator=g).to(torch.int32).to(DEV)
+    want_o, got_o = torch.empty((T, H * Dv), device=DEV), torch.full((T, H * Dv), math.nan, device=DEV)
+    want_s, got_s = start.clone(), start.clone()
+    ops.gla_scan(rows, 0, H * D, 2 * H * D, decay, want_o, want_s, ints([sum(LENGTHS[:i]) for i in range(S + 1)]), slots, S, H, D, Dv, 1.0)
+    cu, first, n = _chunk_table(LENGTHS)
+    ops.retention_chunk_scan(rows, decay, got_o, got_s, cu, first, n, slots, S, H, D, Dv)
+    close(got_o.cpu(), want_o.cpu(), torch.float32, "results")
+    close(got_s.cpu(), want_s.cpu(), torch.float32, "states")
+    assert torch.equal(got_s[S], start[S]), "a slot of nobody's"
+
+
+@pytest.mark.parametrize("dt", DTS)
+@pytest.mark.parametrize("channel", [True, False])
+@pytest.mark.parametrize("H,G_,D,Dv,taps", [(4, 2, 12, 20, 4), (2, 2, 64, 48, 2), (6, 3, 128, 128, 3), (2, 1, 160, 24, 5), (3, 1, 20, 12, 1), (16, 2, 32, 70, 7)])
+def test_a_single_token_in_one_launch_is_the_same_token_step_by_step(dt, channel, H, G_, D, Dv, taps):
+    """Convolution, norms, decays, recurrence, convolution state and gate as one kernel against the kernels one by one."""
+    from tokenmill_amd.hip import ops
+    assert ops.delta_step_takes(H, G_, D, Dv)
+    g = torch.Generator().manual_seed(D + Dv)
+    n, C = 5, 2 * G_ * D + H * Dv
+    rnd = lambda *shape: torch.randn(*shape, generator=g)      # noqa: E731
+    proj, gate = rnd(n, C + 3).to(dt).to(DEV), rnd(n, H * Dv + 1).to(dt).to(DEV)
+    conv_w = (rnd(C, taps) * 0.5).to(dt).to(DEV)
+    conv_state = rnd(n + 2, taps - 1, C).to(dt).to(DEV) if taps > 1 else None
+    ba, z = rnd(n, 2 * H).to(DEV), rnd(n, H * D).to(DEV) if channel else None
+    a_log, dt_bias, norm_w = (rnd(H) - 1).to(DEV), rnd(H * D if channel else H).to(DEV), (torch.rand(Dv, generator=g) + 0.5).to(DEV)
+    state = rnd(n + 2, H, D, Dv).to(DEV)
+    slots = ints([4, 0, 6, 1, 3])
+    cu, seqs = ints(list(range(n + 1))), ints(list(range(n)))
+    s1, c1 = state.clone(), conv_state.clone() if taps > 1 else None
+    rows = torch.empty((n, ops.delta_row_width(H, G_, D, Dv, channel)), device=DEV)
+    o, want = torch.empty((n, H * Dv), device=DEV), torch.empty((n, H * Dv), dtype=dt, device=DEV)
+    ops.delta_prepare(proj, conv_w, c1, ba, a_log, dt_bias, cu, slots, seqs, n, rows, H, G_, D, Dv, 1e-6, z=z)
+    if taps > 1:
+        ops.delta_conv_state(proj, C, c1, cu, slots, n)
+    ops.delta_scan(rows, o, s1, cu, slots, n, H, G_, D, Dv, per_channel=channel)
+    ops.gla_out_gate(o, gate, norm_w, want, H, Dv, 1e-5, sigmoid=channel)
+    s2, c2, got = state.clone(), conv_state.clone() if taps > 1 else None, torch.full((n, H * Dv), math.nan, dtype=dt, device=DEV)
+    ops.delta_step(proj, conv_w, c2, ba, z, a_log, dt_bias, gate, norm_w, s2, slots, got, H, G_, D, Dv, 1e-6, 1e-5, channel)
+    close(got.float().cpu(), want.float().cpu(), dt, "result", bf16=2.0 ** -7)
+    close(s2.cpu(), s1.cpu(), torch.float32, "state")
+    assert taps == 1 or torch.equal(c2, c1), "convolution state"
+
+
+@pytest.mark.parametrize("dt", DTS)
+@pytest.mark.parametrize("H,D,Dv,rot", [(3, 20, 12, 8), (2, 64, 70, 64), (1, 160, 24, 0), (4, 128, 256, 32), (2, 30, 600, 30)])
+def test_a_single_token_of_a_retention_in_one_launch(dt, H, D, Dv, rot):
+    from tokenmill_amd.hip import ops
+    from tokenmill_amd.parts import RotaryEmbedding
+    g = torch.Generator().manual_seed(D + Dv)
+    n = 5
+    proj = torch.randn(n, 2 * H * (D + Dv), generator=g).to(dt).to(DEV)
+    table = None
+    if rot:
+        table = RotaryEmbedding(D, 1e4, 300, rotary_dim=rot, exact=True)
+        table.build_tables(DEV)
+    cos, sin = (table.cos, table.sin) if rot else (None, None)
+    places, slots = ints([0, 7, 299, 64, 1]), ints([4, 0, 6, 1, 3])
+    decay = torch.tensor([0.999, 0.9, 0.5, 0.97][:H]).repeat_interleave(D)[None].contiguous().to(DEV)
+    state = torch.randn(n + 2, H, D, Dv, generator=g).to(DEV)
+    s1, s2 = state.clone(), state.clone()
+    rows, o = torch.empty((n, ops.retention_row_width(H, D, Dv)), device=DEV), torch.empty((n, H * Dv), device=DEV)
+    want, got = torch.empty((n, H * Dv), dtype=dt, device=DEV), torch.full((n, H * Dv), math.nan, dtype=dt, device=DEV)
+    ops.retention_prepare(proj, cos, sin, places, rows, H, D, Dv, D ** -0.5)
+    ops.gla_scan(rows, 0, H * D, 2 * H * D, decay, o, s1, ints(list(range(n + 1))), slots, n, H, D, Dv, 1.0)
+    ops.gla_out_gate(o, proj[:, H * (2 * D + Dv):], None, want, H, Dv, 1e-5)
+    ops.retention_step(proj, cos, sin, places, decay, s2, slots, got, H, D, Dv, D ** -0.5, 1e-5)
+    close(got.float().cpu(), want.float().cpu(), dt, "result", bf16=2.0 ** -7)
+    close(s2.cpu(), s1.cpu(), torch.float32, "state")
 
 
 @pytest.mark.parametrize("dt", DTS)
