@@ -31,6 +31,7 @@ class _WindowOnly:
     """A group described by its window alone."""
     window: int | None
     chunk = None
+    keep = 0
 
     @property
     def keeps_all(self) -> bool:
@@ -52,7 +53,7 @@ class RequestCache:
     request_id: str
     tables: list[list[int]]                     # per group: page ids by logical page index
     state_slot: int
-    released: list[int] = field(default_factory=list)   # per group: leading pages already given back
+    released: list[int] = field(default_factory=list)   # per group: leading pages already looked at (given back, or kept)
     fresh: bool = True                          # state slot not yet zeroed for this admission
 
     def capacity(self, page_size: int) -> int:
@@ -159,7 +160,8 @@ class CacheManager:
         """Give back, in groups that keep a window or only the current chunk, the pages that no later token
         can see: with ``num_computed`` tokens cached, the next query sits at position >= num_computed and sees
         keys from num_computed - W + 1 on, and none from before the start of the chunk that holds position
-        num_computed. Returns the number of pages given back."""
+        num_computed. Pages of the first tokens that a windowed group keeps beside its window stay. Returns the number of
+        pages given back."""
         given = 0
         if not self.any_window:
             return given
@@ -169,8 +171,9 @@ class CacheManager:
             first_needed = spec.first_needed(num_computed)
             upto = min(first_needed // self.page_size, len(rc.tables[g]))
             table = rc.tables[g]
-            back = [table[i] for i in range(rc.released[g], upto) if table[i] != RELEASED]
-            for i in range(rc.released[g], upto):
+            kept = -(-getattr(spec, "keep", 0) // self.page_size)
+            back = [table[i] for i in range(max(rc.released[g], kept), upto) if table[i] != RELEASED]
+            for i in range(max(rc.released[g], kept), upto):
                 table[i] = RELEASED
             if upto > rc.released[g]:
                 rc.released[g] = upto

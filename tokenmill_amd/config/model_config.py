@@ -738,6 +738,117 @@ class KasovikConfig:
                 raise ConfigError(f"layers[{i}]: the feed-forward's ff and limit must be positive")
 
 
+@dataclass(frozen=True)
+class SanazenLayer:
+    type: str                       # "parallel"
+    mixer: dict                     # the mixer's sizes and constants, as config.json gives them
+    mlp: dict | None                # {"ff", "limit", "experts", "top", "shared": {"ff", "limit"} | None} | None
+
+
+@dataclass
+class SanazenConfig:
+    """The Sanazen decoder: token embedding times a constant plus waves of the position; layers whose mixer and feed-forward read two
+    norms of the same stream; a mixer of two side by side, softmax attention (short convolutions, whole-projection norms, a window
+    with kept first tokens, a gate per channel) and lightning attention (fixed decays), added with constant weights; experts with
+    clamped gates on their weighted input, chosen by a sigmoid router, beside a gated shared expert, or no feed-forward; an output
+    head of its own whose logits are scaled and capped. Every size and constant that can differ between two models is read from
+    config.json; the model has no position limit of its own (``max_positions`` if the file gives one)."""
+
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    embedding_scale: float
+    logit_scale: float
+    logit_softcap: float | None
+    layers: tuple[SanazenLayer, ...]
+    max_position_embeddings: int | None = None
+    eos_token_ids: tuple[int, ...] = field(default_factory=tuple)
+
+    architecture = "Sanazen"
+    MIXERS = ("parallel",)
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @classmethod
+    def from_dict(cls, raw: dict, generation: dict | None = None) -> "SanazenConfig":
+        norm, embedding = _require(raw, "norm"), _require(raw, "embedding")
+        layers: list[SanazenLayer] = []
+        for i, entry in enumerate(_require(raw, "layers")):
+            kind = entry.get("type")
+            if kind not in cls.MIXERS:
+                raise ConfigError(f"layers[{i}]: type '{kind}' is not one of {list(cls.MIXERS)}")
+            mixer = entry.get("mixer")
+            left, right = (mixer.get("left"), mixer.get("right")) if isinstance(mixer, dict) else (None, None)
+            if not isinstance(left, dict) or not isinstance(right, dict):
+                raise ConfigError(f"layers[{i}]: a parallel mixer has 'left' and 'right' sizes")
+            for where, key, what in [(mixer, k, "parallel mixer") for k in ("left_scale", "right_scale")] + \
+                    [(left, k, "left mixer") for k in ("heads", "kv_heads", "dim", "vdim", "scale", "conv")] + \
+                    [(right, k, "right mixer") for k in ("heads", "dim", "vdim", "decay")]:
+                if where.get(key) is None:
+                    raise ConfigError(f"layers[{i}]: the {what} has no '{key}'")
+            mlp = entry.get("mlp")
+            if mlp is not None:
+                if mlp.get("kind", "moe") != "moe":
+                    raise ConfigError(f"layers[{i}]: feed-forward kind '{mlp.get('kind')}' is not 'moe'")
+                expert, router, shared = mlp.get("expert") or {}, mlp.get("router") or {}, mlp.get("shared")
+                wanted = [(expert, "ff", "expert"), (expert, "limit", "expert"), (router, "experts", "router"), (router, "top", "router")]
+                if shared is not None:
+                    wanted += [(shared, "ff", "shared expert"), (shared, "limit", "shared expert")]
+                for where, key, what in wanted:
+                    if where.get(key) is None:
+                        raise ConfigError(f"layers[{i}]: the {what} has no '{key}'")
+                mlp = {"ff": int(expert["ff"]), "limit": float(expert["limit"]), "experts": int(router["experts"]), "top": int(router["top"]),
+                       "shared": {"ff": int(shared["ff"]), "limit": float(shared["limit"])} if shared is not None else None}
+            layers.append(SanazenLayer(kind, dict(mixer), mlp))
+        most, cap = raw.get("max_positions"), raw.get("logit_softcap")
+        cfg = cls(vocab_size=int(_require(raw, "vocab")), hidden_size=int(_require(raw, "width")), norm_eps=float(_require(norm, "eps")),
+                  embedding_scale=float(_require(embedding, "scale")), logit_scale=float(raw.get("logit_scale") if raw.get("logit_scale") is not None else 1.0),
+                  logit_softcap=float(cap) if cap else None, layers=tuple(layers),
+                  max_position_embeddings=int(most) if most is not None else None,
+                  eos_token_ids=collect_eos_ids(([generation] if generation else []) + [raw]))
+        cfg.validate()
+        return cfg
+
+    def validate(self) -> None:
+        for name in ("vocab_size", "hidden_size"):
+            if getattr(self, name) <= 0:
+                raise ConfigError(f"{name} must be positive, got {getattr(self, name)}")
+        if self.max_position_embeddings is not None and self.max_position_embeddings <= 0:
+            raise ConfigError("max_positions must be positive")
+        if not self.norm_eps > 0:
+            raise ConfigError("norm.eps must be positive")
+        if self.logit_softcap is not None and not self.logit_softcap > 0:
+            raise ConfigError("logit_softcap must be positive")
+        if not self.layers:
+            raise ConfigError("a model needs at least one layer")
+        for i, layer in enumerate(self.layers):
+            left, right = layer.mixer["left"], layer.mixer["right"]
+            for side, part, keys in (("left", left, ("heads", "kv_heads", "dim", "vdim")), ("right", right, ("heads", "dim", "vdim"))):
+                for key in keys:
+                    if int(part[key]) <= 0:
+                        raise ConfigError(f"layers[{i}]: {side}.{key} must be positive")
+            if int(left["heads"]) % int(left["kv_heads"]):
+                raise ConfigError(f"layers[{i}]: left: {left['heads']} heads do not divide into {left['kv_heads']} kv_heads")
+            if int(left["conv"]) < 1:
+                raise ConfigError(f"layers[{i}]: left.conv must be at least 1")
+            mask = left.get("mask") or {}
+            if mask.get("size") is not None and int(mask["size"]) < 1:
+                raise ConfigError(f"layers[{i}]: left: mask.size must be at least 1")
+            if int(mask.get("keep_first") or 0) < 0:
+                raise ConfigError(f"layers[{i}]: left: mask.keep_first must not be negative")
+            if len(right["decay"]) != int(right["heads"]):
+                raise ConfigError(f"layers[{i}]: right: {len(right['decay'])} decays for {right['heads']} heads")
+            mlp = layer.mlp
+            if mlp is not None:
+                for part in (mlp, mlp["shared"]):
+                    if part is not None and (part["ff"] <= 0 or not part["limit"] > 0):
+                        raise ConfigError(f"layers[{i}]: an expert's ff and limit must be positive")
+                if not 0 < mlp["top"] <= mlp["experts"]:
+                    raise ConfigError(f"layers[{i}]: {mlp['top']} of {mlp['experts']} experts")
+
+
 def read_json(path: Path) -> dict:
     try:
         return json.loads(path.read_text())

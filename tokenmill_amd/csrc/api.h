@@ -41,30 +41,38 @@ int tm_attn_paged_generic(const void* q, int q_stride, void* out, int out_stride
                           const int* positions, int T, int H, int KVH, int D, int page, float scale, int window,
                           int dtype, hipStream_t stream);
 
-// The same with keys and values of different sizes (D, DV), scores capped smoothly at +-softcap (0: as they are) and a gate
+// The same with keys and values of different sizes (D, DV), with a window the first `keep` keys of a request besides, scores capped smoothly at +-softcap (0: as they are) and a gate
 // per (token, head) (float32, rows ldg apart; null: none) whose sigmoid multiplies the head's result;
 // sink (float32 [H]; null: none): one more term exp(sink[h]) in the denominator of head h's softmax, with no key behind it.
 int tm_attn_paged_generic_ext(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                               const int* block_tables, int table_width, const int* seq_of_token, const int* positions, int T, int H,
-                              int KVH, int D, int DV, int page, float scale, int window, float softcap, const float* gate, int ldg,
+                              int KVH, int D, int DV, int page, float scale, int window, int keep, float softcap, const float* gate, int ldg,
                               const float* sink, int dtype, hipStream_t stream);
 
 // The matrix-unit attention kernels with capped scores (softcap > 0: s <- softcap * tanh(s / softcap); 0: as the plain entries)
 // and a sink per head (as above; null: none).
 int tm_attn_prefill_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                              const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH, int D, int page,
-                             float scale, int window, float softcap, const float* sink, hipStream_t stream);
+                             float scale, int window, int keep, float softcap, const float* sink, hipStream_t stream);
 int tm_attn_prefill_shared_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                                const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH, int D, int page,
-                               float scale, int window, float softcap, const float* sink, hipStream_t stream);
+                               float scale, int window, int keep, float softcap, const float* sink, hipStream_t stream);
 int tm_attn_prefill_f32_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                             const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH, int D, int page,
-                            float scale, int window, float softcap, const float* sink, hipStream_t stream);
+                            float scale, int window, int keep, float softcap, const float* sink, hipStream_t stream);
 int tm_attn_decode_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                             const int* block_tables, int table_width, const int* context_lens, float* part_o, float* part_ml,
-                            int max_chunks, int S, int H, int KVH, int D, int page, float scale, int window, float softcap,
+                            int max_chunks, int S, int H, int KVH, int D, int page, float scale, int window, int keep, float softcap,
                             const float* sink, hipStream_t stream);
 
+// The same work behind a short convolution over time (attention_prepare_conv.hip): see the head of that file.
+int tm_conv_norm_rope_store(const void* proj, int ld, int dtype, const void* conv_w, void* conv_state, int taps, const int* cu_q_lens,
+                            const int* state_slots, const int* seq_of_token, int T, int first_single, int n_portions, void* q_out, int H,
+                            int G, int D, int Dv, int rot, int interleaved, const float* q_w, const float* k_w, float eps, int per_head,
+                            const float* cos_t, const float* sin_t, const int* positions, const int* slots, void* k_pool, void* v_pool,
+                            int page, hipStream_t stream);
+// x[t, c] *= sigmoid(gate[t * ldg + c]), gate of x's type
+int tm_channel_gate(void* x, int dtype, const void* gate, int ldg, int T, int N, hipStream_t stream);
 // q and k normed over the whole projection, rotated and stored (attention_prepare.hip): see the head of that file.
 int tm_whole_norm_rope_store(const float* proj, int ld, void* q_out, int dtype, int T, int H, int G, int D, int Dv, int rot,
                              int interleaved, const float* q_w, const float* k_w, float eps, const float* cos_t, const float* sin_t,
@@ -247,7 +255,7 @@ int tm_chunk_chain(const float* Wm, const float* Qm, const float* Km, const floa
 // (recurrence_step.hip): see the head of that file. tm_delta_step_takes: whether the sizes are taken.
 int tm_retention_step(const void* proj, int ld, int dtype, const float* cos_t, const float* sin_t, int rot, const int* positions,
                       const float* decay, float* state, const int* state_slots, void* y, int n, int H, int D, int Dv, float k_scale,
-                      float eps, hipStream_t stream);
+                      float eps, int silu, float* o_out, hipStream_t stream);
 int tm_delta_step_takes(int H, int G, int D, int Dv);
 int tm_delta_step(const void* proj, int ld, const void* conv_w, void* conv_state, const float* ba, int ldba, const float* z, int ldz,
                   const float* a_log, const float* dt_bias, const void* gate, int ldg, int sigmoid, const float* norm_w, float* state,
@@ -256,11 +264,19 @@ int tm_delta_step(const void* proj, int ld, const void* conv_w, void* conv_state
 // A weighted sum of up to three results added to the residual stream, and the RMS norm of the sum (sum_norm.hip): see there.
 int tm_sum_norm(float* resid, const void* y0, float s0, const void* y1, float s1, const void* y2, float s2, const int* rows,
                 const void* w, int w_dtype, void* out, int dtype, int R, int hidden, float eps, hipStream_t stream);
+int tm_sum_norm2(float* resid, const void* y0, float s0, const void* y1, float s1, const void* y2, float s2, const int* rows,
+                 const void* w, const void* w2, int w_dtype, void* out, void* out2, int dtype, int R, int hidden, float eps,
+                 hipStream_t stream);
 // q, k and v of a retention as 32-bit rows, q and k rotated, k scaled (retention.hip): see there.
 int tm_retention_prepare(const void* proj, int ld, int dtype, const float* cos_t, const float* sin_t, int rot, const int* positions,
-                         float* rows, int ldr, int T, int H, int D, int Dv, float k_scale, hipStream_t stream);
+                         float* rows, int ldr, int T, int H, int D, int Dv, float k_scale, int silu,
+                         hipStream_t stream);
 int tm_embed_gather_scaled(const void* table, int dtype, const int* ids, float* out, int T, int hidden, int vocab, float scale,
                            hipStream_t stream);
+// Embedding rows with waves of the position (elementwise.hip), and an output head's scaled and capped logits: see there.
+int tm_embed_waves(const void* table, int dtype, const int* ids, const int* positions, const float* f, float* out, int T, int hidden,
+                   int vocab, float scale, hipStream_t stream);
+int tm_scale_cap(float* x, long long n, float scale, float cap, hipStream_t stream);
 
 // Attention over a shared latent (latent.hip): see the head of that file.
 int tm_latent_prepare(const float* low, int ld, int Lq, int Lk, int Dr, int rot, const float* wq, const float* wk, float eps,
@@ -298,11 +314,17 @@ int tm_moe_combine(const float* part, const int* pair_slot, void* y, int T, int 
 
 // Experts chosen by a router, experts without a gate, experts that stand for the input itself, a shared expert (moe.hip).
 int tm_moe_router(const float* z, int ldz, const float* correction, int T, int E, int top, int* chosen, float* weight,
-                  int over_chosen, hipStream_t stream);
+                  int over_chosen, int sigmoid, hipStream_t stream);
 int tm_moe_route_chosen(const int* ids, const int* table, int T, int top, int E, int real, int tile_rows, int* slot_pair,
                         int* pair_slot, int* tiles, int* n_tiles, hipStream_t stream);
 int tm_moe_up_act(const void* x, int ldx, const int* slot_pair, int top, const void* W, void* act, const int* tiles,
                   const int* n_tiles, int max_tiles, int K, int F, int dtype, hipStream_t stream);
+int tm_moe_clamped(const void* x, int ldx, const int* slot_pair, int top, const float* pair_weight, const void* W, void* act,
+                   const int* tiles, const int* n_tiles, int max_tiles, int K, int F, float limit, float alpha, int dtype,
+                   hipStream_t stream);
+int tm_moe_clamped_mfma(const void* x, int ldx, const int* slot_pair, int top, const float* pair_weight, const void* W, void* act,
+                        const int* tiles, const int* n_tiles, int max_tiles, int tile_rows, int K, int F, float limit, float alpha,
+                        hipStream_t stream);
 int tm_moe_combine_weighted(const float* part, const int* pair_slot, const float* weight, const void* x, int ldx, const float* shared,
                             const float* shared_gate, int ldg, void* y, int T, int top, int N, int dtype, hipStream_t stream);
 int tm_moe_up_act_mfma(const void* x, int ldx, const int* slot_pair, int top, const void* W, void* act, const int* tiles,

@@ -84,13 +84,13 @@ __device__ __forceinline__ void load_table_entries(int (&entry)[4], const int* _
 template <int D>
 __device__ __forceinline__ void load_keys64(Keys64<D>& kv, const bf16_t* __restrict__ k_pool,
                                             const bf16_t* __restrict__ v_pool, const int (&entry)[4], int wbase,
-                                            int ctx, int lo, int kvh, int KVH, int page_shift, int r, int g) {
+                                            int ctx, int keep, int lo, int kvh, int KVH, int page_shift, int r, int g) {
     constexpr int NDC = D / 32, NDT = D / 16;
     const int page_mask = (1 << page_shift) - 1;
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
         const int first = wbase + 16 * q;
-        kv.group_page[q] = (first < ctx && first + 16 > lo) ? entry[q] : -1;                        // wave-uniform
+        kv.group_page[q] = (first < ctx && (first + 16 > lo || first < keep)) ? entry[q] : -1;                        // wave-uniform
     }
     // Every load is unconditional, so that none of them has to be waited for before the next is
     // issued: positions nobody may see read page 0 instead, and keys beyond the context read the rest of
@@ -124,7 +124,7 @@ __device__ __forceinline__ void load_keys64(Keys64<D>& kv, const bf16_t* __restr
 // m is in units of score * scale * log2(e).
 template <int D>
 __device__ __forceinline__ void attend_keys64(const Keys64<D>& kv, const Bf16x8Bits (&qreg)[D / 32], int wbase, int ctx,
-                                              int lo, float scale_log2, float cap_in, float cap_out, int g, float& m, float& l,
+                                              int keep, int lo, float scale_log2, float cap_in, float cap_out, int g, float& m, float& l,
                                               f32x4_t (&o)[D / 16]) {
     constexpr int NDC = D / 32, NDT = D / 16;
     float sc[4][4];                                                 // [tile][row 4g+i of the tile] for head r
@@ -139,7 +139,7 @@ __device__ __forceinline__ void attend_keys64(const Keys64<D>& kv, const Bf16x8B
             const int kj = wbase + tile_key(t, 4 * g + i);
             // cap_in > 0: capped scores, cap * tanh(score * scale / cap), in units of log2 like the plain ones
             const float sv = cap_in > 0.f ? cap_out * tanh_fast(acc[i] * cap_in) : acc[i] * scale_log2;
-            sc[t][i] = (kj < ctx && kj >= lo) ? sv : -INFINITY;
+            sc[t][i] = (kj < ctx && (kj >= lo || kj < keep)) ? sv : -INFINITY;
         }
     }
     m = -INFINITY;
@@ -170,17 +170,17 @@ __device__ __forceinline__ void attend_keys64(const Keys64<D>& kv, const Bf16x8B
         pt.u = u32x4_t{pack_bf16(pr[2 * b][0], pr[2 * b][1]), pack_bf16(pr[2 * b][2], pr[2 * b][3]),
                        pack_bf16(pr[2 * b + 1][0], pr[2 * b + 1][1]), pack_bf16(pr[2 * b + 1][2], pr[2 * b + 1][3])};
         // which of this lane's 8 keys exist (a value beyond the context may hold anything)
-        uint32_t keep[4];
+        uint32_t mask[4];
 #pragma unroll
         for (int w2 = 0; w2 < 4; ++w2) {
             const int ka = wbase + 32 * b + 8 * g + 2 * w2, kb = ka + 1;
-            keep[w2] = ((ka < ctx && ka >= lo) ? 0x0000ffffu : 0u) | ((kb < ctx && kb >= lo) ? 0xffff0000u : 0u);
+            mask[w2] = ((ka < ctx && (ka >= lo || ka < keep)) ? 0x0000ffffu : 0u) | ((kb < ctx && (kb >= lo || kb < keep)) ? 0xffff0000u : 0u);
         }
 #pragma unroll
         for (int dt = 0; dt < NDT; ++dt) {
             Bf16x8Bits vf;
-            vf.u = u32x4_t{kv.v[dt][b][0] & keep[0], kv.v[dt][b][1] & keep[1], kv.v[dt][b][2] & keep[2],
-                           kv.v[dt][b][3] & keep[3]};
+            vf.u = u32x4_t{kv.v[dt][b][0] & mask[0], kv.v[dt][b][1] & mask[1], kv.v[dt][b][2] & mask[2],
+                           kv.v[dt][b][3] & mask[3]};
             o[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf.b, pt.b, o[dt], 0, 0, 0);
         }
     }
@@ -190,14 +190,14 @@ __device__ __forceinline__ void attend_keys64(const Keys64<D>& kv, const Bf16x8B
 template <int D>
 __device__ __forceinline__ void wave_keys64(const Bf16x8Bits (&qreg)[D / 32], const bf16_t* __restrict__ k_pool,
                                             const bf16_t* __restrict__ v_pool, const int* __restrict__ table,
-                                            int table_width, int wbase, int ctx, int lo, int kvh, int KVH,
+                                            int table_width, int wbase, int ctx, int keep, int lo, int kvh, int KVH,
                                             int page_shift, float scale_log2, float cap_in, float cap_out, int r, int g, float& m, float& l,
                                             f32x4_t (&o)[D / 16]) {
     int entry[4];
     load_table_entries(entry, table, table_width, wbase, page_shift);
     Keys64<D> kv;
-    load_keys64<D>(kv, k_pool, v_pool, entry, wbase, ctx, lo, kvh, KVH, page_shift, r, g);
-    attend_keys64<D>(kv, qreg, wbase, ctx, lo, scale_log2, cap_in, cap_out, g, m, l, o);
+    load_keys64<D>(kv, k_pool, v_pool, entry, wbase, ctx, keep, lo, kvh, KVH, page_shift, r, g);
+    attend_keys64<D>(kv, qreg, wbase, ctx, keep, lo, scale_log2, cap_in, cap_out, g, m, l, o);
 }
 
 template <int D>
@@ -221,7 +221,7 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_block_kernel(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
     const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ context_lens, int H, int KVH, int page_shift, float scale_log2, float cap_in, float cap_out,
-    int window, const float* __restrict__ sink) {
+    int window, int keep, const float* __restrict__ sink) {
     constexpr int NDT = D / 16;
     __shared__ float s_m[WAVES][16], s_l[WAVES][16];
     __shared__ float s_o[WAVES][16][16 + 1];                         // one 16-wide d tile at a time
@@ -241,7 +241,9 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_block_kernel(
     f32x4_t o[NDT];
 #pragma unroll
     for (int dt = 0; dt < NDT; ++dt) o[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    const int first = (lo / AD_WKEYS) * AD_WKEYS;                   // aligned to 64 positions
+    // runs of 64 aligned positions: those of the kept first keys, then those of the window
+    const int kept = lo > 0 ? (keep + AD_WKEYS - 1) / AD_WKEYS : 0;
+    const int resume = lo / AD_WKEYS > kept ? lo / AD_WKEYS : kept;
     auto fold = [&](float mi, float li, const f32x4_t (&oi)[NDT]) {  // add a partial to the running one
         const float mn = fmaxf(m, mi);
         const float f0 = (m == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f(m - mn);
@@ -253,10 +255,13 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_block_kernel(
             for (int i = 0; i < 4; ++i) o[dt][i] = o[dt][i] * f0 + oi[dt][i] * f1;
         m = mn;
     };
-    for (int wbase = first + wave * AD_WKEYS; wbase < ctx; wbase += WAVES * AD_WKEYS) {
+    for (int run = wave;; run += WAVES) {
+        const int wbase = (run < kept ? run : resume + run - kept) * AD_WKEYS;
+        if (wbase >= ctx) break;
         float mi, li;
         f32x4_t oi[NDT];
-        wave_keys64<D>(qreg, k_pool, v_pool, table, table_width, wbase, ctx, lo, kvh, KVH, page_shift, scale_log2, cap_in, cap_out, r, g, mi, li, oi);
+        wave_keys64<D>(qreg, k_pool, v_pool, table, table_width, wbase, ctx, keep, lo, kvh, KVH, page_shift, scale_log2, cap_in, cap_out,
+                       r, g, mi, li, oi);
         fold(mi, li, oi);
     }
     // merge the wavefronts in wavefront order; lane: head r, d = 16 dt + 4 g + i
@@ -314,7 +319,7 @@ __global__ __launch_bounds__(256) void attn_decode_split_kernel(
     const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ k_pool,
     const bf16_t* __restrict__ v_pool, const int* __restrict__ block_tables, int table_width,
     const int* __restrict__ context_lens, float* __restrict__ part_o, float* __restrict__ part_ml,
-    int max_chunks, int H, int KVH, int page_shift, float scale_log2, float cap_in, float cap_out, int window) {
+    int max_chunks, int H, int KVH, int page_shift, float scale_log2, float cap_in, float cap_out, int window, int keep) {
     constexpr int NDT = D / 16;
     __shared__ float s_m[4][16], s_l[4][16];
     __shared__ float s_o[4][16][D + 1];
@@ -332,13 +337,13 @@ __global__ __launch_bounds__(256) void attn_decode_split_kernel(
     load_q_operand<D>(qreg, q + (size_t)s * q_stride, G, kvh, r, g);
     const int p = ctx - 1;
     const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
-    if (chunk_lo >= ctx || chunk_lo + AD_CHUNK <= lo) return;       // nothing of this chunk is visible
+    if (chunk_lo >= ctx || (chunk_lo + AD_CHUNK <= lo && chunk_lo >= keep)) return;       // nothing of this chunk is visible
     float m, l;
     f32x4_t o[NDT];
     {
         Keys64<D> kv;
-        load_keys64<D>(kv, k_pool, v_pool, entry, wbase, ctx, lo, kvh, KVH, page_shift, r, g);
-        attend_keys64<D>(kv, qreg, wbase, ctx, lo, scale_log2, cap_in, cap_out, g, m, l, o);
+        load_keys64<D>(kv, k_pool, v_pool, entry, wbase, ctx, keep, lo, kvh, KVH, page_shift, r, g);
+        attend_keys64<D>(kv, qreg, wbase, ctx, keep, lo, scale_log2, cap_in, cap_out, g, m, l, o);
     }
     if (g == 0) {
         s_m[wave][r] = m;
@@ -381,7 +386,7 @@ __global__ __launch_bounds__(256) void attn_decode_split_kernel(
 #define AD_MERGE_WAVES 4
 __global__ __launch_bounds__(64 * AD_MERGE_WAVES) void attn_decode_merge_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, const int* __restrict__ context_lens,
-    bf16_t* __restrict__ out, int out_stride, int max_chunks, int H, int D, int window, const float* __restrict__ sink) {
+    bf16_t* __restrict__ out, int out_stride, int max_chunks, int H, int D, int window, int keep, const float* __restrict__ sink) {
     __shared__ float s_l[AD_MERGE_WAVES], s_o[AD_MERGE_WAVES][128];
     const int s = blockIdx.x, h = blockIdx.y;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / TM_WAVE), lane = threadIdx.x % TM_WAVE;
@@ -400,12 +405,12 @@ __global__ __launch_bounds__(64 * AD_MERGE_WAVES) void attn_decode_merge_kernel(
     }
     const int p = ctx - 1;
     const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
-    const int c0 = lo / AD_CHUNK, c1 = (ctx - 1) / AD_CHUNK;
-    const float mm = wave_max((lane >= c0 && lane <= c1) ? ml[0] : -INFINITY);
+    const int c0 = lo / AD_CHUNK, c1 = (ctx - 1) / AD_CHUNK, ck = (keep + AD_CHUNK - 1) / AD_CHUNK;    // chunks c0 .. c1 and those before ck count
+    const float mm = wave_max(((lane >= c0 || lane < ck) && lane <= c1) ? ml[0] : -INFINITY);
     float ll = 0.f, o0 = 0.f, o1 = 0.f;
     auto add_chunk = [&](int c, float v0, float v1) {               // c is the same in every lane
         const float mc = __shfl(ml[0], c, TM_WAVE), lc = __shfl(ml[1], c, TM_WAVE);
-        const bool in = c >= c0 && c <= c1 && mc != -INFINITY;
+        const bool in = (c >= c0 || c < ck) && c <= c1 && mc != -INFINITY;
         const float f = in ? __builtin_amdgcn_exp2f(mc - mm) : 0.f;
         ll = fmaf(in ? lc : 0.f, f, ll);
         o0 = fmaf(in ? v0 : 0.f, f, o0);
@@ -446,20 +451,24 @@ __global__ __launch_bounds__(64 * AD_MERGE_WAVES) void attn_decode_merge_kernel(
 }
 
 // The same for any number of chunks (contexts beyond 64 chunks): the maxima are found in a pass of
-// their own, and wavefront w adds the chunks c0 + w, c0 + w + 4, ...
+// their own, and wavefront w adds every fourth of those that count
 __global__ __launch_bounds__(64 * AD_MERGE_WAVES) void attn_decode_merge_long_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, const int* __restrict__ context_lens,
-    bf16_t* __restrict__ out, int out_stride, int max_chunks, int H, int D, int window, const float* __restrict__ sink) {
+    bf16_t* __restrict__ out, int out_stride, int max_chunks, int H, int D, int window, int keep, const float* __restrict__ sink) {
     __shared__ float s_m[AD_MERGE_WAVES], s_l[AD_MERGE_WAVES], s_o[AD_MERGE_WAVES][128];
     const int s = blockIdx.x, h = blockIdx.y;
     const int wave = threadIdx.x / TM_WAVE, lane = threadIdx.x % TM_WAVE;
     const int ctx = context_lens[s];
     const int p = ctx - 1;
     const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
-    const int c0 = lo / AD_CHUNK, c1 = (ctx - 1) / AD_CHUNK;
+    const int c1 = (ctx - 1) / AD_CHUNK;
+    // the chunks that count: those of the kept first keys, then those of the window
+    const int kept = lo > 0 ? (keep + AD_CHUNK - 1) / AD_CHUNK : 0, resume = lo / AD_CHUNK > kept ? lo / AD_CHUNK : kept;
+    const int runs = kept + c1 - resume + 1;
+    auto chunk = [&](int i) { return i < kept ? i : resume + i - kept; };
     const size_t base = ((size_t)s * H + h) * max_chunks;
     float mm = -INFINITY;
-    for (int c = c0 + (int)threadIdx.x; c <= c1; c += 64 * AD_MERGE_WAVES) mm = fmaxf(mm, part_ml[(base + c) * 2]);
+    for (int i = (int)threadIdx.x; i < runs; i += 64 * AD_MERGE_WAVES) mm = fmaxf(mm, part_ml[(base + chunk(i)) * 2]);
     mm = wave_max(mm);
     if (lane == 0) s_m[wave] = mm;
     __syncthreads();
@@ -469,7 +478,8 @@ __global__ __launch_bounds__(64 * AD_MERGE_WAVES) void attn_decode_merge_long_ke
     const bool two = lane + 64 < D;
     float ll = 0.f, o0 = 0.f, o1 = 0.f;
 #pragma unroll 4
-    for (int c = c0 + wave; c <= c1; c += AD_MERGE_WAVES) {
+    for (int i = wave; i < runs; i += AD_MERGE_WAVES) {
+        const int c = chunk(i);
         const float mc = part_ml[(base + c) * 2];
         const float lc = part_ml[(base + c) * 2 + 1];
         const float a0 = lane < D ? part_o[(base + c) * D + lane] : 0.f;
@@ -503,7 +513,7 @@ template <int D>
 static int launch_decode(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                          const void* v_pool, const int* block_tables, int table_width, const int* context_lens,
                          float* part_o, float* part_ml, int max_chunks, int S, int H, int KVH, int page,
-                         float scale, int window, float softcap, const float* sink, hipStream_t stream) {
+                         float scale, int window, int keep, float softcap, const float* sink, hipStream_t stream) {
     int page_shift = 0;
     while ((1 << page_shift) < page) ++page_shift;
     const float scale_log2 = scale * 1.4426950408889634f;
@@ -515,20 +525,20 @@ static int launch_decode(const void* q, int q_stride, void* out, int out_stride,
     if (!split) {
         attn_decode_block_kernel<D, WAVES><<<dim3(S, KVH), 64 * WAVES, 0, stream>>>(
             (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool,
-            block_tables, table_width, context_lens, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, sink);
+            block_tables, table_width, context_lens, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, keep, sink);
         TM_CHECK_LAUNCH();
         return TM_OK;
     }
     attn_decode_split_kernel<D><<<dim3(S, KVH, max_chunks), 256, 0, stream>>>(
         (const bf16_t*)q, q_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_tables, table_width,
-        context_lens, part_o, part_ml, max_chunks, H, KVH, page_shift, scale_log2, cap_in, cap_out, window);
+        context_lens, part_o, part_ml, max_chunks, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, keep);
     TM_CHECK_LAUNCH();
     if (max_chunks <= TM_WAVE)
         attn_decode_merge_kernel<<<dim3(S, H), 64 * AD_MERGE_WAVES, 0, stream>>>(
-            part_o, part_ml, context_lens, (bf16_t*)out, out_stride, max_chunks, H, D, window, sink);
+            part_o, part_ml, context_lens, (bf16_t*)out, out_stride, max_chunks, H, D, window, keep, sink);
     else
         attn_decode_merge_long_kernel<<<dim3(S, H), 64 * AD_MERGE_WAVES, 0, stream>>>(
-            part_o, part_ml, context_lens, (bf16_t*)out, out_stride, max_chunks, H, D, window, sink);
+            part_o, part_ml, context_lens, (bf16_t*)out, out_stride, max_chunks, H, D, window, keep, sink);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
@@ -542,10 +552,11 @@ static int launch_decode(const void* q, int q_stride, void* out, int out_stride,
 extern "C" int tm_attn_decode_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                        const void* v_pool, const int* block_tables, int table_width,
                                        const int* context_lens, float* part_o, float* part_ml, int max_chunks, int S,
-                                       int H, int KVH, int D, int page, float scale, int window, float softcap,
+                                       int H, int KVH, int D, int page, float scale, int window, int keep, float softcap,
                                        const float* sink, hipStream_t stream) {
     if (S <= 0) return TM_OK;
-    if (!(softcap >= 0.f)) return TM_ERR_ARG;
+    if (!(softcap >= 0.f) || keep < 0) return TM_ERR_ARG;
+    if (window == 0) keep = 0;
     if (H <= 0 || KVH <= 0 || H % KVH || H / KVH > 16 || page < 16 || (page & (page - 1)) || max_chunks <= 0 ||
         !(scale > 0.f) || max_chunks > 65535 || KVH > 65535 || window < 0 || table_width <= 0 || (q_stride % 8) ||
         ((uintptr_t)q % 16) || (out_stride % 4) || ((uintptr_t)out % 8) || q_stride < H * D || out_stride < H * D)
@@ -553,7 +564,7 @@ extern "C" int tm_attn_decode_mfma_cap(const void* q, int q_stride, void* out, i
 #define TM_DECODE_CASE(DD)                                                                                        \
     case DD:                                                                                                      \
         return launch_decode<DD>(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width,         \
-                                 context_lens, part_o, part_ml, max_chunks, S, H, KVH, page, scale, window, softcap, sink,  \
+                                 context_lens, part_o, part_ml, max_chunks, S, H, KVH, page, scale, window, keep, softcap, sink,  \
                                  stream)
     switch (D) {
         TM_DECODE_CASE(32);
@@ -571,5 +582,5 @@ extern "C" int tm_attn_decode_mfma(const void* q, int q_stride, void* out, int o
                                    const int* context_lens, float* part_o, float* part_ml, int max_chunks, int S,
                                    int H, int KVH, int D, int page, float scale, int window, hipStream_t stream) {
     return tm_attn_decode_mfma_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, context_lens, part_o, part_ml,
-                                   max_chunks, S, H, KVH, D, page, scale, window, 0.f, nullptr, stream);
+                                   max_chunks, S, H, KVH, D, page, scale, window, 0, 0.f, nullptr, stream);
 }

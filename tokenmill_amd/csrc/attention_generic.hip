@@ -1,7 +1,7 @@
 // Paged attention over the cache, generic form: one wavefront per (query token, query head).
 //
 //   scores = (q . k) * scale ; a query at position p of its request sees the keys of that request
-//   at positions lo..p, lo = 0 or p - window + 1 ; softmax in 32-bit ; out = weights . v
+//   at positions lo..p, lo = 0 or p - window + 1, and with a window also the first `keep` ; softmax in 32-bit ; out = weights . v
 //                               (reference src/infer/model/layers.py:72-124, mask rules
 //                                src/infer/kv/context.py:73-74 and src/infer/model/layers.py:122)
 //   query head h reads kv head h / (H / KVH)         (reference src/infer/model/layers.py:86-87,119)
@@ -13,7 +13,7 @@
 // It takes every head size that is a multiple of 4 up to 256 and any q length and start position,
 // in 32-bit and in bfloat16; it is the attention of the true 32-bit path, and the bfloat16 path
 // uses it for shapes its MFMA kernels refuse. Keys are visited in ascending position in groups of
-// 64 starting at lo, so a token's result depends on its own request only (and, in the last bits, on
+// 64 of the visible ones in order (the kept first keys, then lo and on), so a token's result depends on its own request only (and, in the last bits, on
 // whether the step was small enough for the wavefronts of a block to share a token's keys).
 #include "common.h"
 #include "api.h"
@@ -55,7 +55,7 @@ __global__ __launch_bounds__((SPLIT ? AG_SPLIT_WAVES : AG_WAVES) * TM_WAVE) void
     const T* __restrict__ q, int q_stride, T* __restrict__ out, int out_stride,
     const T* __restrict__ k_pool, const T* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ seq_of_token, const int* __restrict__ positions, int T_tokens,
-    int H, int KVH, int D, int DV, int page, float scale, int window, float softcap, const float* __restrict__ gate, int ldg,
+    int H, int KVH, int D, int DV, int page, float scale, int window, int keep, float softcap, const float* __restrict__ gate, int ldg,
     const float* __restrict__ sink) {
     constexpr int WAVES = SPLIT ? AG_SPLIT_WAVES : AG_WAVES;
     constexpr bool STAGED = DMAX > 0 && sizeof(T) == 4;         // 32-bit keys through LDS (see the key loop)
@@ -71,6 +71,8 @@ __global__ __launch_bounds__((SPLIT ? AG_SPLIT_WAVES : AG_WAVES) * TM_WAVE) void
     const int s = seq_of_token[t];
     const int p = positions[t];
     const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    // the visible keys in order: the first `kept`, then lo .. p; place i of that list is position i, or i + gap behind the kept ones
+    const int kept = keep < lo ? keep : lo, gap = lo - kept, last = p - gap;
     const int* table = block_tables + (size_t)s * table_width;
     float* qs = q_s[SPLIT ? 0 : wave];
 
@@ -91,11 +93,11 @@ __global__ __launch_bounds__((SPLIT ? AG_SPLIT_WAVES : AG_WAVES) * TM_WAVE) void
 #pragma unroll
     for (int d = 0; d < (DMAX > 0 ? DMAX : 1); ++d) part[d] = 0.f;
 
-    const int first = SPLIT ? lo + wave * TM_WAVE : lo;
+    const int first = SPLIT ? wave * TM_WAVE : 0;
     const int stride = SPLIT ? WAVES * TM_WAVE : TM_WAVE;
-    for (int j0 = first; j0 <= p; j0 += stride) {
-        const int j = j0 + lane;
-        const bool valid = j <= p;
+    for (int j0 = first; j0 <= last; j0 += stride) {
+        const bool valid = j0 + lane <= last;
+        const int j = j0 + lane < kept ? j0 + lane : j0 + lane + gap;
         long long row = 0;
         float sc = -INFINITY;
         if constexpr (STAGED) {
@@ -174,7 +176,7 @@ __global__ __launch_bounds__((SPLIT ? AG_SPLIT_WAVES : AG_WAVES) * TM_WAVE) void
         }
 #pragma unroll
         for (int i = 0; i < AG_MAXD / TM_WAVE; ++i) acc[i] *= corr;
-        const int n = (p - j0 + 1) < TM_WAVE ? (p - j0 + 1) : TM_WAVE;
+        const int n = (last - j0 + 1) < TM_WAVE ? (last - j0 + 1) : TM_WAVE;
         for (int jj = 0; jj < n; ++jj) {
             const float pj = __shfl(pr_v, jj, TM_WAVE);
             const long long rj = __shfl(row, jj, TM_WAVE);
@@ -238,27 +240,27 @@ template <typename T, int DMAX>
 static void launch_generic_d(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                              const void* v_pool, const int* block_tables, int table_width, const int* seq_of_token,
                              const int* positions, int T_tokens, int H, int KVH, int D, int DV, int page, float scale,
-                             int window, float softcap, const float* gate, int ldg, const float* sink, hipStream_t stream) {
+                             int window, int keep, float softcap, const float* gate, int ldg, const float* sink, hipStream_t stream) {
     const long long pairs = (long long)T_tokens * H;
     if (pairs < 1024)           // too few (token, head) pairs to fill the chip: the wavefronts of a block split the keys
         attn_paged_generic_kernel<T, true, DMAX><<<(unsigned)pairs, AG_SPLIT_WAVES * TM_WAVE, 0, stream>>>(
             (const T*)q, q_stride, (T*)out, out_stride, (const T*)k_pool, (const T*)v_pool, block_tables,
-            table_width, seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, softcap, gate, ldg, sink);
+            table_width, seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink);
     else
         attn_paged_generic_kernel<T, false, DMAX><<<(unsigned)((pairs + AG_WAVES - 1) / AG_WAVES),
                                                     AG_WAVES * TM_WAVE, 0, stream>>>(
             (const T*)q, q_stride, (T*)out, out_stride, (const T*)k_pool, (const T*)v_pool, block_tables,
-            table_width, seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, softcap, gate, ldg, sink);
+            table_width, seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink);
 }
 
 template <typename T>
 static void launch_generic(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                            const void* v_pool, const int* block_tables, int table_width, const int* seq_of_token,
                            const int* positions, int T_tokens, int H, int KVH, int D, int DV, int page, float scale,
-                           int window, float softcap, const float* gate, int ldg, const float* sink, hipStream_t stream) {
+                           int window, int keep, float softcap, const float* gate, int ldg, const float* sink, hipStream_t stream) {
 #define TM_GENERIC(DMAX)                                                                                       \
     launch_generic_d<T, DMAX>(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width,         \
-                              seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, softcap, gate, ldg, sink, stream)
+                              seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink, stream)
     const int widest = D > DV ? D : DV;
     if (widest <= 64) TM_GENERIC(64);
     else if (widest <= 128) TM_GENERIC(128);
@@ -267,26 +269,26 @@ static void launch_generic(const void* q, int q_stride, void* out, int out_strid
 }
 
 // D: size of a key, DV: of a value (the V pool is [pages, KVH, DV, page], out rows H * DV); softcap > 0: a score s becomes
-// softcap * tanh(s / softcap); gate (float32 [T, >= H], rows ldg apart) or null: head h of token t is multiplied by
+// softcap * tanh(s / softcap); with a window, `keep`: the first keys of a request that every token sees beside its window; gate (float32 [T, >= H], rows ldg apart) or null: head h of token t is multiplied by
 // sigmoid(gate[t][h]); sink (float32 [H]) or null: one more term exp(sink[h]) in the denominator of head h's softmax.
 extern "C" int tm_attn_paged_generic_ext(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                          const void* v_pool, const int* block_tables, int table_width,
                                          const int* seq_of_token, const int* positions, int T, int H, int KVH, int D, int DV,
-                                         int page, float scale, int window, float softcap, const float* gate, int ldg,
+                                         int page, float scale, int window, int keep, float softcap, const float* gate, int ldg,
                                          const float* sink, int dtype, hipStream_t stream) {
     if (T <= 0) return TM_OK;
     if (H <= 0 || KVH <= 0 || H % KVH || D <= 0 || D > AG_MAXD || D % 4 || DV <= 0 || DV > AG_MAXD || page <= 0 ||
-        table_width <= 0 || window < 0 || q_stride < H * D || out_stride < H * DV || !(softcap >= 0.f) || (gate && ldg < H))
+        table_width <= 0 || window < 0 || keep < 0 || q_stride < H * D || out_stride < H * DV || !(softcap >= 0.f) || (gate && ldg < H))
         return TM_ERR_ARG;
     if (((long long)T * H + AG_WAVES - 1) / AG_WAVES > 0x7fffffffLL) return TM_ERR_ARG;
     if (dtype == TM_F32) {
         if (((uintptr_t)k_pool % 16)) return TM_ERR_ARG;
         launch_generic<float>(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, seq_of_token,
-                              positions, T, H, KVH, D, DV, page, scale, window, softcap, gate, ldg, sink, stream);
+                              positions, T, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink, stream);
     } else if (dtype == TM_BF16) {
         if (((uintptr_t)k_pool % 8)) return TM_ERR_ARG;
         launch_generic<bf16_t>(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, seq_of_token,
-                               positions, T, H, KVH, D, DV, page, scale, window, softcap, gate, ldg, sink, stream);
+                               positions, T, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink, stream);
     } else {
         return TM_ERR_ARG;
     }
@@ -299,5 +301,5 @@ extern "C" int tm_attn_paged_generic(const void* q, int q_stride, void* out, int
                                      const int* seq_of_token, const int* positions, int T, int H, int KVH, int D,
                                      int page, float scale, int window, int dtype, hipStream_t stream) {
     return tm_attn_paged_generic_ext(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, seq_of_token,
-                                     positions, T, H, KVH, D, D, page, scale, window, 0.f, nullptr, 0, nullptr, dtype, stream);
+                                     positions, T, H, KVH, D, D, page, scale, window, 0, 0.f, nullptr, 0, nullptr, dtype, stream);
 }

@@ -5,7 +5,7 @@
 //   four of the query heads that share it, so that every key and value fragment it loads feeds up
 //   to four heads. Keys and values are read in place through the block table, this step's own
 //   tokens included (they were stored before this kernel runs). A query at position p sees keys
-//   lo..p, lo = 0 or p - window + 1                (reference src/infer/kv/context.py:70-75,
+//   lo..p, lo = 0 or p - window + 1, and with a window also the first `keep` (reference src/infer/kv/context.py:70-75,
 //                                                   src/infer/model/layers.py:100-107).
 //   Key blocks are aligned to absolute positions (multiples of 32) and visited in ascending order,
 //   so a token's result does not depend on how its prompt was cut into portions nor on the rest of
@@ -38,16 +38,25 @@ __device__ __forceinline__ __amdgpu_buffer_rsrc_t uniform_buffer(const void* bas
     return __builtin_amdgcn_make_buffer_rsrc(const_cast<void*>(base), 0, 0x7fffffff, 0x00020000);
 }
 
-// The pages of the next 32 key blocks of a wavefront (blocks kb, kb + KS, ...), one 16-key tile per
-// lane: lane 2 i + t holds the page of tile t of block kb + i * KS. A tile that holds no key any
+// The key blocks of a wavefront: blocks `kept` and up are left out until `resume` (the gap between the kept first keys and the
+// windows; without one kept = 0 and resume is the first block there is).
+struct BlockWalk {
+    int kept, resume;
+    // block b of the walk that goes on by steps of KS from a block of it as if there were no gap
+    template <int KS>
+    __device__ __forceinline__ int at(int from, int b) const { return from < kept && b >= kept ? resume + (b - kept) / KS * KS : b; }
+};
+
+// The pages of the next 32 key blocks of a wavefront (blocks kb, kb + KS, ... of its walk), one 16-key tile per
+// lane: lane 2 i + t holds the page of tile t of the i-th of them. A tile that holds no key any
 // query of this wavefront may see (beyond the newest key, or wholly behind the window) is replaced
 // by the nearest tile that does: its table entry may name no page. The caller masks every score of
 // such a tile by the key's real position and clears its values (the tile in its place may hold keys beyond the newest one).
 template <int KS>
-__device__ __forceinline__ int2 lane_pages(int kb, int lane, int first_tile, int last_tile,
+__device__ __forceinline__ int2 lane_pages(int kb, const BlockWalk& walk, int lane, int kept_tiles, int first_tile, int last_tile,
                                            const int* __restrict__ table, int page_shift) {
-    int tile = 2 * (kb + (lane >> 1) * KS) + (lane & 1);
-    tile = tile < first_tile ? first_tile : (tile > last_tile ? last_tile : tile);
+    int tile = 2 * walk.at<KS>(kb, kb + (lane >> 1) * KS) + (lane & 1);
+    tile = (tile < first_tile && tile >= kept_tiles) ? first_tile : (tile > last_tile ? last_tile : tile);
     const int tile0 = 16 * tile;
     return int2{table[tile0 >> page_shift], tile0 & ((1 << page_shift) - 1)};
 }
@@ -81,12 +90,11 @@ __device__ __forceinline__ void attend_block(KVBlock<D>& blk, HeadState<D, HPW>&
     constexpr int NDC = D / 32, NDT = D / 16;
     // values of keys nobody may see (beyond the newest key, or behind every window: see lane_pages) can hold anything: clear them
     if (key0 + 31 > tv.last_key || key0 < tv.first_key) {
-        auto seen = [&](int k) { return k <= tv.last_key && k >= tv.first_key; };
 #pragma unroll
         for (int t = 0; t < 2; ++t) {
             const int k0 = key0 + 16 * t + 4 * g;
-            const uint32_t keep0 = (seen(k0) ? 0x0000ffffu : 0u) | (seen(k0 + 1) ? 0xffff0000u : 0u);
-            const uint32_t keep1 = (seen(k0 + 2) ? 0x0000ffffu : 0u) | (seen(k0 + 3) ? 0xffff0000u : 0u);
+            const uint32_t keep0 = (tv.seen(k0) ? 0x0000ffffu : 0u) | (tv.seen(k0 + 1) ? 0xffff0000u : 0u);
+            const uint32_t keep1 = (tv.seen(k0 + 2) ? 0x0000ffffu : 0u) | (tv.seen(k0 + 3) ? 0xffff0000u : 0u);
 #pragma unroll
             for (int dt = 0; dt < NDT; ++dt) {
                 blk.v[dt][t][0] &= keep0;
@@ -125,7 +133,7 @@ __device__ __forceinline__ void attend_block(KVBlock<D>& blk, HeadState<D, HPW>&
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const int kj = key0 + 16 * t + 4 * g + i;
-                    if (kj > tv.my_pos || kj < tv.my_lo) sc[hh][t][i] = -INFINITY;
+                    if (!tv.mine(kj)) sc[hh][t][i] = -INFINITY;
                 }
         }
         // this lane's largest score of the block (scale > 0: the maximum commutes with it)
@@ -189,7 +197,7 @@ __global__ __launch_bounds__(64 * KS) void attn_prefill_mfma_kernel(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
     const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ tiles, int n_tiles, int pair, int H, int KVH, int page_shift,
-    float scale_log2, float cap_in, float cap_out, int window, const float* __restrict__ sink) {
+    float scale_log2, float cap_in, float cap_out, int window, int keep, const float* __restrict__ sink) {
     constexpr int NDC = D / 32, NDT = D / 16;
     __shared__ float s_m[KS][16], s_l[KS][16];
     __shared__ float s_o[KS][16][D + 1];
@@ -213,16 +221,14 @@ __global__ __launch_bounds__(64 * KS) void attn_prefill_mfma_kernel(
         const int* tl = tiles + (size_t)(which ? other : (int)blockIdx.x) * 4;
         const int s = tl[0], row0 = tl[1], valid = tl[2], pos0 = tl[3];
         const int* table = block_tables + (size_t)s * table_width;
-        TileView tv;
-        tv.pos0 = pos0;
-        tv.last_key = pos0 + valid - 1;
-        tv.my_pos = pos0 + r < tv.last_key ? pos0 + r : tv.last_key;
-        tv.my_lo = (window > 0 && tv.my_pos - window + 1 > 0) ? tv.my_pos - window + 1 : 0;
-        tv.last_lo = (window > 0 && tv.last_key - window + 1 > 0) ? tv.last_key - window + 1 : 0;
-        const int first_key = (window > 0 && pos0 - window + 1 > 0) ? pos0 - window + 1 : 0;
-        tv.first_key = first_key;
-        const int kb0 = first_key / 32, kb1 = tv.last_key / 32;
-        const int first_tile = first_key / 16, last_tile = tv.last_key / 16;
+        const TileView tv = tile_view(pos0, valid, r, window, keep);
+        const int kb0 = tv.first_key / 32, kb1 = tv.last_key / 32;
+        const int first_tile = tv.first_key / 16, last_tile = tv.last_key / 16;
+        BlockWalk walk;
+        walk.kept = tv.first_key > 0 ? (tv.keep + 31) / 32 : 0;
+        const int kept_tiles = tv.first_key > 0 ? (tv.keep + 15) / 16 : 0;
+        const int behind = kb0 > walk.kept ? kb0 : walk.kept;        // the first block >= behind of this wavefront:
+        walk.resume = behind + ((wave - behind) & (KS - 1));
 
         PFrag qf[HPW][NDC];
 #pragma unroll
@@ -245,28 +251,28 @@ __global__ __launch_bounds__(64 * KS) void attn_prefill_mfma_kernel(
 
         // Two register sets take turns: one is worked on while the other's loads are in flight. The
         // load after the last block repeats it, unused, so that no load hides behind a branch.
-        int kb = kb0 + ((wave - kb0) & (KS - 1));                    // first block >= kb0 of this wavefront
+        int kb = wave < walk.kept ? wave : walk.resume;
         KVBlock<D> ba, bb;
-        int2 pages = lane_pages<KS>(kb, lane, first_tile, last_tile, table, page_shift);
+        int2 pages = lane_pages<KS>(kb, walk, lane, kept_tiles, first_tile, last_tile, table, page_shift);
         int slot = 0;                                                // block kb is slot `slot` of `pages`
         if (kb <= kb1) load_kv_block<D>(ba, pages, 0, k_pool, v_pool, kvh, KVH, page_shift, off);
         while (kb <= kb1) {
             if (slot == 31) {                                        // the next block starts a new set of pages
-                pages = lane_pages<KS>(kb + KS, lane, first_tile, last_tile, table, page_shift);
+                pages = lane_pages<KS>(walk.at<KS>(kb, kb + KS), walk, lane, kept_tiles, first_tile, last_tile, table, page_shift);
                 slot = -1;
             }
             load_kv_block<D>(bb, pages, slot + 1, k_pool, v_pool, kvh, KVH, page_shift, off);
             attend_block<D, HPW>(ba, st, qf, kb * 32, nh, tv, g, scale_log2, cap_in, cap_out);
-            kb += KS;
+            kb = walk.at<KS>(kb, kb + KS);
             ++slot;
             if (kb > kb1) break;
             if (slot == 31) {
-                pages = lane_pages<KS>(kb + KS, lane, first_tile, last_tile, table, page_shift);
+                pages = lane_pages<KS>(walk.at<KS>(kb, kb + KS), walk, lane, kept_tiles, first_tile, last_tile, table, page_shift);
                 slot = -1;
             }
             load_kv_block<D>(ba, pages, slot + 1, k_pool, v_pool, kvh, KVH, page_shift, off);
             attend_block<D, HPW>(bb, st, qf, kb * 32, nh, tv, g, scale_log2, cap_in, cap_out);
-            kb += KS;
+            kb = walk.at<KS>(kb, kb + KS);
             ++slot;
         }
 
@@ -318,7 +324,7 @@ template <int D> struct PrefillShape { static constexpr int HPW = D <= 64 ? 4 : 
 template <int D, int HPW>
 static void launch_split_keys(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                               const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH,
-                              int page_shift, float scale_log2, float cap_in, float cap_out, int window, const float* sink,
+                              int page_shift, float scale_log2, float cap_in, float cap_out, int window, int keep, const float* sink,
                               hipStream_t stream) {
     constexpr int KS = PrefillShape<D>::KS;
     const int splits = (H / KVH + HPW - 1) / HPW;
@@ -327,17 +333,18 @@ static void launch_split_keys(const void* q, int q_stride, void* out, int out_st
     dim3 grid(pair ? (n_tiles + 1) / 2 : n_tiles, KVH * splits);
     attn_prefill_mfma_kernel<D, HPW, KS><<<grid, 64 * KS, 0, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_tables,
-        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, sink);
+        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, keep, sink);
 }
 
 // softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax; sink (float32 [H]) or null: one more term
-// exp(sink[h]) in the denominator of head h's softmax, with no key behind it
+// exp(sink[h]) in the denominator of head h's softmax, with no key behind it; with a window, `keep`: the first keys of a request that
+// every query sees beside its window
 extern "C" int tm_attn_prefill_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                         const void* v_pool, const int* block_tables, int table_width, const int* tiles,
-                                        int n_tiles, int H, int KVH, int D, int page, float scale, int window, float softcap,
+                                        int n_tiles, int H, int KVH, int D, int page, float scale, int window, int keep, float softcap,
                                         const float* sink, hipStream_t stream) {
     if (n_tiles <= 0) return TM_OK;
-    if (!(softcap >= 0.f)) return TM_ERR_ARG;
+    if (!(softcap >= 0.f) || keep < 0) return TM_ERR_ARG;
     const float cap_in = softcap > 0.f ? scale / softcap : 0.f, cap_out = softcap > 0.f ? softcap / scale : 0.f;
     if (H <= 0 || KVH <= 0 || H % KVH || page < 16 || (page & (page - 1)) || window < 0 || table_width <= 0 ||
         (q_stride % 8) || ((uintptr_t)q % 16) || (out_stride % 2) || ((uintptr_t)out % 4) || q_stride < H * D ||
@@ -349,7 +356,7 @@ extern "C" int tm_attn_prefill_mfma_cap(const void* q, int q_stride, void* out, 
     const float scale_log2 = scale * 1.4426950408889634f;
     if ((long long)KVH * ((G + 1) / 2) > 65535) return TM_ERR_ARG;
 #define TM_SPLIT_ARGS q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, \
-                      page_shift, scale_log2, cap_in, cap_out, window, sink, stream
+                      page_shift, scale_log2, cap_in, cap_out, window, keep, sink, stream
 #define TM_PREFILL_CASE(DD)                                                                                       \
     case DD: {                                                                                                    \
         constexpr int HPW = PrefillShape<DD>::HPW;                                                                \
@@ -378,5 +385,5 @@ extern "C" int tm_attn_prefill_mfma(const void* q, int q_stride, void* out, int 
                                     int n_tiles, int H, int KVH, int D, int page, float scale, int window,
                                     hipStream_t stream) {
     return tm_attn_prefill_mfma_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, D,
-                                    page, scale, window, 0.f, nullptr, stream);
+                                    page, scale, window, 0, 0.f, nullptr, stream);
 }

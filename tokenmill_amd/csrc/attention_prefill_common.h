@@ -53,7 +53,26 @@ struct HeadState {
 struct TileView {
     int pos0;               // position of the tile's first query
     int last_key;           // newest key any query of the tile sees
-    int first_key;          // oldest key any query of the tile sees (0 without a window)
-    int last_lo;            // oldest key the tile's last query sees (0 without a window)
-    int my_pos, my_lo;      // this lane's query column: its position and the oldest key it sees
+    int first_key;          // oldest key of the windows of the tile's queries (0 without a window, or where the kept keys reach up to it)
+    int last_lo;            // oldest key of the window of the tile's last query (0 without a window)
+    int keep;               // with a window: the first keys of the request, which every query sees too
+    int my_pos, my_lo;      // this lane's query column: its position and the oldest key of its window
+
+    // does this lane's query see key k?
+    __device__ __forceinline__ bool mine(int k) const { return k <= my_pos && (k >= my_lo || k < keep); }
+    // does any query of the tile?
+    __device__ __forceinline__ bool seen(int k) const { return k <= last_key && (k >= first_key || k < keep); }
 };
+
+__device__ __forceinline__ TileView tile_view(int pos0, int valid, int r, int window, int keep) {
+    TileView tv;
+    tv.pos0 = pos0;
+    tv.last_key = pos0 + valid - 1;
+    tv.my_pos = pos0 + r < tv.last_key ? pos0 + r : tv.last_key;
+    tv.my_lo = (window > 0 && tv.my_pos - window + 1 > 0) ? tv.my_pos - window + 1 : 0;
+    tv.last_lo = (window > 0 && tv.last_key - window + 1 > 0) ? tv.last_key - window + 1 : 0;
+    tv.first_key = (window > 0 && pos0 - window + 1 > 0) ? pos0 - window + 1 : 0;
+    tv.keep = window > 0 ? keep : 0;
+    if (tv.first_key <= tv.keep) tv.first_key = 0;          // no gap between the kept keys and the windows
+    return tv;
+}

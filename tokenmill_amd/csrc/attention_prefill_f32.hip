@@ -5,7 +5,7 @@
 //   the tile may see are cut into blocks of 16 at absolute positions; the block's four wavefronts take
 //   every fourth key block each (key block kb goes to wavefront kb % 4), in ascending position with an
 //   online softmax of their own, and their four partial results are merged through LDS in the order of
-//   the wavefronts: a query at position p sees keys lo..p, lo = 0 or p - window + 1
+//   the wavefronts: a query at position p sees keys lo..p, lo = 0 or p - window + 1, and with a window also the first `keep`
 //                               (reference src/infer/kv/context.py:70-75, src/infer/model/layers.py:100-107).
 //   Which wavefront takes a key block hangs on the key's position only, so a token's result depends
 //   on its request only. The longest tile of a 2,048-token prompt walks 32 key blocks a wavefront
@@ -30,7 +30,7 @@ template <int D>
 __global__ __launch_bounds__(64 * AF_SPLIT) void attn_prefill_f32_kernel(
     const float* __restrict__ q, int q_stride, float* __restrict__ out, int out_stride,
     const float* __restrict__ k_pool, const float* __restrict__ v_pool, const int* __restrict__ block_tables,
-    int table_width, const int* __restrict__ tiles, int H, int KVH, int page_shift, float scale, int window, float softcap,
+    int table_width, const int* __restrict__ tiles, int H, int KVH, int page_shift, float scale, int window, int keep, float softcap,
     const float* __restrict__ sink) {
     constexpr int DQ = D / 4;           // values of a key (or query) a lane holds
     constexpr int NDT = D / 16;         // 16-row tiles of d
@@ -60,14 +60,18 @@ __global__ __launch_bounds__(64 * AF_SPLIT) void attn_prefill_f32_kernel(
 #pragma unroll
     for (int dt = 0; dt < NDT; ++dt) o[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 
+    // key blocks: those of the kept first keys, then those from the oldest window's start on
     const int kb_first = first_key >> 4, kb_last = last_key >> 4;
-    int kb = kb_first + ((wave - kb_first) & (AF_SPLIT - 1));
+    const int kb_kept = keep > 0 && first_key > 0 ? (keep + 15) >> 4 : 0;
+    auto behind_gap = [&](int b) { return (b >= kb_kept && b < kb_first) ? kb_first + ((wave - kb_first) & (AF_SPLIT - 1)) : b; };
+    int kb = behind_gap(wave);
     // a key block's page id is asked for one block ahead (always at an entry this tile may see)
     int pg_next = table[((kb <= kb_last ? kb : kb_last) << 4) >> page_shift];
-    for (; kb <= kb_last; kb += AF_SPLIT) {
+    for (int next; kb <= kb_last; kb = next) {
         const int key0 = kb << 4;
         const int pg = pg_next;
-        pg_next = table[((kb + AF_SPLIT <= kb_last ? kb + AF_SPLIT : kb) << 4) >> page_shift];
+        next = behind_gap(kb + AF_SPLIT);
+        pg_next = table[((next <= kb_last ? next : kb) << 4) >> page_shift];
         const int in_page = key0 & (page - 1);
         // keys: lane (r, g) holds K[key0 + r][16 c + 4 g .. + 3], c = 0 .. D/16 - 1
         const float* kr = k_pool + ((((size_t)pg << page_shift) + in_page + r) * KVH + kvh) * D + 4 * g;
@@ -101,7 +105,7 @@ __global__ __launch_bounds__(64 * AF_SPLIT) void attn_prefill_f32_kernel(
             if (softcap > 0.f) sc[i] = softcap * tanhf(sc[i] / softcap);
             if (edge) {
                 const int kj = key0 + 4 * g + i;
-                if (kj > my_pos || kj < my_lo) sc[i] = -INFINITY;
+                if (kj > my_pos || (kj < my_lo && kj >= keep)) sc[i] = -INFINITY;
             }
         }
         float bm = fmaxf(fmaxf(sc[0], sc[1]), fmaxf(sc[2], sc[3]));
@@ -174,13 +178,14 @@ __global__ __launch_bounds__(64 * AF_SPLIT) void attn_prefill_f32_kernel(
 // tiles int32 [n_tiles][4] = (request index, first row, tokens (1..16), position of the first token).
 // Needs D % 16 == 0 (at most 128), page a power of two >= 16, 16-byte aligned q, out and pools, strides % 4 == 0.
 // softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax; sink (float32 [H]) or null: one more term
-// exp(sink[h]) in the denominator of head h's softmax, with no key behind it.
+// exp(sink[h]) in the denominator of head h's softmax, with no key behind it; with a window, `keep`: the first keys of a request
+// that every token sees beside its window.
 extern "C" int tm_attn_prefill_f32_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                        const void* v_pool, const int* block_tables, int table_width, const int* tiles,
-                                       int n_tiles, int H, int KVH, int D, int page, float scale, int window, float softcap,
+                                       int n_tiles, int H, int KVH, int D, int page, float scale, int window, int keep, float softcap,
                                        const float* sink, hipStream_t stream) {
     if (n_tiles <= 0) return TM_OK;
-    if (!(softcap >= 0.f)) return TM_ERR_ARG;
+    if (!(softcap >= 0.f) || keep < 0) return TM_ERR_ARG;
     if (H <= 0 || KVH <= 0 || H % KVH || page < 16 || (page & (page - 1)) || window < 0 || table_width <= 0 ||
         (q_stride % 4) || (out_stride % 4) || ((uintptr_t)q % 16) || ((uintptr_t)out % 16) || ((uintptr_t)k_pool % 16) ||
         ((uintptr_t)v_pool % 16) || q_stride < H * D || out_stride < H * D || !(scale > 0.f))
@@ -193,7 +198,7 @@ extern "C" int tm_attn_prefill_f32_cap(const void* q, int q_stride, void* out, i
     case DD:                                                                                                      \
         attn_prefill_f32_kernel<DD><<<grid, 64 * AF_SPLIT, 0, stream>>>(                                          \
             (const float*)q, q_stride, (float*)out, out_stride, (const float*)k_pool, (const float*)v_pool,       \
-            block_tables, table_width, tiles, H, KVH, page_shift, scale, window, softcap, sink);                           \
+            block_tables, table_width, tiles, H, KVH, page_shift, scale, window, keep, softcap, sink);                     \
         break
     switch (D) {
         TM_PREFILL_F32_CASE(16);
@@ -217,5 +222,5 @@ extern "C" int tm_attn_prefill_f32(const void* q, int q_stride, void* out, int o
                                    int n_tiles, int H, int KVH, int D, int page, float scale, int window,
                                    hipStream_t stream) {
     return tm_attn_prefill_f32_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, D,
-                                   page, scale, window, 0.f, nullptr, stream);
+                                   page, scale, window, 0, 0.f, nullptr, stream);
 }

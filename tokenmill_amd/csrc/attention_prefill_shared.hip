@@ -56,10 +56,10 @@ struct TilePlaces {
     uint64_t k, v;
 };
 
-__device__ __forceinline__ TilePlaces lane_places(int base_stage, int lane, int first_tile, int last_tile,
+__device__ __forceinline__ TilePlaces lane_places(int base_stage, int lane, int kept_tiles, int first_tile, int last_tile,
                                                   const int* __restrict__ table, int page_shift, int kvh, int KVH, int D) {
     int tile = 4 * base_stage + lane;
-    tile = tile < first_tile ? first_tile : (tile > last_tile ? last_tile : tile);
+    tile = (tile < first_tile && tile >= kept_tiles) ? first_tile : (tile > last_tile ? last_tile : tile);
     const int tile0 = 16 * tile;
     const size_t pg = (size_t)table[tile0 >> page_shift];
     const int in_page = tile0 & ((1 << page_shift) - 1);
@@ -101,10 +101,10 @@ struct StageCopy {
         }
     }
 
-    // Store what was loaded into a stage of LDS. Of the stage's 64 positions [from, keys) can be seen: the values of the
+    // Store what was loaded into a stage of LDS. Of the stage's 64 positions [from, keys) and those before `kept` can be seen: the values of the
     // others (beyond the newest key, or behind every window, where another tile stands in; they can hold anything) are cleared here, once for all wavefronts, so that
     // the products need no mask (their weights are zero, but zero times anything is not).
-    __device__ __forceinline__ void store(unsigned char* stage, int tid, int from, int keys) const {
+    __device__ __forceinline__ void store(unsigned char* stage, int tid, int kept, int from, int keys) const {
 #pragma unroll
         for (int i = 0; i < ITERS; ++i) {
             const int idx = tid + i * THREADS;
@@ -118,7 +118,8 @@ struct StageCopy {
 #pragma unroll
                 for (int w = 0; w < 4; ++w) {
                     const int k0 = first + 2 * w, k1 = k0 + 1;
-                    val[w] &= ((k0 < keys && k0 >= from) ? 0x0000ffffu : 0u) | ((k1 < keys && k1 >= from) ? 0xffff0000u : 0u);
+                    val[w] &= ((k0 < keys && (k0 >= from || k0 < kept)) ? 0x0000ffffu : 0u) |
+                              ((k1 < keys && (k1 >= from || k1 < kept)) ? 0xffff0000u : 0u);
                 }
             }
             *(u32x4_t*)(stage + SharedShape<D>::K_BYTES + d * SharedShape<D>::V_STRIDE + j * 32 + half * 16) = val;
@@ -164,7 +165,7 @@ __device__ __forceinline__ void attend_shared(const unsigned char* stage, int su
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const int kj = key0 + 8 * g + 4 * t + i;        // row 4g+i of tile t of the pair
-                    if (kj > tv.my_pos || kj < tv.my_lo) sc[t][i] = -INFINITY;
+                    if (!tv.mine(kj)) sc[t][i] = -INFINITY;
                 }
         }
         // this lane's largest score of the block (scale > 0: the maximum commutes with it)
@@ -226,7 +227,7 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
     const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ tiles, int n_tiles, int pair, int H, int KVH, int page_shift,
-    float scale_log2, float cap_in, float cap_out, int window, const float* __restrict__ sink) {
+    float scale_log2, float cap_in, float cap_out, int window, int keep, const float* __restrict__ sink) {
     constexpr int NDC = D / 32, NDT = D / 16, THREADS = 64 * WAVES, STAGE = SharedShape<D>::STAGE, HPW = SharedPlan<D>::HPW;
     extern __shared__ __align__(16) unsigned char stages[];          // two stages
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / TM_WAVE);
@@ -244,16 +245,13 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
         const int* tl = tiles + (size_t)(which ? other : (int)blockIdx.x) * 4;
         const int s = tl[0], row0 = tl[1], valid = tl[2], pos0 = tl[3];
         const int* table = block_tables + (size_t)s * table_width;
-        TileView tv;
-        tv.pos0 = pos0;
-        tv.last_key = pos0 + valid - 1;
-        tv.my_pos = pos0 + r < tv.last_key ? pos0 + r : tv.last_key;
-        tv.my_lo = (window > 0 && tv.my_pos - window + 1 > 0) ? tv.my_pos - window + 1 : 0;
-        tv.last_lo = (window > 0 && tv.last_key - window + 1 > 0) ? tv.last_key - window + 1 : 0;
-        const int first_key = (window > 0 && pos0 - window + 1 > 0) ? pos0 - window + 1 : 0;
-        tv.first_key = first_key;
-        const int sb0 = first_key / PS_KEYS, sb1 = tv.last_key / PS_KEYS;
+        const TileView tv = tile_view(pos0, valid, r, window, keep);
+        const int first_key = tv.first_key, sb1 = tv.last_key / PS_KEYS;
         const int first_tile = first_key / 16, last_tile = tv.last_key / 16;
+        // stages: those of the kept first keys (if there is a gap behind them), then those of the windows
+        const int kept_tiles = first_key > 0 ? (tv.keep + 15) / 16 : 0, kept_stages = first_key > 0 ? (tv.keep + PS_KEYS - 1) / PS_KEYS : 0;
+        const int resume = first_key / PS_KEYS > kept_stages ? first_key / PS_KEYS : kept_stages;
+        const int sb0 = kept_stages > 0 ? 0 : resume;
 
         PFrag qf[HPW][NDC];
 #pragma unroll
@@ -278,28 +276,29 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
         // are on their way into registers, and are stored when the work is done. The load after the last stage
         // repeats it, unused, so that no load hides behind a branch.
         int base = sb0;                                              // `places` covers stages base .. base + 15
-        TilePlaces places = lane_places(base, lane, first_tile, last_tile, table, page_shift, kvh, KVH, D);
+        TilePlaces places = lane_places(base, lane, kept_tiles, first_tile, last_tile, table, page_shift, kvh, KVH, D);
         StageCopy<D, THREADS> copy;
         copy.load(places, 0, kp, vp, KVH, page_shift, tid);
-        copy.store(stages, tid, first_key - sb0 * PS_KEYS, tv.last_key + 1 - sb0 * PS_KEYS);
+        copy.store(stages, tid, tv.keep - sb0 * PS_KEYS, first_key - sb0 * PS_KEYS, tv.last_key + 1 - sb0 * PS_KEYS);
         __syncthreads();
-        for (int sb = sb0; sb <= sb1; ++sb) {
-            const int cur = (sb - sb0) & 1;
-            int next = sb + 1 <= sb1 ? sb + 1 : sb1;
-            if (next - base == 16) {
-                base = next;
-                places = lane_places(base, lane, first_tile, last_tile, table, page_shift, kvh, KVH, D);
+        int cur = 0;
+        for (int sb = sb0, next; sb <= sb1; sb = next, cur ^= 1) {
+            next = sb + 1 == kept_stages ? resume : sb + 1;
+            const int ahead = next <= sb1 ? next : sb1;
+            if (ahead - base >= 16) {
+                base = ahead;
+                places = lane_places(base, lane, kept_tiles, first_tile, last_tile, table, page_shift, kvh, KVH, D);
             }
-            copy.load(places, next - base, kp, vp, KVH, page_shift, tid);
+            copy.load(places, ahead - base, kp, vp, KVH, page_shift, tid);
             if (nh > 0) {                                            // wave-uniform
 #pragma unroll
                 for (int sub = 0; sub < 2; ++sub) {
                     const int key0 = sb * PS_KEYS + 32 * sub;
-                    if (key0 > tv.last_key || key0 + 31 < first_key) continue;     // block-uniform: nothing of it is visible
+                    if (key0 > tv.last_key || (key0 + 31 < first_key && key0 >= tv.keep)) continue;     // block-uniform: nothing of it is visible
                     attend_shared<D, HPW>(stages + cur * STAGE, sub, st, qf, key0, tv, r, g, scale_log2, cap_in, cap_out);
                 }
             }
-            copy.store(stages + (cur ^ 1) * STAGE, tid, first_key - next * PS_KEYS, tv.last_key + 1 - next * PS_KEYS);
+            copy.store(stages + (cur ^ 1) * STAGE, tid, tv.keep - ahead * PS_KEYS, first_key - ahead * PS_KEYS, tv.last_key + 1 - ahead * PS_KEYS);
             __syncthreads();
         }
 
@@ -328,7 +327,7 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
 template <int D, int WAVES>
 static int launch_shared(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                          const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH,
-                         int page_shift, float scale_log2, float cap_in, float cap_out, int window, const float* sink,
+                         int page_shift, float scale_log2, float cap_in, float cap_out, int window, int keep, const float* sink,
                          hipStream_t stream) {
     constexpr int lds = 2 * SharedShape<D>::STAGE;
     static bool raised = false;
@@ -343,7 +342,7 @@ static int launch_shared(const void* q, int q_stride, void* out, int out_stride,
     dim3 grid(pair ? (n_tiles + 1) / 2 : n_tiles, KVH);
     attn_prefill_shared_kernel<D, WAVES><<<grid, 64 * WAVES, lds, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_tables,
-        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, sink);
+        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, keep, sink);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
@@ -357,13 +356,14 @@ extern "C" int tm_attn_prefill_shared_takes(int H, int KVH, int D) {
 }
 
 // softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax; sink (float32 [H]) or null: one more term
-// exp(sink[h]) in the denominator of head h's softmax, with no key behind it
+// exp(sink[h]) in the denominator of head h's softmax, with no key behind it; with a window, `keep`: the first keys of a request that
+// every query sees beside its window
 extern "C" int tm_attn_prefill_shared_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                           const void* v_pool, const int* block_tables, int table_width, const int* tiles,
-                                          int n_tiles, int H, int KVH, int D, int page, float scale, int window, float softcap,
+                                          int n_tiles, int H, int KVH, int D, int page, float scale, int window, int keep, float softcap,
                                           const float* sink, hipStream_t stream) {
     if (n_tiles <= 0) return TM_OK;
-    if (!(softcap >= 0.f)) return TM_ERR_ARG;
+    if (!(softcap >= 0.f) || keep < 0) return TM_ERR_ARG;
     const float cap_in = softcap > 0.f ? scale / softcap : 0.f, cap_out = softcap > 0.f ? softcap / scale : 0.f;
     if (!tm_attn_prefill_shared_takes(H, KVH, D) || page < 16 || (page & (page - 1)) || window < 0 || table_width <= 0 ||
         (q_stride % 8) || ((uintptr_t)q % 16) || (out_stride % 4) || ((uintptr_t)out % 8) || q_stride < H * D ||
@@ -375,7 +375,7 @@ extern "C" int tm_attn_prefill_shared_cap(const void* q, int q_stride, void* out
     while ((1 << page_shift) < page) ++page_shift;
     const float scale_log2 = scale * 1.4426950408889634f;
 #define TM_SHARED_ARGS q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, \
-                       page_shift, scale_log2, cap_in, cap_out, window, sink, stream
+                       page_shift, scale_log2, cap_in, cap_out, window, keep, sink, stream
 #define TM_SHARED_CASE(DD)                                                          \
     case DD:                                                                        \
         if (need <= 2) return launch_shared<DD, 2>(TM_SHARED_ARGS);                 \
@@ -400,5 +400,5 @@ extern "C" int tm_attn_prefill_shared(const void* q, int q_stride, void* out, in
                                       int n_tiles, int H, int KVH, int D, int page, float scale, int window,
                                       hipStream_t stream) {
     return tm_attn_prefill_shared_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH,
-                                      D, page, scale, window, 0.f, nullptr, stream);
+                                      D, page, scale, window, 0, 0.f, nullptr, stream);
 }

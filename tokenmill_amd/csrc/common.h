@@ -73,6 +73,13 @@ __device__ __forceinline__ void rotate_pair(float x1, float x2, float c, float s
     y2 = d + e;
 }
 
+// the clamped gated activation g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = up held to +-limit
+__device__ __forceinline__ float clamped_glu_f32(float g, float u, float alpha, float limit) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+}
+
 // tanh from the hardware's exp2 and reciprocal: 1 - 2 / (e^(2x) + 1), exact at both ends (e^(2x) = inf or 0); its absolute
 // error of about 1e-7 is far below a bfloat16 score's own
 __device__ __forceinline__ float tanh_fast(float x) {

@@ -539,12 +539,6 @@ extern "C" int tm_gelu_mul(const void* gu, void* out, int dtype, int T, int I, h
 // out[t, i] = g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = up held to +-limit: the clamped gated activation, computed in
 // 32-bit and rounded once; gu [T, 2I] (gate columns, then up columns). Eight elements a thread where the rows come in whole
 // pieces of eight.
-__device__ __forceinline__ float clamped_glu_f32(float g, float u, float alpha, float limit) {
-    g = fminf(g, limit);
-    u = fminf(fmaxf(u, -limit), limit);
-    return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
-}
-
 template <typename T, int N>
 __global__ __launch_bounds__(256) void clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, float alpha,
                                                           float limit) {
@@ -618,6 +612,62 @@ extern "C" int tm_convert(const void* in, int in_dtype, void* out, int out_dtype
         convert_kernel<bf16_t, float><<<blocks, 256, 0, stream>>>((const bf16_t*)in, (float*)out, (size_t)n);
     else if (in_dtype == TM_F32 && out_dtype == TM_BF16)
         convert_kernel<float, bf16_t><<<blocks, 256, 0, stream>>>((const float*)in, (bf16_t*)out, (size_t)n);
+    else
+        return TM_ERR_ARG;
+    TM_CHECK_LAUNCH();
+    return TM_OK;
+}
+
+// ------------------------------------------------------------------------------------------
+// x <- x * scale, then with cap > 0: cap * tanh(x / cap), in place, 32-bit (an output head's scaled and capped logits)
+// ------------------------------------------------------------------------------------------
+__global__ __launch_bounds__(256) void scale_cap_kernel(float* __restrict__ x, size_t n, float scale, float cap) {
+    for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256) {
+        const float v = x[i] * scale;
+        x[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
+    }
+}
+
+extern "C" int tm_scale_cap(float* x, long long n, float scale, float cap, hipStream_t stream) {
+    if (n <= 0) return TM_OK;
+    if (!x || !(cap >= 0.f)) return TM_ERR_ARG;
+    const long long want = (n + 255) / 256;
+    scale_cap_kernel<<<(int)(want < 16384 ? want : 16384), 256, 0, stream>>>(x, (size_t)n, scale, cap);
+    TM_CHECK_LAUNCH();
+    return TM_OK;
+}
+
+// ------------------------------------------------------------------------------------------
+// out[t] = table[ids[t]] * scale + waves, waves[2 i] = sin(p f[i]), waves[2 i + 1] = cos(p f[i]) with p the token's position;
+// angles, sines and the sum in 32-bit. f holds ceil(hidden / 2) frequencies. A thread a pair.
+// ------------------------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void embed_waves_kernel(const T* __restrict__ table, const int* __restrict__ ids,
+                                                         const int* __restrict__ positions, const float* __restrict__ f,
+                                                         float* __restrict__ out, int hidden, int vocab, float scale) {
+    const int t = blockIdx.x;
+    int id = ids[t];
+    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);       // the host rejects such ids; never read outside
+    const float p = (float)positions[t];
+    const T* row = table + (size_t)id * hidden;
+    float* o = out + (size_t)t * hidden;
+    for (int i = blockIdx.y * 256 + threadIdx.x; 2 * i < hidden; i += 256 * gridDim.y) {
+        float s, c;
+        sincosf(p * f[i], &s, &c);
+        o[2 * i] = Elem<T>::load(row + 2 * i) * scale + s;
+        if (2 * i + 1 < hidden) o[2 * i + 1] = Elem<T>::load(row + 2 * i + 1) * scale + c;
+    }
+}
+
+extern "C" int tm_embed_waves(const void* table, int dtype, const int* ids, const int* positions, const float* f, float* out, int T,
+                              int hidden, int vocab, float scale, hipStream_t stream) {
+    if (T <= 0) return TM_OK;
+    if (!table || !ids || !positions || !f || !out || hidden <= 0 || vocab <= 0) return TM_ERR_ARG;
+    const dim3 grid(T, (hidden + 511) / 512 < 8 ? (hidden + 511) / 512 : 8);
+    if (dtype == TM_F32)
+        embed_waves_kernel<float><<<grid, 256, 0, stream>>>((const float*)table, ids, positions, f, out, hidden, vocab, scale);
+    else if (dtype == TM_BF16)
+        embed_waves_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)table, ids, positions, f, out, hidden, vocab, scale);
     else
         return TM_ERR_ARG;
     TM_CHECK_LAUNCH();

@@ -270,10 +270,38 @@ __global__ __launch_bounds__(TM_WAVE) void gla_out_gate_kernel(const float* __re
     }
 }
 
+// One wide head (a norm over all heads of a token at once): a block a token.
+template <typename T>
+__global__ __launch_bounds__(256) void gla_out_gate_wide_kernel(const float* __restrict__ o, const T* __restrict__ gate, int ldg,
+                                                               const float* __restrict__ w, T* __restrict__ y, int N, float eps,
+                                                               int sigmoid) {
+    __shared__ float red[256 / TM_WAVE];
+    const int t = blockIdx.x;
+    const float* orow = o + (size_t)t * N;
+    const T* grow = gate + (size_t)t * ldg;
+    T* yrow = y + (size_t)t * N;
+    float ss = 0.f;
+    for (int e = threadIdx.x; e < N; e += 256) ss += orow[e] * orow[e];
+    const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)N + eps);
+    for (int e = threadIdx.x; e < N; e += 256) {
+        const float g = Elem<T>::load(grow + e);
+        const float v = w ? w[e] * (orow[e] * r) : orow[e] * r;
+        Elem<T>::store(yrow + e, v * ((sigmoid ? 1.f : g) / (1.f + expf(-g))));
+    }
+}
+
 extern "C" int tm_gla_out_gate(const float* o, const void* gate, int ldg, int dtype, const float* w, void* y, int T, int H, int Dv,
                                float eps, int sigmoid, hipStream_t stream) {
     if (T <= 0) return TM_OK;
     if (H <= 0 || H > 65535 || Dv <= 0 || ldg < H * Dv || !o || !gate || !y || !(eps > 0.f)) return TM_ERR_ARG;
+    if (H == 1 && Dv > 4 * TM_WAVE && (dtype == TM_F32 || dtype == TM_BF16)) {
+        if (dtype == TM_F32)
+            gla_out_gate_wide_kernel<float><<<T, 256, 0, stream>>>(o, (const float*)gate, ldg, w, (float*)y, Dv, eps, sigmoid);
+        else
+            gla_out_gate_wide_kernel<bf16_t><<<T, 256, 0, stream>>>(o, (const bf16_t*)gate, ldg, w, (bf16_t*)y, Dv, eps, sigmoid);
+        TM_CHECK_LAUNCH();
+        return TM_OK;
+    }
     const dim3 grid(T, H);
     if (dtype == TM_F32)
         gla_out_gate_kernel<float><<<grid, TM_WAVE, 0, stream>>>(o, (const float*)gate, ldg, w, (float*)y, H, Dv, eps, sigmoid);

@@ -5,7 +5,7 @@
 //   experts : tiles (group, first slot, rows <= 32) from tm_moe_route; a tile's rows are slots first .. first + rows - 1, and
 //             slot i reads row row_src[i] / src_div of A (row_src null: row i).
 // Epilogues: a plain store in bfloat16 or in 32-bit, or, with a matrix of 2 N rows (gate rows, then up rows),
-// silu(gate product) * up product, or the square of relu(product) in bfloat16. A block is RT tiles of 16 rows by 64 columns; its four wavefronts take 16 columns each;
+// silu(gate product) * up product or the clamped gate of moe.hip (each product times the row's pair weight first), or the square of relu(product) in bfloat16. A block is RT tiles of 16 rows by 64 columns; its four wavefronts take 16 columns each;
 // k ascends in steps of 32 through LDS, so an element's sum has one order wherever its row stands.
 #include "common.h"
 #include "api.h"
@@ -15,7 +15,7 @@
 #define GM_BK 32            // k of a step through LDS (BK of the kernel): 32, or 128 for tiles of few rows, whose steps are
                             // latency and not arithmetic: four times the bytes asked for at once, a quarter of the steps
 
-enum { GM_STORE = 0, GM_STORE_F32 = 1, GM_SILU_MUL = 2, GM_RELU2 = 3 };
+enum { GM_STORE = 0, GM_STORE_F32 = 1, GM_SILU_MUL = 2, GM_RELU2 = 3, GM_CLAMPED = 4 };
 
 template <int RT, int MODE, int BK = GM_BK, int BN = GM_BN>
 __global__ __launch_bounds__(256) void grouped_mfma_kernel(const bf16_t* __restrict__ A, int lda, int a_off,
@@ -24,14 +24,16 @@ __global__ __launch_bounds__(256) void grouped_mfma_kernel(const bf16_t* __restr
                                                            const float* __restrict__ gate, int ldg, const int* __restrict__ tiles,
                                                            const int* __restrict__ n_tiles, int T, int K, int N, int tail, int rot_,
                                                            const float* __restrict__ cos_t, const float* __restrict__ sin_t,
-                                                           const int* __restrict__ positions) {
+                                                           const int* __restrict__ positions, const float* __restrict__ pair_weight,
+                                                           float limit, float alpha) {
     constexpr int BM = RT * 16;
-    constexpr bool GATED = MODE == GM_SILU_MUL;
+    constexpr bool GATED = MODE == GM_SILU_MUL || MODE == GM_CLAMPED;
     constexpr int GM_LD = BK + 8, PPR = BK / 8;                 // 16-byte pieces a row of a step
     constexpr int NCG = BN / GM_BN;                             // groups of 64 columns a block: a wavefront has 16 columns of each
     __shared__ __align__(16) bf16_t As[BM][GM_LD];
     __shared__ __align__(16) bf16_t Bs[GATED ? 2 : 1][BN][GM_LD];
     __shared__ int src[BM];
+    __shared__ float wrow[MODE == GM_CLAMPED ? BM : 1];         // the rows' pair weights
     int group, row0, rows;
     if (tiles) {
         if ((int)blockIdx.x >= n_tiles[0]) return;
@@ -45,6 +47,7 @@ __global__ __launch_bounds__(256) void grouped_mfma_kernel(const bf16_t* __restr
     if (threadIdx.x < BM) {
         const int i = threadIdx.x;
         src[i] = i < rows ? (row_src ? row_src[row0 + i] / src_div : row0 + i) : -1;
+        if (MODE == GM_CLAMPED) wrow[i] = i < rows && pair_weight ? pair_weight[row_src[row0 + i]] : 1.f;
     }
     __syncthreads();
     f32x4_t acc[NCG][RT], acu[NCG][GATED ? RT : 1];
@@ -151,7 +154,9 @@ __global__ __launch_bounds__(256) void grouped_mfma_kernel(const bf16_t* __restr
                 if (row >= rows) continue;
                 const size_t at = (size_t)(row0 + row) * ldc + (size_t)group * c_off + n;
                 float v = acc[cg][t][i];
-                if (MODE == GM_SILU_MUL) {
+                if (MODE == GM_CLAMPED) {
+                    ((bf16_t*)Cv)[at] = f32_to_bf16(clamped_glu_f32(wrow[row] * v, wrow[row] * acu[cg][t][i], alpha, limit));
+                } else if (MODE == GM_SILU_MUL) {
                     const float u = acu[cg][t][i];
                     ((bf16_t*)Cv)[at] = f32_to_bf16(v / (1.0f + __expf(-v)) * u);
                 } else if (MODE == GM_RELU2) {
@@ -189,7 +194,7 @@ extern "C" int tm_heads_matmul_mfma(const void* A, int lda, int a_off, const voi
     if (grid.y > 65535) return TM_ERR_ARG;
     grouped_mfma_kernel<4, GM_STORE><<<grid, 256, 0, stream>>>((const bf16_t*)A, lda, a_off, nullptr, 1, (const bf16_t*)W, C, ldc, c_off,
                                                                gate, ldg, nullptr, nullptr, T, K, N, tail, half_pairs ? -rot : rot, cos_t, sin_t,
-                                                               positions);
+                                                               positions, nullptr, 0.f, 0.f);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
@@ -211,9 +216,30 @@ extern "C" int tm_moe_gate_up_mfma(const void* x, int ldx, const int* slot_pair,
     if (grid.y > 65535) return TM_ERR_ARG;
 #define GM_GO(RT_, BK_, BN_)                                                                                                             \
     grouped_mfma_kernel<RT_, GM_SILU_MUL, BK_, BN_><<<dim3(max_tiles, (F + BN_ - 1) / BN_), 256, 0, stream>>>((const bf16_t*)x, ldx, 0, slot_pair, top, (const bf16_t*)W, act, F, \
-                                                                    0, nullptr, 0, tiles, n_tiles, 0, K, F, 0, 0, nullptr, nullptr, nullptr)
+                                                                    0, nullptr, 0, tiles, n_tiles, 0, K, F, 0, 0, nullptr, nullptr, nullptr, nullptr, 0.f, 0.f)
     // (64 columns a block whatever the tile: with a gate a wavefront holds two results a column)
     if (tile_rows == 32) GM_GO(2, 128, GM_BN); else if (tile_rows == 64) GM_GO(4, GM_BK, GM_BN); else GM_GO(8, GM_BK, GM_BN);
+#undef GM_GO
+    TM_CHECK_LAUNCH();
+    return TM_OK;
+}
+
+// Experts with the clamped gate on their weighted input (moe.hip), W [E, 2F, K].
+extern "C" int tm_moe_clamped_mfma(const void* x, int ldx, const int* slot_pair, int top, const float* pair_weight, const void* W, void* act,
+                                   const int* tiles, const int* n_tiles, int max_tiles, int tile_rows, int K, int F, float limit,
+                                   float alpha, hipStream_t stream) {
+    if (tile_rows != 32 && tile_rows != 64 && tile_rows != 128) return TM_ERR_ARG;
+    if (!x || !slot_pair || !W || !act || !tiles || !n_tiles || top <= 0 || K <= 0 || F <= 0 || ldx < K || max_tiles < 0 || K % 8 ||
+        ldx % 8 || !gm_aligned(x) || !gm_aligned(W) || !(limit > 0.f))
+        return TM_ERR_ARG;
+    if (max_tiles == 0) return TM_OK;
+    dim3 grid(max_tiles, (F + GM_BN - 1) / GM_BN);
+    if (grid.y > 65535) return TM_ERR_ARG;
+#define GM_GO(RT_, BK_)                                                                                                                  \
+    grouped_mfma_kernel<RT_, GM_CLAMPED, BK_, GM_BN><<<grid, 256, 0, stream>>>((const bf16_t*)x, ldx, 0, slot_pair, top, (const bf16_t*)W, act, F, \
+                                                                    0, nullptr, 0, tiles, n_tiles, 0, K, F, 0, 0, nullptr, nullptr, nullptr, \
+                                                                    pair_weight, limit, alpha)
+    if (tile_rows == 32) GM_GO(2, 128); else if (tile_rows == 64) GM_GO(4, GM_BK); else GM_GO(8, GM_BK);
 #undef GM_GO
     TM_CHECK_LAUNCH();
     return TM_OK;
@@ -231,7 +257,7 @@ extern "C" int tm_moe_up_act_mfma(const void* x, int ldx, const int* slot_pair, 
     if (grid.y > 65535) return TM_ERR_ARG;
 #define GM_GO(RT_, BK_, BN_)                                                                                                             \
     grouped_mfma_kernel<RT_, GM_RELU2, BK_, BN_><<<dim3(max_tiles, (F + BN_ - 1) / BN_), 256, 0, stream>>>((const bf16_t*)x, ldx, 0, slot_pair, top, (const bf16_t*)W, act, F, \
-                                                                 0, nullptr, 0, tiles, n_tiles, 0, K, F, 0, 0, nullptr, nullptr, nullptr)
+                                                                 0, nullptr, 0, tiles, n_tiles, 0, K, F, 0, 0, nullptr, nullptr, nullptr, nullptr, 0.f, 0.f)
     // tiles of 128 rows take 128 columns a block (a piece of A read from LDS meets two column groups) where that still
     // leaves two blocks a CU to choose from
     if (tile_rows == 32) GM_GO(2, 128, GM_BN); else if (tile_rows == 64) GM_GO(4, GM_BK, GM_BN);
@@ -251,7 +277,7 @@ extern "C" int tm_moe_down_mfma(const void* act, const void* W, float* part, con
     if (grid.y > 65535) return TM_ERR_ARG;
 #define GM_GO(RT_, BK_, BN_)                                                                                                              \
     grouped_mfma_kernel<RT_, GM_STORE_F32, BK_, BN_><<<dim3(max_tiles, (N + BN_ - 1) / BN_), 256, 0, stream>>>((const bf16_t*)act, F, 0, nullptr, 1, (const bf16_t*)W, part, N, 0, \
-                                                                     nullptr, 0, tiles, n_tiles, 0, F, N, 0, 0, nullptr, nullptr, nullptr)
+                                                                     nullptr, 0, tiles, n_tiles, 0, F, N, 0, 0, nullptr, nullptr, nullptr, nullptr, 0.f, 0.f)
     // tiles of 128 rows take 128 columns a block (a piece of A read from LDS meets two column groups) where that still
     // leaves two blocks a CU to choose from
     if (tile_rows == 32) GM_GO(2, 128, GM_BN); else if (tile_rows == 64) GM_GO(4, GM_BK, GM_BN);

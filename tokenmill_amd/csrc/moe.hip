@@ -4,15 +4,18 @@
 //   pair p = (token t = p / top, choice k = p % top) goes to expert e(p) = table[id[t] * top + k]  (ids null: table[p])
 //   tm_moe_router    z [T, E] (32-bit router outputs) -> s = softmax(z); the `top` largest of s + correction are chosen
 //                    (ties: the lower index), chosen[t, k] in descending order, weight[t, k] = s / (sum of the chosen s + 1e-20);
-//                    with `over_chosen` the `top` largest z are chosen and the weights are the softmax over the chosen z only
+//                    with `over_chosen` the `top` largest z are chosen and the weights are the softmax over the chosen z only;
+//                    with `sigmoid` s = sigmoid(z), and the chosen s are the weights as they are
 //   tm_moe_route     sorts the pairs by expert: slot_pair[slot] = p, pair_slot[p] = slot, and cuts every expert's run of
 //                    slots into tiles of `tile_rows` rows: tiles[i] = (expert, first slot, rows), n_tiles[0] = their number
 //   tm_moe_gate_up   act[slot] = silu(x[t] . Wg[e]^T) * (x[t] . Wu[e]^T)          W [E, 2F, K]: gate rows, then up rows
 //   tm_moe_down      part[slot] = act[slot] . Wd[e]^T  (32-bit)                    Wd [E, N, F]
 //   tm_moe_combine   y[t] = sum_k weight * part[pair_slot[t * top + k]], k ascending, rounded once
 //   tm_moe_up_act    act[slot] = relu(x[t] . Wu[e]^T)^2                           W [E, F, K]: experts without a gate
+//   tm_moe_clamped   act[slot] = g sigmoid(alpha g) (u + 1), g = min(z Wg[e] x[t], limit), u = z Wu[e] x[t] held to +-limit, with z the
+//                    pair's weight (null: 1): an expert on its weighted input                 W [E, 2F, K]
 //   tm_moe_combine_weighted   y[t] = sum_k weight[t, k] * (part[slot of the pair], or x[t] for a pair that has no slot: an
-//                    expert >= `real` stands for the input itself) + sigmoid(shared_gate[t]) * shared[t]
+//                    expert >= `real` stands for the input itself; weight null: 1) + sigmoid(shared_gate[t]) * shared[t]
 //
 // All of it runs from device data (no count crosses to the host), so a step can be recorded into a graph. Which slot a
 // pair gets inside its expert's run may differ from run to run (the cursor is an atomic counter); a row's result does not
@@ -95,13 +98,14 @@ extern "C" int tm_moe_route(const int* ids, const int* table, int T, int top, in
 
 // MODE 1 (gated): C[slot, n] = silu(a . W[e][n]) * (a . W[e][F + n]), a = A[slot_pair[slot] / top]; C of type T.
 // MODE 2         : C[slot, n] = relu(a . W[e][n])^2, the same a; C of type T.
+// MODE 3 (gated): the clamped gate of tm_moe_clamped, the same a; C of type T.
 // MODE 0         : C[slot, n] = A[slot] . W[e][n]; C float32.
 template <typename T, int MODE>
 __global__ __launch_bounds__(256) void moe_product_kernel(const T* __restrict__ A, int lda, const int* __restrict__ slot_pair, int top,
                                                           const T* __restrict__ W, void* __restrict__ Cv, int ldc,
                                                           const int* __restrict__ tiles, const int* __restrict__ n_tiles, int K,
-                                                          int N) {
-    constexpr bool GATED = MODE == 1, GATHER = MODE != 0;
+                                                          int N, const float* __restrict__ pair_weight, float limit, float alpha) {
+    constexpr bool GATED = MODE == 1 || MODE == 3, GATHER = MODE != 0;
     if ((int)blockIdx.x >= n_tiles[0]) return;
     __shared__ float As[MG_TM][MG_TK + 1];
     __shared__ float Bs[GATED ? 2 : 1][MG_TK][MG_TN + 1];
@@ -151,7 +155,10 @@ __global__ __launch_bounds__(256) void moe_product_kernel(const T* __restrict__ 
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
             if (n >= N) continue;
-            if (GATED) {
+            if (MODE == 3) {
+                const float z = pair_weight ? pair_weight[slot_pair[slot0 + r]] : 1.f;
+                Elem<T>::store((T*)Cv + (size_t)(slot0 + r) * ldc + n, clamped_glu_f32(z * acc[i][j], z * acu[i][j], alpha, limit));
+            } else if (GATED) {
                 const float g = acc[i][j], u = acu[i][j];
                 Elem<T>::store((T*)Cv + (size_t)(slot0 + r) * ldc + n, g / (1.0f + __expf(-g)) * u);
             } else if (MODE == 2) {
@@ -173,10 +180,10 @@ extern "C" int tm_moe_gate_up(const void* x, int ldx, const int* slot_pair, int 
     if (grid.y > 65535) return TM_ERR_ARG;
     if (dtype == TM_F32)
         moe_product_kernel<float, 1><<<grid, 256, 0, stream>>>((const float*)x, ldx, slot_pair, top, (const float*)W, act, F, tiles,
-                                                                  n_tiles, K, F);
+                                                                  n_tiles, K, F, nullptr, 0.f, 0.f);
     else
         moe_product_kernel<bf16_t, 1><<<grid, 256, 0, stream>>>((const bf16_t*)x, ldx, slot_pair, top, (const bf16_t*)W, act, F, tiles,
-                                                                   n_tiles, K, F);
+                                                                   n_tiles, K, F, nullptr, 0.f, 0.f);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
@@ -190,10 +197,29 @@ extern "C" int tm_moe_up_act(const void* x, int ldx, const int* slot_pair, int t
     if (grid.y > 65535) return TM_ERR_ARG;
     if (dtype == TM_F32)
         moe_product_kernel<float, 2><<<grid, 256, 0, stream>>>((const float*)x, ldx, slot_pair, top, (const float*)W, act, F, tiles,
-                                                               n_tiles, K, F);
+                                                               n_tiles, K, F, nullptr, 0.f, 0.f);
     else
         moe_product_kernel<bf16_t, 2><<<grid, 256, 0, stream>>>((const bf16_t*)x, ldx, slot_pair, top, (const bf16_t*)W, act, F, tiles,
-                                                                n_tiles, K, F);
+                                                                n_tiles, K, F, nullptr, 0.f, 0.f);
+    TM_CHECK_LAUNCH();
+    return TM_OK;
+}
+
+extern "C" int tm_moe_clamped(const void* x, int ldx, const int* slot_pair, int top, const float* pair_weight, const void* W, void* act,
+                              const int* tiles, const int* n_tiles, int max_tiles, int K, int F, float limit, float alpha, int dtype,
+                              hipStream_t stream) {
+    if (!x || !slot_pair || !W || !act || !tiles || !n_tiles || top <= 0 || K <= 0 || F <= 0 || ldx < K || max_tiles < 0 || !(limit > 0.f))
+        return TM_ERR_ARG;
+    if (dtype != TM_F32 && dtype != TM_BF16) return TM_ERR_ARG;
+    if (max_tiles == 0) return TM_OK;
+    dim3 grid(max_tiles, (F + MG_TN - 1) / MG_TN);
+    if (grid.y > 65535) return TM_ERR_ARG;
+    if (dtype == TM_F32)
+        moe_product_kernel<float, 3><<<grid, 256, 0, stream>>>((const float*)x, ldx, slot_pair, top, (const float*)W, act, F, tiles,
+                                                               n_tiles, K, F, pair_weight, limit, alpha);
+    else
+        moe_product_kernel<bf16_t, 3><<<grid, 256, 0, stream>>>((const bf16_t*)x, ldx, slot_pair, top, (const bf16_t*)W, act, F, tiles,
+                                                                n_tiles, K, F, pair_weight, limit, alpha);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
@@ -207,10 +233,10 @@ extern "C" int tm_moe_down(const void* act, const void* W, float* part, const in
     if (grid.y > 65535) return TM_ERR_ARG;
     if (dtype == TM_F32)
         moe_product_kernel<float, 0><<<grid, 256, 0, stream>>>((const float*)act, F, nullptr, 1, (const float*)W, part, N, tiles,
-                                                                   n_tiles, F, N);
+                                                                   n_tiles, F, N, nullptr, 0.f, 0.f);
     else
         moe_product_kernel<bf16_t, 0><<<grid, 256, 0, stream>>>((const bf16_t*)act, F, nullptr, 1, (const bf16_t*)W, part, N, tiles,
-                                                                    n_tiles, F, N);
+                                                                    n_tiles, F, N, nullptr, 0.f, 0.f);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
@@ -246,7 +272,7 @@ extern "C" int tm_moe_combine(const float* part, const int* pair_slot, void* y, 
 template <int RT_MAX_PER_LANE>
 __global__ __launch_bounds__(TM_WAVE) void moe_router_kernel(const float* __restrict__ z, int ldz, const float* __restrict__ correction,
                                                              int E, int top, int* __restrict__ chosen, float* __restrict__ weight,
-                                                             int over_chosen) {
+                                                             int over_chosen, int sigmoid) {
     const int t = blockIdx.x, lane = threadIdx.x;
     const float* zr = z + (size_t)t * ldz;
     float s[RT_MAX_PER_LANE], c[RT_MAX_PER_LANE];
@@ -257,13 +283,13 @@ __global__ __launch_bounds__(TM_WAVE) void moe_router_kernel(const float* __rest
         s[i] = e < E ? zr[e] : -INFINITY;
         m = fmaxf(m, s[i]);
     }
-    m = wave_max(m);
+    m = sigmoid ? 0.f : wave_max(m);
     float sum = 0.f;
 #pragma unroll
     for (int i = 0; i < RT_MAX_PER_LANE; ++i) {
         const int e = lane + i * TM_WAVE;
         c[i] = s[i];                             // the output itself: what `over_chosen` ranks
-        s[i] = e < E ? expf(s[i] - m) : 0.f;     // m is the largest output, which is chosen first: these are the chosen ones' terms too
+        s[i] = e >= E ? 0.f : sigmoid ? 1.f / (1.f + expf(-s[i])) : expf(s[i] - m);     // m is the largest output, which is chosen first: these are the chosen ones' terms too
         sum += s[i];
     }
     sum = wave_sum(sum);
@@ -271,7 +297,7 @@ __global__ __launch_bounds__(TM_WAVE) void moe_router_kernel(const float* __rest
 #pragma unroll
         for (int i = 0; i < RT_MAX_PER_LANE; ++i) {
             const int e = lane + i * TM_WAVE;
-            s[i] = s[i] / sum;
+            if (!sigmoid) s[i] = s[i] / sum;
             c[i] = e < E ? s[i] + (correction ? correction[e] : 0.f) : -INFINITY;
         }
     }
@@ -297,19 +323,20 @@ __global__ __launch_bounds__(TM_WAVE) void moe_router_kernel(const float* __rest
             weight[(size_t)t * top + k] = sc;
         }
     }
+    if (sigmoid) return;
     __syncthreads();                         // lane 0's scores, seen by the lanes that scale them
     const float inv = over_chosen ? 1.f / total : 1.f / (total + 1e-20f);
     for (int k = lane; k < top; k += TM_WAVE) weight[(size_t)t * top + k] *= inv;
 }
 
 extern "C" int tm_moe_router(const float* z, int ldz, const float* correction, int T, int E, int top, int* chosen, float* weight,
-                             int over_chosen, hipStream_t stream) {
+                             int over_chosen, int sigmoid, hipStream_t stream) {
     if (!z || !chosen || !weight || T < 0 || E <= 0 || E > MOE_MAX_EXPERTS || top <= 0 || top > E || ldz < E) return TM_ERR_ARG;
     if (T == 0) return TM_OK;
-    if (over_chosen && correction) return TM_ERR_ARG;
-    if (E <= TM_WAVE) moe_router_kernel<1><<<T, TM_WAVE, 0, stream>>>(z, ldz, correction, E, top, chosen, weight, over_chosen);
-    else if (E <= 4 * TM_WAVE) moe_router_kernel<4><<<T, TM_WAVE, 0, stream>>>(z, ldz, correction, E, top, chosen, weight, over_chosen);
-    else moe_router_kernel<MOE_MAX_EXPERTS / TM_WAVE><<<T, TM_WAVE, 0, stream>>>(z, ldz, correction, E, top, chosen, weight, over_chosen);
+    if (over_chosen && (correction || sigmoid)) return TM_ERR_ARG;
+    if (E <= TM_WAVE) moe_router_kernel<1><<<T, TM_WAVE, 0, stream>>>(z, ldz, correction, E, top, chosen, weight, over_chosen, sigmoid);
+    else if (E <= 4 * TM_WAVE) moe_router_kernel<4><<<T, TM_WAVE, 0, stream>>>(z, ldz, correction, E, top, chosen, weight, over_chosen, sigmoid);
+    else moe_router_kernel<MOE_MAX_EXPERTS / TM_WAVE><<<T, TM_WAVE, 0, stream>>>(z, ldz, correction, E, top, chosen, weight, over_chosen, sigmoid);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
@@ -328,7 +355,7 @@ __global__ __launch_bounds__(256) void moe_combine_weighted_kernel(const float* 
     for (int k = 0; k < top; ++k) {
         const int slot = pair_slot[t * top + k];
         const float v = slot >= 0 ? part[(size_t)slot * N + c] : Elem<T>::load(x + (size_t)t * ldx + c);
-        s += weight[(size_t)t * top + k] * v;
+        s += weight ? weight[(size_t)t * top + k] * v : v;
     }
     if (shared) s += sg * shared[(size_t)t * N + c];
     Elem<T>::store(y + (size_t)t * N + c, s);
@@ -338,7 +365,7 @@ __global__ __launch_bounds__(256) void moe_combine_weighted_kernel(const float* 
 extern "C" int tm_moe_combine_weighted(const float* part, const int* pair_slot, const float* weight, const void* x, int ldx,
                                        const float* shared, const float* shared_gate, int ldg, void* y, int T, int top, int N, int dtype,
                                        hipStream_t stream) {
-    if (!part || !pair_slot || !weight || !x || !y || T < 0 || top <= 0 || N <= 0 || ldx < N || (shared_gate && ldg < 1)) return TM_ERR_ARG;
+    if (!part || !pair_slot || !x || !y || T < 0 || top <= 0 || N <= 0 || ldx < N || (shared_gate && ldg < 1)) return TM_ERR_ARG;
     if (dtype != TM_F32 && dtype != TM_BF16) return TM_ERR_ARG;
     if (T == 0) return TM_OK;
     const dim3 grid(T, (N + 255) / 256);

@@ -1,6 +1,7 @@
 // Single tokens through a recurrent mixer in one launch: everything between the input projections and the output projection.
 //
-//   tm_retention_step   rotation, S <- decay S + k v^T, o = S^T q, o / rms(o) * silu(g)
+//   tm_retention_step   rotation, S <- decay S + k v^T, o = S^T q, o / rms(o) * silu(g); with `silu` q, k and v are silu of the
+//                       projection; with o_out the heads' o go there in 32-bit as they are (a norm over all heads follows)
 //   tm_delta_step       short convolutions and their state, silu, unit norms, step sizes and decays,
 //                       S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q,   rms norm with a weight, gate
 //
@@ -28,7 +29,11 @@ __global__ __launch_bounds__(RS_THREADS) void retention_step_kernel(const T* __r
                                                                    const float* __restrict__ sin_t, int rot, const int* __restrict__ positions,
                                                                    const float* __restrict__ decay, float* __restrict__ state,
                                                                    const int* __restrict__ slots, T* __restrict__ y, int H, int D, int Dv,
-                                                                   float k_scale, float eps) {
+                                                                   float k_scale, float eps, int silu, float* __restrict__ o_out) {
+    auto in = [&](const T* p) {
+        const float z = Elem<T>::load(p);
+        return silu ? rs_silu(z) : z;
+    };
     __shared__ float q_s[RS_MAX_D], k_s[RS_MAX_D], part[RS_THREADS], red[RS_WAVES];
     const int h = blockIdx.x, t = blockIdx.y, tid = threadIdx.x, wave = tid / TM_WAVE, lane = tid % TM_WAVE;
     const T* row = proj + (size_t)t * ld;
@@ -38,22 +43,22 @@ __global__ __launch_bounds__(RS_THREADS) void retention_step_kernel(const T* __r
     for (int j = tid; j < half; j += RS_THREADS) {
         const float c = cos_t[(size_t)positions[t] * half + j], s = sin_t[(size_t)positions[t] * half + j];
         float a, b;
-        rotate_pair(Elem<T>::load(q + j), Elem<T>::load(q + j + half), c, s, a, b);
+        rotate_pair(in(q + j), in(q + j + half), c, s, a, b);
         q_s[j] = a;
         q_s[j + half] = b;
-        rotate_pair(Elem<T>::load(k + j), Elem<T>::load(k + j + half), c, s, a, b);
+        rotate_pair(in(k + j), in(k + j + half), c, s, a, b);
         k_s[j] = a * k_scale;
         k_s[j + half] = b * k_scale;
     }
     for (int d = rot + tid; d < D; d += RS_THREADS) {
-        q_s[d] = Elem<T>::load(q + d);
-        k_s[d] = Elem<T>::load(k + d) * k_scale;
+        q_s[d] = in(q + d);
+        k_s[d] = in(k + d) * k_scale;
     }
     const int nc = (Dv + TM_WAVE - 1) / TM_WAVE, RG = RS_WAVES / nc;
     const int cg = wave % nc, rg = wave / nc;
     const int e = cg * TM_WAVE + lane;
     const bool mine = rg < RG && e < Dv;
-    const float v = mine ? Elem<T>::load(row + 2 * H * D + h * Dv + e) : 0.f;
+    const float v = mine ? in(row + 2 * H * D + h * Dv + e) : 0.f;
     const float a = decay[h * D];
     float* st = state + (((size_t)slots[t] * H + h) * D) * Dv + (mine ? e : 0);
     __syncthreads();
@@ -85,6 +90,10 @@ __global__ __launch_bounds__(RS_THREADS) void retention_step_kernel(const T* __r
     const bool out = tid < Dv;
     if (out)
         for (int i = 0; i < RG; ++i) o += part[i * nc * TM_WAVE + tid];
+    if (o_out) {
+        if (out) o_out[((size_t)t * H + h) * Dv + tid] = o;
+        return;
+    }
     const float ss = block_sum<RS_THREADS>(o * o, red);
     if (out) {
         const float g = Elem<T>::load(row + 2 * H * D + H * Dv + h * Dv + tid);
@@ -94,18 +103,18 @@ __global__ __launch_bounds__(RS_THREADS) void retention_step_kernel(const T* __r
 
 extern "C" int tm_retention_step(const void* proj, int ld, int dtype, const float* cos_t, const float* sin_t, int rot, const int* positions,
                                  const float* decay, float* state, const int* state_slots, void* y, int n, int H, int D, int Dv,
-                                 float k_scale, float eps, hipStream_t stream) {
+                                 float k_scale, float eps, int silu, float* o_out, hipStream_t stream) {
     if (n <= 0) return TM_OK;
-    if (!proj || !decay || !state || !state_slots || !y || H <= 0 || D <= 0 || D > RS_MAX_D || Dv <= 0 || Dv > RS_THREADS || rot < 0 || rot > D ||
-        (rot & 1) || (rot && (!cos_t || !sin_t || !positions)) || ld < 2 * H * (D + Dv) || n > 65535 || !(eps > 0.f))
+    if (!proj || !decay || !state || !state_slots || (!y && !o_out) || H <= 0 || D <= 0 || D > RS_MAX_D || Dv <= 0 || Dv > RS_THREADS || rot < 0 || rot > D ||
+        (rot & 1) || (rot && (!cos_t || !sin_t || !positions)) || ld < (o_out ? H * (2 * D + Dv) : 2 * H * (D + Dv)) || n > 65535 || !(eps > 0.f))
         return TM_ERR_ARG;
     const dim3 grid(H, n);
     if (dtype == TM_F32)
         retention_step_kernel<float><<<grid, RS_THREADS, 0, stream>>>((const float*)proj, ld, cos_t, sin_t, rot, positions, decay, state,
-                                                                      state_slots, (float*)y, H, D, Dv, k_scale, eps);
+                                                                      state_slots, (float*)y, H, D, Dv, k_scale, eps, silu, o_out);
     else if (dtype == TM_BF16)
         retention_step_kernel<bf16_t><<<grid, RS_THREADS, 0, stream>>>((const bf16_t*)proj, ld, cos_t, sin_t, rot, positions, decay, state,
-                                                                       state_slots, (bf16_t*)y, H, D, Dv, k_scale, eps);
+                                                                       state_slots, (bf16_t*)y, H, D, Dv, k_scale, eps, silu, o_out);
     else
         return TM_ERR_ARG;
     TM_CHECK_LAUNCH();

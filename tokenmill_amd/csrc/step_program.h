@@ -54,6 +54,7 @@ struct TmAttentionOp {          // resid += o(attention(rope(qkv(norm(resid)))))
     float softcap;              // > 0: a scaled score s becomes softcap * tanh(s / softcap) before the softmax
     int outside;                // 1: q always comes projected, encoded and stored (TmStream.qkv); `qkv` and `norm` are not looked at
     const float* sink;          // [H]: one more term exp(sink[h]) in the denominator of head h's softmax, with no key behind it; or null
+    int keep;                   // with a window: the first keys of a request that every token sees beside its window
 };
 
 struct TmFfnOp {                // resid += down(silu(gate(n)) * up(n)), n = norm(resid)
@@ -97,6 +98,8 @@ struct TmStream {
     int qkv_stride;             // elements between the rows of `qkv` (0: (H + 2 KVH) D); a caller that hands in q alone says H D
     const float* gate;          // with `qkv`: a gate per (token, head), rows `ldg` apart: head h of token t is multiplied by
     int ldg;                    // sigmoid(gate[t * ldg + h]) between the attention and the output projection; or null
+    const void* channel_gate;   // with `qkv`: a gate per channel (model type), rows `ldcg` apart: channel c of the attention's result is
+    int ldcg;                   // multiplied by sigmoid(channel_gate[t * ldcg + c]) before the output projection; or null
 };
 
 struct TmProgram;

@@ -192,6 +192,8 @@ struct Run {
     int qkv_in_stride = 0;              // its row stride (0: the whole q|k|v)
     const float* gate_in = nullptr;     // a gate per (token, head) for that operation's result
     int gate_ld = 0;
+    const void* cgate_in = nullptr;     // a gate per channel for it
+    int cgate_ld = 0;
     bool accumulate;
     // workspace
     void *x, *qkv, *attn, *gu, *act, *delta_buf, *hnorm;
@@ -357,17 +359,17 @@ struct Run {
                     HD % 4 == 0 && aligned(attn, 8)) {
                     ++p->taken[TM_PREFILL_SHARED_KEYS];
                     rc = tm_attn_prefill_shared_cap(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->prefill_tiles,
-                                                    s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.softcap, a.sink, stream);
+                                                    s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.keep, a.softcap, a.sink, stream);
                 } else {
                     ++p->taken[TM_PREFILL_SPLIT_KEYS];
                     rc = tm_attn_prefill_mfma_cap(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->prefill_tiles,
-                                                  s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.softcap, a.sink, stream);
+                                                  s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.keep, a.softcap, a.sink, stream);
                 }
                 done_prefill = true;
             } else if (tp && s->n_tiles > 0 && s->prefill_tiles && dtype == TM_F32 && a.D % 16 == 0 && a.D >= 16 &&
                        a.D <= 128 && page_ok && q_stride % 4 == 0 && aligned(q, 16)) {
                 rc = tm_attn_prefill_f32_cap(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->prefill_tiles, s->n_tiles, a.H,
-                                             a.KVH, a.D, a.page, a.scale, a.window, a.softcap, a.sink, stream);
+                                             a.KVH, a.D, a.page, a.scale, a.window, a.keep, a.softcap, a.sink, stream);
                 done_prefill = true;
             }
             if (rc) return rc;
@@ -377,24 +379,29 @@ struct Run {
                 const bool split = tm_decode_splits(nd, a.KVH, s->max_decode_context);
                 rc = tm_attn_decode_mfma_cap(q_dec, q_stride, out_dec, HD, a.k_pool, a.v_pool, tables + (size_t)(S - nd) * W, W,
                                              s->context_lens + (S - nd), split ? part_o : nullptr, split ? part_ml : nullptr,
-                                             tm_decode_chunks(s->max_decode_context), nd, a.H, a.KVH, a.D, a.page, a.scale, a.window,
+                                             tm_decode_chunks(s->max_decode_context), nd, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.keep,
                                              a.softcap, a.sink, stream);
                 done_decode = true;
             }
             if (rc) return rc;
             if (tp && !done_prefill && nd && !done_decode) {
                 rc = tm_attn_paged_generic_ext(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->seq_of_token, s->positions, T,
-                                               a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.softcap, nullptr, 0, a.sink, dtype, stream);
+                                               a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.keep, a.softcap, nullptr, 0, a.sink, dtype, stream);
             } else {
                 if (tp && !done_prefill)
                     rc = tm_attn_paged_generic_ext(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->seq_of_token, s->positions,
-                                                   tp, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.softcap, nullptr, 0, a.sink, dtype, stream);
+                                                   tp, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.keep, a.softcap, nullptr, 0, a.sink, dtype, stream);
                 if (!rc && nd && !done_decode)
                     rc = tm_attn_paged_generic_ext(q_dec, q_stride, out_dec, HD, a.k_pool, a.v_pool, tables, W, s->seq_of_token + tp,
-                                                   s->positions + tp, nd, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.softcap, nullptr, 0, a.sink,
+                                                   s->positions + tp, nd, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.keep, a.softcap, nullptr, 0, a.sink,
                                                    dtype, stream);
             }
             if (rc) return rc;
+            if (cgate_in) {                 // a gate per channel on the way to the output projection
+                rc = tm_channel_gate(attn, dtype, cgate_in, cgate_ld, T, HD, stream);
+                cgate_in = nullptr;
+                if (rc) return rc;
+            }
             if (gate_in) {                  // a gate per (token, head) on the way to the output projection
                 rc = tm_head_gate(attn, dtype, gate_in, gate_ld, T, a.H, a.D, stream);
                 gate_in = nullptr;
@@ -519,7 +526,7 @@ int tm_program_add_attention(TmProgram* p, const TmAttentionOp* a) {
     if (!p || !a || a->H <= 0 || a->KVH <= 0 || a->H % a->KVH || a->D <= 0 || !a->k_pool || !a->v_pool || a->page <= 0 ||
         !linear_fits(p, a->o) || a->o.K != a->H * a->D || a->o.N != p->hidden || !(a->softcap >= 0.f) ||
         (!a->outside && (!linear_fits(p, a->qkv) || a->qkv.K != p->hidden || a->qkv.N != (a->H + 2 * a->KVH) * a->D)) ||
-        a->window < 0 || a->rot < 0 || a->rot > a->D || (a->rot > 0 && (!a->cos_t || !a->sin_t)))
+        a->window < 0 || a->keep < 0 || a->rot < 0 || a->rot > a->D || (a->rot > 0 && (!a->cos_t || !a->sin_t)))
         return -1;
     Op op{};
     op.kind = OP_ATTENTION;
@@ -610,6 +617,8 @@ int tm_program_run(const TmProgram* p, int first, int count, const TmStep* s, Tm
     r.resid = io->resid; r.delta = io->delta; r.x_in = io->x; r.qkv_in = io->qkv; r.accumulate = io->accumulate != 0;
     r.qkv_in_stride = io->qkv_stride; r.gate_in = io->qkv ? io->gate : nullptr; r.gate_ld = io->ldg;
     if (r.gate_in && r.gate_ld < p->ops[first].att.H) return TM_ERR_ARG;
+    r.cgate_in = io->qkv ? io->channel_gate : nullptr; r.cgate_ld = io->ldcg;
+    if (r.cgate_in && r.cgate_ld < p->ops[first].att.H * p->ops[first].att.D) return TM_ERR_ARG;
     r.x = take((size_t)T * p->hidden * es);
     r.qkv = take((size_t)T * p->max_qkv * es);
     r.attn = take((size_t)T * p->max_heads_d * es);

@@ -604,9 +604,10 @@ def attn_decode_mfma_supported(dtype, H: int, KVH: int, D: int, page: int) -> bo
 def attn_decode_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                      block_tables: torch.Tensor, context_lens: torch.Tensor, H: int, KVH: int, D: int, scale: float,
                      window: int, max_context: int, workspace: tuple[torch.Tensor, torch.Tensor] | None = None,
-                     split: bool | None = None, softcap: float = 0.0, sink: torch.Tensor | None = None):
+                     split: bool | None = None, softcap: float = 0.0, sink: torch.Tensor | None = None, keep: int = 0):
     """Attention of one new token per request over its cache (the token's own key included); ``softcap`` > 0: a scaled
-    score s becomes softcap * tanh(s / softcap); ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator.
+    score s becomes softcap * tanh(s / softcap); ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator;
+    ``keep``: with a window, the first keys of a request that every token sees beside it.
     q: [S, >= H*D] rows (unit inner stride), out [S, H*D] view; block_tables int32 [S, W];
     context_lens int32 [S] (new token counted); max_context >= every context length. ``split``: None runs
     the kernel the library's rule names for this many requests (contexts split over blocks and merged, or one
@@ -643,7 +644,7 @@ def attn_decode_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v
     _check(library().tm_attn_decode_mfma_cap(_p(q), c_int(q_stride), _p(out), c_int(out_stride), _p(k_pool), _p(v_pool),
                                              _p(block_tables), c_int(W), _p(context_lens), _p(part_o), _p(part_ml),
                                              c_int(chunks), c_int(S), c_int(H), c_int(KVH), c_int(D), c_int(page),
-                                             c_float(scale), c_int(window), c_float(softcap), _p(sink), _stream()), "attn_decode_mfma")
+                                             c_float(scale), c_int(window), c_int(keep), c_float(softcap), _p(sink), _stream()), "attn_decode_mfma")
     return out
 
 
@@ -657,9 +658,11 @@ def attn_prefill_mfma_supported(dtype, H: int, KVH: int, D: int, page: int) -> b
 
 def attn_prefill_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                       block_tables: torch.Tensor, tiles: torch.Tensor, H: int, KVH: int, D: int, scale: float,
-                      window: int, shared: bool = False, softcap: float = 0.0, sink: torch.Tensor | None = None) -> torch.Tensor:
+                      window: int, shared: bool = False, softcap: float = 0.0, sink: torch.Tensor | None = None,
+                      keep: int = 0) -> torch.Tensor:
     """Attention of prompt portions over the cache (``softcap`` > 0: a scaled score s becomes softcap * tanh(s / softcap);
-    ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator). q: [T, >= H*D] rows, out [T, H*D]; tiles int32
+    ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator; ``keep``: with a window, the first keys of a request
+    that every token sees beside it). q: [T, >= H*D] rows, out [T, H*D]; tiles int32
     [n, 4] = (request index, first row, tokens (1..16), position of the first token) cover the rows
     to compute; every row of a tile belongs to one request at consecutive positions. ``shared``: the kernel
     that stages a tile's keys and values through LDS for all heads of a kv head, instead of the one whose
@@ -687,7 +690,7 @@ def attn_prefill_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, 
     _check(entry(_p(q), c_int(q_stride), _p(out), c_int(out_stride), _p(k_pool), _p(v_pool),
                  _p(block_tables), c_int(block_tables.shape[1]), _p(tiles),
                  c_int(tiles.shape[0]), c_int(H), c_int(KVH), c_int(D), c_int(page),
-                 c_float(scale), c_int(window), c_float(softcap), _p(sink), _stream()), "attn_prefill_shared" if shared else "attn_prefill_mfma")
+                 c_float(scale), c_int(window), c_int(keep), c_float(softcap), _p(sink), _stream()), "attn_prefill_shared" if shared else "attn_prefill_mfma")
     return out
 
 
@@ -698,7 +701,7 @@ def attn_prefill_f32_supported(dtype, H: int, KVH: int, D: int, page: int) -> bo
 
 def attn_prefill_f32(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                      block_tables: torch.Tensor, tiles: torch.Tensor, H: int, KVH: int, D: int, scale: float,
-                     window: int, softcap: float = 0.0, sink: torch.Tensor | None = None) -> torch.Tensor:
+                     window: int, softcap: float = 0.0, sink: torch.Tensor | None = None, keep: int = 0) -> torch.Tensor:
     """Attention of prompt portions over the cache in true 32-bit (32-bit MFMA). Operands as for
     ``attn_prefill_mfma``, all float32."""
     _gpu(q, out, k_pool, v_pool, block_tables, tiles, sink)
@@ -719,7 +722,7 @@ def attn_prefill_f32(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v
     _check(library().tm_attn_prefill_f32_cap(_p(q), c_int(q_stride), _p(out), c_int(out_stride), _p(k_pool), _p(v_pool),
                                              _p(block_tables), c_int(block_tables.shape[1]), _p(tiles),
                                              c_int(tiles.shape[0]), c_int(H), c_int(KVH), c_int(D), c_int(page),
-                                             c_float(scale), c_int(window), c_float(softcap), _p(sink), _stream()), "attn_prefill_f32")
+                                             c_float(scale), c_int(window), c_int(keep), c_float(softcap), _p(sink), _stream()), "attn_prefill_f32")
     return out
 
 
@@ -1754,11 +1757,12 @@ def whole_norm_rope_store(proj: torch.Tensor, q_out: torch.Tensor, H: int, G: in
 def attn_paged_softmax(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, block_tables: torch.Tensor,
                        seq_of_token: torch.Tensor, positions: torch.Tensor, H: int, G: int, D: int, Dv: int, scale: float,
                        window: int = 0, softcap: float = 0.0, gate: torch.Tensor | None = None,
-                       sink: torch.Tensor | None = None) -> torch.Tensor:
+                       sink: torch.Tensor | None = None, keep: int = 0) -> torch.Tensor:
     """Softmax attention of every token of the step over its request's cached keys (its own included), a token and a head a
     wavefront: keys of D channels, values of Dv; a score s becomes softcap * tanh(s / softcap) if ``softcap`` > 0; head h of
     token t is multiplied by sigmoid(gate[t, h]) (gate: a float32 view [T, >= H] with unit inner stride; None: no gate);
-    ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator. q [T, >= H*D] with unit inner stride, out [T, H*Dv]."""
+    ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator; ``keep``: with a window, the first keys of a request
+    that every token sees beside it. q [T, >= H*D] with unit inner stride, out [T, H*Dv]."""
     _gpu(q, out, k_pool, v_pool, block_tables, seq_of_token, positions, gate, sink)
     _check_sink(sink, H)
     T = q.shape[0]
@@ -1771,7 +1775,7 @@ def attn_paged_softmax(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor,
           "attention: block_tables must be contiguous int32 [S, W]")
     _ints(seq_of_token, T, "seq_of_token")
     _ints(positions, T, "positions")
-    _need(window >= 0 and softcap >= 0, "attention: window and softcap must be >= 0 (0 = none)")
+    _need(window >= 0 and softcap >= 0 and keep >= 0, "attention: window, keep and softcap must be >= 0 (0 = none)")
     ldg = 0
     if gate is not None:
         _need(gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape[0] == T and gate.shape[1] >= H and gate.stride(1) == 1,
@@ -1781,22 +1785,115 @@ def attn_paged_softmax(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor,
     _check(library().tm_attn_paged_generic_ext(_p(q), c_int(q_stride), _p(out), c_int(H * Dv), _p(k_pool), _p(v_pool), _p(block_tables),
                                                c_int(block_tables.shape[1]), _p(seq_of_token), _p(positions), c_int(T), c_int(H),
                                                c_int(G), c_int(D), c_int(Dv), c_int(page), c_float(scale), c_int(window),
-                                               c_float(softcap), _p(gate), c_int(ldg), _p(sink), code(q.dtype), _stream()), "attn_paged_generic_ext")
+                                               c_int(keep), c_float(softcap), _p(gate), c_int(ldg), _p(sink), code(q.dtype), _stream()), "attn_paged_generic_ext")
+    return out
+
+
+CONV_PREPARE_MAX_FLOATS = 36 * 1024     # q and k channels of a token, and their heads, that ``conv_norm_rope_store`` takes
+
+
+def conv_norm_rope_store(proj: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Tensor | None, cu_q_lens: torch.Tensor,
+                         state_slots: torch.Tensor, seq_of_token: torch.Tensor, num_seqs: int, num_single: int, q_out: torch.Tensor, H: int,
+                         G: int, D: int, Dv: int, q_w: torch.Tensor | None, k_w: torch.Tensor | None, eps: float, cos: torch.Tensor | None,
+                         sin: torch.Tensor | None, interleaved: bool, positions: torch.Tensor, slots: torch.Tensor, k_pool: torch.Tensor,
+                         v_pool: torch.Tensor, per_head: bool = False) -> torch.Tensor:
+    """``whole_norm_rope_store`` behind a short causal convolution over time on every channel of q | k | v (proj [T, >= H*D + G*D +
+    G*Dv] of the model's type; conv_w [channels, taps] of the same type): rows before a request's first row of the step come from its
+    conv_state [slots, taps - 1, channels] (None with one tap), which becomes the last taps - 1 rows the request has seen. The
+    step's last ``num_single`` rows and requests are single tokens."""
+    _gpu(proj, conv_w, conv_state, cu_q_lens, state_slots, seq_of_token, q_out, q_w, k_w, cos, sin, positions, slots, k_pool, v_pool)
+    T = proj.shape[0]
+    C = (H + G) * D + G * Dv
+    _need(proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= C, f"conv_norm_rope_store: proj is [T, >= {C}]")
+    _need(conv_w.dim() == 2 and conv_w.shape[0] == C and conv_w.is_contiguous() and conv_w.dtype == proj.dtype,
+          f"conv_norm_rope_store: conv_w is [{C}, taps] of proj's type")
+    taps = conv_w.shape[1]
+    _need(1 <= taps <= 16, "conv_norm_rope_store: 1 to 16 taps")
+    _need((conv_state is None) == (taps == 1), "conv_norm_rope_store: a state goes with more than one tap")
+    if conv_state is not None:
+        _need(conv_state.dim() == 3 and tuple(conv_state.shape[1:]) == (taps - 1, C) and conv_state.is_contiguous() and conv_state.dtype == proj.dtype,
+              f"conv_norm_rope_store: the state is [slots, {taps - 1}, {C}] of proj's type")
+    _need(tuple(q_out.shape) == (T, H * D) and q_out.is_contiguous() and q_out.dtype == proj.dtype, f"conv_norm_rope_store: q_out is [{T}, {H * D}] of proj's type")
+    _need((H + G) * (D + 1) <= CONV_PREPARE_MAX_FLOATS, "conv_norm_rope_store: too many channels of q and k for the kernel's LDS")
+    for w, n in ((q_w, D if per_head else H * D), (k_w, D if per_head else G * D)):
+        if w is not None:
+            _need(w.dtype == torch.float32 and tuple(w.shape) == (n,) and w.is_contiguous(), f"conv_norm_rope_store: a norm weight is float32 [{n}]")
+    _need((q_w is None) == (k_w is None) and eps > 0, "conv_norm_rope_store: q and k are normed together or not at all")
+    rot = 0
+    if cos is not None:
+        rot = 2 * cos.shape[1]
+        _need(sin is not None and cos.dtype == sin.dtype == torch.float32 and cos.shape == sin.shape and cos.is_contiguous()
+              and sin.is_contiguous() and rot <= D, "conv_norm_rope_store: cos/sin float32 [max_pos, rot/2], rot <= D")
+    page = _check_pools_kv(k_pool, v_pool, G, D, Dv, proj.dtype, "conv_norm_rope_store")
+    _need(0 <= num_single <= min(T, num_seqs), "conv_norm_rope_store: single tokens are rows and requests of the step")
+    _ints(positions, T, "positions")
+    _ints(slots, T, "slots")
+    _ints(seq_of_token, T, "seq_of_token")
+    _ints(cu_q_lens, num_seqs + 1, "cu_q_lens")
+    _ints(state_slots, num_seqs, "state_slots")
+    ld = proj.stride(0) if T > 1 else max(C, proj.stride(0))
+    portions = num_seqs - num_single
+    _check(library().tm_conv_norm_rope_store(_p(proj), c_int(ld), c_int(code(proj.dtype)), _p(conv_w), _p(conv_state), c_int(taps),
+                                             _p(cu_q_lens), _p(state_slots), _p(seq_of_token), c_int(T), c_int(T - num_single),
+                                             c_int(portions), _p(q_out), c_int(H), c_int(G), c_int(D), c_int(Dv), c_int(rot),
+                                             c_int(1 if interleaved else 0), _p(q_w), _p(k_w), c_float(eps), c_int(1 if per_head else 0),
+                                             _p(cos), _p(sin), _p(positions), _p(slots), _p(k_pool), _p(v_pool), c_int(page), _stream()),
+           "conv_norm_rope_store")
+    if conv_state is not None and portions:
+        delta_conv_state(proj, C, conv_state, cu_q_lens, state_slots, portions)
+    return q_out
+
+
+def channel_gate(x: torch.Tensor, gate: torch.Tensor) -> torch.Tensor:
+    """x[t, c] *= sigmoid(gate[t, c]) in place: x contiguous [T, N], gate a view [T, >= N] of x's type with unit inner stride."""
+    _gpu(x, gate)
+    T, N = x.shape
+    _need(x.is_contiguous() and gate.dim() == 2 and gate.shape[0] == T and gate.shape[1] >= N and gate.stride(1) == 1 and gate.dtype == x.dtype,
+          f"channel_gate: gate is [{T}, >= {N}] of x's type")
+    _check(library().tm_channel_gate(_p(x), c_int(code(x.dtype)), _p(gate), c_int(gate.stride(0) if T > 1 else max(gate.stride(0), N)),
+                                     c_int(T), c_int(N), _stream()), "channel_gate")
+    return x
+
+
+def scale_cap(x: torch.Tensor, scale: float, cap: float = 0.0) -> torch.Tensor:
+    """x (contiguous float32) becomes x * scale, and with ``cap`` > 0 then cap * tanh(x / cap), in place."""
+    _gpu(x)
+    _need(x.dtype == torch.float32 and x.is_contiguous() and cap >= 0, "scale_cap: x is contiguous float32, cap >= 0")
+    _check(library().tm_scale_cap(_p(x), c_longlong(x.numel()), c_float(scale), c_float(cap), _stream()), "scale_cap")
+    return x
+
+
+def embed_waves(table: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor, freq: torch.Tensor, out: torch.Tensor,
+                scale: float = 1.0) -> torch.Tensor:
+    """out[t] = table[ids[t]] * scale + the waves of the token's position: channel 2i is sin(p freq[i]), channel 2i + 1 cos(p freq[i]).
+    table [V, hidden]; ids, positions int32 [T]; freq float32 [ceil(hidden / 2)]; out float32 [T, hidden]."""
+    _gpu(table, ids, positions, freq, out)
+    T = ids.numel()
+    V, hidden = table.shape
+    _need(table.is_contiguous() and out.is_contiguous() and out.dtype == torch.float32 and tuple(out.shape) == (T, hidden),
+          "embed_waves: out is contiguous float32 [T, hidden]")
+    _need(freq.dtype == torch.float32 and freq.is_contiguous() and tuple(freq.shape) == ((hidden + 1) // 2,), "embed_waves: freq is float32 [ceil(hidden / 2)]")
+    _ints(ids, T, "ids")
+    _ints(positions, T, "positions")
+    _check(library().tm_embed_waves(_p(table), code(table.dtype), _p(ids), _p(positions), _p(freq), _p(out), c_int(T), c_int(hidden),
+                                    c_int(V), c_float(scale), _stream()), "embed_waves")
     return out
 
 
 # -------------------------------------------------------------------------------------------- experts by router
 
-def moe_router(z: torch.Tensor, experts: int, top: int, correction: torch.Tensor | None = None, over_chosen: bool = False):
+def moe_router(z: torch.Tensor, experts: int, top: int, correction: torch.Tensor | None = None, over_chosen: bool = False,
+               sigmoid: bool = False):
     """z: float32 view [T, >= experts] (the router's outputs). s = softmax over the first ``experts`` columns; the ``top``
     largest of s + correction are chosen (descending; of equals the lower index). Returns (chosen int32 [T, top], weight
     float32 [T, top] = the chosen experts' s divided by their sum + 1e-20). ``over_chosen``: the ``top`` largest z themselves are
-    chosen and the weights are the softmax over the chosen z only (no correction)."""
+    chosen and the weights are the softmax over the chosen z only (no correction). ``sigmoid``: s = sigmoid(z), and the chosen
+    experts' s are the weights as they are."""
     _gpu(z, correction)
     T = z.shape[0]
     _need(z.dtype == torch.float32 and z.dim() == 2 and z.stride(1) == 1 and z.shape[1] >= experts, f"moe_router: z is float32 [T, >= {experts}]")
     _need(0 < top <= experts <= MOE_MAX_EXPERTS, f"moe_router: {top} of {experts} experts (up to {MOE_MAX_EXPERTS})")
-    _need(not (over_chosen and correction is not None), "moe_router: a correction shifts a choice among softmax scores only")
+    _need(not (over_chosen and (correction is not None or sigmoid)), "moe_router: a correction shifts a choice among scores, not among the logits themselves")
     if correction is not None:
         _need(correction.dtype == torch.float32 and tuple(correction.shape) == (experts,) and correction.is_contiguous(),
               f"moe_router: correction is float32 [{experts}]")
@@ -1804,7 +1901,7 @@ def moe_router(z: torch.Tensor, experts: int, top: int, correction: torch.Tensor
     weight = torch.empty((T, top), dtype=torch.float32, device=z.device)
     ldz = z.stride(0) if T > 1 else max(z.stride(0), experts)
     _check(library().tm_moe_router(_p(z), c_int(ldz), _p(correction), c_int(T), c_int(experts), c_int(top), _p(chosen), _p(weight),
-                                   c_int(1 if over_chosen else 0), _stream()), "moe_router")
+                                   c_int(1 if over_chosen else 0), c_int(1 if sigmoid else 0), _stream()), "moe_router")
     return chosen, weight
 
 
@@ -1827,11 +1924,13 @@ def moe_route_chosen(chosen: torch.Tensor, experts: int, real: int, tile_rows: i
 
 def moe_experts_weighted(x: torch.Tensor, routed, weight: torch.Tensor, w_up: torch.Tensor | None, w_down: torch.Tensor | None, top: int,
                          out: torch.Tensor, shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None,
-                         gated: bool = False) -> torch.Tensor:
+                         gated: bool = False, clamped: tuple[float, float] | None = None, weigh_input: bool = False) -> torch.Tensor:
     """out[t] = sum over the token's ``top`` pairs of weight[t, k] * (Wd[e] relu(Wu[e] x[t])^2, or x[t] itself for a pair
     without a slot) + sigmoid(shared_gate[t]) * shared[t]. w_up [E, F, K], w_down [E, N, F] (both None: every expert stands
     for the input); ``routed`` from ``moe_route_chosen``; shared float32 [T, N] or None; shared_gate a float32 view [T, >= 1].
-    ``gated``: an expert is Wd[e] (silu(Wg[e] x) * (Wu[e] x)) and w_up is [E, 2F, K], an expert's gate rows, then its up rows."""
+    ``gated``: an expert is Wd[e] (silu(Wg[e] x) * (Wu[e] x)) and w_up is [E, 2F, K], an expert's gate rows, then its up rows.
+    ``clamped`` (limit, alpha), with ``gated``: Wd[e] (g sigmoid(alpha g) (u + 1)), g = min(Wg[e] x, limit), u = Wu[e] x held to
+    +-limit. ``weigh_input``, with ``clamped``: a pair's weight multiplies the expert's input and not its output."""
     slot_pair, pair_slot, tiles, n_tiles, tile_rows = routed
     _gpu(x, w_up, w_down, out, weight, shared, shared_gate)
     T, K = x.shape
@@ -1841,6 +1940,9 @@ def moe_experts_weighted(x: torch.Tensor, routed, weight: torch.Tensor, w_up: to
           "moe_experts_weighted: x [T, K], out contiguous [T, K], one type")
     _need(weight.dtype == torch.float32 and tuple(weight.shape) == (T, top) and weight.is_contiguous(), "moe_experts_weighted: weight is float32 [T, top]")
     _need(slot_pair.numel() == P and pair_slot.numel() == P, "moe_experts_weighted: the routing belongs to another step")
+    _need(clamped is None or (gated and clamped[0] > 0), "moe_experts_weighted: a clamped gate has a positive limit")
+    _need(not weigh_input or (clamped is not None and w_up is not None), "moe_experts_weighted: weights on the input are for experts with a clamped gate")
+    on_input, on_output = (weight, None) if weigh_input else (None, weight)
     if shared is not None:
         _need(shared.dtype == torch.float32 and tuple(shared.shape) == (T, N) and shared.is_contiguous(), "moe_experts_weighted: shared is float32 [T, N]")
     ldg = 0
@@ -1861,19 +1963,29 @@ def moe_experts_weighted(x: torch.Tensor, routed, weight: torch.Tensor, w_up: to
               and x.dtype == w_up.dtype == w_down.dtype, "moe_experts_weighted: w_up [E, F, K], w_down [E, N, F], one type")
         act = torch.empty((P, F), dtype=x.dtype, device=x.device)
         if x.dtype == torch.bfloat16 and lib.tm_moe_mfma_takes(_p(x), c_int(ldx), _p(w_up), _p(w_down), _p(act), c_int(K), c_int(F)):
-            first = lib.tm_moe_gate_up_mfma if gated else lib.tm_moe_up_act_mfma
-            _check(first(_p(x), c_int(ldx), _p(slot_pair), c_int(top), _p(w_up), _p(act), _p(tiles), _p(n_tiles),
-                         c_int(most), c_int(tile_rows), c_int(K), c_int(F), _stream()), "moe_up_act_mfma")
+            if clamped is not None:
+                _check(lib.tm_moe_clamped_mfma(_p(x), c_int(ldx), _p(slot_pair), c_int(top), _p(on_input), _p(w_up), _p(act), _p(tiles),
+                                               _p(n_tiles), c_int(most), c_int(tile_rows), c_int(K), c_int(F), c_float(clamped[0]),
+                                               c_float(clamped[1]), _stream()), "moe_clamped_mfma")
+            else:
+                first = lib.tm_moe_gate_up_mfma if gated else lib.tm_moe_up_act_mfma
+                _check(first(_p(x), c_int(ldx), _p(slot_pair), c_int(top), _p(w_up), _p(act), _p(tiles), _p(n_tiles),
+                             c_int(most), c_int(tile_rows), c_int(K), c_int(F), _stream()), "moe_up_act_mfma")
             _check(lib.tm_moe_down_mfma(_p(act), _p(w_down), _p(part), _p(tiles), _p(n_tiles), c_int(most), c_int(tile_rows), c_int(F),
                                         c_int(N), _stream()), "moe_down_mfma")
         else:
             _need(tile_rows == MOE_TILE_ROWS, "moe_experts_weighted: these products take tiles of 32 rows")
-            first = lib.tm_moe_gate_up if gated else lib.tm_moe_up_act
-            _check(first(_p(x), c_int(ldx), _p(slot_pair), c_int(top), _p(w_up), _p(act), _p(tiles), _p(n_tiles), c_int(most),
-                         c_int(K), c_int(F), dt, _stream()), "moe_up_act")
+            if clamped is not None:
+                _check(lib.tm_moe_clamped(_p(x), c_int(ldx), _p(slot_pair), c_int(top), _p(on_input), _p(w_up), _p(act), _p(tiles),
+                                          _p(n_tiles), c_int(most), c_int(K), c_int(F), c_float(clamped[0]), c_float(clamped[1]), dt,
+                                          _stream()), "moe_clamped")
+            else:
+                first = lib.tm_moe_gate_up if gated else lib.tm_moe_up_act
+                _check(first(_p(x), c_int(ldx), _p(slot_pair), c_int(top), _p(w_up), _p(act), _p(tiles), _p(n_tiles), c_int(most),
+                             c_int(K), c_int(F), dt, _stream()), "moe_up_act")
             _check(lib.tm_moe_down(_p(act), _p(w_down), _p(part), _p(tiles), _p(n_tiles), c_int(most), c_int(F), c_int(N), dt, _stream()),
                    "moe_down")
-    _check(lib.tm_moe_combine_weighted(_p(part), _p(pair_slot), _p(weight), _p(x), c_int(ldx), _p(shared), _p(shared_gate), c_int(ldg),
+    _check(lib.tm_moe_combine_weighted(_p(part), _p(pair_slot), _p(on_output), _p(x), c_int(ldx), _p(shared), _p(shared_gate), c_int(ldg),
                                        _p(out), c_int(T), c_int(top), c_int(N), dt, _stream()), "moe_combine_weighted")
     return out
 
@@ -2040,29 +2152,33 @@ def embed_pairs(table: torch.Tensor, pairs: torch.Tensor, ids: torch.Tensor, pos
 
 
 def sum_norm(resid: torch.Tensor, parts: list, w: torch.Tensor | None, out: torch.Tensor | None, eps: float,
-             rows: torch.Tensor | None = None) -> torch.Tensor | None:
-    """v = resid + sum of scale * y over ``parts`` [(y, scale), ...] (one to three, [T, hidden] of one type); with ``rows`` None
-    every row runs and v is written back to resid (float32 [T, hidden]); out = v / sqrt(mean(v^2) + eps) * w (out None: the add
-    alone). With ``rows`` (int32 [R]) only those rows are read, resid stays as it is and out is [R, hidden]."""
+             rows: torch.Tensor | None = None, w2: torch.Tensor | None = None, out2: torch.Tensor | None = None) -> torch.Tensor | None:
+    """v = resid + sum of scale * y over ``parts`` [(y, scale), ...] (up to three, [T, hidden] of one type; none only with an
+    ``out``); with ``rows`` None every row runs and v is written back to resid (float32 [T, hidden]); out = v / sqrt(mean(v^2) +
+    eps) * w (out None: the add alone), and with ``out2`` likewise out2 with the weights w2. With ``rows`` (int32 [R]) only those
+    rows are read, resid stays as it is and out is [R, hidden]."""
     T, hidden = resid.shape
-    _need(1 <= len(parts) <= 3, "sum_norm: one to three results")
+    _need(len(parts) <= 3 and (parts or out is not None), "sum_norm: up to three results, or a norm alone")
     ys = [y for y, _ in parts]
-    _gpu(resid, w, out, rows, *ys)
+    dtype = ys[0].dtype if ys else out.dtype
+    _gpu(resid, w, out, rows, w2, out2, *ys)
     _need(resid.dtype == torch.float32 and resid.is_contiguous(), "sum_norm: resid is contiguous float32")
     for y in ys:
-        _need(y.is_contiguous() and tuple(y.shape) == (T, hidden) and y.dtype == ys[0].dtype, f"sum_norm: the results are contiguous [{T}, {hidden}] of one type")
+        _need(y.is_contiguous() and tuple(y.shape) == (T, hidden) and y.dtype == dtype, f"sum_norm: the results are contiguous [{T}, {hidden}] of one type")
     n = T if rows is None else rows.numel()
     if rows is not None:
         _ints(rows, n, "rows")
         _need(out is not None, "sum_norm: rows are only read for a norm")
-    if out is not None:
-        _need(out.is_contiguous() and tuple(out.shape) == (n, hidden) and out.dtype == ys[0].dtype, f"sum_norm: out is [{n}, {hidden}] of the results' type")
-        _need(w is not None and w.is_contiguous() and tuple(w.shape) == (hidden,), f"sum_norm: w is [{hidden}]")
+    _need((w2 is None) == (out2 is None) and (out2 is None or out is not None), "sum_norm: a second norm has weights and stands beside a first")
+    for o, weight in ((out, w), (out2, w2)):
+        if o is not None:
+            _need(o.is_contiguous() and tuple(o.shape) == (n, hidden) and o.dtype == dtype, f"sum_norm: out is [{n}, {hidden}] of the results' type")
+            _need(weight is not None and weight.is_contiguous() and tuple(weight.shape) == (hidden,) and weight.dtype == w.dtype, f"sum_norm: w is [{hidden}]")
     scales = [float(s) for _, s in parts] + [0.0] * (3 - len(parts))
     ys = ys + [None] * (3 - len(ys))
-    _check(library().tm_sum_norm(_p(resid), _p(ys[0]), c_float(scales[0]), _p(ys[1]), c_float(scales[1]), _p(ys[2]), c_float(scales[2]),
-                                 _p(rows), _p(w if out is not None else None), c_int(code(w.dtype) if w is not None else 0), _p(out),
-                                 c_int(code(parts[0][0].dtype)), c_int(n), c_int(hidden), c_float(eps), _stream()), "sum_norm")
+    _check(library().tm_sum_norm2(_p(resid), _p(ys[0]), c_float(scales[0]), _p(ys[1]), c_float(scales[1]), _p(ys[2]), c_float(scales[2]),
+                                  _p(rows), _p(w if out is not None else None), _p(w2), c_int(code(w.dtype) if w is not None else 0), _p(out),
+                                  _p(out2), c_int(code(dtype)), c_int(n), c_int(hidden), c_float(eps), _stream()), "sum_norm")
     return out
 
 
@@ -2072,9 +2188,10 @@ def retention_row_width(H: int, D: int, Dv: int) -> int:
 
 
 def retention_prepare(proj: torch.Tensor, cos: torch.Tensor | None, sin: torch.Tensor | None, positions: torch.Tensor, rows: torch.Tensor,
-                      H: int, D: int, Dv: int, k_scale: float) -> torch.Tensor:
+                      H: int, D: int, Dv: int, k_scale: float, silu: bool = False) -> torch.Tensor:
     """rows float32 [T, retention_row_width] = [q | k * k_scale | v] from proj [T, >= H (2 D + Dv)] (q, k, v in this order), the first
-    2 * cos.shape[1] channels of every head of q and k turned by the token's position (pairs half that width apart)."""
+    2 * cos.shape[1] channels of every head of q and k turned by the token's position (pairs half that width apart). ``silu``:
+    of silu(proj) instead."""
     _gpu(proj, cos, sin, positions, rows)
     T = proj.shape[0]
     width = H * (2 * D + Dv)
@@ -2089,8 +2206,8 @@ def retention_prepare(proj: torch.Tensor, cos: torch.Tensor | None, sin: torch.T
     _ints(positions, T, "positions")
     ld = proj.stride(0) if T > 1 else max(proj.stride(0), proj.shape[1])
     _check(library().tm_retention_prepare(_p(proj), c_int(ld), c_int(code(proj.dtype)), _p(cos), _p(sin), c_int(rot), _p(positions), _p(rows),
-                                          c_int(rows.shape[1]), c_int(T), c_int(H), c_int(D), c_int(Dv), c_float(k_scale), _stream()),
-           "retention_prepare")
+                                          c_int(rows.shape[1]), c_int(T), c_int(H), c_int(D), c_int(Dv), c_float(k_scale),
+                                          c_int(1 if silu else 0), _stream()), "retention_prepare")
     return rows
 
 
@@ -2197,15 +2314,20 @@ def retention_step_takes(D: int, Dv: int) -> bool:
 
 
 def retention_step(proj: torch.Tensor, cos: torch.Tensor | None, sin: torch.Tensor | None, positions: torch.Tensor, decay: torch.Tensor,
-                   state: torch.Tensor, state_slots: torch.Tensor, y: torch.Tensor, H: int, D: int, Dv: int, k_scale: float,
-                   eps: float) -> torch.Tensor:
+                   state: torch.Tensor, state_slots: torch.Tensor, y: torch.Tensor | None, H: int, D: int, Dv: int, k_scale: float,
+                   eps: float, silu: bool = False, o: torch.Tensor | None = None) -> torch.Tensor:
     """Single tokens, one a request: ``retention_prepare``, the recurrence over one row and ``gla_out_gate`` (silu, no weight) in one
-    launch. proj [n, >= 2 H (D + Dv)] = q | k | v | g; positions and state_slots int32 [n]; y [n, H * Dv] of proj's type."""
-    _gpu(proj, cos, sin, positions, decay, state, state_slots, y)
+    launch. proj [n, >= 2 H (D + Dv)] = q | k | v | g; positions and state_slots int32 [n]; y [n, H * Dv] of proj's type. ``silu``: q, k
+    and v are silu of the projection. ``o`` (float32 [n, H * Dv]) in place of y: the recurrence's result as it is (g is not read)."""
+    _gpu(proj, cos, sin, positions, decay, state, state_slots, y, o)
     n = proj.shape[0]
-    ld = _rows_of(proj, n, 2 * H * (D + Dv), "retention_step: proj")
+    _need((y is None) != (o is None), "retention_step: one of y and o")
+    ld = _rows_of(proj, n, H * (2 * D + Dv) if y is None else 2 * H * (D + Dv), "retention_step: proj")
     _need(retention_step_takes(D, Dv), "retention_step: sizes the kernel does not take")
-    _need(tuple(y.shape) == (n, H * Dv) and y.is_contiguous() and y.dtype == proj.dtype, f"retention_step: y is [{n}, {H * Dv}] of proj's type")
+    if o is not None:
+        _need(tuple(o.shape) == (n, H * Dv) and o.is_contiguous() and o.dtype == torch.float32, f"retention_step: o is float32 [{n}, {H * Dv}]")
+    else:
+        _need(tuple(y.shape) == (n, H * Dv) and y.is_contiguous() and y.dtype == proj.dtype, f"retention_step: y is [{n}, {H * Dv}] of proj's type")
     _need(decay.dtype == torch.float32 and decay.is_contiguous() and decay.numel() == H * D, f"retention_step: decay is float32 [{H * D}]")
     rot = 0
     if cos is not None:
@@ -2217,8 +2339,8 @@ def retention_step(proj: torch.Tensor, cos: torch.Tensor | None, sin: torch.Tens
     _ints(state_slots, n, "state_slots")
     _check(library().tm_retention_step(_p(proj), c_int(ld), c_int(code(proj.dtype)), _p(cos), _p(sin), c_int(rot), _p(positions), _p(decay),
                                        _p(state), _p(state_slots), _p(y), c_int(n), c_int(H), c_int(D), c_int(Dv), c_float(k_scale),
-                                       c_float(eps), _stream()), "retention_step")
-    return y
+                                       c_float(eps), c_int(1 if silu else 0), _p(o), _stream()), "retention_step")
+    return y if o is None else o
 
 
 def delta_step_takes(H: int, G: int, D: int, Dv: int) -> bool:

@@ -7,7 +7,7 @@ from tokenmill_amd.parts.base import (FeedForward, GroupStep, KVCacheSpec, KVCac
 from tokenmill_amd.parts.block import GatedResidualBlock, PreNormBlock, SandwichBlock, SharedNormBlock
 from tokenmill_amd.parts.conv import ShortConvolution
 from tokenmill_amd.parts.delta_rule import GatedDeltaRule
-from tokenmill_amd.parts.embedding import LearnedPositions, OutputHead, PairRows, TokenEmbedding
+from tokenmill_amd.parts.embedding import LearnedPositions, OutputHead, PairRows, PositionWaves, TokenEmbedding
 from tokenmill_amd.parts.gla import GatedLinearAttention
 from tokenmill_amd.parts.linear import Linear
 from tokenmill_amd.parts.mlp import DenseFeedForward, GatedFeedForward, SwiGLU
@@ -22,4 +22,4 @@ __all__ = ["GQAttention", "FeedForward", "GroupStep", "KVCacheSpec", "KVCacheVie
            "TokenEmbedding", "Linear", "SwiGLU", "RMSNorm", "SigmoidAttention", "SandwichBlock", "LearnedPositions", "GatedLinearAttention",
            "DenseFeedForward", "GroupRMSNorm", "LatentAttention", "LayerCacheSpec", "GatedResidualBlock", "ShortConvolution",
            "TableRoutedExperts", "GatedAdd", "SoftmaxAttention", "RoutedExperts", "PassThrough", "LayerNorm", "NoPositionEncoding", "RotaryEmbedding",
-           "GatedDeltaRule", "ParallelMixer", "GatedFeedForward", "SharedNormBlock", "PairRows", "WeightedAdd", "Retention"]
+           "GatedDeltaRule", "ParallelMixer", "GatedFeedForward", "SharedNormBlock", "PairRows", "PositionWaves", "WeightedAdd", "Retention"]

@@ -25,13 +25,15 @@ class KVCacheSpec:
     """Keys and values in pages. ``window``: None keeps every token; W keeps the last W. ``chunk``: C means that a
     token never reads a key from before the start of its own chunk of C positions (counted from position 0), so the
     pages of finished chunks can be given back. ``v_head_dim``: size of a value where it differs from a key's.
-    ``values``: False for a mixer whose values are part of its key rows (a shared latent): the group has no value pool."""
+    ``values``: False for a mixer whose values are part of its key rows (a shared latent): the group has no value pool.
+    ``keep``: with a window, the first ``keep`` tokens of a request stay beside it."""
     kv_heads: int
     head_dim: int
     window: int | None = None
     v_head_dim: int | None = None
     chunk: int | None = None
     values: bool = True
+    keep: int = 0
 
     @property
     def value_dim(self) -> int:
@@ -39,7 +41,7 @@ class KVCacheSpec:
 
     def first_needed(self, num_computed: int) -> int:
         """With ``num_computed`` tokens cached, the next query sits at position num_computed or later: the first
-        position whose key it, or any later token, may still read."""
+        position, behind the kept ones, whose key it, or any later token, may still read."""
         first = 0
         if self.window is not None:
             first = max(first, num_computed - self.window + 1)
@@ -217,6 +219,13 @@ class NormedInput:
                 self._tensor = self.norm.add_norm(self.resid, self.delta, self.dtype)
             self.delta = self.delta_norm = None
         return self._tensor
+
+    def pair(self, second: Norm) -> tuple[torch.Tensor, torch.Tensor]:
+        """This input and another norm's of the same stream (sublayers side by side)."""
+        from tokenmill_amd.parts.norm import norm_pair
+        self._tensor, other = norm_pair(self.norm, second, self.resid, self.delta, self.dtype, self.delta_norm)
+        self.delta = self.delta_norm = None
+        return self._tensor, other
 
     def fusable_rms(self) -> tuple[torch.Tensor, float] | None:
         """(weight, eps) when nothing is pending on the residual and the norm is an RMS norm."""

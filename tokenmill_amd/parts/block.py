@@ -242,18 +242,23 @@ class GatedResidualBlock(Block):
 
 
 class SharedNormBlock(Block):
-    """One norm, and both sublayers read its result:
+    """Sublayers side by side. One norm, and both read its result:
 
         h = norm(x);   x += mixer(h) + ffn(h)            (``ffn`` None: the mixer alone)
+
+    or, with ``norm_fed``, two norms of the same x: x += mixer(norm(x)) + ffn(norm_fed(x)).
 
     A mixer of several results (``forward_parts``) brings them with their weights. Everything that goes into the stream stays
     pending together (``WeightedAdd``), so the norm of the next block adds it all and norms the sum in one kernel."""
 
-    def __init__(self, norm: Norm, mixer: Mixer, ffn: FeedForward | None = None, names: tuple[str, str, str] = ("norm1", "mix.", "mlp.")):
-        self.norm, self.mixer, self.ffn, self.names = norm, mixer, ffn, names
+    def __init__(self, norm: Norm, mixer: Mixer, ffn: FeedForward | None = None,
+                 names: tuple[str, ...] = ("norm1", "mix.", "mlp.", "norm2"), norm_fed: Norm | None = None):
+        if norm_fed is not None and ffn is None:
+            raise ValueError("a norm for a feed-forward that is not there")
+        self.norm, self.mixer, self.ffn, self.norm_fed, self.names = norm, mixer, ffn, norm_fed, names
 
     def _parts(self):
-        return [(p, n) for p, n in zip((self.norm, self.mixer, self.ffn), self.names) if p is not None]
+        return [(p, n) for p, n in zip((self.norm, self.mixer, self.ffn, self.norm_fed), self.names) if p is not None]
 
     def tensor_specs(self, prefix: str):
         specs = {}
@@ -272,11 +277,11 @@ class SharedNormBlock(Block):
     def _results(self, x: NormedInput, step: StepContext, cache):
         """(first result, how it and the others go into the stream)."""
         from tokenmill_amd.parts.norm import WeightedAdd
-        h = x.tensor()
+        h, fed = (x.tensor(),) * 2 if self.norm_fed is None else x.pair(self.norm_fed)
         split = getattr(self.mixer, "forward_parts", None)
         parts = split(h, step, cache) if split is not None else [(self.mixer.forward(h, step, cache), 1.0)]
         if self.ffn is not None:
-            parts = [*parts, (self.ffn.forward(h, step), 1.0)]
+            parts = [*parts, (self.ffn.forward(fed, step), 1.0)]
         (first, scale), *others = parts
         return first, WeightedAdd(scale, others)
 

@@ -15,14 +15,17 @@ from tokenmill_amd.weights.loader import TensorSpec
 
 class Linear(Part):
     def __init__(self, in_features: int, out_features: list[int] | int, names: list[str] | str,
-                 bias: bool = False, library_first: bool = False, suffixes: tuple[str, str] = (".weight", ".bias"),
+                 bias: bool | list[bool] = False, library_first: bool = False, suffixes: tuple[str, str] = (".weight", ".bias"),
                  wide_bias: bool = False, activation: str | None = None):
         self.in_features = in_features
         self.out_splits = [out_features] if isinstance(out_features, int) else list(out_features)
         self.names = [names] if isinstance(names, str) else list(names)
         assert len(self.names) == len(self.out_splits)
         self.out_features = sum(self.out_splits)
-        self.has_bias = bias
+        # a list: which of the stacked matrices have a bias in the checkpoint (the others add zeros)
+        self.biases = [bool(b) for b in bias] if isinstance(bias, (list, tuple)) else [bool(bias)] * len(self.names)
+        assert len(self.biases) == len(self.names)
+        self.has_bias = any(self.biases)
         self.bias_init_zero = False
         self.library_first = library_first              # a wide matrix the library reads fastest at any row count
         self.wide_bias = wide_bias                      # the bias is kept in 32-bit (a product whose 32-bit result is wanted)
@@ -38,9 +41,9 @@ class Linear(Part):
     def tensor_specs(self, prefix: str) -> dict[str, TensorSpec]:
         specs = {}
         sw, sb = self.suffixes
-        for name, n in zip(self.names, self.out_splits):
+        for name, n, has in zip(self.names, self.out_splits, self.biases):
             specs[f"{prefix}{name}{sw}"] = TensorSpec((n, self.in_features))
-            if self.has_bias:
+            if has:
                 specs[f"{prefix}{name}{sb}"] = TensorSpec((n,), init="zeros" if self.bias_init_zero else "normal")
         return specs
 
@@ -49,7 +52,7 @@ class Linear(Part):
         ws = [tensors[f"{prefix}{name}{sw}"] for name in self.names]
         self.weight = ws[0] if len(ws) == 1 else torch.cat(ws, dim=0).contiguous()
         if self.has_bias:
-            bs = [tensors[f"{prefix}{name}{sb}"] for name in self.names]
+            bs = [tensors[f"{prefix}{name}{sb}"] if has else w.new_zeros(w.shape[0]) for name, w, has in zip(self.names, ws, self.biases)]
             self.bias = bs[0] if len(bs) == 1 else torch.cat(bs, dim=0).contiguous()
             if (self.weight.dtype == torch.float32 or self.wide_bias) and self.bias.dtype != torch.float32:
                 self.bias = self.bias.float()          # a 32-bit product, or one with a 32-bit result, adds a 32-bit bias

@@ -155,7 +155,7 @@ class GatedFeedForward(FeedForward):
     def cost(self, label: str, step: StepContext | None, rows: int) -> tuple[int, int]:
         return self.gate_up.cost(rows) if label == "gate_up" else self.down.cost(rows)
 
-    def forward(self, x, step: StepContext | None = None, residual: torch.Tensor | None = None):
+    def forward(self, x, step: StepContext | None = None, residual: torch.Tensor | None = None, out_dtype: torch.dtype | None = None):
         from tokenmill_amd import profiling
         x = as_tensor(x)
         with profiling.label("gate_up", lambda: self.gate_up.cost(x.shape[0])):
@@ -166,4 +166,4 @@ class GatedFeedForward(FeedForward):
             else:
                 (ops.gelu_mul if self.activation == "gelu_tanh" else ops.silu_mul)(gu, a)
         with profiling.label("down", lambda: self.down.cost(x.shape[0])):
-            return self.down.forward(a)
+            return self.down.forward(a, out_dtype=out_dtype)

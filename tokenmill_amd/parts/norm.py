@@ -130,6 +130,26 @@ class GroupRMSNorm(Norm):
             ops.group_norm(resid, y, self.weight, None, None, self.groups, self.eps)
 
 
+def norm_pair(first: Norm, second: Norm, resid, delta, out_dtype, delta_norm=None):
+    """(first(v), second(v)) with v the stream and what is pending on it, which is added (resid is updated): two norms of one sum, in
+    one kernel where both are plain RMS norms that agree on eps."""
+    if isinstance(first, GroupRMSNorm) and isinstance(second, GroupRMSNorm) and first.groups == second.groups == 1 \
+            and first.eps == second.eps and first.weight.dtype == second.weight.dtype and not first.one_plus and not second.one_plus \
+            and (delta is None or delta_norm is None or (isinstance(delta_norm, WeightedAdd) and len(delta_norm.others) <= 2)):
+        n = resid.shape[0]
+        out, out2 = (torch.empty((n, first.hidden), dtype=out_dtype, device=resid.device) for _ in range(2))
+        parts = [] if delta is None else delta_norm.parts(delta) if delta_norm is not None else [(delta, 1.0)]
+        moved = sum(n * first.hidden * y.element_size() for y, _ in parts)
+        with profiling.label("norm", lambda: (n * first.hidden * ((8 if parts else 4) + 2 * out.element_size()) + moved, 0)):
+            ops.sum_norm(resid, parts, first.weight, out, first.eps, w2=second.weight, out2=out2)
+        return out, out2
+    if delta_norm is not None:
+        a = first.add_norm(resid, delta, out_dtype, delta_norm=delta_norm)
+    else:
+        a = first.add_norm(resid, delta, out_dtype)
+    return a, second.add_norm(resid, None, out_dtype)
+
+
 class PassThrough(Norm):
     """No norm in front of a sublayer: its input is the residual stream itself, rounded to the model's type. What is still
     pending on the stream (a sublayer's result and the norm it has to pass) is added by the same kernel."""

@@ -9,8 +9,8 @@ or the results are added with two constant weights (``scales``),
 
 which a block that takes several results at once (``forward_parts``) adds into the residual stream in 32-bit.
 
-The two may be any mixers of which at most one keeps pages and at most one keeps state slots (an attention beside a
-recurrence): the layer's cache is then the pages of the one with the state of the other beside them.
+The two may be any mixers of which at most one keeps pages (an attention beside a recurrence); each may keep state slots. The
+layer's cache is then those pages with the states of the left and then of the right mixer beside them.
 """
 from __future__ import annotations
 
@@ -44,11 +44,17 @@ class ParallelMixer(Mixer):
         self.scales = (float(scales[0]), float(scales[1])) if scales is not None else None
         self.prefixes, self.norm_names = prefixes, norm_names if scales is None else ()
         (lk, ls), (rk, rs) = _split(left.cache_spec()), _split(right.cache_spec())
-        if (lk is not None and rk is not None) or (ls is not None and rs is not None):
-            raise ValueError("of two mixers side by side, one may keep pages and one may keep state")
+        if lk is not None and rk is not None:
+            raise ValueError("of two mixers side by side, one may keep pages")
         self.pages_of = 0 if lk is not None else 1 if rk is not None else None
         self.state_of = 0 if ls is not None else 1 if rs is not None else None
-        self._spec = LayerCacheSpec(lk or rk, ls if ls is not None else rs) if (self.pages_of is not None or self.state_of is not None) else None
+        # with state on both sides the layer holds a tuple: the left mixer's, then the right one's
+        self.states_of = tuple(len(s) if isinstance(s, tuple) else 1 for s in (ls, rs)) if ls is not None and rs is not None else None
+        self._single = (not isinstance(ls, tuple), not isinstance(rs, tuple))
+        states = ls if ls is not None else rs
+        if self.states_of is not None:
+            states = tuple(s for side in (ls, rs) for s in (side if isinstance(side, tuple) else (side,)))
+        self._spec = LayerCacheSpec(lk or rk, states) if (self.pages_of is not None or self.state_of is not None) else None
         self.w_left: torch.Tensor | None = None
         self.w_right: torch.Tensor | None = None
 
@@ -80,6 +86,13 @@ class ParallelMixer(Mixer):
         """What mixer ``which`` is handed of the layer's cache: the pages, the state, or nothing."""
         if cache is None:
             return None
+        if self.states_of is not None:
+            n = self.states_of[0]
+            mine = cache.state[:n] if which == 0 else cache.state[n:]
+            mine = mine[0] if self._single[which] else mine
+            if isinstance(cache, KVCacheView) and which == self.pages_of:
+                return KVCacheView(cache.k, cache.v, cache.group, cache.write, mine)
+            return StateView(mine)
         if isinstance(cache, KVCacheView):
             if which == self.pages_of:
                 return cache

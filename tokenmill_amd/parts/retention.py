@@ -6,6 +6,10 @@
     o_t = S_t^T q_t
     y_t = W_o (concat over heads of unit_rms(o_t) * silu(g_t))
 
+What another model may ask for, each a constructor parameter: q, k and v that are silu of their projection (``silu``); another
+scale of k (``k_scale``); one norm over the heads side by side with a weight per channel in place of a norm per head
+(``whole_norm``); a sigmoid gate (``sigmoid_gate``).
+
 with the rotation of ``rotary`` (by the token's position, over the first channels of a head) or none. The state is the mixer's
 cache: a ``StateSpec`` slot per request, advanced in token order inside a step's portion and carried from step to step. What
 lies between the projections and the norm of the result is 32-bit. It is gated linear attention with decays that do not
@@ -22,12 +26,15 @@ from tokenmill_amd.parts.base import Mixer, StateSpec, StateView, StepContext, a
 from tokenmill_amd.parts.gla import MAX_KEY_DIM
 from tokenmill_amd.parts.linear import Linear
 from tokenmill_amd.parts.position import RotaryEmbedding
+from tokenmill_amd.weights.loader import TensorSpec
 
 
 class Retention(Mixer):
     def __init__(self, hidden: int, num_heads: int, key_dim: int, value_dim: int, decay: list[float], norm_eps: float,
                  rotary: RotaryEmbedding | None = None, names: tuple[str, ...] = ("q", "k", "v", "g", "o"),
-                 suffixes: tuple[str, str] = ("", ".b")):
+                 suffixes: tuple[str, str] = ("", ".b"), silu: bool = False, k_scale: float | None = None, whole_norm: bool = False,
+                 sigmoid_gate: bool = False, norm_name: str = "norm"):
+        """``k_scale``: None for 1 / sqrt(key size)."""
         if not 0 < key_dim <= MAX_KEY_DIM or value_dim <= 0:
             raise ValueError(f"key size {key_dim}: the recurrence kernel takes up to {MAX_KEY_DIM}")
         if len(decay) != num_heads:
@@ -36,19 +43,27 @@ class Retention(Mixer):
             raise ValueError("a retention rotates pairs half the rotated width apart, inside a head")
         self.hidden, self.num_heads, self.key_dim, self.value_dim = hidden, num_heads, key_dim, value_dim
         self.norm_eps, self.rotary, self.decay_values = float(norm_eps), rotary, [float(d) for d in decay]
+        self.silu, self.k_scale, self.whole_norm, self.sigmoid_gate = silu, float(k_scale) if k_scale is not None else key_dim ** -0.5, whole_norm, sigmoid_gate
+        self.norm_name = norm_name
+        self.norm_w: torch.Tensor | None = None         # float32 [H * Dv] with a norm over all heads
         self.k_size, self.v_size = num_heads * key_dim, num_heads * value_dim
         self.proj = Linear(hidden, [self.k_size, self.k_size, self.v_size, self.v_size], list(names[:4]), bias=False, suffixes=suffixes)
         self.o = Linear(self.v_size, hidden, names[4], bias=False, suffixes=suffixes)
         self.decay: torch.Tensor | None = None          # float32 [1, H * D]: every token's
 
     def tensor_specs(self, prefix: str):
-        return {**self.proj.tensor_specs(prefix), **self.o.tensor_specs(prefix)}
+        specs = {**self.proj.tensor_specs(prefix), **self.o.tensor_specs(prefix)}
+        if self.whole_norm:
+            specs[prefix + self.norm_name] = TensorSpec((self.v_size,), init="ones")
+        return specs
 
     def load(self, tensors, prefix: str) -> None:
         self.proj.load(tensors, prefix)
         self.o.load(tensors, prefix)
         if self.rotary is not None:
             self.rotary.load(tensors, prefix)
+        if self.whole_norm:
+            self.norm_w = tensors[prefix + self.norm_name].float().contiguous()
         per_head = torch.tensor(self.decay_values, dtype=torch.float32)
         self.decay = per_head.repeat_interleave(self.key_dim)[None].contiguous().to(self.o.weight.device)
 
@@ -87,18 +102,24 @@ class Retention(Mixer):
         y = torch.empty((T, self.v_size), dtype=x.dtype, device=x.device)
         cos, sin = (rot.cos, rot.sin) if rot is not None else (None, None)
         # the step's single tokens (its last rows and requests) go through one kernel from here to y, where it takes the sizes
-        singles = step.num_decode if ops.retention_step_takes(D, Dv) else 0
+        singles = step.num_decode if ops.retention_step_takes(D, Dv) and (self.whole_norm or not self.sigmoid_gate) else 0
         P, Tp = step.num_seqs - singles, T - singles
         with profiling.label("recurrence", lambda: self.cost("attention", step, T)):
+            o = torch.empty((T if self.whole_norm else Tp, self.v_size), dtype=torch.float32, device=x.device)
             if Tp:
-                o = torch.empty((Tp, self.v_size), dtype=torch.float32, device=x.device)
                 rows = torch.empty((Tp, ops.retention_row_width(H, D, Dv)), dtype=torch.float32, device=x.device)
-                ops.retention_prepare(proj[:Tp], cos, sin, step.positions, rows, H, D, Dv, D ** -0.5)
-                self._scan(rows, o, cache.state, step, P)
-                ops.gla_out_gate(o, proj[:Tp, 2 * self.k_size + self.v_size:], None, y[:Tp], H, Dv, self.norm_eps)
-            if singles:
+                ops.retention_prepare(proj[:Tp], cos, sin, step.positions, rows, H, D, Dv, self.k_scale, silu=self.silu)
+                self._scan(rows, o[:Tp], cache.state, step, P)
+                if not self.whole_norm:
+                    ops.gla_out_gate(o, proj[:Tp, 2 * self.k_size + self.v_size:], None, y[:Tp], H, Dv, self.norm_eps, sigmoid=self.sigmoid_gate)
+            if singles and self.whole_norm:
+                ops.retention_step(proj[Tp:], cos, sin, step.positions[Tp:], self.decay, cache.state, step.state_slots[P:], None, H, D, Dv,
+                                   self.k_scale, self.norm_eps, silu=self.silu, o=o[Tp:])
+            elif singles:
                 ops.retention_step(proj[Tp:], cos, sin, step.positions[Tp:], self.decay, cache.state, step.state_slots[P:], y[Tp:], H, D, Dv,
-                                   D ** -0.5, self.norm_eps)
+                                   self.k_scale, self.norm_eps, silu=self.silu)
+            if self.whole_norm:                     # the heads side by side as one
+                ops.gla_out_gate(o, proj[:, 2 * self.k_size + self.v_size:], self.norm_w, y, 1, self.v_size, self.norm_eps, sigmoid=self.sigmoid_gate)
         with profiling.label("o_proj", lambda: self.o.cost(T)):
             return self.o.forward(y)
 
