@@ -3,7 +3,7 @@ weights, synthetic token ids, on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--dtype bfloat16|float32] [--layers L]
                     [--config CONFIG.json|NAME]      another shape of the architecture (7b, 32b, a file)
-                    [--part all|decode|prefill|offline|mixed7b|preempt32b|modinex|lusolix|gaborax|luzevik|kasovik]
+                    [--part all|decode|prefill|offline|mixed7b|preempt32b|modinex|lusolix|gaborax|luzevik|kasovik|sanazen]
                     [--part decode --contexts 8192,32768 --batches 8,64]     decode steps over long contexts
 
 A "step" is one decode step of the engine (scheduling, metadata upload, the forward pass and greedy
@@ -19,6 +19,8 @@ of their operations has to move and do), not from formulas of one architecture.
                         (portions of prompts beside decoding requests, budget 2,048), up to 64 at a time
     --part preempt32b   the 32B shape, context 8,192: 64 prompts of 2,048 ids on 8,192 pages of 16, so
                         that growth during decoding evicts requests; reports evictions and tok/s
+    --part sanazen      the Sanazen design at two such sizes (sanazen-1k, sanazen-2k) beside the Gaborax and Kasovik models of those
+                        sizes (the closest designs: whole-projection norms and routed experts; mixers side by side with a retention)
     --part kasovik      the Kasovik design at two such sizes (kasovik-1k, kasovik-2k) beside the Luzevik and Modinex models of those
                         sizes (the closest designs: mixers side by side with a delta rule; a decayed linear recurrence)
     --part luzevik      the Luzevik design at two such sizes (luzevik-1k, luzevik-2k) beside the Lusolix models of those sizes (the
@@ -63,7 +65,7 @@ class _Matrices:
 
 # a design's comparison (--part <design>): the shipped shapes <design>-1k and <design>-2k, each beside these models of its size
 DESIGNS = {"modinex": ("qwen2-like",), "lusolix": ("qwen2-like",), "gaborax": ("qwen2-like",), "luzevik": ("lusolix", "qwen2-like"),
-           "kasovik": ("luzevik", "modinex")}
+           "kasovik": ("luzevik", "modinex"), "sanazen": ("gaborax", "kasovik")}
 
 
 def _linears(model):
@@ -111,7 +113,7 @@ def main() -> int:
                     help="captured shapes also try every algorithm the library holds, not only its heuristic's candidates")
     ap.add_argument("--skip-points", action="store_true", help="only the headline batch and the prefill")
     ap.add_argument("--skip-kernels", action="store_true", help="no per-operation kernel trace")
-    ap.add_argument("--part", default="all", choices=["all", "decode", "prefill", "offline", "mixed7b", "preempt32b", "modinex", "lusolix", "gaborax", "luzevik", "kasovik"],
+    ap.add_argument("--part", default="all", choices=["all", "decode", "prefill", "offline", "mixed7b", "preempt32b", "modinex", "lusolix", "gaborax", "luzevik", "kasovik", "sanazen"],
                     help="all: the headline line. decode / prefill: only that (for profiling one of them). offline: "
                          "--requests prompts of --offline-prompt tokens submitted at once. mixed7b / preempt32b: see above")
     ap.add_argument("--requests", type=int, default=None, help="requests of the offline, mixed7b and preempt32b parts")
