@@ -90,53 +90,44 @@ def test_scaled_and_capped_logits():
             assert head.emit(None, None) is None
 
 
-@pytest.mark.parametrize("dt", DTS)
-@pytest.mark.parametrize("T,N,extra", [(5, 72, 0), (3, 129, 4), (70, 2048, 8), (1, 20, 3)])
-def test_a_gate_per_channel(dt, T, N, extra):
-    from tokenmill_amd.hip import ops
-    torch.manual_seed(N)
-    x, g = q(torch.randn(T, N), dt), q(torch.randn(T, extra + N) * 4, dt)
-    g[0, extra], g[0, extra + 1] = 200.0, -200.0
-    got = ops.channel_gate(x.to(dt).to(DEV), g.to(dt).to(DEV)[:, extra:])
-    close(got.float().cpu(), q(x * torch.sigmoid(g[:, extra:]), dt), dt, "gated", bf16=2.0 ** -8)
-
-
 # ----------------------------------------------------------------------------------------------- window attention with kept tokens
 
 MASKS = [(6, 2, 64, 16, 40, 4, 150), (4, 1, 32, 16, 1, 33, 90), (8, 8, 128, 16, 100, 70, 330), (5, 1, 96, 32, 64, 1, 150), (3, 3, 20, 8, 9, 3, 60),
          (2, 1, 160, 16, 33, 17, 80), (4, 2, 64, 16, 300, 65, 700), (3, 1, 64, 16, 20, 0, 70), (2, 2, 32, 64, 24, 600, 640), (4, 4, 32, 16, 50, 257, 650)]
 
 
-def _every_kernel(qa, k_pool, v_pool, tab, n, H, G_, D, page, scale, window, keep, at):
+def _every_kernel(qa, k_pool, v_pool, tab, n, H, G_, D, page, scale, window, keep, at, gate=None):
     """The attention of positions ``at`` (a run up to n - 1) by every kernel that takes the sizes: name -> [len(at), H * D]."""
     from tokenmill_amd.hip import ops
     dt = qa.dtype
     m, places = len(at), ints(list(at))
     new = lambda rows=m: torch.full((rows, H * D), math.nan, dtype=dt, device=DEV)     # noqa: E731
     results, which = {}, {}
+    g = lambda rows=slice(None): gate[rows] if gate is not None else None     # noqa: E731
     out = new()
-    ops.attn_paged_softmax(qa[:m], out, k_pool, v_pool, tab, ints([0] * m), places, H, G_, D, D, scale, window, keep=keep)
+    ops.attn_paged_softmax(qa[:m], out, k_pool, v_pool, tab, ints([0] * m), places, H, G_, D, D, scale, window, keep=keep, channel_gate=g())
     results["a token and head alone"] = out
     some = sorted({0, m // 2, m - 1})
     out = new(len(some))
     ops.attn_paged_softmax(qa[:len(some)], out, k_pool, v_pool, tab, ints([0] * len(some)), places[some].contiguous(), H, G_, D, D, scale,
-                           window, keep=keep)
+                           window, keep=keep, channel_gate=g(some))
     results["few tokens, keys over wavefronts"] = out
     which["few tokens, keys over wavefronts"] = some
     tiles = torch.tensor([[0, i, min(16, m - i), at[i]] for i in range(0, m, 16)], dtype=torch.int32, device=DEV)
     if ops.attn_prefill_mfma_supported(dt, H, G_, D, page):
         for shared in (False, True):
             out = new()
-            ops.attn_prefill_mfma(qa[:m], out, k_pool, v_pool, tab, tiles, H, G_, D, scale, window, shared=shared, keep=keep)
+            ops.attn_prefill_mfma(qa[:m], out, k_pool, v_pool, tab, tiles, H, G_, D, scale, window, shared=shared, keep=keep, channel_gate=g())
             results[f"prompt tiles, shared keys {shared}"] = out
         tabs = tab.expand(m, -1).contiguous()
         for split in (False, True):
             out = new()
-            ops.attn_decode_mfma(qa[:m], out, k_pool, v_pool, tabs, ints([p + 1 for p in at]), H, G_, D, scale, window, n, split=split, keep=keep)
+            ops.attn_decode_mfma(qa[:m], out, k_pool, v_pool, tabs, ints([p + 1 for p in at]), H, G_, D, scale, window, n, split=split, keep=keep,
+                                 channel_gate=g())
             results[f"single tokens, split {split}"] = out
     if ops.attn_prefill_f32_supported(dt, H, G_, D, page):
         out = new()
-        ops.attn_prefill_f32(qa[:m], out, k_pool, v_pool, tab, tiles, H, G_, D, scale, window, keep=keep)
+        ops.attn_prefill_f32(qa[:m], out, k_pool, v_pool, tab, tiles, H, G_, D, scale, window, keep=keep, channel_gate=g())
         results["prompt tiles in 32-bit"] = out
     return {k: (v.float().cpu(), which.get(k, range(m))) for k, v in results.items()}
 
@@ -205,6 +196,28 @@ def test_far_keys_at_the_edges_of_what_is_kept(dt, D):
             if "few" in how:
                 continue                                   # (its rows of q are the first ones)
             close(got.view(-1, H, D), want[200:], dt, f"key {far}, {how}", bf16=2.0 ** -6)
+
+
+@pytest.mark.parametrize("dt", DTS)
+@pytest.mark.parametrize("H,G_,D", [(4, 2, 32), (6, 1, 64), (3, 3, 20), (2, 1, 128), (2, 2, 160)])
+def test_a_gate_per_channel_in_every_kernel(dt, H, G_, D):
+    """The gate's rows are a view into wider rows; wide open, shut, and in between."""
+    n, page, window, keep = 90, 16, 30, 3
+    g = torch.Generator().manual_seed(D)
+    k, v, qa = (q(torch.randn(n, h, D, generator=g), dt) for h in (G_, G_, H))
+    gate = q(torch.randn(n, 8 + H * D, generator=g) * 3, dt)
+    gate[5, 8:10], gate[6, 8:10] = 200.0, -200.0
+    pages = n // page + 1
+    pool = [torch.zeros((pages * page, G_, D), dtype=dt) for _ in range(2)]
+    pool[0][:n], pool[1][:n] = k.to(dt), v.to(dt)
+    k_pool = pool[0].view(pages, page, G_, D).to(DEV)
+    v_pool = pool[1].view(pages, page, G_, D).permute(0, 2, 3, 1).contiguous().to(DEV)
+    spread = lambda x: x.repeat_interleave(H // G_, 1)     # noqa: E731
+    want = P.kept_window_attention(qa, spread(k), spread(v), 0.2, window, keep).reshape(n, -1) * torch.sigmoid(gate[:, 8:])
+    for how, (got, which) in _every_kernel(qa.reshape(n, -1).to(dt).to(DEV), k_pool, v_pool, ints([list(range(pages))]), n, H, G_, D, page, 0.2, window,
+                                           keep, list(range(n)), gate.to(dt).to(DEV)[:, 8:]).items():
+        if "few" not in how:                               # (its rows of q are the first ones)
+            close(got, want, dt, how, bf16=2.0 ** -6)
 
 
 ATTENTIONS = [(6, 2, 20, 12, 4, 9, 3), (4, 2, 32, 32, 3, 24, 5), (8, 1, 64, 64, 2, 40, 18), (5, 1, 96, 96, 5, 1, 35), (2, 2, 128, 128, 4, 70, 1),

@@ -41,29 +41,31 @@ int tm_attn_paged_generic(const void* q, int q_stride, void* out, int out_stride
                           const int* positions, int T, int H, int KVH, int D, int page, float scale, int window,
                           int dtype, hipStream_t stream);
 
-// The same with keys and values of different sizes (D, DV), with a window the first `keep` keys of a request besides, scores capped smoothly at +-softcap (0: as they are) and a gate
+// The same with keys and values of different sizes (D, DV), scores capped smoothly at +-softcap (0: as they are) and a gate
 // per (token, head) (float32, rows ldg apart; null: none) whose sigmoid multiplies the head's result;
-// sink (float32 [H]; null: none): one more term exp(sink[h]) in the denominator of head h's softmax, with no key behind it.
+// sink (float32 [H]; null: none): one more term exp(sink[h]) in the denominator of head h's softmax, with no key behind it;
+// keep: with a window, the first keys of a request that every token sees beside it; cgate (the tensors' type, a row a token, ldcg
+// apart; null: none): a gate per channel of the result, likewise.
 int tm_attn_paged_generic_ext(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                               const int* block_tables, int table_width, const int* seq_of_token, const int* positions, int T, int H,
                               int KVH, int D, int DV, int page, float scale, int window, int keep, float softcap, const float* gate, int ldg,
-                              const float* sink, int dtype, hipStream_t stream);
+                              const float* sink, const void* cgate, int ldcg, int dtype, hipStream_t stream);
 
 // The matrix-unit attention kernels with capped scores (softcap > 0: s <- softcap * tanh(s / softcap); 0: as the plain entries)
-// and a sink per head (as above; null: none).
+// and a sink per head (as above; null: none), kept first keys and a gate per channel (as above).
 int tm_attn_prefill_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                              const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH, int D, int page,
-                             float scale, int window, int keep, float softcap, const float* sink, hipStream_t stream);
+                             float scale, int window, int keep, float softcap, const float* sink, const void* cgate, int ldcg, hipStream_t stream);
 int tm_attn_prefill_shared_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                                const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH, int D, int page,
-                               float scale, int window, int keep, float softcap, const float* sink, hipStream_t stream);
+                               float scale, int window, int keep, float softcap, const float* sink, const void* cgate, int ldcg, hipStream_t stream);
 int tm_attn_prefill_f32_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                             const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH, int D, int page,
-                            float scale, int window, int keep, float softcap, const float* sink, hipStream_t stream);
+                            float scale, int window, int keep, float softcap, const float* sink, const void* cgate, int ldcg, hipStream_t stream);
 int tm_attn_decode_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                             const int* block_tables, int table_width, const int* context_lens, float* part_o, float* part_ml,
                             int max_chunks, int S, int H, int KVH, int D, int page, float scale, int window, int keep, float softcap,
-                            const float* sink, hipStream_t stream);
+                            const float* sink, const void* cgate, int ldcg, hipStream_t stream);
 
 // The same work behind a short convolution over time (attention_prepare_conv.hip): see the head of that file.
 int tm_conv_norm_rope_store(const void* proj, int ld, int dtype, const void* conv_w, void* conv_state, int taps, const int* cu_q_lens,
@@ -71,8 +73,6 @@ int tm_conv_norm_rope_store(const void* proj, int ld, int dtype, const void* con
                             int G, int D, int Dv, int rot, int interleaved, const float* q_w, const float* k_w, float eps, int per_head,
                             const float* cos_t, const float* sin_t, const int* positions, const int* slots, void* k_pool, void* v_pool,
                             int page, hipStream_t stream);
-// x[t, c] *= sigmoid(gate[t * ldg + c]), gate of x's type
-int tm_channel_gate(void* x, int dtype, const void* gate, int ldg, int T, int N, hipStream_t stream);
 // q and k normed over the whole projection, rotated and stored (attention_prepare.hip): see the head of that file.
 int tm_whole_norm_rope_store(const float* proj, int ld, void* q_out, int dtype, int T, int H, int G, int D, int Dv, int rot,
                              int interleaved, const float* q_w, const float* k_w, float eps, const float* cos_t, const float* sin_t,

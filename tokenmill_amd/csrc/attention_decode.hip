@@ -221,7 +221,7 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_block_kernel(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
     const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ context_lens, int H, int KVH, int page_shift, float scale_log2, float cap_in, float cap_out,
-    int window, int keep, const float* __restrict__ sink) {
+    int window, int keep, const float* __restrict__ sink, const bf16_t* __restrict__ cgate, int ldcg) {
     constexpr int NDT = D / 16;
     __shared__ float s_m[WAVES][16], s_l[WAVES][16];
     __shared__ float s_o[WAVES][16][16 + 1];                         // one 16-wide d tile at a time
@@ -300,6 +300,13 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_block_kernel(
                 }
                 if (sink) lsum += __builtin_amdgcn_exp2f(sink[kvh * G + n] * 1.4426950408889634f - mx);     // a term of the denominator without a key
                 const float iv = 1.f / lsum;
+                if (cgate) {                                        // a gate per channel
+                    const uint2 gp = *(const uint2*)(cgate + (size_t)s * ldcg + (size_t)(kvh * G + n) * D + 16 * dt + d4);
+                    acc[0] *= sigmoid_fast(__uint_as_float(gp.x << 16));
+                    acc[1] *= sigmoid_fast(__uint_as_float(gp.x & 0xffff0000u));
+                    acc[2] *= sigmoid_fast(__uint_as_float(gp.y << 16));
+                    acc[3] *= sigmoid_fast(__uint_as_float(gp.y & 0xffff0000u));
+                }
                 uint2 pk;
                 pk.x = pack_bf16(acc[0] * iv, acc[1] * iv);
                 pk.y = pack_bf16(acc[2] * iv, acc[3] * iv);
@@ -386,7 +393,8 @@ __global__ __launch_bounds__(256) void attn_decode_split_kernel(
 #define AD_MERGE_WAVES 4
 __global__ __launch_bounds__(64 * AD_MERGE_WAVES) void attn_decode_merge_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, const int* __restrict__ context_lens,
-    bf16_t* __restrict__ out, int out_stride, int max_chunks, int H, int D, int window, int keep, const float* __restrict__ sink) {
+    bf16_t* __restrict__ out, int out_stride, int max_chunks, int H, int D, int window, int keep, const float* __restrict__ sink,
+    const bf16_t* __restrict__ cgate, int ldcg) {
     __shared__ float s_l[AD_MERGE_WAVES], s_o[AD_MERGE_WAVES][128];
     const int s = blockIdx.x, h = blockIdx.y;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / TM_WAVE), lane = threadIdx.x % TM_WAVE;
@@ -446,6 +454,11 @@ __global__ __launch_bounds__(64 * AD_MERGE_WAVES) void attn_decode_merge_kernel(
     }
     if (sink) ll += __builtin_amdgcn_exp2f(sink[h] * 1.4426950408889634f - mm);      // a term of the denominator without a key
     bf16_t* orow = out + (size_t)s * out_stride + (size_t)h * D;
+    if (cgate) {                                                    // a gate per channel
+        const bf16_t* gp = cgate + (size_t)s * ldcg + (size_t)h * D;
+        if (lane < D) o0 *= sigmoid_fast(bf16_to_f32(gp[lane]));
+        if (lane + 64 < D) o1 *= sigmoid_fast(bf16_to_f32(gp[lane + 64]));
+    }
     if (lane < D) orow[lane] = f32_to_bf16(o0 / ll);
     if (lane + 64 < D) orow[lane + 64] = f32_to_bf16(o1 / ll);
 }
@@ -454,7 +467,8 @@ __global__ __launch_bounds__(64 * AD_MERGE_WAVES) void attn_decode_merge_kernel(
 // their own, and wavefront w adds every fourth of those that count
 __global__ __launch_bounds__(64 * AD_MERGE_WAVES) void attn_decode_merge_long_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, const int* __restrict__ context_lens,
-    bf16_t* __restrict__ out, int out_stride, int max_chunks, int H, int D, int window, int keep, const float* __restrict__ sink) {
+    bf16_t* __restrict__ out, int out_stride, int max_chunks, int H, int D, int window, int keep, const float* __restrict__ sink,
+    const bf16_t* __restrict__ cgate, int ldcg) {
     __shared__ float s_m[AD_MERGE_WAVES], s_l[AD_MERGE_WAVES], s_o[AD_MERGE_WAVES][128];
     const int s = blockIdx.x, h = blockIdx.y;
     const int wave = threadIdx.x / TM_WAVE, lane = threadIdx.x % TM_WAVE;
@@ -505,6 +519,11 @@ __global__ __launch_bounds__(64 * AD_MERGE_WAVES) void attn_decode_merge_long_ke
     }
     if (sink) ll += __builtin_amdgcn_exp2f(sink[h] * 1.4426950408889634f - mm);      // a term of the denominator without a key
     bf16_t* orow = out + (size_t)s * out_stride + (size_t)h * D;
+    if (cgate) {                                                    // a gate per channel
+        const bf16_t* gp = cgate + (size_t)s * ldcg + (size_t)h * D;
+        if (lane < D) o0 *= sigmoid_fast(bf16_to_f32(gp[lane]));
+        if (lane + 64 < D) o1 *= sigmoid_fast(bf16_to_f32(gp[lane + 64]));
+    }
     if (lane < D) orow[lane] = f32_to_bf16(o0 / ll);
     if (two) orow[lane + 64] = f32_to_bf16(o1 / ll);
 }
@@ -513,7 +532,8 @@ template <int D>
 static int launch_decode(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                          const void* v_pool, const int* block_tables, int table_width, const int* context_lens,
                          float* part_o, float* part_ml, int max_chunks, int S, int H, int KVH, int page,
-                         float scale, int window, int keep, float softcap, const float* sink, hipStream_t stream) {
+                         float scale, int window, int keep, float softcap, const float* sink, const bf16_t* cgate, int ldcg,
+                         hipStream_t stream) {
     int page_shift = 0;
     while ((1 << page_shift) < page) ++page_shift;
     const float scale_log2 = scale * 1.4426950408889634f;
@@ -525,7 +545,8 @@ static int launch_decode(const void* q, int q_stride, void* out, int out_stride,
     if (!split) {
         attn_decode_block_kernel<D, WAVES><<<dim3(S, KVH), 64 * WAVES, 0, stream>>>(
             (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool,
-            block_tables, table_width, context_lens, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, keep, sink);
+            block_tables, table_width, context_lens, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, keep, sink,
+            cgate, ldcg);
         TM_CHECK_LAUNCH();
         return TM_OK;
     }
@@ -535,10 +556,10 @@ static int launch_decode(const void* q, int q_stride, void* out, int out_stride,
     TM_CHECK_LAUNCH();
     if (max_chunks <= TM_WAVE)
         attn_decode_merge_kernel<<<dim3(S, H), 64 * AD_MERGE_WAVES, 0, stream>>>(
-            part_o, part_ml, context_lens, (bf16_t*)out, out_stride, max_chunks, H, D, window, keep, sink);
+            part_o, part_ml, context_lens, (bf16_t*)out, out_stride, max_chunks, H, D, window, keep, sink, cgate, ldcg);
     else
         attn_decode_merge_long_kernel<<<dim3(S, H), 64 * AD_MERGE_WAVES, 0, stream>>>(
-            part_o, part_ml, context_lens, (bf16_t*)out, out_stride, max_chunks, H, D, window, keep, sink);
+            part_o, part_ml, context_lens, (bf16_t*)out, out_stride, max_chunks, H, D, window, keep, sink, cgate, ldcg);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
@@ -548,14 +569,16 @@ static int launch_decode(const void* q, int q_stride, void* out, int out_stride,
 // are scratch for the split kernels, which run when both are given (the caller gives them when the
 // (request, kv head) pairs alone are too few blocks for the chip); without them the block kernel runs.
 // softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax; sink (float32 [H]) or null: one more term
-// exp(sink[h]) in the denominator of head h's softmax, with no key behind it (added once, where a request's partials meet).
+// exp(sink[h]) in the denominator of head h's softmax, with no key behind it (added once, where a request's partials meet); with a window, `keep`: the first
+// keys of a request that every token sees beside its window; cgate (rows ldcg apart, a row a request) or null: channel c of the result is
+// multiplied by sigmoid(cgate[c]).
 extern "C" int tm_attn_decode_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                        const void* v_pool, const int* block_tables, int table_width,
                                        const int* context_lens, float* part_o, float* part_ml, int max_chunks, int S,
                                        int H, int KVH, int D, int page, float scale, int window, int keep, float softcap,
-                                       const float* sink, hipStream_t stream) {
+                                       const float* sink, const void* cgate, int ldcg, hipStream_t stream) {
     if (S <= 0) return TM_OK;
-    if (!(softcap >= 0.f) || keep < 0) return TM_ERR_ARG;
+    if (!(softcap >= 0.f) || keep < 0 || (cgate && (ldcg < H * D || ldcg % 4 || (uintptr_t)cgate % 8))) return TM_ERR_ARG;
     if (window == 0) keep = 0;
     if (H <= 0 || KVH <= 0 || H % KVH || H / KVH > 16 || page < 16 || (page & (page - 1)) || max_chunks <= 0 ||
         !(scale > 0.f) || max_chunks > 65535 || KVH > 65535 || window < 0 || table_width <= 0 || (q_stride % 8) ||
@@ -565,7 +588,7 @@ extern "C" int tm_attn_decode_mfma_cap(const void* q, int q_stride, void* out, i
     case DD:                                                                                                      \
         return launch_decode<DD>(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width,         \
                                  context_lens, part_o, part_ml, max_chunks, S, H, KVH, page, scale, window, keep, softcap, sink,  \
-                                 stream)
+                                 (const bf16_t*)cgate, ldcg, stream)
     switch (D) {
         TM_DECODE_CASE(32);
         TM_DECODE_CASE(64);
@@ -582,5 +605,5 @@ extern "C" int tm_attn_decode_mfma(const void* q, int q_stride, void* out, int o
                                    const int* context_lens, float* part_o, float* part_ml, int max_chunks, int S,
                                    int H, int KVH, int D, int page, float scale, int window, hipStream_t stream) {
     return tm_attn_decode_mfma_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, context_lens, part_o, part_ml,
-                                   max_chunks, S, H, KVH, D, page, scale, window, 0, 0.f, nullptr, stream);
+                                   max_chunks, S, H, KVH, D, page, scale, window, 0, 0.f, nullptr, nullptr, 0, stream);
 }

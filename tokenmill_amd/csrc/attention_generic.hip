@@ -56,7 +56,7 @@ __global__ __launch_bounds__((SPLIT ? AG_SPLIT_WAVES : AG_WAVES) * TM_WAVE) void
     const T* __restrict__ k_pool, const T* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ seq_of_token, const int* __restrict__ positions, int T_tokens,
     int H, int KVH, int D, int DV, int page, float scale, int window, int keep, float softcap, const float* __restrict__ gate, int ldg,
-    const float* __restrict__ sink) {
+    const float* __restrict__ sink, const T* __restrict__ cgate, int ldcg) {
     constexpr int WAVES = SPLIT ? AG_SPLIT_WAVES : AG_WAVES;
     constexpr bool STAGED = DMAX > 0 && sizeof(T) == 4;         // 32-bit keys through LDS (see the key loop)
     __shared__ __align__(16) float k_tile[STAGED ? WAVES : 1][STAGED ? TM_WAVE * AG_KSTRIDE : 4];
@@ -200,13 +200,16 @@ __global__ __launch_bounds__((SPLIT ? AG_SPLIT_WAVES : AG_WAVES) * TM_WAVE) void
     T* orow = out + (size_t)t * out_stride + (size_t)h * DV;
     // a gate per (token, head): the result times the sigmoid of the gate's 32-bit value, before its one rounding
     const float gated = gate ? 1.f / (1.f + expf(-gate[(size_t)t * ldg + h])) : 1.f;
+    // a gate per channel
+    const T* crow = cgate ? cgate + (size_t)t * ldcg + (size_t)h * DV : nullptr;
+    auto channel = [&](int d) { return crow ? 1.f / (1.f + expf(-Elem<T>::load(crow + d))) : 1.f; };
     if (!SPLIT) {
         if (sink) l += expf(sink[h] - m);                // a term of the denominator without a key
         const float inv = gated / l;
 #pragma unroll
         for (int i = 0; i < AG_MAXD / TM_WAVE; ++i) {
             const int d = lane + i * TM_WAVE;
-            if (d < DV) Elem<T>::store(orow + d, acc[i] * inv);
+            if (d < DV) Elem<T>::store(orow + d, acc[i] * inv * channel(d));
         }
         return;
     }
@@ -232,7 +235,7 @@ __global__ __launch_bounds__((SPLIT ? AG_SPLIT_WAVES : AG_WAVES) * TM_WAVE) void
         float oo = 0.f;
 #pragma unroll
         for (int ww = 0; ww < WAVES; ++ww) oo += (s_m[ww] == -INFINITY) ? 0.f : s_acc[ww][d] * expf(s_m[ww] - mm);
-        Elem<T>::store(orow + d, oo / ll * gated);
+        Elem<T>::store(orow + d, oo / ll * gated * channel(d));
     }
 }
 
@@ -240,27 +243,31 @@ template <typename T, int DMAX>
 static void launch_generic_d(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                              const void* v_pool, const int* block_tables, int table_width, const int* seq_of_token,
                              const int* positions, int T_tokens, int H, int KVH, int D, int DV, int page, float scale,
-                             int window, int keep, float softcap, const float* gate, int ldg, const float* sink, hipStream_t stream) {
+                             int window, int keep, float softcap, const float* gate, int ldg, const float* sink, const void* cgate, int ldcg,
+                           hipStream_t stream) {
     const long long pairs = (long long)T_tokens * H;
     if (pairs < 1024)           // too few (token, head) pairs to fill the chip: the wavefronts of a block split the keys
         attn_paged_generic_kernel<T, true, DMAX><<<(unsigned)pairs, AG_SPLIT_WAVES * TM_WAVE, 0, stream>>>(
             (const T*)q, q_stride, (T*)out, out_stride, (const T*)k_pool, (const T*)v_pool, block_tables,
-            table_width, seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink);
+            table_width, seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink,
+            (const T*)cgate, ldcg);
     else
         attn_paged_generic_kernel<T, false, DMAX><<<(unsigned)((pairs + AG_WAVES - 1) / AG_WAVES),
                                                     AG_WAVES * TM_WAVE, 0, stream>>>(
             (const T*)q, q_stride, (T*)out, out_stride, (const T*)k_pool, (const T*)v_pool, block_tables,
-            table_width, seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink);
+            table_width, seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink,
+            (const T*)cgate, ldcg);
 }
 
 template <typename T>
 static void launch_generic(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                            const void* v_pool, const int* block_tables, int table_width, const int* seq_of_token,
                            const int* positions, int T_tokens, int H, int KVH, int D, int DV, int page, float scale,
-                           int window, int keep, float softcap, const float* gate, int ldg, const float* sink, hipStream_t stream) {
+                           int window, int keep, float softcap, const float* gate, int ldg, const float* sink, const void* cgate, int ldcg,
+                           hipStream_t stream) {
 #define TM_GENERIC(DMAX)                                                                                       \
     launch_generic_d<T, DMAX>(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width,         \
-                              seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink, stream)
+                              seq_of_token, positions, T_tokens, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink, cgate, ldcg, stream)
     const int widest = D > DV ? D : DV;
     if (widest <= 64) TM_GENERIC(64);
     else if (widest <= 128) TM_GENERIC(128);
@@ -270,25 +277,26 @@ static void launch_generic(const void* q, int q_stride, void* out, int out_strid
 
 // D: size of a key, DV: of a value (the V pool is [pages, KVH, DV, page], out rows H * DV); softcap > 0: a score s becomes
 // softcap * tanh(s / softcap); with a window, `keep`: the first keys of a request that every token sees beside its window; gate (float32 [T, >= H], rows ldg apart) or null: head h of token t is multiplied by
-// sigmoid(gate[t][h]); sink (float32 [H]) or null: one more term exp(sink[h]) in the denominator of head h's softmax.
+// sigmoid(gate[t][h]); sink (float32 [H]) or null: one more term exp(sink[h]) in the denominator of head h's softmax; cgate (T's
+// type, rows ldcg apart) or null: channel c of token t is multiplied by sigmoid(cgate[t][c]).
 extern "C" int tm_attn_paged_generic_ext(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                          const void* v_pool, const int* block_tables, int table_width,
                                          const int* seq_of_token, const int* positions, int T, int H, int KVH, int D, int DV,
                                          int page, float scale, int window, int keep, float softcap, const float* gate, int ldg,
-                                         const float* sink, int dtype, hipStream_t stream) {
+                                         const float* sink, const void* cgate, int ldcg, int dtype, hipStream_t stream) {
     if (T <= 0) return TM_OK;
     if (H <= 0 || KVH <= 0 || H % KVH || D <= 0 || D > AG_MAXD || D % 4 || DV <= 0 || DV > AG_MAXD || page <= 0 ||
-        table_width <= 0 || window < 0 || keep < 0 || q_stride < H * D || out_stride < H * DV || !(softcap >= 0.f) || (gate && ldg < H))
+        table_width <= 0 || window < 0 || keep < 0 || q_stride < H * D || out_stride < H * DV || !(softcap >= 0.f) || (gate && ldg < H) || (cgate && ldcg < H * DV))
         return TM_ERR_ARG;
     if (((long long)T * H + AG_WAVES - 1) / AG_WAVES > 0x7fffffffLL) return TM_ERR_ARG;
     if (dtype == TM_F32) {
         if (((uintptr_t)k_pool % 16)) return TM_ERR_ARG;
         launch_generic<float>(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, seq_of_token,
-                              positions, T, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink, stream);
+                              positions, T, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink, cgate, ldcg, stream);
     } else if (dtype == TM_BF16) {
         if (((uintptr_t)k_pool % 8)) return TM_ERR_ARG;
         launch_generic<bf16_t>(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, seq_of_token,
-                               positions, T, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink, stream);
+                               positions, T, H, KVH, D, DV, page, scale, window, keep, softcap, gate, ldg, sink, cgate, ldcg, stream);
     } else {
         return TM_ERR_ARG;
     }
@@ -301,5 +309,5 @@ extern "C" int tm_attn_paged_generic(const void* q, int q_stride, void* out, int
                                      const int* seq_of_token, const int* positions, int T, int H, int KVH, int D,
                                      int page, float scale, int window, int dtype, hipStream_t stream) {
     return tm_attn_paged_generic_ext(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, seq_of_token,
-                                     positions, T, H, KVH, D, D, page, scale, window, 0, 0.f, nullptr, 0, nullptr, dtype, stream);
+                                     positions, T, H, KVH, D, D, page, scale, window, 0, 0.f, nullptr, 0, nullptr, nullptr, 0, dtype, stream);
 }

@@ -197,7 +197,8 @@ __global__ __launch_bounds__(64 * KS) void attn_prefill_mfma_kernel(
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
     const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ tiles, int n_tiles, int pair, int H, int KVH, int page_shift,
-    float scale_log2, float cap_in, float cap_out, int window, int keep, const float* __restrict__ sink) {
+    float scale_log2, float cap_in, float cap_out, int window, int keep, const float* __restrict__ sink,
+    const bf16_t* __restrict__ cgate, int ldcg) {
     constexpr int NDC = D / 32, NDT = D / 16;
     __shared__ float s_m[KS][16], s_l[KS][16];
     __shared__ float s_o[KS][16][D + 1];
@@ -283,6 +284,14 @@ __global__ __launch_bounds__(64 * KS) void attn_prefill_mfma_kernel(
             float lsum = st.l[hh];
             lsum += __shfl_xor(lsum, 16, TM_WAVE);
             lsum += __shfl_xor(lsum, 32, TM_WAVE);
+            // a gate per channel: this thread's pieces, on their way while the partials meet
+            constexpr int GP = (16 * (D / 2) + 64 * KS - 1) / (64 * KS);
+            uint32_t gv[GP];
+#pragma unroll
+            for (int u = 0; u < GP; ++u) {
+                const int idx = threadIdx.x + u * 64 * KS, col = idx / (D / 2) < valid ? idx / (D / 2) : valid - 1;
+                gv[u] = cgate ? *(const uint32_t*)(cgate + (size_t)(row0 + col) * ldcg + (size_t)(h0 + hh) * D + 2 * (idx % (D / 2))) : 0u;
+            }
             if (g == 0) {
                 s_m[wave][r] = st.m[hh];
                 s_l[wave][r] = lsum;
@@ -292,7 +301,9 @@ __global__ __launch_bounds__(64 * KS) void attn_prefill_mfma_kernel(
 #pragma unroll
                 for (int i = 0; i < 4; ++i) s_o[wave][r][16 * dt + 4 * g + i] = st.o[hh][dt][i];
             __syncthreads();
-            for (int idx = threadIdx.x; idx < 16 * (D / 2); idx += 64 * KS) {
+#pragma unroll
+            for (int u = 0; u < GP; ++u) {
+                const int idx = threadIdx.x + u * 64 * KS;
                 const int col = idx / (D / 2), d = 2 * (idx % (D / 2));
                 if (col >= valid) continue;
                 float mm = s_m[0][col];
@@ -308,6 +319,10 @@ __global__ __launch_bounds__(64 * KS) void attn_prefill_mfma_kernel(
                 }
                 if (sink) ll += __builtin_amdgcn_exp2f(sink[h0 + hh] * 1.4426950408889634f - mm);      // a term of the denominator without a key
                 const float inv = 1.f / ll;
+                if (cgate) {
+                    o0 *= sigmoid_fast(__uint_as_float(gv[u] << 16));
+                    o1 *= sigmoid_fast(__uint_as_float(gv[u] & 0xffff0000u));
+                }
                 *(uint32_t*)(out + (size_t)(row0 + col) * out_stride + (size_t)(h0 + hh) * D + d) = pk_bf16(o0 * inv, o1 * inv);
             }
             __syncthreads();
@@ -325,7 +340,7 @@ template <int D, int HPW>
 static void launch_split_keys(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                               const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH,
                               int page_shift, float scale_log2, float cap_in, float cap_out, int window, int keep, const float* sink,
-                              hipStream_t stream) {
+                              const bf16_t* cgate, int ldcg, hipStream_t stream) {
     constexpr int KS = PrefillShape<D>::KS;
     const int splits = (H / KVH + HPW - 1) / HPW;
     // fold the table in two once the folded launch still gives every CU a block
@@ -333,18 +348,19 @@ static void launch_split_keys(const void* q, int q_stride, void* out, int out_st
     dim3 grid(pair ? (n_tiles + 1) / 2 : n_tiles, KVH * splits);
     attn_prefill_mfma_kernel<D, HPW, KS><<<grid, 64 * KS, 0, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_tables,
-        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, keep, sink);
+        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, keep, sink, cgate, ldcg);
 }
 
 // softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax; sink (float32 [H]) or null: one more term
 // exp(sink[h]) in the denominator of head h's softmax, with no key behind it; with a window, `keep`: the first keys of a request that
-// every query sees beside its window
+// every query sees beside its window; cgate (rows of the flat batch, ldcg apart) or null: channel c of the result is multiplied by
+// sigmoid(cgate[c])
 extern "C" int tm_attn_prefill_mfma_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                         const void* v_pool, const int* block_tables, int table_width, const int* tiles,
                                         int n_tiles, int H, int KVH, int D, int page, float scale, int window, int keep, float softcap,
-                                        const float* sink, hipStream_t stream) {
+                                        const float* sink, const void* cgate, int ldcg, hipStream_t stream) {
     if (n_tiles <= 0) return TM_OK;
-    if (!(softcap >= 0.f) || keep < 0) return TM_ERR_ARG;
+    if (!(softcap >= 0.f) || keep < 0 || (cgate && (ldcg < H * D || ldcg % 2 || (uintptr_t)cgate % 4))) return TM_ERR_ARG;
     const float cap_in = softcap > 0.f ? scale / softcap : 0.f, cap_out = softcap > 0.f ? softcap / scale : 0.f;
     if (H <= 0 || KVH <= 0 || H % KVH || page < 16 || (page & (page - 1)) || window < 0 || table_width <= 0 ||
         (q_stride % 8) || ((uintptr_t)q % 16) || (out_stride % 2) || ((uintptr_t)out % 4) || q_stride < H * D ||
@@ -356,7 +372,7 @@ extern "C" int tm_attn_prefill_mfma_cap(const void* q, int q_stride, void* out, 
     const float scale_log2 = scale * 1.4426950408889634f;
     if ((long long)KVH * ((G + 1) / 2) > 65535) return TM_ERR_ARG;
 #define TM_SPLIT_ARGS q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, \
-                      page_shift, scale_log2, cap_in, cap_out, window, keep, sink, stream
+                      page_shift, scale_log2, cap_in, cap_out, window, keep, sink, (const bf16_t*)cgate, ldcg, stream
 #define TM_PREFILL_CASE(DD)                                                                                       \
     case DD: {                                                                                                    \
         constexpr int HPW = PrefillShape<DD>::HPW;                                                                \
@@ -385,5 +401,5 @@ extern "C" int tm_attn_prefill_mfma(const void* q, int q_stride, void* out, int 
                                     int n_tiles, int H, int KVH, int D, int page, float scale, int window,
                                     hipStream_t stream) {
     return tm_attn_prefill_mfma_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, D,
-                                    page, scale, window, 0, 0.f, nullptr, stream);
+                                    page, scale, window, 0, 0.f, nullptr, nullptr, 0, stream);
 }

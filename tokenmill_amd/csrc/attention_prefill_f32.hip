@@ -31,7 +31,7 @@ __global__ __launch_bounds__(64 * AF_SPLIT) void attn_prefill_f32_kernel(
     const float* __restrict__ q, int q_stride, float* __restrict__ out, int out_stride,
     const float* __restrict__ k_pool, const float* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ tiles, int H, int KVH, int page_shift, float scale, int window, int keep, float softcap,
-    const float* __restrict__ sink) {
+    const float* __restrict__ sink, const float* __restrict__ cgate, int ldcg) {
     constexpr int DQ = D / 4;           // values of a key (or query) a lane holds
     constexpr int NDT = D / 16;         // 16-row tiles of d
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / TM_WAVE);
@@ -169,6 +169,9 @@ __global__ __launch_bounds__(64 * AF_SPLIT) void attn_prefill_f32_kernel(
 #pragma unroll
                 for (int i = 0; i < 4; ++i) acc[i] += part[i] * sw[w];
             }
+            if (cgate)                                                  // a gate per channel
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc[i] *= 1.f / (1.f + expf(-cgate[(size_t)(row0 + tok) * ldcg + (size_t)h * D + d + i]));
             *(f32x4_t*)(orow + d) = f32x4_t{acc[0] * inv, acc[1] * inv, acc[2] * inv, acc[3] * inv};
         }
     }
@@ -179,13 +182,14 @@ __global__ __launch_bounds__(64 * AF_SPLIT) void attn_prefill_f32_kernel(
 // Needs D % 16 == 0 (at most 128), page a power of two >= 16, 16-byte aligned q, out and pools, strides % 4 == 0.
 // softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax; sink (float32 [H]) or null: one more term
 // exp(sink[h]) in the denominator of head h's softmax, with no key behind it; with a window, `keep`: the first keys of a request
-// that every token sees beside its window.
+// that every token sees beside its window; cgate (rows of the flat batch, ldcg apart) or null: channel c of the result is multiplied by
+// sigmoid(cgate[c]).
 extern "C" int tm_attn_prefill_f32_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                        const void* v_pool, const int* block_tables, int table_width, const int* tiles,
                                        int n_tiles, int H, int KVH, int D, int page, float scale, int window, int keep, float softcap,
-                                       const float* sink, hipStream_t stream) {
+                                       const float* sink, const void* cgate, int ldcg, hipStream_t stream) {
     if (n_tiles <= 0) return TM_OK;
-    if (!(softcap >= 0.f) || keep < 0) return TM_ERR_ARG;
+    if (!(softcap >= 0.f) || keep < 0 || (cgate && ldcg < H * D)) return TM_ERR_ARG;
     if (H <= 0 || KVH <= 0 || H % KVH || page < 16 || (page & (page - 1)) || window < 0 || table_width <= 0 ||
         (q_stride % 4) || (out_stride % 4) || ((uintptr_t)q % 16) || ((uintptr_t)out % 16) || ((uintptr_t)k_pool % 16) ||
         ((uintptr_t)v_pool % 16) || q_stride < H * D || out_stride < H * D || !(scale > 0.f))
@@ -198,7 +202,7 @@ extern "C" int tm_attn_prefill_f32_cap(const void* q, int q_stride, void* out, i
     case DD:                                                                                                      \
         attn_prefill_f32_kernel<DD><<<grid, 64 * AF_SPLIT, 0, stream>>>(                                          \
             (const float*)q, q_stride, (float*)out, out_stride, (const float*)k_pool, (const float*)v_pool,       \
-            block_tables, table_width, tiles, H, KVH, page_shift, scale, window, keep, softcap, sink);                     \
+            block_tables, table_width, tiles, H, KVH, page_shift, scale, window, keep, softcap, sink, (const float*)cgate, ldcg); \
         break
     switch (D) {
         TM_PREFILL_F32_CASE(16);
@@ -222,5 +226,5 @@ extern "C" int tm_attn_prefill_f32(const void* q, int q_stride, void* out, int o
                                    int n_tiles, int H, int KVH, int D, int page, float scale, int window,
                                    hipStream_t stream) {
     return tm_attn_prefill_f32_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, D,
-                                   page, scale, window, 0, 0.f, nullptr, stream);
+                                   page, scale, window, 0, 0.f, nullptr, nullptr, 0, stream);
 }

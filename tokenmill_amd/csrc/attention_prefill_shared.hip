@@ -227,7 +227,8 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
     const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
     const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool, const int* __restrict__ block_tables,
     int table_width, const int* __restrict__ tiles, int n_tiles, int pair, int H, int KVH, int page_shift,
-    float scale_log2, float cap_in, float cap_out, int window, int keep, const float* __restrict__ sink) {
+    float scale_log2, float cap_in, float cap_out, int window, int keep, const float* __restrict__ sink,
+    const bf16_t* __restrict__ cgate, int ldcg) {
     constexpr int NDC = D / 32, NDT = D / 16, THREADS = 64 * WAVES, STAGE = SharedShape<D>::STAGE, HPW = SharedPlan<D>::HPW;
     extern __shared__ __align__(16) unsigned char stages[];          // two stages
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / TM_WAVE);
@@ -315,6 +316,13 @@ __global__ __launch_bounds__(64 * WAVES, SharedPlan<D>::WAVES_PER_SIMD) void att
             bf16_t* orow = out + (size_t)(row0 + r) * out_stride + (size_t)(h0 + hh) * D + 4 * g;
 #pragma unroll
             for (int dt = 0; dt < NDT; ++dt) {
+                if (cgate) {                                         // a gate per channel
+                    const uint2 gp = *(const uint2*)(cgate + (size_t)(row0 + r) * ldcg + (size_t)(h0 + hh) * D + 4 * g + 16 * dt);
+                    st.o[hh][dt][0] *= sigmoid_fast(__uint_as_float(gp.x << 16));
+                    st.o[hh][dt][1] *= sigmoid_fast(__uint_as_float(gp.x & 0xffff0000u));
+                    st.o[hh][dt][2] *= sigmoid_fast(__uint_as_float(gp.y << 16));
+                    st.o[hh][dt][3] *= sigmoid_fast(__uint_as_float(gp.y & 0xffff0000u));
+                }
                 uint2 pk;
                 pk.x = pk_bf16(st.o[hh][dt][0] * inv, st.o[hh][dt][1] * inv);
                 pk.y = pk_bf16(st.o[hh][dt][2] * inv, st.o[hh][dt][3] * inv);
@@ -328,7 +336,7 @@ template <int D, int WAVES>
 static int launch_shared(const void* q, int q_stride, void* out, int out_stride, const void* k_pool, const void* v_pool,
                          const int* block_tables, int table_width, const int* tiles, int n_tiles, int H, int KVH,
                          int page_shift, float scale_log2, float cap_in, float cap_out, int window, int keep, const float* sink,
-                         hipStream_t stream) {
+                         const bf16_t* cgate, int ldcg, hipStream_t stream) {
     constexpr int lds = 2 * SharedShape<D>::STAGE;
     static bool raised = false;
     if (lds > 48 * 1024 && !raised) {
@@ -342,7 +350,7 @@ static int launch_shared(const void* q, int q_stride, void* out, int out_stride,
     dim3 grid(pair ? (n_tiles + 1) / 2 : n_tiles, KVH);
     attn_prefill_shared_kernel<D, WAVES><<<grid, 64 * WAVES, lds, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_tables,
-        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, keep, sink);
+        table_width, tiles, n_tiles, pair, H, KVH, page_shift, scale_log2, cap_in, cap_out, window, keep, sink, cgate, ldcg);
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
@@ -357,13 +365,14 @@ extern "C" int tm_attn_prefill_shared_takes(int H, int KVH, int D) {
 
 // softcap > 0: a score s (scaled) becomes softcap * tanh(s / softcap) before the softmax; sink (float32 [H]) or null: one more term
 // exp(sink[h]) in the denominator of head h's softmax, with no key behind it; with a window, `keep`: the first keys of a request that
-// every query sees beside its window
+// every query sees beside its window; cgate (rows of the flat batch, ldcg apart) or null: channel c of the result is multiplied by
+// sigmoid(cgate[c])
 extern "C" int tm_attn_prefill_shared_cap(const void* q, int q_stride, void* out, int out_stride, const void* k_pool,
                                           const void* v_pool, const int* block_tables, int table_width, const int* tiles,
                                           int n_tiles, int H, int KVH, int D, int page, float scale, int window, int keep, float softcap,
-                                          const float* sink, hipStream_t stream) {
+                                          const float* sink, const void* cgate, int ldcg, hipStream_t stream) {
     if (n_tiles <= 0) return TM_OK;
-    if (!(softcap >= 0.f) || keep < 0) return TM_ERR_ARG;
+    if (!(softcap >= 0.f) || keep < 0 || (cgate && (ldcg < H * D || ldcg % 4 || (uintptr_t)cgate % 8))) return TM_ERR_ARG;
     const float cap_in = softcap > 0.f ? scale / softcap : 0.f, cap_out = softcap > 0.f ? softcap / scale : 0.f;
     if (!tm_attn_prefill_shared_takes(H, KVH, D) || page < 16 || (page & (page - 1)) || window < 0 || table_width <= 0 ||
         (q_stride % 8) || ((uintptr_t)q % 16) || (out_stride % 4) || ((uintptr_t)out % 8) || q_stride < H * D ||
@@ -375,7 +384,7 @@ extern "C" int tm_attn_prefill_shared_cap(const void* q, int q_stride, void* out
     while ((1 << page_shift) < page) ++page_shift;
     const float scale_log2 = scale * 1.4426950408889634f;
 #define TM_SHARED_ARGS q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH, \
-                       page_shift, scale_log2, cap_in, cap_out, window, keep, sink, stream
+                       page_shift, scale_log2, cap_in, cap_out, window, keep, sink, (const bf16_t*)cgate, ldcg, stream
 #define TM_SHARED_CASE(DD)                                                          \
     case DD:                                                                        \
         if (need <= 2) return launch_shared<DD, 2>(TM_SHARED_ARGS);                 \
@@ -400,5 +409,5 @@ extern "C" int tm_attn_prefill_shared(const void* q, int q_stride, void* out, in
                                       int n_tiles, int H, int KVH, int D, int page, float scale, int window,
                                       hipStream_t stream) {
     return tm_attn_prefill_shared_cap(q, q_stride, out, out_stride, k_pool, v_pool, block_tables, table_width, tiles, n_tiles, H, KVH,
-                                      D, page, scale, window, 0, 0.f, nullptr, stream);
+                                      D, page, scale, window, 0, 0.f, nullptr, nullptr, 0, stream);
 }

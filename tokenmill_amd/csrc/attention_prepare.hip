@@ -228,48 +228,3 @@ extern "C" int tm_head_gate(void* x, int dtype, const float* gate, int ldg, int 
     TM_CHECK_LAUNCH();
     return TM_OK;
 }
-
-// x[t, c] *= sigmoid(gate[t * ldg + c]): a gate per channel of an attention's result, of the result's own type. Four channels a thread
-// where the rows allow it (VEC).
-template <typename T, int VEC>
-__global__ __launch_bounds__(256) void channel_gate_kernel(T* __restrict__ x, const T* __restrict__ gate, int ldg, int N) {
-    const int c = (blockIdx.x * 256 + threadIdx.x) * VEC;
-    if (c >= N) return;
-    T* xp = x + (size_t)blockIdx.y * N + c;
-    const T* gp = gate + (size_t)blockIdx.y * ldg + c;
-    T xv[VEC], gv[VEC];
-    if constexpr (VEC == 1) {
-        xv[0] = *xp;
-        gv[0] = *gp;
-    } else if constexpr (sizeof(T) == 4) {
-        *(uint4*)xv = *(const uint4*)xp;
-        *(uint4*)gv = *(const uint4*)gp;
-    } else {
-        *(uint2*)xv = *(const uint2*)xp;
-        *(uint2*)gv = *(const uint2*)gp;
-    }
-#pragma unroll
-    for (int e = 0; e < VEC; ++e) Elem<T>::store(&xv[e], Elem<T>::load(&xv[e]) * (1.f / (1.f + expf(-Elem<T>::load(&gv[e])))));
-    if constexpr (VEC == 1) *xp = xv[0];
-    else if constexpr (sizeof(T) == 4) *(uint4*)xp = *(const uint4*)xv;
-    else *(uint2*)xp = *(const uint2*)xv;
-}
-
-extern "C" int tm_channel_gate(void* x, int dtype, const void* gate, int ldg, int T, int N, hipStream_t stream) {
-    if (T <= 0) return TM_OK;
-    if (!x || !gate || N <= 0 || ldg < N || (dtype != TM_F32 && dtype != TM_BF16)) return TM_ERR_ARG;
-    const size_t e = dtype == TM_F32 ? 4 : 2;
-    const bool vec = N % 4 == 0 && ldg % 4 == 0 && (uintptr_t)x % (4 * e) == 0 && (uintptr_t)gate % (4 * e) == 0;
-    const int per = 256 * (vec ? 4 : 1);
-    for (int t0 = 0; t0 < T; t0 += 65535) {
-        const dim3 grid((N + per - 1) / per, T - t0 < 65535 ? T - t0 : 65535);
-        char* xp = (char*)x + (size_t)t0 * N * e;
-        const char* gp = (const char*)gate + (size_t)t0 * ldg * e;
-        if (dtype == TM_F32 && vec) channel_gate_kernel<float, 4><<<grid, 256, 0, stream>>>((float*)xp, (const float*)gp, ldg, N);
-        else if (dtype == TM_F32) channel_gate_kernel<float, 1><<<grid, 256, 0, stream>>>((float*)xp, (const float*)gp, ldg, N);
-        else if (vec) channel_gate_kernel<bf16_t, 4><<<grid, 256, 0, stream>>>((bf16_t*)xp, (const bf16_t*)gp, ldg, N);
-        else channel_gate_kernel<bf16_t, 1><<<grid, 256, 0, stream>>>((bf16_t*)xp, (const bf16_t*)gp, ldg, N);
-        TM_CHECK_LAUNCH();
-    }
-    return TM_OK;
-}

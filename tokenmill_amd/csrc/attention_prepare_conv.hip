@@ -6,14 +6,15 @@
 //   q and k of u normed over the whole projection (or head by head, `per_head`), the first `rot` channels of every head turned by
 //   the token's position, q to q_out, k and v to the token's cache slot: the operands and layouts of attention_prepare.hip
 //
-// Everything between the loads and the stores is 32-bit. A block a token; a token's sums have one order whatever else is in the
-// step. The rows from first_single on are the step's single tokens, one a request (request n_portions + row - first_single): a
+// Everything between the loads and the stores is 32-bit. A block a token, of more threads in a step of few tokens (a token's sums are
+// then ordered otherwise). The rows from first_single on are the step's single tokens, one a request (request n_portions + row - first_single): a
 // single token's block is the only one that touches its request's state, and moves it on itself. The state of the requests with
 // longer portions is moved on by tm_delta_conv_state afterwards (other blocks still read it here).
 #include "common.h"
 #include "api.h"
 
 #define CP_THREADS 256
+#define CP_WIDE 1024                    // threads of a token's block in a step of few tokens
 #define CP_MAX_TAPS 16
 #define CP_MAX_FLOATS (36 * 1024)       // q and k of a token in LDS, and a norm per head of theirs
 
@@ -78,15 +79,15 @@ __device__ __forceinline__ void cp_conv(const T* __restrict__ proj, int ld, cons
     }
 }
 
-template <typename T, int VEC, int TAPS>
-__global__ __launch_bounds__(CP_THREADS) void conv_norm_rope_store_kernel(
+template <typename T, int VEC, int TAPS, int NT>
+__global__ __launch_bounds__(NT) void conv_norm_rope_store_kernel(
     const T* __restrict__ proj, int ld, const T* __restrict__ conv_w, T* __restrict__ conv_state, int taps, const int* __restrict__ cu,
     const int* __restrict__ state_slots, const int* __restrict__ seq_of_token, int first_single, int n_portions, T* __restrict__ q_out, int H,
     int G, int D, int Dv, int rot, int interleaved, const float* __restrict__ q_w, const float* __restrict__ k_w, float eps, int per_head,
     const float* __restrict__ cos_t, const float* __restrict__ sin_t, const int* __restrict__ positions, const int* __restrict__ slots,
     T* __restrict__ k_pool, T* __restrict__ v_pool, int page) {
     extern __shared__ __align__(16) float lds[];
-    __shared__ float red[CP_THREADS / TM_WAVE];
+    __shared__ float red[NT / TM_WAVE];
     const int t = blockIdx.x, tid = threadIdx.x;
     const int Q = H * D, K = G * D, QK = Q + K, V = G * Dv, C = QK + V;
     float* xs = lds;                                // q and k behind the convolution
@@ -97,7 +98,7 @@ __global__ __launch_bounds__(CP_THREADS) void conv_norm_rope_store_kernel(
     T* st = conv_state + (size_t)state_slots[s] * (taps - 1) * C;
     const int slot = slots[t];
     float sq = 0.f, sk = 0.f;
-    for (int c = tid * VEC; c < QK; c += CP_THREADS * VEC) {        // (Q is a multiple of VEC: a piece is all of q or all of k)
+    for (int c = tid * VEC; c < QK; c += NT * VEC) {        // (Q is a multiple of VEC: a piece is all of q or all of k)
         float u[VEC];
         cp_conv<T, VEC, TAPS>(proj, ld, conv_w, st, C, taps, first, i, c, single, u);
         float ss = 0.f;
@@ -111,7 +112,7 @@ __global__ __launch_bounds__(CP_THREADS) void conv_norm_rope_store_kernel(
     }
     if (slot >= 0 || single) {
         const size_t vbase = slot >= 0 ? (size_t)(slot / page) * V * page + slot % page : 0;
-        for (int c = tid * VEC; c < V; c += CP_THREADS * VEC) {
+        for (int c = tid * VEC; c < V; c += NT * VEC) {
             float u[VEC];
             cp_conv<T, VEC, TAPS>(proj, ld, conv_w, st, C, taps, first, i, QK + c, single, u);
             if (slot >= 0)
@@ -124,15 +125,15 @@ __global__ __launch_bounds__(CP_THREADS) void conv_norm_rope_store_kernel(
     if (normed && per_head) {                       // a wavefront a head
         __syncthreads();
         const int wave = tid / TM_WAVE, lane = tid % TM_WAVE;
-        for (int hh = wave; hh < H + G; hh += CP_THREADS / TM_WAVE) {
+        for (int hh = wave; hh < H + G; hh += NT / TM_WAVE) {
             float ss = 0.f;
             for (int d = lane; d < D; d += TM_WAVE) ss += xs[hh * D + d] * xs[hh * D + d];
             ss = wave_sum(ss);
             if (lane == 0) inv_head[hh] = 1.0f / sqrtf(ss / (float)D + eps);
         }
     } else if (normed) {
-        rq = 1.0f / sqrtf(block_sum<CP_THREADS>(sq, red) / (float)Q + eps);
-        rk = 1.0f / sqrtf(block_sum<CP_THREADS>(sk, red) / (float)K + eps);
+        rq = 1.0f / sqrtf(block_sum<NT>(sq, red) / (float)Q + eps);
+        rk = 1.0f / sqrtf(block_sum<NT>(sk, red) / (float)K + eps);
     }
     __syncthreads();
     const int half = cos_t ? rot / 2 : 0;
@@ -154,7 +155,7 @@ __global__ __launch_bounds__(CP_THREADS) void conv_norm_rope_store_kernel(
         else if (ko) Elem<T>::store(ko + (c - Q), y);
     };
     if (half) {
-        for (int idx = tid; idx < (H + G) * half; idx += CP_THREADS) {
+        for (int idx = tid; idx < (H + G) * half; idx += NT) {
             const int hh = idx / half, j = idx % half;
             const int a = hh * D + (interleaved ? 2 * j : j), b = hh * D + (interleaved ? 2 * j + 1 : j + half);
             float y1, y2;
@@ -163,13 +164,13 @@ __global__ __launch_bounds__(CP_THREADS) void conv_norm_rope_store_kernel(
             put(b, y2);
         }
         const int rest = D - 2 * half;
-        for (int idx = tid; idx < (H + G) * rest; idx += CP_THREADS) {
+        for (int idx = tid; idx < (H + G) * rest; idx += NT) {
             const int c = idx / rest * D + 2 * half + idx % rest;
             put(c, value(c));
         }
         return;
     }
-    for (int c = tid * VEC; c < QK; c += CP_THREADS * VEC) {
+    for (int c = tid * VEC; c < QK; c += NT * VEC) {
         if (c >= Q && !ko) continue;
         Vec<T, VEC> y;
 #pragma unroll
@@ -195,14 +196,19 @@ extern "C" int tm_conv_norm_rope_store(const void* proj, int ld, int dtype, cons
     auto al = [&](const void* p) { return ((uintptr_t)p % b) == 0; };
     const bool vec = D % 4 == 0 && (G * Dv) % 4 == 0 && ld % 4 == 0 && al(proj) && al(conv_w) && al(conv_state) && al(q_out) && al(k_pool);
     const size_t bytes = (size_t)floats * sizeof(float);
-#define CP_GO(T_, V_, TAPS_)                                                                                                              \
+#define CP_RUN(T_, V_, TAPS_, NT_)                                                                                                            \
     do {                                                                                                                                  \
-        auto fn = conv_norm_rope_store_kernel<T_, V_, TAPS_>;                                                                             \
+        auto fn = conv_norm_rope_store_kernel<T_, V_, TAPS_, NT_>;                                                                         \
         if (bytes > 48 * 1024 && hipFuncSetAttribute((const void*)fn, hipFuncAttributeMaxDynamicSharedMemorySize, CP_MAX_FLOATS * 4) != hipSuccess) \
             return TM_ERR_LAUNCH;                                                                                                         \
-        fn<<<T, CP_THREADS, bytes, stream>>>((const T_*)proj, ld, (const T_*)conv_w, (T_*)conv_state, taps, cu_q_lens, state_slots,       \
+        fn<<<T, NT_, bytes, stream>>>((const T_*)proj, ld, (const T_*)conv_w, (T_*)conv_state, taps, cu_q_lens, state_slots,       \
                                              seq_of_token, first_single, n_portions, (T_*)q_out, H, G, D, Dv, rot, interleaved, q_w, k_w, \
                                              eps, per_head, cos_t, sin_t, positions, slots, (T_*)k_pool, (T_*)v_pool, page);              \
+    } while (0)
+#define CP_GO(T_, V_, TAPS_)                     \
+    do {                                         \
+        if (T < 256) CP_RUN(T_, V_, TAPS_, CP_WIDE); \
+        else CP_RUN(T_, V_, TAPS_, CP_THREADS);  \
     } while (0)
 #define CP_TAPS(T_)                                     \
     if (!vec) CP_GO(T_, 1, 0);                          \
@@ -216,6 +222,7 @@ extern "C" int tm_conv_norm_rope_store(const void* proj, int ld, int dtype, cons
     if (dtype == TM_F32) { CP_TAPS(float) } else { CP_TAPS(bf16_t) }
 #undef CP_TAPS
 #undef CP_GO
+#undef CP_RUN
     TM_CHECK_LAUNCH();
     return TM_OK;
 }

@@ -73,6 +73,9 @@ __device__ __forceinline__ void rotate_pair(float x1, float x2, float c, float s
     y2 = d + e;
 }
 
+// sigmoid from the hardware's exponential
+__device__ __forceinline__ float sigmoid_fast(float x) { return 1.0f / (1.0f + __expf(-x)); }
+
 // the clamped gated activation g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = up held to +-limit
 __device__ __forceinline__ float clamped_glu_f32(float g, float u, float alpha, float limit) {
     g = fminf(g, limit);

@@ -639,9 +639,10 @@ extern "C" int tm_scale_cap(float* x, long long n, float scale, float cap, hipSt
 
 // ------------------------------------------------------------------------------------------
 // out[t] = table[ids[t]] * scale + waves, waves[2 i] = sin(p f[i]), waves[2 i + 1] = cos(p f[i]) with p the token's position;
-// angles, sines and the sum in 32-bit. f holds ceil(hidden / 2) frequencies. A thread a pair.
+// angles, sines and the sum in 32-bit. f holds ceil(hidden / 2) frequencies. A thread has two pairs where the rows come in pieces of
+// four (WIDE), else one.
 // ------------------------------------------------------------------------------------------
-template <typename T>
+template <typename T, bool WIDE>
 __global__ __launch_bounds__(256) void embed_waves_kernel(const T* __restrict__ table, const int* __restrict__ ids,
                                                          const int* __restrict__ positions, const float* __restrict__ f,
                                                          float* __restrict__ out, int hidden, int vocab, float scale) {
@@ -651,7 +652,21 @@ __global__ __launch_bounds__(256) void embed_waves_kernel(const T* __restrict__ 
     const float p = (float)positions[t];
     const T* row = table + (size_t)id * hidden;
     float* o = out + (size_t)t * hidden;
-    for (int i = blockIdx.y * 256 + threadIdx.x; 2 * i < hidden; i += 256 * gridDim.y) {
+    if constexpr (WIDE) {
+        const int c = 4 * (blockIdx.y * 256 + threadIdx.x);
+        if (c >= hidden) return;
+        const float2 fr = *(const float2*)(f + c / 2);
+        T x[4];
+        if constexpr (sizeof(T) == 4) *(uint4*)x = *(const uint4*)(row + c);
+        else *(uint2*)x = *(const uint2*)(row + c);
+        float s0, c0, s1, c1;
+        sincosf(p * fr.x, &s0, &c0);
+        sincosf(p * fr.y, &s1, &c1);
+        *(float4*)(o + c) = float4{Elem<T>::load(x) * scale + s0, Elem<T>::load(x + 1) * scale + c0, Elem<T>::load(x + 2) * scale + s1,
+                                   Elem<T>::load(x + 3) * scale + c1};
+    } else {
+        const int i = blockIdx.y * 256 + threadIdx.x;
+        if (2 * i >= hidden) return;
         float s, c;
         sincosf(p * f[i], &s, &c);
         o[2 * i] = Elem<T>::load(row + 2 * i) * scale + s;
@@ -659,15 +674,24 @@ __global__ __launch_bounds__(256) void embed_waves_kernel(const T* __restrict__ 
     }
 }
 
+template <typename T>
+static void launch_embed_waves(const T* table, const int* ids, const int* positions, const float* f, float* out, int n, int hidden,
+                               int vocab, float scale, hipStream_t stream) {
+    const bool wide = hidden % 4 == 0 && (uintptr_t)table % (4 * sizeof(T)) == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)f % 8 == 0;
+    const int per = wide ? 1024 : 512;
+    const dim3 grid(n, (hidden + per - 1) / per);
+    if (wide) embed_waves_kernel<T, true><<<grid, 256, 0, stream>>>(table, ids, positions, f, out, hidden, vocab, scale);
+    else embed_waves_kernel<T, false><<<grid, 256, 0, stream>>>(table, ids, positions, f, out, hidden, vocab, scale);
+}
+
 extern "C" int tm_embed_waves(const void* table, int dtype, const int* ids, const int* positions, const float* f, float* out, int T,
                               int hidden, int vocab, float scale, hipStream_t stream) {
     if (T <= 0) return TM_OK;
-    if (!table || !ids || !positions || !f || !out || hidden <= 0 || vocab <= 0) return TM_ERR_ARG;
-    const dim3 grid(T, (hidden + 511) / 512 < 8 ? (hidden + 511) / 512 : 8);
+    if (!table || !ids || !positions || !f || !out || hidden <= 0 || hidden > 65535 * 512 || vocab <= 0) return TM_ERR_ARG;
     if (dtype == TM_F32)
-        embed_waves_kernel<float><<<grid, 256, 0, stream>>>((const float*)table, ids, positions, f, out, hidden, vocab, scale);
+        launch_embed_waves<float>((const float*)table, ids, positions, f, out, T, hidden, vocab, scale, stream);
     else if (dtype == TM_BF16)
-        embed_waves_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)table, ids, positions, f, out, hidden, vocab, scale);
+        launch_embed_waves<bf16_t>((const bf16_t*)table, ids, positions, f, out, T, hidden, vocab, scale, stream);
     else
         return TM_ERR_ARG;
     TM_CHECK_LAUNCH();

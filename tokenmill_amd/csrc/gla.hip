@@ -270,24 +270,74 @@ __global__ __launch_bounds__(TM_WAVE) void gla_out_gate_kernel(const float* __re
     }
 }
 
-// One wide head (a norm over all heads of a token at once): a block a token.
-template <typename T>
-__global__ __launch_bounds__(256) void gla_out_gate_wide_kernel(const float* __restrict__ o, const T* __restrict__ gate, int ldg,
-                                                               const float* __restrict__ w, T* __restrict__ y, int N, float eps,
-                                                               int sigmoid) {
-    __shared__ float red[256 / TM_WAVE];
+// One wide head (a norm over all heads of a token at once): a block a token. VEC 4: a thread's pieces of four channels of the result,
+// the gate and the weight are asked for at once and stay in registers (up to NT * 4 * GW_PIECES channels); VEC 1: any width, read twice.
+#define GW_PIECES 4
+template <typename T, int VEC, int NT>
+__global__ __launch_bounds__(NT) void gla_out_gate_wide_kernel(const float* __restrict__ o, const T* __restrict__ gate, int ldg,
+                                                              const float* __restrict__ w, T* __restrict__ y, int N, float eps,
+                                                              int sigmoid) {
+    __shared__ float red[NT / TM_WAVE];
     const int t = blockIdx.x;
     const float* orow = o + (size_t)t * N;
     const T* grow = gate + (size_t)t * ldg;
     T* yrow = y + (size_t)t * N;
     float ss = 0.f;
-    for (int e = threadIdx.x; e < N; e += 256) ss += orow[e] * orow[e];
-    const float r = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)N + eps);
-    for (int e = threadIdx.x; e < N; e += 256) {
-        const float g = Elem<T>::load(grow + e);
-        const float v = w ? w[e] * (orow[e] * r) : orow[e] * r;
-        Elem<T>::store(yrow + e, v * ((sigmoid ? 1.f : g) / (1.f + expf(-g))));
+    if constexpr (VEC == 4) {
+        float4 ov[GW_PIECES], wv[GW_PIECES];
+        T gv[GW_PIECES][4];
+#pragma unroll
+        for (int i = 0; i < GW_PIECES; ++i) {
+            const int e = 4 * (threadIdx.x + i * NT);
+            ov[i] = wv[i] = float4{0.f, 0.f, 0.f, 0.f};
+            if (e < N) {
+                ov[i] = *(const float4*)(orow + e);
+                wv[i] = w ? *(const float4*)(w + e) : float4{1.f, 1.f, 1.f, 1.f};
+                if constexpr (sizeof(T) == 4) *(uint4*)gv[i] = *(const uint4*)(grow + e);
+                else *(uint2*)gv[i] = *(const uint2*)(grow + e);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < GW_PIECES; ++i) ss += ov[i].x * ov[i].x + ov[i].y * ov[i].y + ov[i].z * ov[i].z + ov[i].w * ov[i].w;
+        const float r = 1.0f / sqrtf(block_sum<NT>(ss, red) / (float)N + eps);
+#pragma unroll
+        for (int i = 0; i < GW_PIECES; ++i) {
+            const int e = 4 * (threadIdx.x + i * NT);
+            if (e >= N) continue;
+            const float* op = &ov[i].x;
+            const float* wp = &wv[i].x;
+            T out[4];
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+                const float g = Elem<T>::load(&gv[i][k]);
+                Elem<T>::store(&out[k], wp[k] * (op[k] * r) * ((sigmoid ? 1.f : g) / (1.f + expf(-g))));
+            }
+            if constexpr (sizeof(T) == 4) *(uint4*)(yrow + e) = *(const uint4*)out;
+            else *(uint2*)(yrow + e) = *(const uint2*)out;
+        }
+    } else {
+        for (int e = threadIdx.x; e < N; e += NT) ss += orow[e] * orow[e];
+        const float r = 1.0f / sqrtf(block_sum<NT>(ss, red) / (float)N + eps);
+        for (int e = threadIdx.x; e < N; e += NT) {
+            const float g = Elem<T>::load(grow + e);
+            const float v = w ? w[e] * (orow[e] * r) : orow[e] * r;
+            Elem<T>::store(yrow + e, v * ((sigmoid ? 1.f : g) / (1.f + expf(-g))));
+        }
     }
+}
+
+template <typename T>
+static void launch_out_gate_wide(const float* o, const T* gate, int ldg, const float* w, T* y, int n, int N, float eps, int sigmoid,
+                                 hipStream_t stream) {
+    const size_t b = 4 * sizeof(T);
+    const bool vec = N % 4 == 0 && ldg % 4 == 0 && (uintptr_t)o % 16 == 0 && (uintptr_t)gate % b == 0 && (uintptr_t)y % b == 0 &&
+                     (uintptr_t)w % 16 == 0;
+    if (vec && N <= 256 * 4 * GW_PIECES)
+        gla_out_gate_wide_kernel<T, 4, 256><<<n, 256, 0, stream>>>(o, gate, ldg, w, y, N, eps, sigmoid);
+    else if (vec && N <= 1024 * 4 * GW_PIECES)
+        gla_out_gate_wide_kernel<T, 4, 1024><<<n, 1024, 0, stream>>>(o, gate, ldg, w, y, N, eps, sigmoid);
+    else
+        gla_out_gate_wide_kernel<T, 1, 256><<<n, 256, 0, stream>>>(o, gate, ldg, w, y, N, eps, sigmoid);
 }
 
 extern "C" int tm_gla_out_gate(const float* o, const void* gate, int ldg, int dtype, const float* w, void* y, int T, int H, int Dv,
@@ -296,9 +346,9 @@ extern "C" int tm_gla_out_gate(const float* o, const void* gate, int ldg, int dt
     if (H <= 0 || H > 65535 || Dv <= 0 || ldg < H * Dv || !o || !gate || !y || !(eps > 0.f)) return TM_ERR_ARG;
     if (H == 1 && Dv > 4 * TM_WAVE && (dtype == TM_F32 || dtype == TM_BF16)) {
         if (dtype == TM_F32)
-            gla_out_gate_wide_kernel<float><<<T, 256, 0, stream>>>(o, (const float*)gate, ldg, w, (float*)y, Dv, eps, sigmoid);
+            launch_out_gate_wide<float>(o, (const float*)gate, ldg, w, (float*)y, T, Dv, eps, sigmoid, stream);
         else
-            gla_out_gate_wide_kernel<bf16_t><<<T, 256, 0, stream>>>(o, (const bf16_t*)gate, ldg, w, (bf16_t*)y, Dv, eps, sigmoid);
+            launch_out_gate_wide<bf16_t>(o, (const bf16_t*)gate, ldg, w, (bf16_t*)y, T, Dv, eps, sigmoid, stream);
         TM_CHECK_LAUNCH();
         return TM_OK;
     }

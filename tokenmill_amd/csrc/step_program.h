@@ -7,7 +7,7 @@
 
 #include "api.h"
 
-#define TM_MAX_GROUPS 8
+#define TM_MAX_GROUPS 32
 
 extern "C" {
 

@@ -354,22 +354,25 @@ struct Run {
             const bool head_mfma = a.D == 32 || a.D == 64 || a.D == 96 || a.D == 128;
             const bool q_ok = aligned(q, 16) && q_stride % 8 == 0;
             bool done_prefill = false, done_decode = false;
+            const void* cg = cgate_in;      // a gate per channel, applied where a kernel stores its result
+            const void* cg_dec = cg ? (const char*)cg + (size_t)tp * cgate_ld * es : nullptr;
+            cgate_in = nullptr;
             if (tp && s->n_tiles > 0 && s->prefill_tiles && dtype == TM_BF16 && head_mfma && page_ok && q_ok) {
                 if (tm_prefill_shares_keys(a.D, a.H, a.KVH, s->n_tiles) && tm_attn_prefill_shared_takes(a.H, a.KVH, a.D) &&
                     HD % 4 == 0 && aligned(attn, 8)) {
                     ++p->taken[TM_PREFILL_SHARED_KEYS];
                     rc = tm_attn_prefill_shared_cap(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->prefill_tiles,
-                                                    s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.keep, a.softcap, a.sink, stream);
+                                                    s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.keep, a.softcap, a.sink, cg, cgate_ld, stream);
                 } else {
                     ++p->taken[TM_PREFILL_SPLIT_KEYS];
                     rc = tm_attn_prefill_mfma_cap(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->prefill_tiles,
-                                                  s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.keep, a.softcap, a.sink, stream);
+                                                  s->n_tiles, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.keep, a.softcap, a.sink, cg, cgate_ld, stream);
                 }
                 done_prefill = true;
             } else if (tp && s->n_tiles > 0 && s->prefill_tiles && dtype == TM_F32 && a.D % 16 == 0 && a.D >= 16 &&
                        a.D <= 128 && page_ok && q_stride % 4 == 0 && aligned(q, 16)) {
                 rc = tm_attn_prefill_f32_cap(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->prefill_tiles, s->n_tiles, a.H,
-                                             a.KVH, a.D, a.page, a.scale, a.window, a.keep, a.softcap, a.sink, stream);
+                                             a.KVH, a.D, a.page, a.scale, a.window, a.keep, a.softcap, a.sink, cg, cgate_ld, stream);
                 done_prefill = true;
             }
             if (rc) return rc;
@@ -380,28 +383,25 @@ struct Run {
                 rc = tm_attn_decode_mfma_cap(q_dec, q_stride, out_dec, HD, a.k_pool, a.v_pool, tables + (size_t)(S - nd) * W, W,
                                              s->context_lens + (S - nd), split ? part_o : nullptr, split ? part_ml : nullptr,
                                              tm_decode_chunks(s->max_decode_context), nd, a.H, a.KVH, a.D, a.page, a.scale, a.window, a.keep,
-                                             a.softcap, a.sink, stream);
+                                             a.softcap, a.sink, cg_dec, cgate_ld, stream);
                 done_decode = true;
             }
             if (rc) return rc;
             if (tp && !done_prefill && nd && !done_decode) {
                 rc = tm_attn_paged_generic_ext(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->seq_of_token, s->positions, T,
-                                               a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.keep, a.softcap, nullptr, 0, a.sink, dtype, stream);
+                                               a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.keep, a.softcap, nullptr, 0, a.sink, cg, cgate_ld, dtype,
+                                               stream);
             } else {
                 if (tp && !done_prefill)
                     rc = tm_attn_paged_generic_ext(q, q_stride, attn, HD, a.k_pool, a.v_pool, tables, W, s->seq_of_token, s->positions,
-                                                   tp, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.keep, a.softcap, nullptr, 0, a.sink, dtype, stream);
+                                                   tp, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.keep, a.softcap, nullptr, 0, a.sink, cg, cgate_ld, dtype,
+                                               stream);
                 if (!rc && nd && !done_decode)
                     rc = tm_attn_paged_generic_ext(q_dec, q_stride, out_dec, HD, a.k_pool, a.v_pool, tables, W, s->seq_of_token + tp,
                                                    s->positions + tp, nd, a.H, a.KVH, a.D, a.D, a.page, a.scale, a.window, a.keep, a.softcap, nullptr, 0, a.sink,
-                                                   dtype, stream);
+                                                   cg_dec, cgate_ld, dtype, stream);
             }
             if (rc) return rc;
-            if (cgate_in) {                 // a gate per channel on the way to the output projection
-                rc = tm_channel_gate(attn, dtype, cgate_in, cgate_ld, T, HD, stream);
-                cgate_in = nullptr;
-                if (rc) return rc;
-            }
             if (gate_in) {                  // a gate per (token, head) on the way to the output projection
                 rc = tm_head_gate(attn, dtype, gate_in, gate_ld, T, a.H, a.D, stream);
                 gate_in = nullptr;

@@ -7,7 +7,7 @@ from ctypes import CFUNCTYPE, POINTER, Structure, c_char_p, c_float, c_int, c_si
 
 from tokenmill_amd.hip.library import library
 
-MAX_GROUPS = 8
+MAX_GROUPS = 32
 
 
 class TmTune(Structure):

@@ -596,6 +596,16 @@ def _gemm_skinny_packed(a, w: PackedWeight, bias, out, silu: bool, accum) -> tor
     return accum if accum is not None else out
 
 
+def _channel_gate(gate: torch.Tensor | None, T: int, N: int, dtype) -> tuple[torch.Tensor | None, int]:
+    """A gate per channel of an attention's result as the kernels take it: (tensor, elements between its rows)."""
+    if gate is None:
+        return None, 0
+    _gpu(gate)
+    _need(gate.dtype == dtype and gate.dim() == 2 and gate.shape[0] == T and gate.shape[1] >= N and gate.stride(1) == 1,
+          f"attention: a gate per channel is {dtype} [{T}, >= {N}] with unit inner stride")
+    return gate, (gate.stride(0) if T > 1 else max(gate.stride(0), N))
+
+
 def attn_decode_mfma_supported(dtype, H: int, KVH: int, D: int, page: int) -> bool:
     return (dtype == torch.bfloat16 and D in (32, 64, 96, 128) and page >= 16 and page & (page - 1) == 0
             and H % KVH == 0 and H // KVH <= 16)
@@ -604,10 +614,12 @@ def attn_decode_mfma_supported(dtype, H: int, KVH: int, D: int, page: int) -> bo
 def attn_decode_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                      block_tables: torch.Tensor, context_lens: torch.Tensor, H: int, KVH: int, D: int, scale: float,
                      window: int, max_context: int, workspace: tuple[torch.Tensor, torch.Tensor] | None = None,
-                     split: bool | None = None, softcap: float = 0.0, sink: torch.Tensor | None = None, keep: int = 0):
+                     split: bool | None = None, softcap: float = 0.0, sink: torch.Tensor | None = None, keep: int = 0,
+                     channel_gate: torch.Tensor | None = None):
     """Attention of one new token per request over its cache (the token's own key included); ``softcap`` > 0: a scaled
     score s becomes softcap * tanh(s / softcap); ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator;
-    ``keep``: with a window, the first keys of a request that every token sees beside it.
+    ``keep``: with a window, the first keys of a request that every token sees beside it; ``channel_gate`` (a view [S, >= H*D] of q's
+    type): channel c of the result is multiplied by sigmoid of it.
     q: [S, >= H*D] rows (unit inner stride), out [S, H*D] view; block_tables int32 [S, W];
     context_lens int32 [S] (new token counted); max_context >= every context length. ``split``: None runs
     the kernel the library's rule names for this many requests (contexts split over blocks and merged, or one
@@ -615,6 +627,7 @@ def attn_decode_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v
     _gpu(q, out, k_pool, v_pool, block_tables, context_lens, sink)
     _check_sink(sink, H)
     S = q.shape[0]
+    cgate, ldcg = _channel_gate(channel_gate, S, H * D, q.dtype)
     page = _check_pools(k_pool, v_pool, KVH, D, torch.bfloat16, "attn_decode")
     _need(attn_decode_mfma_supported(q.dtype, H, KVH, D, page), "attn_decode: unsupported head size, group or page size")
     _need(q.stride(1) == 1 and out.stride(1) == 1 and out.dtype == torch.bfloat16 and out.shape[0] == S
@@ -644,7 +657,7 @@ def attn_decode_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v
     _check(library().tm_attn_decode_mfma_cap(_p(q), c_int(q_stride), _p(out), c_int(out_stride), _p(k_pool), _p(v_pool),
                                              _p(block_tables), c_int(W), _p(context_lens), _p(part_o), _p(part_ml),
                                              c_int(chunks), c_int(S), c_int(H), c_int(KVH), c_int(D), c_int(page),
-                                             c_float(scale), c_int(window), c_int(keep), c_float(softcap), _p(sink), _stream()), "attn_decode_mfma")
+                                             c_float(scale), c_int(window), c_int(keep), c_float(softcap), _p(sink), _p(cgate), c_int(ldcg), _stream()), "attn_decode_mfma")
     return out
 
 
@@ -659,10 +672,11 @@ def attn_prefill_mfma_supported(dtype, H: int, KVH: int, D: int, page: int) -> b
 def attn_prefill_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                       block_tables: torch.Tensor, tiles: torch.Tensor, H: int, KVH: int, D: int, scale: float,
                       window: int, shared: bool = False, softcap: float = 0.0, sink: torch.Tensor | None = None,
-                      keep: int = 0) -> torch.Tensor:
+                      keep: int = 0, channel_gate: torch.Tensor | None = None) -> torch.Tensor:
     """Attention of prompt portions over the cache (``softcap`` > 0: a scaled score s becomes softcap * tanh(s / softcap);
     ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator; ``keep``: with a window, the first keys of a request
-    that every token sees beside it). q: [T, >= H*D] rows, out [T, H*D]; tiles int32
+    that every token sees beside it; ``channel_gate`` (a view [T, >= H*D] of q's type): channel c of the result is multiplied by
+    sigmoid of it). q: [T, >= H*D] rows, out [T, H*D]; tiles int32
     [n, 4] = (request index, first row, tokens (1..16), position of the first token) cover the rows
     to compute; every row of a tile belongs to one request at consecutive positions. ``shared``: the kernel
     that stages a tile's keys and values through LDS for all heads of a kv head, instead of the one whose
@@ -670,6 +684,7 @@ def attn_prefill_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, 
     _gpu(q, out, k_pool, v_pool, block_tables, tiles, sink)
     _check_sink(sink, H)
     T = q.shape[0]
+    cgate, ldcg = _channel_gate(channel_gate, T, H * D, q.dtype)
     page = _check_pools(k_pool, v_pool, KVH, D, torch.bfloat16, "attn_prefill")
     _need(attn_prefill_mfma_supported(q.dtype, H, KVH, D, page), "attn_prefill: unsupported head size or page size")
     _need(q.stride(1) == 1 and out.stride(1) == 1 and out.dtype == torch.bfloat16 and out.shape[0] == T
@@ -690,7 +705,7 @@ def attn_prefill_mfma(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, 
     _check(entry(_p(q), c_int(q_stride), _p(out), c_int(out_stride), _p(k_pool), _p(v_pool),
                  _p(block_tables), c_int(block_tables.shape[1]), _p(tiles),
                  c_int(tiles.shape[0]), c_int(H), c_int(KVH), c_int(D), c_int(page),
-                 c_float(scale), c_int(window), c_int(keep), c_float(softcap), _p(sink), _stream()), "attn_prefill_shared" if shared else "attn_prefill_mfma")
+                 c_float(scale), c_int(window), c_int(keep), c_float(softcap), _p(sink), _p(cgate), c_int(ldcg), _stream()), "attn_prefill_shared" if shared else "attn_prefill_mfma")
     return out
 
 
@@ -701,12 +716,14 @@ def attn_prefill_f32_supported(dtype, H: int, KVH: int, D: int, page: int) -> bo
 
 def attn_prefill_f32(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                      block_tables: torch.Tensor, tiles: torch.Tensor, H: int, KVH: int, D: int, scale: float,
-                     window: int, softcap: float = 0.0, sink: torch.Tensor | None = None, keep: int = 0) -> torch.Tensor:
+                     window: int, softcap: float = 0.0, sink: torch.Tensor | None = None, keep: int = 0,
+                     channel_gate: torch.Tensor | None = None) -> torch.Tensor:
     """Attention of prompt portions over the cache in true 32-bit (32-bit MFMA). Operands as for
     ``attn_prefill_mfma``, all float32."""
     _gpu(q, out, k_pool, v_pool, block_tables, tiles, sink)
     _check_sink(sink, H)
     T = q.shape[0]
+    cgate, ldcg = _channel_gate(channel_gate, T, H * D, q.dtype)
     page = _check_pools(k_pool, v_pool, KVH, D, torch.float32, "attn_prefill_f32")
     _need(attn_prefill_f32_supported(q.dtype, H, KVH, D, page), "attn_prefill_f32: unsupported head size or page size")
     _need(q.stride(1) == 1 and out.stride(1) == 1 and out.dtype == torch.float32 and out.shape[0] == T
@@ -722,7 +739,7 @@ def attn_prefill_f32(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v
     _check(library().tm_attn_prefill_f32_cap(_p(q), c_int(q_stride), _p(out), c_int(out_stride), _p(k_pool), _p(v_pool),
                                              _p(block_tables), c_int(block_tables.shape[1]), _p(tiles),
                                              c_int(tiles.shape[0]), c_int(H), c_int(KVH), c_int(D), c_int(page),
-                                             c_float(scale), c_int(window), c_int(keep), c_float(softcap), _p(sink), _stream()), "attn_prefill_f32")
+                                             c_float(scale), c_int(window), c_int(keep), c_float(softcap), _p(sink), _p(cgate), c_int(ldcg), _stream()), "attn_prefill_f32")
     return out
 
 
@@ -1757,15 +1774,17 @@ def whole_norm_rope_store(proj: torch.Tensor, q_out: torch.Tensor, H: int, G: in
 def attn_paged_softmax(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, block_tables: torch.Tensor,
                        seq_of_token: torch.Tensor, positions: torch.Tensor, H: int, G: int, D: int, Dv: int, scale: float,
                        window: int = 0, softcap: float = 0.0, gate: torch.Tensor | None = None,
-                       sink: torch.Tensor | None = None, keep: int = 0) -> torch.Tensor:
+                       sink: torch.Tensor | None = None, keep: int = 0, channel_gate: torch.Tensor | None = None) -> torch.Tensor:
     """Softmax attention of every token of the step over its request's cached keys (its own included), a token and a head a
     wavefront: keys of D channels, values of Dv; a score s becomes softcap * tanh(s / softcap) if ``softcap`` > 0; head h of
     token t is multiplied by sigmoid(gate[t, h]) (gate: a float32 view [T, >= H] with unit inner stride; None: no gate);
     ``sink`` (float32 [H]): one more term exp(sink[h]) in the denominator; ``keep``: with a window, the first keys of a request
-    that every token sees beside it. q [T, >= H*D] with unit inner stride, out [T, H*Dv]."""
+    that every token sees beside it; ``channel_gate`` (a view [T, >= H*Dv] of q's type): channel c of the result is multiplied by
+    sigmoid of it. q [T, >= H*D] with unit inner stride, out [T, H*Dv]."""
     _gpu(q, out, k_pool, v_pool, block_tables, seq_of_token, positions, gate, sink)
     _check_sink(sink, H)
     T = q.shape[0]
+    cgate, ldcg = _channel_gate(channel_gate, T, H * Dv, q.dtype)
     _need(q.stride(1) == 1 and q.shape[1] >= H * D and out.is_contiguous() and tuple(out.shape) == (T, H * Dv),
           f"attention: q [T, >={H * D}] unit inner stride, out contiguous [T, {H * Dv}]")
     _need(q.dtype == out.dtype, "attention: q and out share one type")
@@ -1785,7 +1804,8 @@ def attn_paged_softmax(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor,
     _check(library().tm_attn_paged_generic_ext(_p(q), c_int(q_stride), _p(out), c_int(H * Dv), _p(k_pool), _p(v_pool), _p(block_tables),
                                                c_int(block_tables.shape[1]), _p(seq_of_token), _p(positions), c_int(T), c_int(H),
                                                c_int(G), c_int(D), c_int(Dv), c_int(page), c_float(scale), c_int(window),
-                                               c_int(keep), c_float(softcap), _p(gate), c_int(ldg), _p(sink), code(q.dtype), _stream()), "attn_paged_generic_ext")
+                                               c_int(keep), c_float(softcap), _p(gate), c_int(ldg), _p(sink), _p(cgate), c_int(ldcg), code(q.dtype), _stream()),
+           "attn_paged_generic_ext")
     return out
 
 
@@ -1842,17 +1862,6 @@ def conv_norm_rope_store(proj: torch.Tensor, conv_w: torch.Tensor, conv_state: t
     if conv_state is not None and portions:
         delta_conv_state(proj, C, conv_state, cu_q_lens, state_slots, portions)
     return q_out
-
-
-def channel_gate(x: torch.Tensor, gate: torch.Tensor) -> torch.Tensor:
-    """x[t, c] *= sigmoid(gate[t, c]) in place: x contiguous [T, N], gate a view [T, >= N] of x's type with unit inner stride."""
-    _gpu(x, gate)
-    T, N = x.shape
-    _need(x.is_contiguous() and gate.dim() == 2 and gate.shape[0] == T and gate.shape[1] >= N and gate.stride(1) == 1 and gate.dtype == x.dtype,
-          f"channel_gate: gate is [{T}, >= {N}] of x's type")
-    _check(library().tm_channel_gate(_p(x), c_int(code(x.dtype)), _p(gate), c_int(gate.stride(0) if T > 1 else max(gate.stride(0), N)),
-                                     c_int(T), c_int(N), _stream()), "channel_gate")
-    return x
 
 
 def scale_cap(x: torch.Tensor, scale: float, cap: float = 0.0) -> torch.Tensor:

@@ -222,9 +222,7 @@ class SoftmaxAttention(Mixer):
                 return program.run_one(op, step, qkv=q, gate=gate, channel_gate=cgate)
         out = torch.empty((T, H * Dv), dtype=x.dtype, device=x.device)
         with profiling.label("attention", lambda: self.cost("attention", step, T)):
-            self._attend(q, out, gate, step, cache, group)
-            if cgate is not None:
-                ops.channel_gate(out, cgate)
+            self._attend(q, out, gate, cgate, step, cache, group)
         with profiling.label("o_proj", lambda: self.o.cost(T)):
             return self.o.forward(out)
 
@@ -238,8 +236,8 @@ class SoftmaxAttention(Mixer):
         entry = self._own[key]
         return entry[:2] if entry is not None else None
 
-    def _attend(self, q, out, gate, step: StepContext, cache: KVCacheView, group) -> None:
+    def _attend(self, q, out, gate, cgate, step: StepContext, cache: KVCacheView, group) -> None:
         """Keys and values of different sizes: a token and a head a wavefront."""
         H, G, D, Dv = self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim
         ops.attn_paged_softmax(q, out, cache.k, cache.v, group.block_tables, step.seq_of_token, step.positions, H, G, D, Dv,
-                               self.scale, self.window or 0, self.softcap, gate, sink=self.sink, keep=self.keep_first)
+                               self.scale, self.window or 0, self.softcap, gate, sink=self.sink, keep=self.keep_first, channel_gate=cgate)
